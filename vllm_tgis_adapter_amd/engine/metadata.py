@@ -8,7 +8,7 @@ decode kernel over the rest without re-gathering.
 
 from __future__ import annotations
 
-from dataclasses import dataclass
+from dataclasses import dataclass, field
 from typing import Optional
 
 import torch
@@ -41,6 +41,10 @@ class AttnMetadata:
     seq_start_loc: Optional[torch.Tensor] = None   # [ns+1] int32 device
     seq_lens: Optional[torch.Tensor] = None        # [ns] int32 device
     state_slots: Optional[torch.Tensor] = None     # [ns] int32 device
+
+    # Values one layer computes and later layers of the same step read again
+    # (rotation tables); dropped with the step.
+    step_values: dict = field(default_factory=dict)
 
     @property
     def num_tokens(self) -> int:

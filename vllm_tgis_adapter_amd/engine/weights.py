@@ -66,3 +66,19 @@ def load_safetensors_weights(path: str) -> dict[str, torch.Tensor]:
             weights.update(torch.load(os.path.join(path, fn), map_location="cpu", weights_only=True))
         return weights
     raise FileNotFoundError(f"No safetensors/bin weights under {path}")
+
+
+def safetensors_shapes(path: str) -> dict[str, tuple]:
+    """Names and shapes of the tensors in a model dir's safetensors files, from
+    their headers alone; empty when the dir has none."""
+    from safetensors import safe_open
+
+    shapes: dict[str, tuple] = {}
+    if not os.path.isdir(path):
+        return shapes
+    for fn in sorted(os.listdir(path)):
+        if fn.endswith(".safetensors"):
+            with safe_open(os.path.join(path, fn), framework="pt") as f:
+                for name in f.keys():
+                    shapes[name] = tuple(f.get_slice(name).get_shape())
+    return shapes

@@ -34,6 +34,10 @@ def get_model(cfg: ModelConfig):
         from .gumozen import GumozenForCausalLM
 
         return GumozenForCausalLM(cfg)
+    if cfg.architecture == "balenex":
+        from .balenex import BalenexForCausalLM
+
+        return BalenexForCausalLM(cfg)
     raise ValueError(f"Unsupported architecture: {cfg.architecture}")
 
 
@@ -55,4 +59,8 @@ def native_extensions(cfg: ModelConfig) -> list[str]:
         from .gumozen import native_extensions as gz
 
         return gz(cfg)
+    if cfg.architecture == "balenex":
+        from .balenex import native_extensions as bx
+
+        return bx(cfg)
     return ["_C"]

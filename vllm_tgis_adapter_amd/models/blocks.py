@@ -48,6 +48,16 @@ that another design can assemble them differently:
 - ``stepped_rotary_frequencies``  rotation frequencies divided by a factor
                         for long wavelengths, kept for short ones, blended
                         linearly in between
+- ``SpanAttention``     grouped-query attention over a sliding window plus a
+                        prefix (the sequence's first tokens, or pooled blocks
+                        of older tokens); optional biases, short convolution,
+                        query/key norm with or without weights, rotation of
+                        queries and keys, rotated values turned back at the
+                        output
+- ``GLAMixer``          gated linear attention: a matrix state per head with a
+                        data-dependent decay per key channel from a low-rank
+                        projection
+- ``BiasedGatedMLP``    down(silu(gate h + b) * (up h + b)) + b
 
 The recurrent mixers keep their state (f32) and the last inputs of their short
 convolutions in per-sequence slots; a sequence that starts in a step starts
@@ -661,25 +671,37 @@ class MLSTMMixer(_Mixer):
 
 class ParallelMixer(nn.Module):
     """Two mixers fed one input through a single merged projection; result =
-    left_scale * left + right_scale * right.  Returns the two outputs
-    and their scales; the caller's residual kernel forms the sum in f32."""
+    left_scale * left + right_scale * right.  Returns the two outputs; the
+    caller's residual kernel forms the sum in f32 with the scales, after an RMS
+    norm of each output over the width when ``out_norms`` gives them weights.
+    ``row_multiple``: the merged product gets zero rows up to a multiple of
+    that many."""
 
     def __init__(self, width: int, left: _Mixer, right: _Mixer, left_scale: float,
-                 right_scale: float, dtype: torch.dtype):
+                 right_scale: float, dtype: torch.dtype, out_norms: bool = False,
+                 row_multiple: int = 1):
         super().__init__()
         if left.has_in_bias or right.has_in_bias:
             raise ValueError("merged projection of mixers with input bias is not supported")
         self.left, self.right = left, right
         self.left_scale, self.right_scale = left_scale, right_scale
-        self.in_weight = _randn_param((left.in_rows + right.in_rows, width), dtype)
+        rows = left.in_rows + right.in_rows
+        self.in_weight = _randn_param((rows + -rows % row_multiple, width), dtype)
+        self.left_norm = _f32_param(width, fill=1.0) if out_norms else None
+        self.right_norm = _f32_param(width, fill=1.0) if out_norms else None
 
     def load(self, left_tensors: dict, right_tensors: dict) -> None:
         n = self.left.in_rows
+        m = n + self.right.in_rows
+        self.in_weight.data[m:].zero_()
         for mod, rows, t in ((self.left, self.in_weight.data[:n], left_tensors),
-                             (self.right, self.in_weight.data[n:], right_tensors)):
+                             (self.right, self.in_weight.data[n:m], right_tensors)):
             mod.load_in(rows, None, t)
             mod.o_weight.data.copy_(t["o"].to(mod.dtype))
             mod.load_rest(t)
+        if self.left_norm is not None:
+            self.left_norm.data.copy_(left_tensors["out"].float())
+            self.right_norm.data.copy_(right_tensors["out"].float())
 
     def cache_shapes(self, block_size: int) -> list:
         return self.left.cache_shapes(block_size) + self.right.cache_shapes(block_size)
@@ -690,8 +712,8 @@ class ParallelMixer(nn.Module):
         nl = len(self.left.cache_shapes(1))
         a = ops.linear(self.left.mix(proj[:, :n], positions, cache[:nl], meta),
                        self.left.o_weight)
-        b = ops.linear(self.right.mix(proj[:, n:], positions, cache[nl:], meta),
-                       self.right.o_weight)
+        b = ops.linear(self.right.mix(proj[:, n:n + self.right.in_rows], positions, cache[nl:],
+                                      meta), self.right.o_weight)
         return a, b
 
 
@@ -1138,3 +1160,225 @@ class GatedRoutedExperts(nn.Module):
         a = ops.moe_gemm(xs, self.gate_up, seg, gated=True)
         ye = ops.moe_gemm(a, self.down, seg, gated=False)
         return ops.moe_combine(ye, pos, ids, torch.ones_like(w), ne)
+
+
+# ---------------------------------------------------------------------------
+# Attention over a window plus a prefix with everything that may happen to its
+# inputs in one pass, gated linear attention, biased gated feed-forward.
+# ---------------------------------------------------------------------------
+
+
+class SpanAttention(_Mixer):
+    """Causal grouped-query softmax attention in which a query at position i
+    sees the last ``window`` tokens (0: all) and, in the same softmax, either
+    the first ``keep_first`` tokens of the sequence (at their true positions)
+    or, with ``pool`` > 0, the mean key and mean value of every block of
+    ``pool`` positions that ends at or before i - window.
+
+    Projected rows: [q | k | v], plus ``qkv_bias``.  In order: a short causal
+    convolution over time per channel (``taps`` > 0), RMS norm of every query
+    and key head over dim (with a weight shared by the heads when
+    ``norm_weights``), rotation of the first ``rot_dims`` dims of queries and
+    keys (dim i with i + rot_dims/2).  ``rotate_values``: the value of position
+    j is turned by j's angles over all of vdim and cached so; the output of
+    position i is turned back by i's angles.  score = q . k * scale.
+    ``o_bias``: the output projection's bias, left to the caller's residual
+    kernel.
+
+    Cache: keys and values per token; with ``pool`` also the pooled keys and
+    values, block b in the cache block that holds its last token; with a
+    convolution the last taps-1 projected rows per sequence."""
+
+    def __init__(self, width: int, *, heads: int, kv_heads: int, dim: int, vdim: int,
+                 scale: float, eps: float, window: int = 0, keep_first: int = 0,
+                 pool: int = 0, taps: int = 0, norm_weights: bool = True,
+                 rot_base: float = 10000.0, rot_dims: int = 0, rotate_values: bool = False,
+                 qkv_bias: bool = True, o_bias: bool = False, own_in: bool = True,
+                 dtype: torch.dtype = torch.bfloat16):
+        super().__init__()
+        if heads % kv_heads:
+            raise ValueError("heads must be a multiple of kv_heads")
+        if rot_dims % 2 or rot_dims > dim or (rotate_values and vdim % 2):
+            raise ValueError("rotated dims must be even and at most the head size")
+        if min(window, keep_first, pool, taps) < 0 or (keep_first and pool):
+            raise ValueError("the prefix is either kept first tokens or pooled blocks")
+        if pool and not window:
+            raise ValueError("pooled blocks need a window")
+        self.heads, self.kv_heads, self.dim, self.vdim = heads, kv_heads, dim, vdim
+        self.scale, self.eps = scale, eps
+        self.window, self.keep_first, self.pool, self.taps = window, keep_first, pool, taps
+        self.rot_base, self.rot_dims, self.rotate_values = rot_base, rot_dims, rotate_values
+        self.channels = heads * dim + kv_heads * (dim + vdim)
+        self.in_rows = self.channels
+        self.out_rows = heads * vdim
+        self._alloc(width, own_in, dtype)
+        self.qkv_bias = _f32_param(self.channels) if qkv_bias else None
+        self.o_bias = _f32_param(width) if o_bias else None
+        self.q_norm = _f32_param(dim, fill=1.0) if norm_weights else None
+        self.k_norm = _f32_param(dim, fill=1.0) if norm_weights else None
+        # stored [taps, channels]: a thread's neighbouring channels are contiguous
+        self.conv_weight = None
+        if taps:
+            w = torch.empty(taps, self.channels, dtype=torch.float32).normal_(0.0, 0.2)
+            w[-1] += 0.7
+            self.conv_weight = nn.Parameter(w, requires_grad=False)
+        for name, dims in (("inv_freq", rot_dims), ("v_inv_freq", vdim if rotate_values else 0)):
+            freqs, _ = scaled_rotary_frequencies(rot_base, max(dims, 2))
+            self.register_buffer(name, torch.tensor(freqs, dtype=torch.float64).to(torch.float32),
+                                 persistent=False)
+
+    def load_in(self, weight, bias, t) -> None:
+        off = 0
+        for name in ("q", "k", "v"):
+            n = t[name].shape[0]
+            weight[off:off + n].copy_(t[name].to(weight.dtype))
+            if self.qkv_bias is not None:
+                self.qkv_bias.data[off:off + n].copy_(t[name + ".b"].float())
+            if self.conv_weight is not None:
+                self.conv_weight.data[:, off:off + n].copy_(t[name + ".conv"].float().T)
+            off += n
+        if off != self.in_rows:
+            raise ValueError("projection tensors do not add up to the mixer's rows")
+
+    def load_rest(self, t) -> None:
+        if self.q_norm is not None:
+            self.q_norm.data.copy_(t["q.norm"].float())
+            self.k_norm.data.copy_(t["k.norm"].float())
+        if self.o_bias is not None:
+            self.o_bias.data.copy_(t["o.b"].float())
+
+    def cache_shapes(self, block_size: int) -> list:
+        ng, d, dv = self.kv_heads, self.dim, self.vdim
+        out = [("paged", (block_size, ng, d), self.dtype),
+               ("paged", (block_size, ng, dv), self.dtype)]
+        if self.pool:
+            n = ops.pool_slots_per_block(block_size, self.pool)
+            out += [("paged", (n, ng, d), self.dtype), ("paged", (n, ng, dv), self.dtype)]
+        if self.taps:
+            out.append(("slot", (max(self.taps - 1, 0), self.channels), self.dtype))
+        return out
+
+    def _table(self, positions, inv_freq, dims: int, meta: AttnMetadata):
+        if not dims:
+            return None
+        key = ("rotary", self.rot_base, dims)
+        if key not in meta.step_values:
+            meta.step_values[key] = ops.rotary_table(positions, inv_freq)
+        return meta.step_values[key]
+
+    def mix(self, proj, positions, cache, meta: AttnMetadata) -> torch.Tensor:
+        t, nh, dv = proj.shape[0], self.heads, self.vdim
+        k_cache, v_cache = cache[0], cache[1]
+        k_pool, v_pool = (cache[2], cache[3]) if self.pool else (None, None)
+        table = self._table(positions, self.inv_freq, self.rot_dims, meta)
+        v_table = self._table(positions, self.v_inv_freq, dv if self.rotate_values else 0, meta)
+        npt = meta.num_prefill_tokens
+        q = ops.attn_inputs_cache_write(
+            proj, self.qkv_bias, nh, self.kv_heads, self.dim, dv, self.eps, self.q_norm,
+            self.k_norm, self.conv_weight, cache[-1] if self.taps else None, table, v_table,
+            k_cache, v_cache, meta.slot_mapping, meta.seq_start_loc, meta.seq_lens,
+            meta.state_slots, has_portions=npt > 0)
+        out = torch.empty((t, nh, dv), dtype=proj.dtype, device=proj.device)
+        back = lambda rows: None if v_table is None else v_table[rows]
+        if npt:
+            if self.pool:
+                ops.pool_cache_write(k_cache, v_cache, k_pool, v_pool, self.pool,
+                                     meta.prefill_block_tables, meta.prefill_query_start_loc,
+                                     meta.prefill_seq_lens)
+            ops.span_attention_prefill(
+                q[:npt], k_cache, v_cache, k_pool, v_pool, meta.prefill_block_tables,
+                meta.prefill_query_start_loc, meta.prefill_seq_lens, self.scale,
+                meta.max_prefill_query_len, self.window, self.keep_first, self.pool,
+                back(slice(0, npt)), out=out[:npt])
+        if meta.num_decode_seqs:
+            if self.pool:
+                ops.pool_cache_write(k_cache, v_cache, k_pool, v_pool, self.pool,
+                                     meta.decode_block_tables, None, meta.decode_seq_lens)
+            ops.span_attention_decode(
+                q[npt:], k_cache, v_cache, k_pool, v_pool, meta.decode_block_tables,
+                meta.decode_seq_lens, self.scale, self.window, self.keep_first, self.pool,
+                back(slice(npt, t)), out=out[npt:])
+        return out.view(t, nh * dv)
+
+
+class GLAMixer(_Mixer):
+    """Gated linear attention.  q = W_q h / sqrt(dim), k, v per head; decay per
+    key channel alpha = sigmoid(W_a2 (W_a1 h) + b)^(1/tau); S_t = diag(alpha_t)
+    S_(t-1) + k_t v_t^T, o_t = S_t^T q_t; each head's o is RMS-normed over vdim
+    with one weight for all heads, times silu(W_g h).  Projected rows: [q | k |
+    v | g | a1]; the second, low-rank product of the decay runs in f32 with the
+    scan's gates."""
+
+    def __init__(self, width: int, *, heads: int, dim: int, vdim: int, rank: int, tau: float,
+                 eps: float, own_in: bool = True, dtype: torch.dtype = torch.bfloat16):
+        super().__init__()
+        self.heads, self.dim, self.vdim, self.rank = heads, dim, vdim, rank
+        self.tau, self.eps = tau, eps
+        self.in_rows = 2 * heads * dim + 2 * heads * vdim + rank
+        self.out_rows = heads * vdim
+        self._alloc(width, own_in, dtype)
+        # stored [rank, channels]: a channel's products read neighbouring columns
+        self.a2_t = nn.Parameter(
+            torch.empty(rank, heads * dim, dtype=torch.float32).normal_(0.0, rank ** -0.5),
+            requires_grad=False)
+        self.a2_bias = _f32_param(heads * dim)
+        self.norm = _f32_param(heads * vdim, fill=1.0)   # the head weight, repeated
+
+    def load_in(self, weight, bias, t) -> None:
+        off = 0
+        for name in ("q", "k", "v", "g", "a1"):
+            n = t[name].shape[0]
+            weight[off:off + n].copy_(t[name].to(weight.dtype))
+            off += n
+        if off != self.in_rows:
+            raise ValueError("projection tensors do not add up to the mixer's rows")
+
+    def load_rest(self, t) -> None:
+        self.a2_t.data.copy_(t["a2"].float().T)
+        self.a2_bias.data.copy_(t["a2.b"].float())
+        self.norm.data.copy_(t["norm"].float().repeat(self.heads))
+
+    def cache_shapes(self, block_size: int) -> list:
+        return [("slot", (self.heads, self.vdim, self.dim), torch.float32)]
+
+    def mix(self, proj, positions, cache, meta: AttnMetadata) -> torch.Tensor:
+        t, nh, d, dv = proj.shape[0], self.heads, self.dim, self.vdim
+        a = nh * d
+        b = 2 * a + nh * dv
+        c = b + nh * dv
+        o = ops.gla_scan(
+            proj[:, :a].view(t, nh, d), proj[:, a:2 * a].view(t, nh, d),
+            proj[:, 2 * a:b].view(t, nh, dv), proj[:, c:c + self.rank], self.a2_t,
+            self.a2_bias, 1.0 / self.tau, d ** -0.5, cache[0], meta.seq_start_loc,
+            meta.seq_lens, meta.state_slots)
+        return ops.gated_group_norm(o, proj[:, b:c], self.norm, nh, self.eps,
+                                    gate_first=False, out_dtype=self.dtype, silu_after=True)
+
+
+class BiasedGatedMLP(nn.Module):
+    """down(silu(gate h + b) * (up h + b)); gate and up are one merged product.
+    The down-projection's bias ``down_bias`` is left to the caller's residual
+    kernel."""
+
+    def __init__(self, width: int, ff: int, dtype: torch.dtype):
+        super().__init__()
+        if get_tp_world_size() != 1:
+            raise ValueError("BiasedGatedMLP is not sharded; run it with one rank")
+        self.ff = ff
+        self.gate_up = _randn_param((2 * ff, width), dtype, std=width ** -0.5)
+        self.gate_up_bias = _f32_param(2 * ff)
+        self.down = _randn_param((width, ff), dtype, std=ff ** -0.5)
+        self.down_bias = _f32_param(width)
+
+    def load(self, t: dict) -> None:
+        ff = self.ff
+        for i, name in enumerate(("gate", "up")):
+            rows = slice(i * ff, (i + 1) * ff)
+            self.gate_up.data[rows].copy_(t[name].to(self.gate_up.dtype))
+            self.gate_up_bias.data[rows].copy_(t[name + ".b"].float())
+        self.down.data.copy_(t["down"].to(self.down.dtype))
+        self.down_bias.data.copy_(t["down.b"].float())
+
+    def forward(self, h: torch.Tensor) -> torch.Tensor:
+        return ops.linear(ops.silu_mul_bias(ops.linear(h, self.gate_up), self.gate_up_bias),
+                          self.down)

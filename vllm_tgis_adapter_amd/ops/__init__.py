@@ -891,16 +891,19 @@ def ssd_scan(xbc, dt, dt_bias, a_log, d_skip, state, seq_start_loc, seq_lens,
 
 
 def gated_group_norm(y, gate, weight, groups: int, eps: float, gate_first: bool,
-                     out_dtype: torch.dtype) -> torch.Tensor:
+                     out_dtype: torch.dtype, silu_after: bool = False) -> torch.Tensor:
     """RMS norm of y [T, C] (f32) in ``groups`` equal parts, times weight, with
-    a gate [T, C]: silu(gate) multiplied in before the norm (gate_first) or
-    sigmoid(gate) after it."""
+    a gate [T, C]: silu(gate) multiplied in before the norm (gate_first), or
+    sigmoid(gate) (``silu_after``: silu(gate)) after it."""
+    if gate_first and silu_after:
+        raise ValueError("the gate comes either before or after the norm")
     if y.numel() and _native_seq(y):
         out = torch.empty(y.shape, dtype=out_dtype, device=y.device)
         _S.gated_group_norm(out, y, gate, weight, int(groups), float(eps),
-                            bool(gate_first))
+                            1 if gate_first else (2 if silu_after else 0))
         return out
-    return reference.gated_group_norm(y, gate, weight, groups, eps, gate_first, out_dtype)
+    return reference.gated_group_norm(y, gate, weight, groups, eps, gate_first, out_dtype,
+                                      silu_after)
 
 
 def rglru_scan(u, r_pre, i_pre, r_bias, i_bias, lam, gate_c, y_branch, state,
@@ -1207,3 +1210,187 @@ def silu_mul_scaled(gu: torch.Tensor, col_scale: torch.Tensor) -> torch.Tensor:
         _S.silu_mul_scaled(out, gu, col_scale)
         return out
     return reference.silu_mul_scaled(gu, col_scale)
+
+
+# ---------------------------------------------------------------------------
+# Grouped RMS norms around both ends of a sublayer, attention inputs with a
+# short convolution, rotated values and pooled key/value blocks, attention over
+# a window plus a prefix, gated linear attention, biased gated feed-forward.
+# Same extension as the stream ops; the matrix-core attention variants live
+# with the other paged attention kernels.
+# ---------------------------------------------------------------------------
+
+
+def stream_add_group_norm(x: torch.Tensor, a: torch.Tensor | None,
+                          w_out: torch.Tensor | None, groups: int, eps: float, *,
+                          a_bias: torch.Tensor | None = None, b: torch.Tensor | None = None,
+                          wa: torch.Tensor | None = None, wb: torch.Tensor | None = None,
+                          mix: float = 0.5, next_w: torch.Tensor | None = None,
+                          out_dtype: torch.dtype = torch.bfloat16) -> torch.Tensor | None:
+    """x (f32 [T, W], in place) += N(y) * w_out, N being an RMS norm of
+    ``groups`` equal parts, with y = a + a_bias, or, when ``b`` is given, y =
+    mix * (a / rms(a) * wa + b / rms(b) * wb) over the whole width; nothing is
+    added when ``a`` is None.  With ``next_w`` the norm that reads the updated
+    stream next, N(x) * next_w, is returned in ``out_dtype``."""
+    if x.numel() and _native_seq(x):
+        out = torch.empty(x.shape, dtype=out_dtype, device=x.device) if next_w is not None else None
+        _S.stream_add_group_norm(x, a, a_bias, b, wa, wb, w_out, int(groups), float(eps),
+                                 float(mix), next_w, out)
+        return out
+    return reference.stream_add_group_norm(x, a, a_bias, b, wa, wb, w_out, groups, eps, mix,
+                                           next_w, out_dtype)
+
+
+def rotary_table(positions: torch.Tensor, inv_freq: torch.Tensor) -> torch.Tensor:
+    """cos and sin of the f32 angles position * inv_freq[i]: [T, pairs, 2] f32,
+    computed once per step and read by every layer that shares the frequencies."""
+    if positions.numel() and _native_seq(positions):
+        out = torch.empty((positions.shape[0], inv_freq.shape[0], 2), dtype=torch.float32,
+                          device=positions.device)
+        _S.rotary_table(out, positions, inv_freq)
+        return out
+    return reference.rotary_table(positions, inv_freq)
+
+
+def attn_inputs_cache_write(proj: torch.Tensor, bias, heads: int, kv_heads: int, dim: int,
+                            vdim: int, eps: float, q_weight, k_weight, conv_weight,
+                            conv_state, rot_table, v_table, k_cache, v_cache, slot_mapping,
+                            seq_start_loc, seq_lens, state_slots,
+                            has_portions: bool = True) -> torch.Tensor:
+    """From projected rows [q | k | v] (proj [T, C], rows may be strided) to the
+    attention's inputs, one pass: + bias [C] f32; a short causal convolution per
+    channel (``conv_weight`` [taps, C] f32 or None) whose last taps-1 projected
+    rows per sequence live in ``conv_state`` [slots, taps-1, C]; RMS norm of
+    every query and key head over dim (weights [dim] f32, or None for none);
+    rotation of queries and keys by ``rot_table`` and of values by ``v_table``
+    (rotary_table rows or None; pairs (i, i + R/2) of the first R dims); keys
+    and values stored in the paged cache.  Returns the queries [T, heads, dim].
+    ``has_portions`` False promises that every sequence brings one row."""
+    if proj.numel() and _native_seq(proj):
+        out = torch.empty((proj.shape[0], heads, dim), dtype=proj.dtype, device=proj.device)
+        _S.attn_inputs_cache_write(out, proj, bias, int(kv_heads), int(vdim), float(eps),
+                                   q_weight, k_weight, conv_weight, conv_state, rot_table,
+                                   v_table, k_cache, v_cache, slot_mapping, seq_start_loc,
+                                   seq_lens, state_slots, bool(has_portions))
+        return out
+    cpu = lambda t: None if t is None else t.cpu()
+    return reference.attn_inputs_cache_write(
+        proj, bias, heads, kv_heads, dim, vdim, eps, q_weight, k_weight, conv_weight,
+        conv_state, rot_table, v_table, k_cache, v_cache, slot_mapping, cpu(seq_start_loc),
+        cpu(seq_lens), cpu(state_slots))
+
+
+pool_slots_per_block = reference.pool_slots_per_block
+
+
+def pool_cache_write(k_cache, v_cache, k_pool, v_pool, pool: int, block_tables,
+                     query_start_loc, seq_lens) -> None:
+    """Means of every block of ``pool`` consecutive cached keys / values that
+    this step's rows complete (the tail of each sequence; ``query_start_loc``
+    None: one row each).  Pooled block b is kept in the cache block that holds
+    its last token: k_pool [blocks, slots, G, dim], v_pool [.., vdim], slots =
+    pool_slots_per_block."""
+    if k_cache.device.type == "cuda" and seq_lens.numel() and _native_seq(k_cache):
+        _S.pool_cache_write(k_cache, v_cache, k_pool, v_pool, int(pool), block_tables,
+                            query_start_loc, seq_lens)
+        return
+    if query_start_loc is None:
+        query_start_loc = torch.arange(seq_lens.numel() + 1, dtype=torch.int32)
+    reference.pool_cache_write(k_cache, v_cache, k_pool, v_pool, pool, block_tables.cpu(),
+                               query_start_loc.cpu(), seq_lens.cpu())
+
+
+def span_attention_uses_matrix_cores(dtype: torch.dtype, heads: int, kv_heads: int,
+                                     dim: int, vdim: int) -> bool:
+    """Shapes the span variants of the MFMA kernels take (prompt portions need
+    size 128, single queries 64 or 128)."""
+    return (dtype == torch.bfloat16 and dim == vdim and dim in (64, 128)
+            and heads % kv_heads == 0 and 1 <= heads // kv_heads <= 8)
+
+
+def _span_matrix_core_fits(q, k_cache, v_cache, out, window: int, single: bool) -> bool:
+    if _attn_ext() is None or _FORCE_REFERENCE or window <= 0:
+        return False
+    return (span_attention_uses_matrix_cores(q.dtype, q.shape[1], k_cache.shape[2],
+                                             q.shape[2], v_cache.shape[3])
+            and (single or q.shape[2] == 128) and q.is_contiguous() and out.is_contiguous())
+
+
+def span_attention_prefill(q, k_cache, v_cache, k_pool, v_pool, block_tables,
+                           query_start_loc, seq_lens, scale, max_query_len, window: int,
+                           keep_first: int, pool: int, back_table, out: torch.Tensor,
+                           general: bool = False) -> torch.Tensor:
+    """Causal grouped-query softmax attention of query portions over the paged
+    cache in which a query at position i sees the tokens j with 0 <= i - j <
+    window (window 0: every j <= i) and, beside them in the same softmax,
+    either the sequence's first ``keep_first`` tokens or (``pool`` > 0) one
+    pooled key and value for every block of ``pool`` positions that ends at or
+    before i - window (pool_cache_write).  ``back_table`` (rotary_table rows of
+    the queries, over the value size): each head's output is turned back by its
+    own position's angles.  ``general``: the any-shape kernel even where a
+    matrix-core kernel would take the shape."""
+    if q.numel() and _native_seq(q):
+        if not general and _span_matrix_core_fits(q, k_cache, v_cache, out, window, False):
+            _attn_ext().span_attention_prefill(
+                out, q, k_cache, v_cache, k_pool, v_pool, block_tables, query_start_loc,
+                seq_lens, float(scale), int(max_query_len), int(window), int(keep_first),
+                int(pool), back_table)
+            return out
+        _S.span_attention(out, q, k_cache, v_cache, k_pool, v_pool, block_tables,
+                          query_start_loc, seq_lens, float(scale), int(window),
+                          int(keep_first), int(pool), back_table)
+        return out
+    out.copy_(reference.span_attention(
+        q, k_cache, v_cache, k_pool, v_pool, block_tables.cpu(), query_start_loc.cpu(),
+        seq_lens.cpu(), scale, window, keep_first, pool, back_table))
+    return out
+
+
+def span_attention_decode(q, k_cache, v_cache, k_pool, v_pool, block_tables, seq_lens, scale,
+                          window: int, keep_first: int, pool: int, back_table,
+                          out: torch.Tensor, general: bool = False) -> torch.Tensor:
+    """Same attention for one new query per sequence (length 0 = padding row,
+    zeros)."""
+    if q.numel() and _native_seq(q):
+        if not general and _span_matrix_core_fits(q, k_cache, v_cache, out, window, True):
+            _attn_ext().span_attention_decode(
+                out, q, k_cache, v_cache, k_pool, v_pool, block_tables, seq_lens,
+                float(scale), int(window), int(keep_first), int(pool), back_table)
+            return out
+        _S.span_attention(out, q, k_cache, v_cache, k_pool, v_pool, block_tables, None,
+                          seq_lens, float(scale), int(window), int(keep_first), int(pool),
+                          back_table)
+        return out
+    qsl = torch.arange(q.shape[0] + 1, dtype=torch.int32)
+    out.copy_(reference.span_attention(
+        q, k_cache, v_cache, k_pool, v_pool, block_tables.cpu(), qsl, seq_lens.cpu(), scale,
+        window, keep_first, pool, back_table))
+    return out
+
+
+def gla_scan(q, k, v, a1, a2_t, a2_bias, inv_tau: float, q_scale: float, state,
+             seq_start_loc, seq_lens, state_slots) -> torch.Tensor:
+    """Gated linear attention over each sequence's new rows.  q, k [T, H, dim],
+    v [T, H, vdim], a1 [T, rank] (may be views into a merged projection); decay
+    per key channel alpha = sigmoid(a1 a2_t + a2_bias)^inv_tau with a2_t [rank,
+    H * dim] f32, all in f32; S_t = diag(alpha_t) S_(t-1) + k_t v_t^T, o_t =
+    S_t^T q_t * q_scale.  State [slots, H, vdim, dim] f32, advanced in place.
+    Returns o [T, H * vdim] f32."""
+    if q.numel() and _native_seq(q):
+        o = torch.empty((q.shape[0], q.shape[1] * v.shape[-1]), dtype=torch.float32,
+                        device=q.device)
+        _S.gla_scan(o, q, k, v, a1, a2_t, a2_bias, float(inv_tau), float(q_scale), state,
+                    seq_start_loc, seq_lens, state_slots)
+        return o
+    return reference.gla_scan(q, k, v, a1, a2_t, a2_bias, inv_tau, q_scale, state,
+                              seq_start_loc.cpu(), seq_lens.cpu(), state_slots.cpu())
+
+
+def silu_mul_bias(gu: torch.Tensor, bias: torch.Tensor | None = None) -> torch.Tensor:
+    """gu [T, 2 ff] (gate columns, then up columns) -> silu(gate + b) * (up + b)
+    [T, ff], bias [2 ff] f32."""
+    if gu.numel() and _native_seq(gu):
+        out = torch.empty((gu.shape[0], gu.shape[1] // 2), dtype=gu.dtype, device=gu.device)
+        _S.silu_mul_bias(out, gu, bias)
+        return out
+    return reference.silu_mul_bias(gu, bias)

@@ -496,10 +496,11 @@ def gated_group_norm(
     eps: float,
     gate_first: bool,
     out_dtype: torch.dtype,
+    silu_after: bool = False,
 ) -> torch.Tensor:
     """gate_first: RMS-norm of y * silu(gate) in ``groups`` equal parts, times
     weight.  Otherwise: RMS-norm of y in parts, times weight, times
-    sigmoid(gate)."""
+    sigmoid(gate) (``silu_after``: silu(gate))."""
     t, c = y.shape
     yf = y.float()
     gf = gate.float()
@@ -510,6 +511,8 @@ def gated_group_norm(
     out = yg.reshape(t, c) * weight.float()
     if not gate_first:
         out = out * torch.sigmoid(gf)
+        if silu_after:
+            out = out * gf
     return out.to(out_dtype)
 
 
@@ -894,3 +897,203 @@ def silu_mul_scaled(gu: torch.Tensor, col_scale: torch.Tensor) -> torch.Tensor:
     z = gu.float().view(t, e, 2, -1) * col_scale.float().view(t, e, 1, 1)
     g, u = z[:, :, 0], z[:, :, 1]
     return (g * torch.sigmoid(g) * u).to(gu.dtype).reshape(t, -1)
+
+
+# ---------------------------------------------------------------------------
+# Grouped RMS norms around both ends of a sublayer, attention inputs with a
+# short convolution, rotated values and pooled key/value blocks, attention over
+# a window plus a prefix (kept first tokens or pooled blocks), gated linear
+# attention, biased gated feed-forward.
+# ---------------------------------------------------------------------------
+
+
+def _group_unit(x: torch.Tensor, groups: int, eps: float) -> torch.Tensor:
+    t, c = x.shape
+    g = x.view(t, groups, c // groups)
+    return (g * torch.rsqrt(g.pow(2).mean(dim=-1, keepdim=True) + eps)).reshape(t, c)
+
+
+def stream_add_group_norm(x: torch.Tensor, a: torch.Tensor | None,
+                          a_bias: torch.Tensor | None, b: torch.Tensor | None,
+                          wa: torch.Tensor | None, wb: torch.Tensor | None,
+                          w_out: torch.Tensor | None, groups: int, eps: float,
+                          mix: float, next_w: torch.Tensor | None,
+                          out_dtype: torch.dtype) -> torch.Tensor | None:
+    """See ops.stream_add_group_norm."""
+    if a is not None:
+        y = a.float()
+        if a_bias is not None:
+            y = y + a_bias.float()
+        if b is not None:
+            y = mix * (_group_unit(y, 1, eps) * wa.float()
+                       + _group_unit(b.float(), 1, eps) * wb.float())
+        x.add_(_group_unit(y, groups, eps) * w_out.float())
+    if next_w is None:
+        return None
+    return (_group_unit(x, groups, eps) * next_w.float()).to(out_dtype)
+
+
+def rotary_table(positions: torch.Tensor, inv_freq: torch.Tensor) -> torch.Tensor:
+    ang = positions.to(torch.float32).unsqueeze(1) * inv_freq.float().unsqueeze(0)
+    return torch.stack([ang.cos(), ang.sin()], dim=-1)
+
+
+def _rotate_rows(x: torch.Tensor, table: torch.Tensor, sign: float = 1.0) -> torch.Tensor:
+    """x [T, H, D] f32, table [T, R/2, 2]: pairs (i, i + R/2) of the first R dims."""
+    half = table.shape[1]
+    c, s = table[:, None, :, 0], sign * table[:, None, :, 1]
+    u, v = x[..., :half], x[..., half:2 * half]
+    return torch.cat([u * c - v * s, v * c + u * s, x[..., 2 * half:]], dim=-1)
+
+
+def attn_inputs_cache_write(proj, bias, heads, kv_heads, dim, vdim, eps, q_weight, k_weight,
+                            conv_weight, conv_state, rot_table, v_table, k_cache, v_cache,
+                            slot_mapping, seq_start_loc, seq_lens, state_slots):
+    """See ops.attn_inputs_cache_write (conv_weight here [taps, C])."""
+    t = proj.shape[0]
+    u = proj.float()
+    if bias is not None:
+        u = u + bias.float()
+    if conv_weight is not None:
+        taps = conv_weight.shape[0]
+        out = torch.zeros_like(u)
+        wf = conv_weight.float()
+        for a, b, start, slot in _seq_iter(seq_start_loc, seq_lens, state_slots):
+            if slot < 0:
+                continue
+            if taps > 1:
+                # state row j is position start - (taps-1) + j, stored before the bias
+                hist = conv_state[slot].float()
+                if bias is not None:
+                    hist = hist + bias.float()
+                valid = (torch.arange(taps - 1) + start - (taps - 1)) >= 0
+                hist = hist * valid.to(hist).unsqueeze(1)
+                raw = torch.cat([conv_state[slot], proj[a:b].to(conv_state.dtype)])
+            else:
+                hist = u.new_zeros((0, u.shape[1]))
+            ext = torch.cat([hist, u[a:b]])
+            for j in range(taps):
+                out[a:b] += wf[j] * ext[j:j + b - a]
+            if taps > 1:
+                conv_state[slot] = raw[b - a:]
+        u = out
+    nq, nk = heads * dim, kv_heads * dim
+    q = u[:, :nq].view(t, heads, dim)
+    k = u[:, nq:nq + nk].view(t, kv_heads, dim)
+    v = u[:, nq + nk:].view(t, kv_heads, vdim)
+
+    def unit(x, w):
+        x = x * torch.rsqrt(x.pow(2).mean(dim=-1, keepdim=True) + eps)
+        return x if w is None else x * w.float()
+
+    q, k = unit(q, q_weight), unit(k, k_weight)
+    if rot_table is not None:
+        q, k = _rotate_rows(q, rot_table), _rotate_rows(k, rot_table)
+    if v_table is not None:
+        v = _rotate_rows(v, v_table)
+    ok = slot_mapping >= 0
+    sm = slot_mapping[ok]
+    bs = k_cache.shape[1]
+    blk = torch.div(sm, bs, rounding_mode="floor")
+    k_cache[blk, sm % bs] = k[ok].to(k_cache.dtype)
+    v_cache[blk, sm % bs] = v[ok].to(v_cache.dtype)
+    return q.to(proj.dtype).contiguous()
+
+
+def pool_slots_per_block(block_size: int, pool: int) -> int:
+    """Most pooled blocks that end inside one cache block."""
+    return (block_size + pool - 1) // pool
+
+
+def pool_entry(b: int, pool: int, block_size: int) -> tuple[int, int]:
+    """(index in the sequence's block table, place inside that cache block) of
+    pooled block b: it lives in the cache block that holds its last token."""
+    page = (b * pool + pool - 1) // block_size
+    return page, b - (page * block_size) // pool
+
+
+def pool_cache_write(k_cache, v_cache, k_pool, v_pool, pool, block_tables, query_start_loc,
+                     seq_lens) -> None:
+    """See ops.pool_cache_write."""
+    bs = k_cache.shape[1]
+    qs, lens = query_start_loc.tolist(), seq_lens.tolist()
+    for i in range(len(lens)):
+        n, end = qs[i + 1] - qs[i], lens[i]
+        if n == 0 or end == 0:
+            continue
+        k, v = _gather_kv(k_cache, v_cache, block_tables[i], end)
+        for b in range((end - n) // pool, end // pool):
+            page, at = pool_entry(b, pool, bs)
+            blk = int(block_tables[i][page])
+            rows = slice(b * pool, (b + 1) * pool)
+            k_pool[blk, at] = k[rows].float().mean(0).to(k_pool.dtype)
+            v_pool[blk, at] = v[rows].float().mean(0).to(v_pool.dtype)
+
+
+def span_attention(q, k_cache, v_cache, k_pool, v_pool, block_tables, query_start_loc,
+                   seq_lens, scale: float, window: int, keep_first: int, pool: int,
+                   back_table) -> torch.Tensor:
+    """See ops.span_attention_prefill; queries are the tail of each sequence."""
+    nh, ng = q.shape[1], k_cache.shape[2]
+    group = nh // ng
+    bs = k_cache.shape[1]
+    out = torch.zeros((q.shape[0], nh, v_cache.shape[-1]), dtype=torch.float32, device=q.device)
+    qs, lens = query_start_loc.tolist(), seq_lens.tolist()
+    for i in range(len(lens)):
+        s, e = qs[i], qs[i + 1]
+        n, ctx = e - s, lens[i]
+        if n == 0 or ctx == 0:
+            continue
+        k, v = _gather_kv(k_cache, v_cache, block_tables[i], ctx)
+        kpos = torch.arange(ctx, device=q.device)
+        qpos = torch.arange(ctx - n, ctx, device=q.device).unsqueeze(1)
+        see = kpos <= qpos
+        if window > 0:
+            see = see & ((qpos - kpos < window) | (kpos < keep_first))
+            nb = max(0, (ctx - window) // pool) if pool > 0 else 0
+            if nb:
+                at = [pool_entry(b, pool, bs) for b in range(nb)]
+                blk = block_tables[i][torch.tensor([p for p, _ in at])].long()
+                off = torch.tensor([o for _, o in at])
+                k = torch.cat([k_pool[blk, off], k])
+                v = torch.cat([v_pool[blk, off], v])
+                last = torch.arange(nb, device=q.device) * pool + pool - 1
+                see = torch.cat([last <= qpos - window, see], dim=1)
+        kf = k.float().repeat_interleave(group, dim=1)
+        vf = v.float().repeat_interleave(group, dim=1)
+        sc = torch.einsum("qhd,shd->hqs", q[s:e].float(), kf) * scale
+        sc.masked_fill_(~see.unsqueeze(0), float("-inf"))
+        out[s:e] = torch.einsum("hqs,shd->qhd", torch.softmax(sc, dim=-1), vf)
+    if back_table is not None:
+        out = _rotate_rows(out, back_table, -1.0)
+    return out.to(q.dtype)
+
+
+def gla_scan(q, k, v, a1, a2_t, a2_bias, inv_tau: float, q_scale: float, state,
+             seq_start_loc, seq_lens, state_slots) -> torch.Tensor:
+    """See ops.gla_scan."""
+    t, nh, d = q.shape
+    dv = v.shape[-1]
+    z = a1.float() @ a2_t.float() + a2_bias.float()
+    alpha = torch.exp(torch.nn.functional.logsigmoid(z) * inv_tau).view(t, nh, d)
+    qf, kf, vf = q.float() * q_scale, k.float(), v.float()
+    out = torch.zeros((t, nh, dv), dtype=torch.float32, device=q.device)
+    for a, b, start, slot in _seq_iter(seq_start_loc, seq_lens, state_slots):
+        if slot < 0:
+            continue
+        s = state[slot].clone() if start > 0 else torch.zeros_like(state[slot])
+        for i in range(a, b):
+            s = alpha[i].unsqueeze(1) * s + vf[i].unsqueeze(2) * kf[i].unsqueeze(1)
+            out[i] = torch.einsum("hvd,hd->hv", s, qf[i])
+        state[slot] = s
+    return out.view(t, nh * dv)
+
+
+def silu_mul_bias(gu: torch.Tensor, bias: torch.Tensor | None) -> torch.Tensor:
+    """gu [T, 2 ff] (gate columns, then up columns), bias [2 ff] f32:
+    silu(gate + b) * (up + b)."""
+    z = gu.float()
+    if bias is not None:
+        z = z + bias.float()
+    g, u = z.chunk(2, dim=-1)
+    return (g * torch.sigmoid(g) * u).to(gu.dtype)
