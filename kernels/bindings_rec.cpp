@@ -174,7 +174,8 @@ void stream_add_vec(torch::Tensor x, c10::optional<torch::Tensor> other,
 
 void gated_group_norm(torch::Tensor out, torch::Tensor y, torch::Tensor gate,
                       torch::Tensor weight, int64_t groups, double eps,
-                      bool gate_first) {
+                      int64_t gate_mode) {
+  TORCH_CHECK(gate_mode >= 0 && gate_mode <= 2, "gate mode");
   check_f32(y, "y");
   check_f32(weight, "weight");
   TORCH_CHECK(y.dim() == 2 && gate.dim() == 2 && gate.is_cuda() &&
@@ -188,7 +189,7 @@ void gated_group_norm(torch::Tensor out, torch::Tensor y, torch::Tensor gate,
     launch_gated_group_norm<scalar_t>(
         ptr<scalar_t>(out), ptr<float>(y), ptr<scalar_t>(gate),
         (long)gate.stride(0), ptr<float>(weight), (float)eps, rows, cols,
-        (int)groups, gate_first ? 1 : 0, stream());
+        (int)groups, (int)gate_mode, stream());
   });
 }
 

@@ -44,6 +44,9 @@ void register_par_ops(pybind11::module& m);
 // token shift, norm + rotation + cache write, chunk-masked attention, the
 // differential combination, HGRN2, weighted gated activation (bindings_mix.cpp)
 void register_mix_ops(pybind11::module& m);
+// span_ops.hip, the window-plus-prefix attention and the gated linear attention
+// scan (bindings_span.cpp)
+void register_span_ops(pybind11::module& m);
 namespace {
 
 hipStream_t stream() { return at::hip::getCurrentHIPStream().stream(); }
@@ -298,4 +301,5 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   register_rec_ops(m);
   register_par_ops(m);
   register_mix_ops(m);
+  register_span_ops(m);
 }

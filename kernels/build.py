@@ -16,9 +16,11 @@ Several extensions, so that a model only builds the ones it uses
             convolution with per-sequence state, grouped-query attention of
             any shape, recurrences with per-sequence state, two-norm blocks,
             rotation + cache write, gates, expert routing, the grouped expert
-            product, token shift, chunk-masked differential attention pieces
+            product, token shift, chunk-masked differential attention pieces,
+            grouped norms around sublayers, attention inputs in one pass,
+            attention over a window plus a prefix, gated linear attention
             + bindings_seq.cpp, bindings_rec.cpp, bindings_par.cpp,
-            bindings_mix.cpp
+            bindings_mix.cpp, bindings_span.cpp
 ``_C_lat``  windowed latent attention with sinks + bindings_lat.cpp
 """
 
@@ -38,7 +40,7 @@ ARCH = os.environ.get("PYTORCH_ROCM_ARCH", "gfx950")
 
 _SEQ_SOURCES = ["stream_ops.hip", "canon_conv.hip", "layer_norm_stream.hip",
                 "paged_attention_any.hip", "recurrent_scan.hip", "gated_block.hip",
-                "mix_ops.hip"]
+                "mix_ops.hip", "span_ops.hip"]
 # kernels without torch types that more than one extension links
 _SHARED_SOURCES = ["moe_gemm.hip"]
 _LAT_SOURCES = ["latent_attention.hip", "latent_attention_mfma.hip"]
@@ -58,7 +60,8 @@ EXTENSIONS = {
     "_C_seq": dict(
         sources=lambda: [KERNELS / n for n in _SEQ_SOURCES + _SHARED_SOURCES]
         + [KERNELS / "bindings_seq.cpp", KERNELS / "bindings_rec.cpp",
-           KERNELS / "bindings_par.cpp", KERNELS / "bindings_mix.cpp"],
+           KERNELS / "bindings_par.cpp", KERNELS / "bindings_mix.cpp",
+           KERNELS / "bindings_span.cpp"],
     ),
     "_C_lat": dict(
         sources=lambda: [KERNELS / n for n in _LAT_SOURCES] + [KERNELS / "bindings_lat.cpp"],

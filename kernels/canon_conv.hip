@@ -153,6 +153,17 @@ __global__ void conv_state_update_kernel(T* __restrict__ state,
   }
 }
 
+// advances the kept inputs of every sequence past its new rows (taps > 1)
+template <typename T>
+void launch_conv_state_update(T* state, const T* h, const int* loc, const int* seq_lens,
+                              const int* slots, int nseq, int width, int taps, long in_st,
+                              hipStream_t stream) {
+  const int block = 256;
+  dim3 g2(nseq, (width + block - 1) / block);
+  conv_state_update_kernel<T><<<g2, block, 0, stream>>>(state, h, loc, seq_lens, slots,
+                                                       width, taps, in_st);
+}
+
 template <typename T>
 void launch_causal_conv_state(T* out, const T* h, const float* w, T* state,
                               const int* loc, const int* seq_lens,
@@ -184,11 +195,9 @@ void launch_causal_conv_state(T* out, const T* h, const float* w, T* state,
         out, h, w, state, loc, seq_lens, slots, nseq, width, taps, add_input,
         in_st, bias, act);
   }
-  if (taps > 1) {
-    dim3 g2(nseq, (width + block - 1) / block);
-    conv_state_update_kernel<T><<<g2, block, 0, stream>>>(
-        state, h, loc, seq_lens, slots, width, taps, in_st);
-  }
+  if (taps > 1)
+    launch_conv_state_update<T>(state, h, loc, seq_lens, slots, nseq, width, taps, in_st,
+                                stream);
 }
 
 template void launch_causal_conv_state<float>(float*, const float*, const float*,
@@ -200,3 +209,9 @@ template void launch_causal_conv_state<__hip_bfloat16>(
     __hip_bfloat16*, const __hip_bfloat16*, const float*, __hip_bfloat16*,
     const int*, const int*, const int*, int, int, int, int, int, long,
     const float*, int, hipStream_t);
+template void launch_conv_state_update<float>(float*, const float*, const int*,
+                                              const int*, const int*, int, int, int,
+                                              long, hipStream_t);
+template void launch_conv_state_update<__hip_bfloat16>(
+    __hip_bfloat16*, const __hip_bfloat16*, const int*, const int*, const int*, int,
+    int, int, long, hipStream_t);

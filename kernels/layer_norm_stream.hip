@@ -6,7 +6,8 @@
 //                            next_out = LN(x) * next_w of the updated row
 //   stream_add_vec           x += other + vec (vec broadcast over rows)
 //   gated_group_norm         RMS norm of an f32 row in equal parts with a gate:
-//                            silu(gate) before the norm or sigmoid(gate) after
+//                            sigmoid(gate) after the norm (gate_mode 0), silu(gate)
+//                            before (1) or after it (2)
 //   qk_norm_cache_write      per-head RMS norm of queries and keys, query
 //                            temperature by position, keys and values stored
 //                            in the paged cache
@@ -232,7 +233,7 @@ template <typename T>
 __global__ __launch_bounds__(256) void gated_group_norm_kernel(
     T* __restrict__ out, const float* __restrict__ y, const T* __restrict__ gate,
     long gate_stride, const float* __restrict__ w, float eps, int cols, int gsize,
-    int gate_first) {
+    int gate_mode) {
   __shared__ float r0[16];
   const long row = blockIdx.x;
   const int c0 = blockIdx.y * gsize;
@@ -241,7 +242,7 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(
   float ss = 0.f;
   for (int c = threadIdx.x; c < gsize; c += blockDim.x) {
     float v = yr[c];
-    if (gate_first) {
+    if (gate_mode == 1) {
       const float g = ScalarOps<T>::to_f32(gr[c]);
       v *= g / (1.0f + expf(-g));
     }
@@ -252,8 +253,8 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(
     const float g = ScalarOps<T>::to_f32(gr[c]);
     const float sg = 1.0f / (1.0f + expf(-g));
     float v = yr[c];
-    if (gate_first) v = v * (g * sg) * inv * w[c0 + c];
-    else v = v * inv * w[c0 + c] * sg;
+    if (gate_mode == 1) v = v * (g * sg) * inv * w[c0 + c];
+    else v = v * inv * w[c0 + c] * (gate_mode == 2 ? g * sg : sg);
     out[row * cols + c0 + c] = ScalarOps<T>::from_f32(v);
   }
 }
@@ -314,7 +315,7 @@ template <typename T, int NCH>
 __global__ __launch_bounds__(256) void gated_group_norm_reg_kernel(
     T* __restrict__ out, const float* __restrict__ y, const T* __restrict__ gate,
     long gate_stride, const float* __restrict__ w, float eps, int cols, int gsize,
-    int gate_first) {
+    int gate_mode) {
   __shared__ float r0[16];
   const long row = blockIdx.x;
   const int c0 = blockIdx.y * gsize;
@@ -332,9 +333,11 @@ __global__ __launch_bounds__(256) void gated_group_norm_reg_kernel(
       const float4 g = ld4<T>(gr + c);
       sg[i] = make_float4(1.0f / (1.0f + expf(-g.x)), 1.0f / (1.0f + expf(-g.y)),
                           1.0f / (1.0f + expf(-g.z)), 1.0f / (1.0f + expf(-g.w)));
-      if (gate_first) {
+      if (gate_mode == 1) {
         v[i].x *= g.x * sg[i].x; v[i].y *= g.y * sg[i].y;
         v[i].z *= g.z * sg[i].z; v[i].w *= g.w * sg[i].w;
+      } else if (gate_mode == 2) {
+        sg[i].x *= g.x; sg[i].y *= g.y; sg[i].z *= g.z; sg[i].w *= g.w;
       }
       ss += (v[i].x * v[i].x + v[i].y * v[i].y) + (v[i].z * v[i].z + v[i].w * v[i].w);
     }
@@ -347,7 +350,7 @@ __global__ __launch_bounds__(256) void gated_group_norm_reg_kernel(
       const float4 ww = ld4<float>(w + c0 + c);
       float4 o = make_float4(v[i].x * inv * ww.x, v[i].y * inv * ww.y,
                              v[i].z * inv * ww.z, v[i].w * inv * ww.w);
-      if (!gate_first) { o.x *= sg[i].x; o.y *= sg[i].y; o.z *= sg[i].z; o.w *= sg[i].w; }
+      if (gate_mode != 1) { o.x *= sg[i].x; o.y *= sg[i].y; o.z *= sg[i].z; o.w *= sg[i].w; }
       st4<T>(out + row * cols + c0 + c, o);
     }
   }
@@ -471,7 +474,7 @@ void launch_stream_add_vec(float* x, const float* other, const float* vec,
 template <typename T>
 void launch_gated_group_norm(T* out, const float* y, const T* gate,
                              long gate_stride, const float* w, float eps,
-                             int rows, int cols, int groups, int gate_first,
+                             int rows, int cols, int groups, int gate_mode,
                              hipStream_t s) {
   const int gsize = cols / groups;
   dim3 grid(rows, groups);
@@ -481,15 +484,15 @@ void launch_gated_group_norm(T* out, const float* y, const T* gate,
     const int vb = q4 <= 64 ? 64 : (q4 <= 128 ? 128 : 256);
     if (q4 <= vb)
       gated_group_norm_reg_kernel<T, 1><<<grid, vb, 0, s>>>(out, y, gate, gate_stride, w,
-                                                           eps, cols, gsize, gate_first);
+                                                           eps, cols, gsize, gate_mode);
     else
       gated_group_norm_reg_kernel<T, 4><<<grid, vb, 0, s>>>(out, y, gate, gate_stride, w,
-                                                           eps, cols, gsize, gate_first);
+                                                           eps, cols, gsize, gate_mode);
     return;
   }
   const int block = gsize <= 64 ? 64 : (gsize <= 128 ? 128 : 256);
   gated_group_norm_kernel<T><<<grid, block, 0, s>>>(out, y, gate, gate_stride, w, eps,
-                                                   cols, gsize, gate_first);
+                                                   cols, gsize, gate_mode);
 }
 
 template <typename T>

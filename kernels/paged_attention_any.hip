@@ -11,7 +11,12 @@
 // chunk size c it sees only keys of its own chunk, floor(j / c) = floor(i / c),
 // chunks counted from position 0.  The value cache may hold fewer heads Gv
 // than the key cache: key head g reads value head g mod Gv.  The output type
-// may be f32 beside a 16-bit cache.  One workgroup per (query row, head).  Per tile of 256 keys:
+// may be f32 beside a 16-bit cache.  With a prefix (SPAN) a query also sees, in
+// the same softmax, keys ahead of its window: the sequence's first `keep`
+// tokens, or one pooled key and value for every block of `pool` positions that
+// ends at or before i - window (block b is kept in the cache block that holds
+// its last token), and its output may be turned back by its position's angles.
+// Prefix and window form one list of keys that is walked in order.  One workgroup per (query row, head).  Per tile of 256 keys:
 //   phase 1  thread j scores key j (q, already multiplied by the score scale,
 //            broadcast from LDS; the key row read with 16-byte loads), block
 //            max / sum give the online-softmax step
@@ -56,7 +61,14 @@ DEVINLINE float pa_reduce_sum(float x, float* scratch) {
   return s;
 }
 
-template <typename T, typename O>
+template <typename T>
+struct SpanPrefix {
+  int keep, pool, per_block;          // pool > 0: pooled blocks, per_block of them per cache block
+  const T* k_pool; const T* v_pool;   // [blocks, per_block, G, dim | vdim]
+  const float2* back;                 // [rows, vdim/2] cos, sin, or null
+};
+
+template <typename T, typename O, bool SPAN>
 __global__ __launch_bounds__(PA_THREADS) void paged_attention_any_kernel(
     O* __restrict__ out, long o_st, const T* __restrict__ q, long q_st,
     const T* __restrict__ k_cache, const T* __restrict__ v_cache,
@@ -64,7 +76,7 @@ __global__ __launch_bounds__(PA_THREADS) void paged_attention_any_kernel(
     const int* __restrict__ qsl, const int* __restrict__ seq_lens, int nseq,
     float scale, int heads, int kv_heads, int dim, int vdim, int block_size,
     int vp /* pow2 >= min(vdim, 256) */, int vec_ok, int window, int has_sink,
-    float sink, int chunk, int v_heads) {
+    float sink, int chunk, int v_heads, SpanPrefix<T> sp) {
   extern __shared__ float smem[];
   float* q_s = smem;                               // [dim]
   float* p_s = q_s + ((dim + 1) & ~1);             // [256]
@@ -116,13 +128,26 @@ __global__ __launch_bounds__(PA_THREADS) void paged_attention_any_kernel(
 
   int first = (window > 0 && ctx > window) ? ctx - window : 0;
   if (chunk > 0) first = max(first, ((ctx - 1) / chunk) * chunk);
-  for (int base = first; base < ctx; base += PA_THREADS) {
-    const int j = base + tid;
+  int npre = 0;   // keys ahead of the window
+  if (SPAN && window > 0)
+    npre = sp.pool > 0 ? max(0, ctx - window) / sp.pool : min(sp.keep, first);
+  const int total = npre + ctx - first;
+  for (int base = 0; base < total; base += PA_THREADS) {
+    const int u = base + tid;
     float s = -INFINITY;
-    if (j < ctx) {
-      const long tok = (long)bt[j / block_size] * block_size + (j % block_size);
-      tok_s[tid] = tok;
-      const T* kr = k_cache + tok * k_tok + (long)g_kv * dim;
+    if (u < total) {
+      const T* kr;
+      if (SPAN && sp.pool > 0 && u < npre) {
+        const int page = (u * sp.pool + sp.pool - 1) / block_size;
+        const long at = (long)bt[page] * sp.per_block + (u - page * block_size / sp.pool);
+        tok_s[tid] = -1 - at;
+        kr = sp.k_pool + at * k_tok + (long)g_kv * dim;
+      } else {
+        const int j = SPAN && u < npre ? u : first + u - npre;
+        const long tok = (long)bt[j / block_size] * block_size + (j % block_size);
+        tok_s[tid] = tok;
+        kr = k_cache + tok * k_tok + (long)g_kv * dim;
+      }
       float a = 0.f;
       if (vec_ok) {
         for (int k = 0; k < dim; k += V) {
@@ -138,17 +163,19 @@ __global__ __launch_bounds__(PA_THREADS) void paged_attention_any_kernel(
     const float m_tile = pa_reduce_max(s, red);
     const float m_new = fmaxf(m_run, m_tile);
     const float alpha = (m_run == -INFINITY) ? 0.f : expf(m_run - m_new);
-    const float p = (j < ctx) ? expf(s - m_new) : 0.f;
+    const float p = (u < total) ? expf(s - m_new) : 0.f;
     p_s[tid] = p;
     const float l_tile = pa_reduce_sum(p, red);   // its barriers also publish p_s / tok_s
     l_run = l_run * alpha + l_tile;
     m_run = m_new;
-    const int nk = min(PA_THREADS, ctx - base);
+    const int nk = min(PA_THREADS, total - base);
 #pragma unroll
     for (int i = 0; i < PA_MAX_DPT; ++i) acc[i] *= alpha;
     for (int jj = g; jj < nk; jj += groups) {
       const float pj = p_s[jj];
-      const T* vr = v_cache + tok_s[jj] * v_tok + (long)g_v * vdim;
+      const long tok = tok_s[jj];
+      const T* vr = (SPAN && tok < 0 ? sp.v_pool + (-1 - tok) * v_tok : v_cache + tok * v_tok) +
+                    (long)g_v * vdim;
 #pragma unroll
       for (int i = 0; i < PA_MAX_DPT; ++i) {
         const int k = k0 + i * vp;
@@ -164,42 +191,62 @@ __global__ __launch_bounds__(PA_THREADS) void paged_attention_any_kernel(
     const float rescale = expf(m_run - m_fin);
     inv = rescale / (l_run * rescale + expf(sink - m_fin));
   }
+  const bool back = SPAN && sp.back != nullptr;
   if (groups > 1) {
     // vdim <= vp <= 128 here: one dim per thread, sum the groups through LDS
     acc_s[tid] = acc[0];
     __syncthreads();
+    float a = 0.f;
     if (g == 0 && k0 < vdim) {
-      float a = 0.f;
       for (int gg = 0; gg < groups; ++gg) a += acc_s[gg * vp + k0];
-      orow[k0] = ScalarOps<O>::from_f32(a * inv);
+      if (!back) orow[k0] = ScalarOps<O>::from_f32(a * inv);
+    }
+    if (back) {
+      __syncthreads();
+      if (g == 0 && k0 < vdim) acc_s[k0] = a * inv;
     }
   } else {
 #pragma unroll
     for (int i = 0; i < PA_MAX_DPT; ++i) {
       const int k = k0 + i * vp;
-      if (k < vdim) orow[k] = ScalarOps<O>::from_f32(acc[i] * inv);
+      if (k >= vdim) continue;
+      if (back) acc_s[k] = acc[i] * inv;
+      else orow[k] = ScalarOps<O>::from_f32(acc[i] * inv);
+    }
+  }
+  if (back) {
+    __syncthreads();
+    const int half = vdim / 2;
+    const float2* tab = sp.back + (long)row * half;
+    for (int k = tid; k < half; k += PA_THREADS) {
+      const float a = acc_s[k], b = acc_s[k + half];
+      const float2 cs = tab[k];
+      orow[k] = ScalarOps<O>::from_f32(a * cs.x + b * cs.y);
+      orow[k + half] = ScalarOps<O>::from_f32(b * cs.x - a * cs.y);
     }
   }
 }
 
 }  // namespace
 
-template <typename T, typename O>
+template <typename T, typename O, bool SPAN = false>
 static void launch_any(O* out, long o_st, const T* q, long q_st, const T* k_cache,
                        const T* v_cache, const int* block_tables, int bt_stride,
                        const int* qsl, const int* seq_lens, int nseq, float scale,
                        int rows, int heads, int kv_heads, int dim, int vdim,
                        int block_size, int vec_ok, int window, int has_sink,
-                       float sink, int chunk, int v_heads, hipStream_t stream) {
+                       float sink, int chunk, int v_heads, hipStream_t stream,
+                       SpanPrefix<T> sp = SpanPrefix<T>{}) {
   int vp = 1;
   while (vp < vdim && vp < PA_THREADS) vp <<= 1;
-  const size_t smem = sizeof(float) * (((dim + 1) & ~1) + PA_THREADS + 16 + PA_THREADS) +
+  const size_t smem = sizeof(float) * (((dim + 1) & ~1) + PA_THREADS + 16 +
+                                       (vdim > PA_THREADS ? vdim : PA_THREADS)) +
                       sizeof(long) * PA_THREADS;
   dim3 grid(rows, heads);
-  paged_attention_any_kernel<T, O><<<grid, PA_THREADS, smem, stream>>>(
+  paged_attention_any_kernel<T, O, SPAN><<<grid, PA_THREADS, smem, stream>>>(
       out, o_st, q, q_st, k_cache, v_cache, block_tables, bt_stride, qsl,
       seq_lens, nseq, scale, heads, kv_heads, dim, vdim, block_size, vp, vec_ok,
-      window, has_sink, sink, chunk, v_heads);
+      window, has_sink, sink, chunk, v_heads, sp);
 }
 
 template <typename T>
@@ -230,6 +277,33 @@ void launch_chunk_attention(float* out, long o_st, const T* q, long q_st,
                        block_size, vec_ok, 0, 0, 0.f, chunk, v_heads, stream);
 }
 
+// window plus a prefix of first tokens or pooled blocks
+template <typename T>
+void launch_span_attention(T* out, long o_st, const T* q, long q_st, const T* k_cache,
+                           const T* v_cache, const T* k_pool, const T* v_pool,
+                           const int* block_tables, int bt_stride, const int* qsl,
+                           const int* seq_lens, int nseq, float scale, int rows,
+                           int heads, int kv_heads, int dim, int vdim, int block_size,
+                           int per_block, int vec_ok, int window, int keep, int pool,
+                           const float* back, hipStream_t stream) {
+  SpanPrefix<T> sp;
+  sp.keep = keep; sp.pool = pool; sp.per_block = per_block;
+  sp.k_pool = k_pool; sp.v_pool = v_pool;
+  sp.back = reinterpret_cast<const float2*>(back);
+  launch_any<T, T, true>(out, o_st, q, q_st, k_cache, v_cache, block_tables, bt_stride, qsl,
+                         seq_lens, nseq, scale, rows, heads, kv_heads, dim, vdim, block_size,
+                         vec_ok, window, 0, 0.f, 0, kv_heads, stream, sp);
+}
+
+template void launch_span_attention<float>(
+    float*, long, const float*, long, const float*, const float*, const float*,
+    const float*, const int*, int, const int*, const int*, int, float, int, int, int, int,
+    int, int, int, int, int, int, int, const float*, hipStream_t);
+template void launch_span_attention<__hip_bfloat16>(
+    __hip_bfloat16*, long, const __hip_bfloat16*, long, const __hip_bfloat16*,
+    const __hip_bfloat16*, const __hip_bfloat16*, const __hip_bfloat16*, const int*, int,
+    const int*, const int*, int, float, int, int, int, int, int, int, int, int, int, int,
+    int, const float*, hipStream_t);
 template void launch_paged_attention_any<float>(
     float*, long, const float*, long, const float*, const float*, const int*, int,
     const int*, const int*, int, float, int, int, int, int, int, int, int, int,

@@ -22,6 +22,10 @@
 //               g = l + (1 - l) sigmoid(f + b) with a lower bound l per
 //               channel, y = S silu(q); a pointwise kernel ahead of the scan
 //               writes g and silu(q) in f32 once per (row, head, channel)
+//   KIND_GLA    a decay per key channel: S_t[j, i] = alpha_t[i] S_(t-1)[j, i] +
+//               k_t[i] v_t[j], y = S q * q_scale; alpha = sigmoid(z)^(1/tau) with z
+//               from a low-rank product, written by a pre-pass in f32 once per
+//               (row, head, channel)
 // alpha, beta (and exp(-m')) are computed once per (row, head) by small gate
 // kernels ahead of the scan (for the mLSTM a sequential pass over the rows
 // carries the maximum), not by every thread of it.
@@ -44,7 +48,7 @@
 namespace {
 
 constexpr int NPT = 16;   // state values per thread along N
-enum { KIND_SSD = 0, KIND_MLSTM = 1, KIND_HGRN2 = 2 };
+enum { KIND_SSD = 0, KIND_MLSTM = 1, KIND_HGRN2 = 2, KIND_GLA = 3 };
 
 DEVINLINE float softplus_f(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
 DEVINLINE float logsigmoid_f(float x) { return fminf(x, 0.f) - log1pf(expf(-fabsf(x))); }
@@ -103,6 +107,7 @@ struct ScanArgs {
   float* y; long y_st;               // [T, H*vdim] f32
   float* s_state; float* n_state; float* m_state;
   const int* loc; const int* seq_lens; const int* slots;
+  const float* decay;                // GLA: [T, H*nk] f32
   int heads, vdim, nk, per_group;    // nk = N (SSD) or dim (mLSTM); heads per k/q group
   int vec_ok;
 };
@@ -212,30 +217,35 @@ __global__ __launch_bounds__(256) void matrix_scan_kernel(ScanArgs a) {
 
   // the next row's inputs are loaded while this row is computed: with two
   // waves per SIMD the load latency is otherwise paid once per token
-  float kk[NPT], qq[NPT], vj[VPT];
+  // constant subscripts only, so that the decay slices of the other kinds vanish
+  constexpr int ND = KIND == KIND_GLA ? NPT : 1;
+  const float* dp = KIND == KIND_GLA ? a.decay + (long)h * a.nk : nullptr;
+  const long d_st = (long)a.heads * a.nk;
+  float kk[NPT], qq[NPT], vj[VPT], dd[ND];
   float4 gt;
-  auto load_row = [&](long row, float* k_, float* q_, float* v_, float4& g_) {
+  auto load_row = [&](long row, float* k_, float* q_, float* v_, float* d_, float4& g_) {
+    if constexpr (KIND == KIND_GLA) load_slice<float>(dp + row * d_st, n0, a.nk, vec, d_);
     load_slice<KQ>(kp + row * a.k_st, n0, a.nk, vec, k_);
     load_slice<KQ>(qp + row * a.q_st, n0, a.nk, vec, q_);
 #pragma unroll
     for (int c = 0; c < VPT; ++c) v_[c] = ScalarOps<T>::to_f32(vp[row * a.v_st + jc[c]]);
-    g_ = KIND == KIND_HGRN2 ? make_float4(0.f, 0.f, 0.f, 0.f) : gp[row * a.heads];
+    g_ = KIND == KIND_HGRN2 || KIND == KIND_GLA ? make_float4(0.f, 0.f, 0.f, 0.f) : gp[row * a.heads];
   };
-  load_row(row0, kk, qq, vj, gt);
+  load_row(row0, kk, qq, vj, dd, gt);
   for (int r = 0; r < n; ++r) {
     const long row = row0 + r;
-    float kn[NPT], qn[NPT], vn[VPT];
+    float kn[NPT], qn[NPT], vn[VPT], dn[ND];
     float4 gn;
     const bool more = r + 1 < n;       // uniform over the workgroup
-    if (more) load_row(row + 1, kn, qn, vn, gn);
+    if (more) load_row(row + 1, kn, qn, vn, dn, gn);
     const float alpha = gt.x, beta = gt.y;
     float dot[VPT], ndot = 0.f;
 #pragma unroll
     for (int c = 0; c < VPT; ++c) dot[c] = 0.f;
 #pragma unroll
     for (int i = 0; i < NPT; ++i) {
-      const float al = KIND == KIND_HGRN2 ? kk[i] : alpha;
-      const float bk = KIND == KIND_HGRN2 ? 1.0f - kk[i] : beta * kk[i];
+      const float al = KIND == KIND_HGRN2 ? kk[i] : KIND == KIND_GLA ? dd[i < ND ? i : 0] : alpha;
+      const float bk = KIND == KIND_HGRN2 ? 1.0f - kk[i] : KIND == KIND_GLA ? kk[i] : beta * kk[i];
       if (KIND == KIND_MLSTM) {
         nst[i] = alpha * nst[i] + bk;
         ndot += nst[i] * qq[i];
@@ -254,13 +264,18 @@ __global__ __launch_bounds__(256) void matrix_scan_kernel(ScanArgs a) {
 #pragma unroll
     for (int c = 0; c < VPT; ++c) {
       const float d = lanes_sum<NSP>(dot[c]);
-      const float yv = KIND == KIND_MLSTM ? d * den : d + c2 * vj[c];
+      const float yv = KIND == KIND_MLSTM ? d * den
+                       : KIND == KIND_GLA ? d * a.q_scale : d + c2 * vj[c];
       if (ns == 0 && jbase + c < a.vdim)
         a.y[row * a.y_st + (long)h * a.vdim + jbase + c] = yv;
     }
     if (more) {
 #pragma unroll
       for (int i = 0; i < NPT; ++i) { kk[i] = kn[i]; qq[i] = qn[i]; }
+      if constexpr (KIND == KIND_GLA) {
+#pragma unroll
+        for (int i = 0; i < ND; ++i) dd[i] = dn[i];
+      }
 #pragma unroll
       for (int c = 0; c < VPT; ++c) vj[c] = vn[c];
       gt = gn;
@@ -327,6 +342,41 @@ __global__ __launch_bounds__(256) void hgrn2_gates_kernel(
   const float qv = ScalarOps<T>::to_f32(q[row * q_st + c]);
   gq[row * 2 * hd + c] = lo + (1.0f - lo) * sigmoid_f(fv);
   gq[row * 2 * hd + hd + c] = qv * sigmoid_f(qv);
+}
+
+// GLA pre-pass: decay [T, channels] f32 = exp(logsigmoid(a1 . a2[:, c] + b) / tau).
+// One thread per channel and GLA_ROWS rows; the rows' inner projections are
+// broadcast from LDS, a channel's column of a2 [rank, channels] is read once.
+constexpr int GLA_ROWS = 16;
+
+template <typename T>
+__global__ __launch_bounds__(256) void gla_decay_kernel(
+    float* __restrict__ decay, const T* __restrict__ a1, long a1_st,
+    const float* __restrict__ a2, const float* __restrict__ bias, float inv_tau, int rows,
+    int channels, int rank) {
+  extern __shared__ float inner[];   // [rank][GLA_ROWS]
+  const int r0 = blockIdx.x * GLA_ROWS;
+  const int n = min(GLA_ROWS, rows - r0);
+  for (int i = threadIdx.x; i < rank * GLA_ROWS; i += blockDim.x) {
+    const int r = i / rank, k = i - r * rank;
+    inner[k * GLA_ROWS + r] =
+        r < n ? ScalarOps<T>::to_f32(a1[(long)(r0 + r) * a1_st + k]) : 0.f;
+  }
+  __syncthreads();
+  const int c = blockIdx.y * blockDim.x + threadIdx.x;
+  if (c >= channels) return;
+  float z[GLA_ROWS];
+  const float b = bias[c];
+#pragma unroll
+  for (int r = 0; r < GLA_ROWS; ++r) z[r] = b;
+  for (int k = 0; k < rank; ++k) {
+    const float w = a2[(long)k * channels + c];
+#pragma unroll
+    for (int r = 0; r < GLA_ROWS; ++r) z[r] += inner[k * GLA_ROWS + r] * w;
+  }
+#pragma unroll
+  for (int r = 0; r < GLA_ROWS; ++r)
+    if (r < n) decay[(long)(r0 + r) * channels + c] = expf(logsigmoid_f(z[r]) * inv_tau);
 }
 
 template <typename T, int KIND>
@@ -474,6 +524,30 @@ void launch_hgrn2_scan(float* o, const T* q, long q_st, const T* f, long f_st,
 }
 
 template <typename T>
+void launch_gla_scan(float* o, const T* q, long q_st, const T* k, long k_st, const T* v,
+                     long v_st, const T* a1, long a1_st, const float* a2,
+                     const float* a2_bias, float inv_tau, float q_scale, float* state,
+                     const int* loc, const int* seq_lens, const int* slots, int nseq,
+                     int heads, int dim, int vdim, int rank, int vec_ok, float* decay,
+                     int rows, hipStream_t stream) {
+  const int hd = heads * dim;
+  const dim3 grid((rows + GLA_ROWS - 1) / GLA_ROWS, (hd + 255) / 256);
+  gla_decay_kernel<T><<<grid, 256, sizeof(float) * GLA_ROWS * rank, stream>>>(
+      decay, a1, a1_st, a2, a2_bias, inv_tau, rows, hd, rank);
+  ScanArgs a{};
+  a.rows = rows;
+  a.q = q; a.q_st = q_st; a.k = k; a.k_st = k_st; a.v = v; a.v_st = v_st;
+  a.decay = decay;
+  a.q_scale = q_scale;
+  a.y = o; a.y_st = (long)heads * vdim;
+  a.s_state = state;
+  a.loc = loc; a.seq_lens = seq_lens; a.slots = slots;
+  a.heads = heads; a.vdim = vdim; a.nk = dim; a.per_group = 1;
+  a.vec_ok = vec_ok;
+  launch_matrix_scan<T, KIND_GLA>(a, nseq, stream);
+}
+
+template <typename T>
 void launch_rglru_scan(T* out, const T* u, const T* r_pre, const T* i_pre,
                        const float* r_bias, const float* i_bias, const float* lam,
                        float gate_c, const T* y_branch, float* state,
@@ -502,6 +576,11 @@ void launch_rglru_scan(T* out, const T* u, const T* r_pre, const T* i_pre,
                                      float*, const int*, const int*, const int*,\
                                      int, int, int, int, int, float*, int,      \
                                      hipStream_t);                              \
+  template void launch_gla_scan<T>(float*, const T*, long, const T*, long,      \
+                                   const T*, long, const T*, long, const float*, \
+                                   const float*, float, float, float*,          \
+                                   const int*, const int*, const int*, int, int, \
+                                   int, int, int, int, float*, int, hipStream_t); \
   template void launch_rglru_scan<T>(T*, const T*, const T*, const T*,          \
                                      const float*, const float*, const float*,  \
                                      float, const T*, float*, const int*,       \

@@ -1284,7 +1284,7 @@ class SpanAttention(_Mixer):
             if self.pool:
                 ops.pool_cache_write(k_cache, v_cache, k_pool, v_pool, self.pool,
                                      meta.prefill_block_tables, meta.prefill_query_start_loc,
-                                     meta.prefill_seq_lens)
+                                     meta.prefill_seq_lens, npt)
             ops.span_attention_prefill(
                 q[:npt], k_cache, v_cache, k_pool, v_pool, meta.prefill_block_tables,
                 meta.prefill_query_start_loc, meta.prefill_seq_lens, self.scale,
@@ -1293,7 +1293,8 @@ class SpanAttention(_Mixer):
         if meta.num_decode_seqs:
             if self.pool:
                 ops.pool_cache_write(k_cache, v_cache, k_pool, v_pool, self.pool,
-                                     meta.decode_block_tables, None, meta.decode_seq_lens)
+                                     meta.decode_block_tables, None, meta.decode_seq_lens,
+                                     t - npt)
             ops.span_attention_decode(
                 q[npt:], k_cache, v_cache, k_pool, v_pool, meta.decode_block_tables,
                 meta.decode_seq_lens, self.scale, self.window, self.keep_first, self.pool,

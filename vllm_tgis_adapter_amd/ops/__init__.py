@@ -1284,15 +1284,15 @@ pool_slots_per_block = reference.pool_slots_per_block
 
 
 def pool_cache_write(k_cache, v_cache, k_pool, v_pool, pool: int, block_tables,
-                     query_start_loc, seq_lens) -> None:
+                     query_start_loc, seq_lens, rows: int) -> None:
     """Means of every block of ``pool`` consecutive cached keys / values that
-    this step's rows complete (the tail of each sequence; ``query_start_loc``
-    None: one row each).  Pooled block b is kept in the cache block that holds
+    this step's ``rows`` rows complete (the tail of each sequence;
+    ``query_start_loc`` None: one row each).  Pooled block b is kept in the cache block that holds
     its last token: k_pool [blocks, slots, G, dim], v_pool [.., vdim], slots =
     pool_slots_per_block."""
     if k_cache.device.type == "cuda" and seq_lens.numel() and _native_seq(k_cache):
         _S.pool_cache_write(k_cache, v_cache, k_pool, v_pool, int(pool), block_tables,
-                            query_start_loc, seq_lens)
+                            query_start_loc, seq_lens, int(rows))
         return
     if query_start_loc is None:
         query_start_loc = torch.arange(seq_lens.numel() + 1, dtype=torch.int32)
