@@ -48,7 +48,19 @@ DEVINLINE bf16x8_t load_kv8<unsigned char>(const unsigned char* p) {
 // CH (chunk variant, on top of WS): the query sees the keys of its own chunk
 // of `chunk` positions only; the value cache holds v_heads <= kvh heads and
 // key head g reads value head g mod v_heads.
-template <int HEAD_DIM, typename CT, bool WS, bool CH = false>
+// PX (prefix variants, on top of WS): keys ahead of the window, in tiles of
+// their own before the window's tiles.  PX_KEEP: the sequence's first `keep`
+// tokens.  PX_POOL: one pooled key and value per block of `pool` positions that
+// ends at or before seq_len - 1 - window; pooled block b is kept in the cache
+// block that holds its last token (per_block places each).
+enum { PX_NONE = 0, PX_KEEP = 1, PX_POOL = 2 };
+struct SpanKeys {
+  int keep, pool, per_block;
+  const __hip_bfloat16* k_pool;
+  const __hip_bfloat16* v_pool;
+};
+
+template <int HEAD_DIM, typename CT, bool WS, bool CH = false, int PX = PX_NONE>
 __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
     float* __restrict__ part_acc,   // [nseq, nheads, P, HEAD_DIM] f32
     float* __restrict__ part_ml,    // [nseq, nheads, P, 2] f32 (m, l)
@@ -65,8 +77,10 @@ __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
     const int max_blocks,
     const int window,
     const int chunk = 0,
-    const int v_heads = 0) {
+    const int v_heads = 0,
+    const SpanKeys sp = SpanKeys{}) {
   static_assert(!CH || WS, "the chunk variant builds on the window variant");
+  static_assert(PX == PX_NONE || (WS && !CH), "prefixes build on the window variant");
   constexpr int KCH = HEAD_DIM / 16;  // k-chunks for the QK^T mfma
   constexpr int DT = HEAD_DIM / 32;   // 32-col output tiles
 
@@ -87,9 +101,15 @@ __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
   const int first_pos = (CH && chunk > 0) ? max(0, seq_len - 1) / chunk * chunk
                         : (WS && window > 0) ? max(0, seq_len - window) : 0;
   const int tile_first = first_pos / KVT;
-  const int tpp = (tiles_total - tile_first + npart - 1) / npart;
-  const int tile_lo = tile_first + part * tpp;
-  const int tile_hi = min(tile_lo + tpp, tiles_total);
+  // prefix tiles come first in this workgroup range's numbering
+  int pre_len = 0;
+  if (PX == PX_KEEP) pre_len = min(sp.keep, first_pos);
+  if (PX == PX_POOL) pre_len = max(0, seq_len - window) / sp.pool;
+  const int pre_tiles = PX == PX_NONE ? 0 : (pre_len + KVT - 1) / KVT;
+  const int shift = tile_first - pre_tiles;   // window tile = numbered tile + shift
+  const int tpp = (tiles_total - shift + npart - 1) / npart;
+  const int tile_lo = (PX == PX_NONE ? tile_first : 0) + part * tpp;
+  const int tile_hi = min(tile_lo + tpp, PX == PX_NONE ? tiles_total : tiles_total - shift);
 
   const int head0 = kv_head * group;
   const int* btable = block_tables + (long)seq * max_blocks;
@@ -122,7 +142,23 @@ __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
   constexpr int VPASS = KVT * HEAD_DIM / 8 / 64;  // V staging passes per wave
 
   for (int t = tile_lo + wave; t < tile_hi; t += NWAVES) {
-    const int kv_base = t * KVT;
+    const bool prefix = PX != PX_NONE && t < pre_tiles;
+    const int kv_base = (PX == PX_NONE || prefix ? t : t + shift) * KVT;
+    const int limit = prefix ? pre_len : seq_len;
+    // cached row of key kv_base + s, in the token or the pooled cache
+    auto row_of = [&](int pos) {
+      if (PX == PX_POOL && prefix) {
+        const int page = (pos * sp.pool + sp.pool - 1) / block_size;
+        return (long)btable[page] * sp.per_block + (pos - page * block_size / sp.pool);
+      }
+      const int block = btable[pos / block_size];
+      return (long)block * block_size + pos % block_size;
+    };
+    const CT* k_src = k_cache;
+    const CT* v_src = v_cache;
+    if constexpr (PX == PX_POOL) {
+      if (prefix) { k_src = sp.k_pool; v_src = sp.v_pool; }
+    }
 
     // ---- issue ALL of this tile's HBM loads first (K frags + V rows) -----
     // K is needed first (QK^T mfma), so its 8 loads go out before V's; the
@@ -133,11 +169,8 @@ __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
     bf16x8_t ka[KCH];
     {
       const int pos = kv_base + col;
-      if (pos < seq_len) {
-        const int block = btable[pos / block_size];
-        const CT* k_row =
-            k_cache + ((long)block * block_size + pos % block_size) * kv_row_stride +
-            (long)kv_head * HEAD_DIM;
+      if (pos < limit) {
+        const CT* k_row = k_src + row_of(pos) * kv_row_stride + (long)kv_head * HEAD_DIM;
 #pragma unroll
         for (int ks = 0; ks < KCH; ++ks)
           ka[ks] = load_kv8<CT>(k_row + ks * 16 + half * 8);
@@ -157,12 +190,9 @@ __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
         const int s = pass * ROWS_PER_PASS + r_in_pass;
         const int pos = kv_base + s;
         vv[pass] = bf16x8_t{};
-        if (pos < seq_len) {
-          const int block = btable[pos / block_size];
-          const long row = ((long)block * block_size + pos % block_size) *
-                               v_row_stride +
-                           (long)v_head * HEAD_DIM + d8;
-          vv[pass] = load_kv8<CT>(v_cache + row);
+        if (pos < limit) {
+          const long row = row_of(pos) * v_row_stride + (long)v_head * HEAD_DIM + d8;
+          vv[pass] = load_kv8<CT>(v_src + row);
         }
       }
 #pragma unroll
@@ -185,7 +215,7 @@ __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
     for (int r = 0; r < 16; ++r) {
       const int kv_pos = kv_base + (r & 3) + 8 * (r >> 2) + 4 * half;
       float sv = acc_s[r] * scale;
-      if (kv_pos >= seq_len || (WS && kv_pos < first_pos)) sv = -FLT_MAX;
+      if (kv_pos >= limit || (WS && !prefix && kv_pos < first_pos)) sv = -FLT_MAX;
       s_val[r] = sv;
       local_max = fmaxf(local_max, sv);
     }
@@ -285,7 +315,9 @@ __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
 }
 
 // Reduce the P partials of each (seq, head) row: out = sum_p f_p acc_p / sum_p f_p l_p
-template <int HEAD_DIM, typename OT = __hip_bfloat16>
+// back (cos, sin per row and pair, or null): dims m and m + HEAD_DIM/2 are turned
+// back by the row's angles before the rounding.
+template <int HEAD_DIM, typename OT = __hip_bfloat16, bool BACK = false>
 __global__ void decode_merge_kernel(
     OT* __restrict__ out,                  // [nseq, nheads, HD]
     const float* __restrict__ part_acc,    // [nseq, nheads, P, HD]
@@ -293,7 +325,8 @@ __global__ void decode_merge_kernel(
     const int nheads,
     const int P,
     const int has_sink,
-    const float sink) {
+    const float sink,
+    const float2* __restrict__ back = nullptr) {
   const int seq = blockIdx.x;
   const int head = blockIdx.y;
   const int d = threadIdx.x;
@@ -314,6 +347,14 @@ __global__ void decode_merge_kernel(
     A += f * acc[(long)p * HEAD_DIM];
   }
   const float inv = L > 0.f ? 1.f / L : 0.f;
+  if constexpr (BACK) {
+    __shared__ float turned[HEAD_DIM];
+    turned[d] = A;
+    __syncthreads();
+    const float2 cs = back[(long)seq * (HEAD_DIM / 2) + d % (HEAD_DIM / 2)];
+    A = d < HEAD_DIM / 2 ? A * cs.x + turned[d + HEAD_DIM / 2] * cs.y
+                         : A * cs.x - turned[d - HEAD_DIM / 2] * cs.y;
+  }
   if constexpr (sizeof(OT) == 4)
     out[row * HEAD_DIM + d] = A * inv;
   else
@@ -352,15 +393,15 @@ static void launch_decode_ct(__hip_bfloat16* out, float* part_acc,
         hipLaunchKernelGGL((paged_decode_mfma_kernel<64, CT, true>), grid, block, 0,
                            stream, part_acc, part_ml, q, kc, vc, bt, sl, scale,
                            nheads, kvh, group, block_size, max_blocks, window);
-        hipLaunchKernelGGL(decode_merge_kernel<64>, mgrid, dim3(64), 0, stream,
-                           out, part_acc, part_ml, nheads, P, has_sink, sink);
+        hipLaunchKernelGGL((decode_merge_kernel<64>), mgrid, dim3(64), 0, stream,
+                           out, part_acc, part_ml, nheads, P, has_sink, sink, nullptr);
         break;
       case 128:
         hipLaunchKernelGGL((paged_decode_mfma_kernel<128, CT, true>), grid, block, 0,
                            stream, part_acc, part_ml, q, kc, vc, bt, sl, scale,
                            nheads, kvh, group, block_size, max_blocks, window);
-        hipLaunchKernelGGL(decode_merge_kernel<128>, mgrid, dim3(128), 0, stream,
-                           out, part_acc, part_ml, nheads, P, has_sink, sink);
+        hipLaunchKernelGGL((decode_merge_kernel<128>), mgrid, dim3(128), 0, stream,
+                           out, part_acc, part_ml, nheads, P, has_sink, sink, nullptr);
         break;
       default:
         abort();
@@ -372,15 +413,15 @@ static void launch_decode_ct(__hip_bfloat16* out, float* part_acc,
       hipLaunchKernelGGL((paged_decode_mfma_kernel<64, CT, false>), grid, block, 0,
                          stream, part_acc, part_ml, q, kc, vc, bt, sl, scale,
                          nheads, kvh, group, block_size, max_blocks, 0);
-      hipLaunchKernelGGL(decode_merge_kernel<64>, mgrid, dim3(64), 0, stream,
-                         out, part_acc, part_ml, nheads, P, 0, 0.f);
+      hipLaunchKernelGGL((decode_merge_kernel<64>), mgrid, dim3(64), 0, stream,
+                         out, part_acc, part_ml, nheads, P, 0, 0.f, nullptr);
       break;
     case 128:
       hipLaunchKernelGGL((paged_decode_mfma_kernel<128, CT, false>), grid, block, 0,
                          stream, part_acc, part_ml, q, kc, vc, bt, sl, scale,
                          nheads, kvh, group, block_size, max_blocks, 0);
-      hipLaunchKernelGGL(decode_merge_kernel<128>, mgrid, dim3(128), 0, stream,
-                         out, part_acc, part_ml, nheads, P, 0, 0.f);
+      hipLaunchKernelGGL((decode_merge_kernel<128>), mgrid, dim3(128), 0, stream,
+                         out, part_acc, part_ml, nheads, P, 0, 0.f, nullptr);
       break;
     default:
       abort();
@@ -445,7 +486,7 @@ void launch_paged_decode_mfma_chunk(float* out, float* part_acc, float* part_ml,
           0, stream, part_acc, part_ml, q, kc, vc, bt, sl, scale, nheads, kvh, group,
           block_size, max_blocks, 0, chunk, v_heads);
       hipLaunchKernelGGL((decode_merge_kernel<64, float>), mgrid, dim3(64), 0, stream,
-                         out, part_acc, part_ml, nheads, P, 0, 0.f);
+                         out, part_acc, part_ml, nheads, P, 0, 0.f, nullptr);
       break;
     case 128:
       hipLaunchKernelGGL(
@@ -453,9 +494,58 @@ void launch_paged_decode_mfma_chunk(float* out, float* part_acc, float* part_ml,
           dim3(256), 0, stream, part_acc, part_ml, q, kc, vc, bt, sl, scale, nheads,
           kvh, group, block_size, max_blocks, 0, chunk, v_heads);
       hipLaunchKernelGGL((decode_merge_kernel<128, float>), mgrid, dim3(128), 0,
-                         stream, out, part_acc, part_ml, nheads, P, 0, 0.f);
+                         stream, out, part_acc, part_ml, nheads, P, 0, 0.f, nullptr);
       break;
     default:
       abort();
   }
+}
+
+// window plus a prefix of first tokens or pooled blocks (bf16 cache)
+template <int HD>
+static void launch_decode_span(__hip_bfloat16* out, float* part_acc, float* part_ml,
+                               const __hip_bfloat16* q, const __hip_bfloat16* kc,
+                               const __hip_bfloat16* vc, const int* bt, const int* sl,
+                               float scale, int nseq, int nheads, int kvh, int block_size,
+                               int max_blocks, int npart, int window, const SpanKeys& sp,
+                               const float2* back, hipStream_t stream) {
+  const int group = nheads / kvh;
+  const dim3 grid(nseq, kvh, npart), mgrid(nseq, nheads);
+  const int P = npart * NWAVES;
+  if (sp.pool > 0)
+    hipLaunchKernelGGL((paged_decode_mfma_kernel<HD, __hip_bfloat16, true, false, PX_POOL>),
+                       grid, dim3(256), 0, stream, part_acc, part_ml, q, kc, vc, bt, sl,
+                       scale, nheads, kvh, group, block_size, max_blocks, window, 0, 0, sp);
+  else
+    hipLaunchKernelGGL((paged_decode_mfma_kernel<HD, __hip_bfloat16, true, false, PX_KEEP>),
+                       grid, dim3(256), 0, stream, part_acc, part_ml, q, kc, vc, bt, sl,
+                       scale, nheads, kvh, group, block_size, max_blocks, window, 0, 0, sp);
+  if (back != nullptr)
+    hipLaunchKernelGGL((decode_merge_kernel<HD, __hip_bfloat16, true>), mgrid, dim3(HD), 0,
+                       stream, out, part_acc, part_ml, nheads, P, 0, 0.f, back);
+  else
+    hipLaunchKernelGGL((decode_merge_kernel<HD>), mgrid, dim3(HD), 0, stream, out, part_acc,
+                       part_ml, nheads, P, 0, 0.f, nullptr);
+}
+
+void launch_paged_decode_mfma_span(__hip_bfloat16* out, float* part_acc, float* part_ml,
+                                   const __hip_bfloat16* q, const __hip_bfloat16* kc,
+                                   const __hip_bfloat16* vc, const __hip_bfloat16* kp,
+                                   const __hip_bfloat16* vp, const int* bt, const int* sl,
+                                   float scale, int nseq, int nheads, int kvh,
+                                   int head_dim, int block_size, int per_block,
+                                   int max_blocks, int npart, int window, int keep,
+                                   int pool, const float* back, hipStream_t stream) {
+  SpanKeys sp;
+  sp.keep = keep; sp.pool = pool; sp.per_block = per_block;
+  sp.k_pool = kp; sp.v_pool = vp;
+  const float2* b2 = reinterpret_cast<const float2*>(back);
+  if (head_dim == 64)
+    launch_decode_span<64>(out, part_acc, part_ml, q, kc, vc, bt, sl, scale, nseq, nheads,
+                           kvh, block_size, max_blocks, npart, window, sp, b2, stream);
+  else if (head_dim == 128)
+    launch_decode_span<128>(out, part_acc, part_ml, q, kc, vc, bt, sl, scale, nseq, nheads,
+                            kvh, block_size, max_blocks, npart, window, sp, b2, stream);
+  else
+    abort();
 }

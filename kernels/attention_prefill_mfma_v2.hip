@@ -67,8 +67,23 @@ __device__ inline float cross_half_sum(float v) {
 // keys j <= i of its own chunk only, floor(j / chunk) = floor(i / chunk); the
 // value cache holds v_heads <= kvh heads and key head g reads value head
 // g mod v_heads; the output is f32.
+// PX (prefix variants, on top of WS without a sink): keys ahead of the window,
+// in tiles of their own before the window's tiles.  PX_KEEP: the sequence's
+// first `keep` tokens.  PX_POOL: one pooled key and value per block of `pool`
+// positions that ends at or before i - window; pooled block b is kept in the
+// cache block that holds its last token (per_block places each).  back (cos,
+// sin per query row and pair): the output's dims m and m + HEAD_DIM/2 are turned
+// back by the row's angles before they are rounded.
+enum { PX_NONE = 0, PX_KEEP = 1, PX_POOL = 2 };
+struct SpanTiles {
+  int keep, pool, per_block;
+  const __hip_bfloat16* k_pool;
+  const __hip_bfloat16* v_pool;
+  const float2* back;
+};
+
 template <int HEAD_DIM, typename CT, int NW, bool WS, bool CH = false,
-          typename OT = __hip_bfloat16>
+          typename OT = __hip_bfloat16, int PX = PX_NONE>
 __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v2_kernel(
     OT* __restrict__ out,                        // [total_q, nheads, HD]
     const __hip_bfloat16* __restrict__ q,        // [total_q, nheads, HD]
@@ -86,8 +101,10 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
     const int has_sink,
     const float sink,
     const int chunk = 0,
-    const int v_heads = 0) {
+    const int v_heads = 0,
+    const SpanTiles sp = SpanTiles{}) {
   static_assert(HEAD_DIM == 128, "v2 is specialised for HD=128");
+  static_assert(PX == PX_NONE || (WS && !CH), "prefixes build on the window variant");
   static_assert(!CH || WS, "the chunk variant builds on the window variant");
   constexpr int KCH = HEAD_DIM / 16;  // QK^T k-chunks (8)
   constexpr int DT = HEAD_DIM / 32;   // 32-col output tiles (4)
@@ -166,20 +183,49 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
     wave_win_lo = wave_q_pos_min / chunk * chunk;
   }
 
+  // prefix: its length for the whole workgroup, its tiles (all keys of a kept
+  // prefix lie before kv_first, so no key is met twice), and how much of it the
+  // first and the last row of this wave see
+  int pre_len = 0, pre_lo = 0, pre_hi = 0;
+  if (PX == PX_KEEP) pre_len = pre_lo = pre_hi = min(sp.keep, kv_first);
+  if (PX == PX_POOL) {
+    pre_len = max(0, wg_max_pos + 1 - window) / sp.pool;
+    pre_lo = max(0, wave_q_pos_min + 1 - window) / sp.pool;
+    pre_hi = max(0, wave_max_pos + 1 - window) / sp.pool;
+  }
+  const int pre_tiles = PX == PX_NONE ? 0 : (pre_len + KVT2 - 1) / KVT2;
+  const int q_pre = PX == PX_POOL ? max(0, q_pos + 1 - window) / sp.pool : pre_len;
+  const int num_tiles = pre_tiles + (kv_limit - kv_first + KVT2 - 1) / KVT2;
+  auto tile_pos = [&](int it) {
+    return PX != PX_NONE && it < pre_tiles ? it * KVT2
+                                           : kv_first + (it - pre_tiles) * KVT2;
+  };
+
   // ---- staging map: thread t covers slot (t % ROWS_PER_PASS, t / RPP * 8)
   // with ROWS_PER_PASS = NTHREADS/16 rows per pass (16 8-elem slots per row)
   constexpr int RPP = NTHREADS / 16;
   const int st_s = tid % RPP;
   const int st_d8 = (tid / RPP) * 8;
   bf16x8_t st_k[ST_PASS], st_v[ST_PASS];
-  auto stage_load = [&](int kv_base) {
+  auto stage_load = [&](int kv_base, bool prefix) {
+    const int limit = PX != PX_NONE && prefix ? pre_len : kv_limit;
 #pragma unroll
     for (int pass = 0; pass < ST_PASS; ++pass) {
       const int s = st_s + pass * RPP;
       const int pos = kv_base + s;
       st_k[pass] = bf16x8_t{};
       st_v[pass] = bf16x8_t{};
-      if (pos < kv_limit) {
+      if (pos < limit) {
+        if (PX == PX_POOL && prefix) {
+          const int page = (pos * sp.pool + sp.pool - 1) / block_size;
+          const long at = (long)btable[page] * sp.per_block +
+                          (pos - page * block_size / sp.pool);
+          st_k[pass] = load_kv8_v2<__hip_bfloat16>(sp.k_pool + at * kv_row_stride +
+                                                   (long)kv_head * HEAD_DIM + st_d8);
+          st_v[pass] = load_kv8_v2<__hip_bfloat16>(sp.v_pool + at * kv_row_stride +
+                                                   (long)kv_head * HEAD_DIM + st_d8);
+          continue;
+        }
         const int block = btable[pos / block_size];
         const long tok = (long)block * block_size + pos % block_size;
         st_k[pass] = load_kv8_v2<CT>(k_cache + tok * kv_row_stride +
@@ -202,20 +248,25 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
     }
   };
 
-  stage_load(kv_first);
-  stage_write((kv_first / KVT2) & 1);
+  stage_load(tile_pos(0), PX != PX_NONE && pre_tiles > 0);
+  stage_write(0);
 
   const float sc2 = scale * LOG2E;  // fold softmax scale into exp2 domain
 
-  for (int kv_base = kv_first; kv_base < kv_limit; kv_base += KVT2) {
-    const int buf = (kv_base / KVT2) & 1;
+  for (int it = 0; it < num_tiles; ++it) {
+    const int kv_base = tile_pos(it);
+    const bool prefix = PX != PX_NONE && it < pre_tiles;
+    const int buf = it & 1;
     __syncthreads();  // publish tile (kv_base) to all waves
 
     // wave-uniform: MFMAs must run with a full EXEC mask — a per-lane guard
     // here drops the masked lanes' K fragments from the score MFMA
     const bool wave_active =
-        (tile_base + wave * 32 < q_len) && (kv_base <= wave_max_pos) &&
-        (!WS || kv_base + KVT2 > wave_win_lo);
+        (tile_base + wave * 32 < q_len) &&
+        (prefix ? kv_base < pre_hi
+                : (kv_base <= wave_max_pos) &&
+                      (!WS || kv_base + KVT2 > wave_win_lo ||
+                       (PX == PX_KEEP && kv_base < sp.keep)));
     const char* k_lds = reinterpret_cast<const char*>(k_lds2[buf]);
     const char* v_lds = v_lds2[buf];
 
@@ -238,21 +289,23 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
     }
 
     // ---- async stage: issue next tile's HBM loads now ------------------
-    const int next_base = kv_base + KVT2;
-    if (next_base < kv_limit) stage_load(next_base);
+    const bool more = it + 1 < num_tiles;
+    if (more) stage_load(tile_pos(it + 1), PX != PX_NONE && it + 1 < pre_tiles);
 
     if (wave_active) {
       // ---- online softmax; the running max m2_state lives in the RAW
       // score domain (sc2 > 0 commutes with max), so the P pass is one
       // fma + exp2 per element: p = exp2(acc*sc2 - m*sc2).
       // fast path: tile strictly below every row's causal diagonal
-      const bool full_tile = (kv_base + KVT2 - 1 <= wave_q_pos_min) &&
-                             (kv_base + KVT2 <= seq_len) &&
-                             (tile_base + wave * 32 + 31 < q_len) &&
-                             (!WS || window == 0 ||
-                              kv_base > wave_q_pos_min + 31 - window) &&
-                             (!CH || chunk == 0 ||
-                              kv_base >= (wave_q_pos_min + 31) / chunk * chunk);
+      const bool full_tile =
+          (tile_base + wave * 32 + 31 < q_len) &&
+          (prefix ? kv_base + KVT2 <= pre_lo
+                  : (kv_base + KVT2 - 1 <= wave_q_pos_min) &&
+                        (kv_base + KVT2 <= seq_len) &&
+                        (!WS || window == 0 ||
+                         kv_base > wave_q_pos_min + 31 - window) &&
+                        (!CH || chunk == 0 ||
+                         kv_base >= (wave_q_pos_min + 31) / chunk * chunk));
       float local_max = -FLT_MAX;
       if (full_tile) {
 #pragma unroll
@@ -268,10 +321,13 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
             const int kv_pos =
                 kv_base + kb * 32 + (r & 3) + 8 * (r >> 2) + 4 * half;
             float v = acc_s[kb][r];
-            if (!q_valid || kv_pos > q_pos || kv_pos >= seq_len ||
-                (WS && window > 0 && kv_pos + window <= q_pos) ||
-                (CH && kv_pos < q_lo))
-              v = -FLT_MAX;
+            const bool hidden =
+                prefix ? kv_pos >= q_pre
+                       : kv_pos > q_pos || kv_pos >= seq_len ||
+                             (WS && window > 0 && kv_pos + window <= q_pos &&
+                              (PX != PX_KEEP || kv_pos >= sp.keep)) ||
+                             (CH && kv_pos < q_lo);
+            if (!q_valid || hidden) v = -FLT_MAX;
             acc_s[kb][r] = v;
             local_max = fmaxf(local_max, v);
           }
@@ -385,7 +441,7 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
     }
 
     // ---- write next tile into the other buffer -------------------------
-    if (next_base < kv_limit) stage_write(buf ^ 1);
+    if (more) stage_write(buf ^ 1);
   }
 
   // ---- epilogue: normalize and store -----------------------------------
@@ -410,6 +466,16 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
     const int q_local = tile_base + wave * 32 + qrow;
     if (q_local >= q_len) continue;
     OT* out_row = out + ((long)(q_start + q_local) * nheads + head) * HEAD_DIM;
+    if (PX != PX_NONE && sp.back != nullptr) {
+      const float2* tab = sp.back + (long)(q_start + q_local) * (HEAD_DIM / 2);
+#pragma unroll
+      for (int dt = 0; dt < DT / 2; ++dt) {
+        const float2 cs = tab[dt * 32 + col];
+        const float a = acc_o[dt][r], b = acc_o[dt + DT / 2][r];
+        acc_o[dt][r] = a * cs.x + b * cs.y;
+        acc_o[dt + DT / 2][r] = b * cs.x - a * cs.y;
+      }
+    }
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
       if constexpr (CH)
@@ -504,4 +570,28 @@ void launch_paged_prefill_mfma_v2_chunk(
       (paged_prefill_mfma_v2_kernel<128, __hip_bfloat16, 8, true, true, float>),
       dim3(nseq, nheads, qtiles), dim3(512), 0, stream, out, q, kc, vc, bt, qsl,
       sl, scale, nheads, kvh, block_size, max_blocks, 0, 0, 0.f, chunk, v_heads);
+}
+
+// window plus a prefix of first tokens or pooled blocks (bf16 cache, HD = 128)
+void launch_paged_prefill_mfma_v2_span(
+    __hip_bfloat16* out, const __hip_bfloat16* q, const __hip_bfloat16* kc,
+    const __hip_bfloat16* vc, const __hip_bfloat16* kp, const __hip_bfloat16* vp,
+    const int* bt, const int* qsl, const int* sl, float scale, int nseq, int nheads,
+    int kvh, int block_size, int per_block, int max_blocks, int max_query_len,
+    int window, int keep, int pool, const float* back, hipStream_t stream) {
+  const dim3 grid(nseq, nheads, (max_query_len + 255) / 256);
+  SpanTiles sp;
+  sp.keep = keep; sp.pool = pool; sp.per_block = per_block;
+  sp.k_pool = kp; sp.v_pool = vp;
+  sp.back = reinterpret_cast<const float2*>(back);
+  if (pool > 0)
+    hipLaunchKernelGGL((paged_prefill_mfma_v2_kernel<128, __hip_bfloat16, 8, true, false,
+                                                     __hip_bfloat16, PX_POOL>),
+                       grid, dim3(512), 0, stream, out, q, kc, vc, bt, qsl, sl, scale,
+                       nheads, kvh, block_size, max_blocks, window, 0, 0.f, 0, 0, sp);
+  else
+    hipLaunchKernelGGL((paged_prefill_mfma_v2_kernel<128, __hip_bfloat16, 8, true, false,
+                                                     __hip_bfloat16, PX_KEEP>),
+                       grid, dim3(512), 0, stream, out, q, kc, vc, bt, qsl, sl, scale,
+                       nheads, kvh, block_size, max_blocks, window, 0, 0.f, 0, 0, sp);
 }

@@ -57,6 +57,18 @@ void launch_paged_decode_mfma_chunk(float*, float*, float*, const __hip_bfloat16
                                     const __hip_bfloat16*, const __hip_bfloat16*,
                                     const int*, const int*, float, int, int, int,
                                     int, int, int, int, int, int, hipStream_t);
+void launch_paged_prefill_mfma_v2_span(__hip_bfloat16*, const __hip_bfloat16*,
+                                       const __hip_bfloat16*, const __hip_bfloat16*,
+                                       const __hip_bfloat16*, const __hip_bfloat16*,
+                                       const int*, const int*, const int*, float, int,
+                                       int, int, int, int, int, int, int, int, int,
+                                       const float*, hipStream_t);
+void launch_paged_decode_mfma_span(__hip_bfloat16*, float*, float*, const __hip_bfloat16*,
+                                   const __hip_bfloat16*, const __hip_bfloat16*,
+                                   const __hip_bfloat16*, const __hip_bfloat16*,
+                                   const int*, const int*, float, int, int, int, int, int,
+                                   int, int, int, int, int, int, const float*,
+                                   hipStream_t);
 void launch_paged_decode_mfma_ws(__hip_bfloat16*, float*, float*,
                                  const __hip_bfloat16*, const __hip_bfloat16*,
                                  const __hip_bfloat16*, const int*, const int*,
@@ -396,9 +408,112 @@ void chunk_attention_decode(torch::Tensor out, torch::Tensor q, torch::Tensor k_
       (int)chunk, current_stream());
 }
 
+// Prefix variants of the bf16 MFMA kernels: a window (> 0) and, beside it, the
+// first `keep` tokens or one pooled key and value per block of `pool` positions
+// that ends at or before the window (pooled block b lives in the cache block of
+// its last token).  back_table [rows, dim/2, 2] f32: the output's dims m and
+// m + dim/2 are turned back by the row's angles.  Sizes as for the window
+// variants.  Returns the places per cache block.
+int check_span(const torch::Tensor& out, const torch::Tensor& q,
+               const torch::Tensor& k_cache, const torch::Tensor& v_cache,
+               const c10::optional<torch::Tensor>& k_pool,
+               const c10::optional<torch::Tensor>& v_pool,
+               const torch::Tensor& block_tables, const torch::Tensor& seq_lens,
+               int64_t window, int64_t keep, int64_t pool,
+               const c10::optional<torch::Tensor>& back) {
+  check_windowed(out, q, k_cache, v_cache, block_tables, seq_lens, window);
+  TORCH_CHECK(window > 0 && keep >= 0 && pool >= 0 && !(keep && pool), "mask");
+  if (back.has_value()) {
+    const auto& b = back.value();
+    TORCH_CHECK(b.is_cuda() && b.is_contiguous() &&
+                b.scalar_type() == at::ScalarType::Float &&
+                b.numel() == q.size(0) * q.size(2), "back_table is [rows, dim / 2, 2]");
+  }
+  if (pool == 0) return 0;
+  TORCH_CHECK(k_pool.has_value() && v_pool.has_value(), "pooled caches missing");
+  const auto &kp = k_pool.value(), &vp = v_pool.value();
+  const int64_t per_block = (k_cache.size(1) + pool - 1) / pool;
+  TORCH_CHECK(kp.is_cuda() && kp.is_contiguous() && vp.is_cuda() && vp.is_contiguous() &&
+              kp.scalar_type() == at::ScalarType::BFloat16 &&
+              vp.scalar_type() == at::ScalarType::BFloat16 && kp.dim() == 4 &&
+              kp.sizes() == vp.sizes() && kp.size(0) == k_cache.size(0) &&
+              kp.size(1) == per_block && kp.size(2) == k_cache.size(2) &&
+              kp.size(3) == k_cache.size(3), "pooled caches do not fit the caches");
+  return (int)per_block;
+}
+
+const __hip_bfloat16* bf16_or_null(const c10::optional<torch::Tensor>& t) {
+  return t.has_value() ? reinterpret_cast<const __hip_bfloat16*>(t.value().data_ptr())
+                       : nullptr;
+}
+
+void span_attention_prefill(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
+                            torch::Tensor v_cache, c10::optional<torch::Tensor> k_pool,
+                            c10::optional<torch::Tensor> v_pool,
+                            torch::Tensor block_tables, torch::Tensor query_start_loc,
+                            torch::Tensor seq_lens, double scale, int64_t max_query_len,
+                            int64_t window, int64_t keep, int64_t pool,
+                            c10::optional<torch::Tensor> back) {
+  const int per_block = check_span(out, q, k_cache, v_cache, k_pool, v_pool, block_tables,
+                                   seq_lens, window, keep, pool, back);
+  TORCH_CHECK(q.size(2) == 128, "prompt portions need key size 128");
+  const int nseq = seq_lens.numel();
+  TORCH_CHECK(query_start_loc.is_cuda() && query_start_loc.is_contiguous() &&
+              query_start_loc.scalar_type() == at::ScalarType::Int &&
+              query_start_loc.numel() == nseq + 1 && max_query_len >= 1);
+  if (q.size(0) == 0 || nseq == 0) return;
+  launch_paged_prefill_mfma_v2_span(
+      reinterpret_cast<__hip_bfloat16*>(out.data_ptr()),
+      reinterpret_cast<const __hip_bfloat16*>(q.data_ptr()),
+      reinterpret_cast<const __hip_bfloat16*>(k_cache.data_ptr()),
+      reinterpret_cast<const __hip_bfloat16*>(v_cache.data_ptr()), bf16_or_null(k_pool),
+      bf16_or_null(v_pool), block_tables.data_ptr<int>(), query_start_loc.data_ptr<int>(),
+      seq_lens.data_ptr<int>(), (float)scale, nseq, (int)q.size(1), (int)k_cache.size(2),
+      (int)k_cache.size(1), per_block, (int)block_tables.size(1), (int)max_query_len,
+      (int)window, (int)keep, (int)pool,
+      back.has_value() ? back.value().data_ptr<float>() : nullptr, current_stream());
+}
+
+void span_attention_decode(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
+                           torch::Tensor v_cache, c10::optional<torch::Tensor> k_pool,
+                           c10::optional<torch::Tensor> v_pool, torch::Tensor block_tables,
+                           torch::Tensor seq_lens, double scale, int64_t window,
+                           int64_t keep, int64_t pool, c10::optional<torch::Tensor> back) {
+  const int per_block = check_span(out, q, k_cache, v_cache, k_pool, v_pool, block_tables,
+                                   seq_lens, window, keep, pool, back);
+  const int nseq = q.size(0), nheads = q.size(1), head_dim = q.size(2);
+  TORCH_CHECK(head_dim == 64 || head_dim == 128, "key size 64 or 128");
+  TORCH_CHECK(seq_lens.numel() == nseq, "one query row per sequence expected");
+  if (nseq == 0) return;
+  const int kvh = k_cache.size(2), block_size = k_cache.size(1);
+  const int max_blocks = block_tables.size(1);
+  // shape-pure split count: window and prefix bound the keys a query reads
+  const int64_t ctx = (int64_t)max_blocks * block_size;
+  const int64_t span = std::min(ctx, window + 32) +
+                       (pool > 0 ? ctx / pool + 32 : std::min(ctx, keep + 32));
+  const int npart = decode_mfma_num_partitions(nseq, kvh, (int)span);
+  const int P = npart * 4;
+  auto opts = q.options().dtype(at::ScalarType::Float);
+  auto part_acc = at::empty({nseq, nheads, P, head_dim}, opts);
+  auto part_ml = at::empty({nseq, nheads, P, 2}, opts);
+  launch_paged_decode_mfma_span(
+      reinterpret_cast<__hip_bfloat16*>(out.data_ptr()), part_acc.data_ptr<float>(),
+      part_ml.data_ptr<float>(), reinterpret_cast<const __hip_bfloat16*>(q.data_ptr()),
+      reinterpret_cast<const __hip_bfloat16*>(k_cache.data_ptr()),
+      reinterpret_cast<const __hip_bfloat16*>(v_cache.data_ptr()), bf16_or_null(k_pool),
+      bf16_or_null(v_pool), block_tables.data_ptr<int>(), seq_lens.data_ptr<int>(),
+      (float)scale, nseq, nheads, kvh, head_dim, block_size, per_block, max_blocks, npart,
+      (int)window, (int)keep, (int)pool,
+      back.has_value() ? back.value().data_ptr<float>() : nullptr, current_stream());
+}
+
 }  // namespace
 
 void register_attention_ops(pybind11::module& m) {
+  m.def("span_attention_prefill", &span_attention_prefill,
+        "paged prefill attention over a window plus a prefix (CDNA4)");
+  m.def("span_attention_decode", &span_attention_decode,
+        "paged decode attention over a window plus a prefix (CDNA4)");
   m.def("chunk_attention_prefill", &chunk_attention_prefill,
         "paged chunk-masked prefill attention, f32 out (CDNA4)");
   m.def("chunk_attention_decode", &chunk_attention_decode,

@@ -1,0 +1,700 @@
+"""Balenex through the engine against the plain oracle (tests/balenex_oracle.py).
+
+Every test builds its own small configuration with random weights.  CPU runs
+use the reference ops, GPU runs (marked) the HIP kernels; both go through the
+engine's request, cache-block and state-slot bookkeeping.
+"""
+
+from __future__ import annotations
+
+import math
+
+import pytest
+import torch
+
+import balenex_oracle as oracle
+from vllm_tgis_adapter_amd import ops
+from vllm_tgis_adapter_amd.engine import EngineConfig, LLMEngine, ModelConfig, SamplingParams
+from vllm_tgis_adapter_amd.engine.config import CacheConfig, SchedulerConfig
+from vllm_tgis_adapter_amd.models import blocks
+
+CPU = pytest.param("cpu", id="cpu")
+GPU = pytest.param("cuda", id="gpu", marks=pytest.mark.gpu)
+DEVICES = [CPU, GPU]
+F64 = torch.float64
+EPS = 1e-5
+
+
+def left_spec(heads=4, kv_heads=2, dim=8, vdim=12, conv=3, size=7, keep=3, base=50.0, rot=6):
+    return {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "conv": conv,
+            "scale": 1.3 / math.sqrt(dim), "mask": {"size": size, "keep_first": keep},
+            "rot": {"base": base, "dims": rot}}
+
+
+def right_spec(heads=3, dim=6, vdim=10, tau=5.0):
+    return {"heads": heads, "dim": dim, "vdim": vdim, "tau": tau}
+
+
+def pooled_spec(heads=4, kv_heads=2, dim=8, vdim=6, size=5, pool=3):
+    return {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim,
+            "scale": 1.3 / math.sqrt(dim), "mask": {"size": size, "pool": pool}}
+
+
+def par(left=None, right=None):
+    return {"left": left or left_spec(), "right": right or right_spec()}
+
+
+def dense(ff=20):
+    return {"kind": "dense", "ff": ff}
+
+
+def make_config(layers=None, width=30, vocab=50, groups=3, eps=EPS):
+    if layers is None:
+        layers = [("attention", pooled_spec(), dense()),
+                  ("parallel", par(), dense(14)),
+                  ("attention", pooled_spec(3, 3, 6, 10, size=4, pool=6), None),
+                  ("parallel", par(left_spec(2, 1, 6, 4, conv=2, size=5, keep=9, rot=4),
+                                   right_spec(2, 4, 4, tau=2.0)), None)]
+    return {"architecture": "Balenex", "vocab": vocab, "width": width,
+            "norm": {"eps": eps, "groups": groups},
+            "layers": [{"type": t, "mixer": m, "mlp": f} for t, m, f in layers]}
+
+
+def _engine(path, device, dtype="float32", blocks=64, slots=4, block_size=4, eager=True):
+    mc = ModelConfig.from_model_arg(path, dtype=dtype)
+    return LLMEngine(EngineConfig(
+        model_config=mc,
+        cache_config=CacheConfig(block_size=block_size, num_gpu_blocks=blocks),
+        scheduler_config=SchedulerConfig(max_num_seqs=slots, max_num_batched_tokens=1 << 20),
+        device=device, enforce_eager=eager))
+
+
+def _tokens(n, vocab, seed):
+    g = torch.Generator().manual_seed(seed)
+    return torch.randint(0, vocab, (n,), generator=g).tolist()
+
+
+def _feed(engine, rid, tokens, cuts):
+    """Feed one request in portions; logits of every position."""
+    rows, at = [], 0
+    for n in cuts:
+        last = at + n == len(tokens)
+        rows.append(engine.replay_step([(rid, tokens[at:at + n], list(range(n)))],
+                                       [rid] if last else []))
+        at += n
+    assert at == len(tokens)
+    return torch.cat(rows).double().cpu()
+
+
+def _close(got, want, dtype="float32", what=""):
+    tol = 3e-4 if dtype == "float32" else 0.05 * max(1.0, float(want.abs().max()))
+    err = float((got - want).abs().max())
+    assert err < tol, f"{what} {err}"
+
+
+@pytest.fixture(scope="module")
+def model(tmp_path_factory):
+    cfg = make_config()
+    w = oracle.random_weights(cfg, seed=1)
+    path = str(tmp_path_factory.mktemp("balenex") / "m")
+    oracle.write_model(path, cfg, w)
+    return cfg, w, path
+
+
+# -- each mechanism alone, as the framework's block, in portions --------------
+
+
+class _Meta:
+    """What a mixer reads of the step metadata, for one sequence fed in
+    portions through block tables and a state slot of its own."""
+
+    def __init__(self, dev, bs, nblocks, slot):
+        self.dev, self.bs, self.slot = dev, bs, slot
+        self.blocks = list(range(nblocks - 1, -1, -1))   # scattered on purpose
+        self.at = 0
+
+    def step(self, n):
+        i32 = lambda v: torch.tensor(v, dtype=torch.int32, device=self.dev)
+        s, e = self.at, self.at + n
+        self.at = e
+        nb = (e + self.bs - 1) // self.bs
+        m = type("M", (), {})()
+        m.step_values = {}
+        m.slot_mapping = torch.tensor(
+            [self.blocks[p // self.bs] * self.bs + p % self.bs for p in range(s, e)],
+            dtype=torch.long, device=self.dev)
+        m.seq_start_loc, m.seq_lens, m.state_slots = i32([0, n]), i32([e]), i32([self.slot])
+        table = i32([self.blocks[:nb]])
+        empty_t, empty = torch.empty((0, 0), dtype=torch.int32, device=self.dev), i32([])
+        if n > 1:
+            m.num_prefill_tokens, m.num_decode_seqs = n, 0
+            m.prefill_block_tables, m.prefill_query_start_loc = table, i32([0, n])
+            m.prefill_seq_lens, m.max_prefill_query_len = i32([e]), n
+            m.decode_block_tables, m.decode_seq_lens = empty_t, empty
+        else:
+            m.num_prefill_tokens, m.num_decode_seqs = 0, 1
+            m.prefill_block_tables, m.prefill_query_start_loc = empty_t, i32([0])
+            m.prefill_seq_lens, m.max_prefill_query_len = empty, 0
+            m.decode_block_tables, m.decode_seq_lens = table, i32([e])
+        return m, torch.arange(s, e, device=self.dev)
+
+
+def _run_block(call, cache_shapes, n, dev, cuts, bs=4):
+    """``call(rows slice, positions, cache list, meta)`` over n rows fed in
+    portions; paged tensors and state slots start dirty."""
+    nblocks = (n + bs - 1) // bs + 2
+    cache = []
+    for kind, shape, dt in cache_shapes:
+        lead = nblocks if kind == "paged" else 3
+        cache.append(torch.full((lead,) + tuple(shape), 3.0, dtype=dt, device=dev))
+    meta = _Meta(dev, bs, nblocks, slot=1)
+    outs, at = [], 0
+    for k in cuts:
+        m, pos = meta.step(k)
+        outs.append(call(slice(at, at + k), pos, cache, m).double().cpu())
+        at += k
+    return torch.cat(outs)
+
+
+CUTS = [[23], [1] * 23, [2] * 11 + [1], [7, 1, 1, 3, 2, 9], [21, 2]]
+
+
+def _mixer_weights(kind, spec, width, seed, rank=5):
+    g = torch.Generator().manual_seed(seed)
+    return {n: oracle.random_tensor(n, s, g)
+            for n, s in oracle.mixer_shapes(kind, spec, width, rank).items()}
+
+
+def _f64(w, prefix=""):
+    return {k[len(prefix):]: v.double() for k, v in w.items() if k.startswith(prefix)}
+
+
+def _own_projection(mod, width):
+    """Give a mixer built for a merged projection one of its own."""
+    mod.in_weight = torch.nn.Parameter(torch.zeros(mod.in_rows, width), requires_grad=False)
+    return mod
+
+
+LEFTS = [
+    left_spec(),
+    left_spec(3, 3, 6, 6, conv=1, size=4, keep=0, rot=6),       # every dim rotated, one tap
+    left_spec(4, 1, 10, 4, conv=2, size=1, keep=2, rot=2),      # a window of one
+    left_spec(2, 2, 16, 16, conv=4, size=40, keep=5, rot=16),   # nothing leaves the window
+    left_spec(6, 2, 12, 20, conv=6, size=3, keep=30, rot=8),    # everything is kept
+    left_spec(2, 1, 16, 8, conv=3, size=9, keep=1, rot=0),      # no key rotation
+]
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("spec", LEFTS)
+def test_conv_attention_alone(device, spec):
+    width = 24
+    g = torch.Generator().manual_seed(4)
+    h = torch.randn(23, width, generator=g)
+    w = {k[5:]: t for k, t in
+         _mixer_weights("parallel", par(spec), width, 5).items() if k.startswith("left.")}
+    want = oracle.conv_attention(h.double(), _f64(w), spec, EPS)
+    mod = _own_projection(blocks.SpanAttention(
+        width, heads=spec["heads"], kv_heads=spec["kv_heads"], dim=spec["dim"],
+        vdim=spec["vdim"], scale=spec["scale"], eps=EPS, window=spec["mask"]["size"],
+        keep_first=spec["mask"]["keep_first"], taps=spec["conv"], rot_base=spec["rot"]["base"],
+        rot_dims=spec["rot"]["dims"], rotate_values=True, own_in=False, dtype=torch.float32),
+        width)
+    mod.load(w)
+    mod = mod.to(device)
+    for cuts in CUTS:
+        got = _run_block(lambda sl, pos, cache, m: mod(h[sl].to(device), pos, cache, m),
+                         mod.cache_shapes(4), 23, device, cuts)
+        _close(got, want, what=f"cuts {cuts}")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("bs", [4, 16])
+@pytest.mark.parametrize("spec", [
+    pooled_spec(), pooled_spec(3, 3, 6, 10, size=1, pool=1), pooled_spec(4, 1, 5, 3, size=2, pool=4),
+    pooled_spec(2, 2, 16, 16, size=30, pool=2), pooled_spec(6, 3, 12, 8, size=3, pool=7),
+    pooled_spec(1, 1, 4, 4, size=6, pool=16)])
+def test_pooled_attention_alone(device, spec, bs):
+    width = 24
+    g = torch.Generator().manual_seed(6)
+    h = torch.randn(23, width, generator=g)
+    w = _mixer_weights("attention", spec, width, 7)
+    want = oracle.pooled_attention(h.double(), _f64(w), spec, EPS) - w["o.b"].double()
+    mod = blocks.SpanAttention(
+        width, heads=spec["heads"], kv_heads=spec["kv_heads"], dim=spec["dim"],
+        vdim=spec["vdim"], scale=spec["scale"], eps=EPS, window=spec["mask"]["size"],
+        pool=spec["mask"]["pool"], norm_weights=False, o_bias=True, dtype=torch.float32)
+    mod.load(w)
+    assert torch.equal(mod.o_bias, w["o.b"])       # added by the residual kernel
+    mod = mod.to(device)
+    for cuts in CUTS:
+        got = _run_block(lambda sl, pos, cache, m: mod(h[sl].to(device), pos, cache, m),
+                         mod.cache_shapes(bs), 23, device, cuts, bs)
+        _close(got, want, what=f"cuts {cuts}")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("spec,rank", [(right_spec(), 5), (right_spec(1, 4, 4, 1.0), 1),
+                                       (right_spec(4, 16, 3, 16.0), 9),
+                                       (right_spec(2, 5, 33, 0.5), 20)])
+def test_gated_linear_attention_alone(device, spec, rank):
+    width = 24
+    g = torch.Generator().manual_seed(8)
+    h = torch.randn(23, width, generator=g)
+    w = {k[6:]: t for k, t in _mixer_weights("parallel", par(right=spec), width, 9, rank).items()
+         if k.startswith("right.")}
+    want = oracle.gated_linear_attention(h.double(), _f64(w), spec, EPS)
+    mod = _own_projection(blocks.GLAMixer(
+        width, heads=spec["heads"], dim=spec["dim"], vdim=spec["vdim"], rank=rank,
+        tau=spec["tau"], eps=EPS, own_in=False, dtype=torch.float32), width)
+    mod.load(w)
+    mod = mod.to(device)
+    for cuts in CUTS:
+        got = _run_block(lambda sl, pos, cache, m: mod(h[sl].to(device), pos, cache, m),
+                         mod.cache_shapes(4), 23, device, cuts)
+        _close(got, want, what=f"cuts {cuts}")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_grouped_norm_and_half_sum_alone(device):
+    g = torch.Generator().manual_seed(10)
+    for width, groups in [(24, 3), (32, 1), (20, 5), (64, 16)]:
+        x, a, b = (torch.randn(9, width, generator=g) for _ in range(3))
+        # one part far larger than the others: a single statistic would flatten them
+        a[:, :width // groups] *= 50.0
+        wa, wb, wo, wn = (torch.randn(width, generator=g) for _ in range(4))
+        d = lambda t: t.to(device)
+        y = 0.5 * (oracle.rms_norm(a.double(), wa.double(), EPS)
+                   + oracle.rms_norm(b.double(), wb.double(), EPS))
+        want = x.double() + oracle.group_norm(y, wo.double(), groups, EPS)
+        xs = d(x.clone())
+        nxt = ops.stream_add_group_norm(xs, d(a), d(wo), groups, EPS, b=d(b), wa=d(wa), wb=d(wb),
+                                        mix=0.5, next_w=d(wn), out_dtype=torch.float32)
+        _close(xs.double().cpu(), want, what="stream")
+        _close(nxt.double().cpu(), oracle.group_norm(want, wn.double(), groups, EPS), what="next")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_gated_ff_alone(device):
+    g = torch.Generator().manual_seed(11)
+    width, ff = 18, 26
+    names = {"gate": (ff, width), "gate.b": (ff,), "up": (ff, width), "up.b": (ff,),
+             "down": (width, ff), "down.b": (width,)}
+    w = {n: oracle.random_tensor(n, s, g) for n, s in names.items()}
+    h = torch.randn(11, width, generator=g)
+    mod = blocks.BiasedGatedMLP(width, ff, torch.float32)
+    mod.load(w)
+    mod = mod.to(device)
+    got = mod(h.to(device)) + mod.down_bias
+    _close(got.double().cpu(), oracle.gated_ff(h.double(), _f64(w)))
+
+
+def test_decay_is_a_power_of_the_gate():
+    """With values only at the first token the state is that value times the
+    product of the later decays; tau stretches them."""
+    spec = right_spec(1, 1, 1, tau=4.0)
+    w = {"q": torch.tensor([[1.0, 0.0]]), "k": torch.tensor([[1.0, 0.0]]),
+         "v": torch.tensor([[0.0, 1.0]]), "g": torch.tensor([[0.0, 0.0]]),
+         "a1": torch.tensor([[1.0, 0.0]]), "a2": torch.tensor([[0.0]]),
+         "a2.b": torch.tensor([-2.0]), "norm": torch.ones(1), "o": torch.ones(1, 1)}
+    h = torch.tensor([[1.0, 3.0]] + [[1.0, 0.0]] * 4)
+    alpha = (1.0 / (1.0 + math.exp(2.0))) ** 0.25
+    state = torch.zeros(1, 1, 1, 1)
+    proj = lambda n: h @ w[n].T
+    i32 = lambda v: torch.tensor(v, dtype=torch.int32)
+    o = ops.gla_scan(proj("q").view(5, 1, 1), proj("k").view(5, 1, 1), proj("v").view(5, 1, 1),
+                     proj("a1"), w["a2"].T.contiguous(), w["a2.b"], 1 / spec["tau"], 1.0, state,
+                     i32([0, 5]), i32([5]), i32([0]))
+    want = torch.tensor([3.0 * alpha ** t for t in range(5)])
+    assert float((o[:, 0] - want).abs().max()) < 1e-6
+
+
+# -- what a query sees: keys far away, at page borders, at every edge -----------
+
+
+def _spike(window, keep, pool, ctx, at, n_new, device, bs=4, dim=8, dtype=torch.float32):
+    """One head; every key is small noise but the one at ``at``, which the last
+    query points at; its value is all 100.  Returns the last query's output
+    through the op and from the definition."""
+    g = torch.Generator().manual_seed(ctx * 31 + at)
+    k = torch.randn(ctx, 1, dim, generator=g) * 0.05
+    v = torch.randn(ctx, 1, dim, generator=g) * 0.05
+    q = torch.randn(n_new, 1, dim, generator=g) * 0.05
+    direction = torch.ones(dim) / math.sqrt(dim)
+    gain = 7.0 * math.sqrt(max(pool, 1))      # a pooled spike is divided by pool
+    k[at, 0] = gain * direction
+    v[at, 0] = 100.0
+    q[-1, 0] = gain * direction
+    k, v, q = k.to(dtype), v.to(dtype), q.to(dtype)
+    nb = (ctx + bs - 1) // bs
+    table = list(range(nb - 1, -1, -1))
+    kc = torch.zeros(nb, bs, 1, dim, dtype=dtype)
+    vc = torch.zeros(nb, bs, 1, dim, dtype=dtype)
+    for p in range(ctx):
+        kc[table[p // bs], p % bs] = k[p]
+        vc[table[p // bs], p % bs] = v[p]
+    dev = lambda t: t.to(device)
+    i32 = lambda x: torch.tensor(x, dtype=torch.int32, device=device)
+    kc, vc, tables = dev(kc), dev(vc), i32([table])
+    kp = vp = None
+    if pool:
+        slots = ops.pool_slots_per_block(bs, pool)
+        kp = torch.full((nb, slots, 1, dim), 50.0, dtype=dtype, device=device)
+        vp = kp.clone()
+        ops.pool_cache_write(kc, vc, kp, vp, pool, tables, i32([0, ctx]), i32([ctx]), ctx)
+    out = torch.empty(n_new, 1, dim, dtype=dtype, device=device)
+    if n_new > 1:
+        ops.span_attention_prefill(dev(q), kc, vc, kp, vp, tables, i32([0, n_new]), i32([ctx]),
+                                   1.0, n_new, window, keep, pool, None, out=out)
+    else:
+        ops.span_attention_decode(dev(q), kc, vc, kp, vp, tables, i32([ctx]), 1.0, window, keep,
+                                  pool, None, out=out)
+    i = ctx - 1
+    seen = oracle.keys_first_and_window(i, window, keep)
+    kk, vv = [k[seen, 0].double()], [v[seen, 0].double()]
+    if pool:
+        for b in range(oracle.pooled_seen(i, window, pool)):
+            rows = slice(b * pool, (b + 1) * pool)
+            kk.append(k[rows, 0].double().mean(0, keepdim=True))
+            vv.append(v[rows, 0].double().mean(0, keepdim=True))
+    want = oracle.attend(q[-1].double(), torch.cat(kk).unsqueeze(0), torch.cat(vv).unsqueeze(0),
+                         1.0)[0]
+    return out[-1, 0].double().cpu(), want
+
+
+def _edges(window, keep, pool, ctx):
+    first = max(0, ctx - window)
+    places = {0, 1, ctx - 1, first, first - 1, first + 1, keep - 1, keep, keep + 1, 3, 4, 7, 8, 15,
+              16}
+    if pool:
+        nb = oracle.pooled_seen(ctx - 1, window, pool)
+        places |= {nb * pool - 1, nb * pool, (nb - 1) * pool, (nb - 1) * pool - 1, pool - 1, pool}
+    return sorted(p for p in places if 0 <= p < ctx)
+
+
+def _expected_height(window, keep, pool, ctx, at):
+    if ctx - 1 - at < window or at < keep:
+        return 100.0
+    if pool and at // pool < oracle.pooled_seen(ctx - 1, window, pool):
+        return 100.0 / pool
+    return 0.0
+
+
+MASKS = [(6, 2, 0), (6, 0, 3), (8, 9, 0), (1, 1, 0), (1, 0, 1), (5, 0, 16), (16, 0, 4), (40, 20, 0),
+         (9, 0, 7)]
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("n_new", [1, 2, 7])
+@pytest.mark.parametrize("window,keep,pool", MASKS)
+def test_edges_and_far_keys(device, n_new, window, keep, pool):
+    for ctx in (7, 30, 31, 64, 150):
+        for at in _edges(window, keep, pool, ctx):
+            got, want = _spike(window, keep, pool, ctx, at, min(n_new, ctx), device)
+            height = _expected_height(window, keep, pool, ctx, at)
+            # the spike decides the output exactly when it is seen
+            assert abs(float(want.mean()) - height) < 1.0 + 0.02 * height, (ctx, at)
+            assert float((got - want).abs().max()) < 2e-3, f"ctx {ctx} spike at {at}"
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("dim", [64, 128])
+@pytest.mark.parametrize("n_new", [1, 5, 300])
+@pytest.mark.parametrize("window,keep,pool", [(64, 10, 0), (100, 0, 16), (100, 150, 0),
+                                              (33, 0, 5), (257, 64, 0), (128, 0, 40), (64, 0, 1)])
+def test_edges_and_far_keys_on_matrix_cores(dim, n_new, window, keep, pool):
+    """The same on the bf16 matrix-core kernels (portions: head size 128)."""
+    for ctx in (130, 700):
+        for at in _edges(window, keep, pool, ctx) + [63, 64]:
+            if at >= ctx:
+                continue
+            got, want = _spike(window, keep, pool, ctx, at, min(n_new, ctx), "cuda", bs=16,
+                               dim=dim, dtype=torch.bfloat16)
+            assert float((got - want).abs().max()) < 0.6, f"ctx {ctx} spike at {at}"
+
+
+# -- the whole model through the engine ----------------------------------------
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_whole_prompt_and_layers_match_oracle(model, device):
+    cfg, w, path = model
+    toks = _tokens(27, cfg["vocab"], 2)
+    layers = []
+    want = oracle.forward(cfg, w, toks, layers)
+    eng = _engine(path, device)
+    probe = eng.worker.model.stream_probe = []
+    got = _feed(eng, "a", toks, [len(toks)])
+    _close(got, want, what="logits")
+    assert len(probe) == len(layers)
+    for i, (a, b) in enumerate(zip(probe, layers)):
+        _close(a.double().cpu(), b, what=f"stream after layer {i}")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_decode_and_portions_equal_whole(model, device):
+    cfg, w, path = model
+    toks = _tokens(31, cfg["vocab"], 3)
+    want = oracle.forward(cfg, w, toks)
+    eng = _engine(path, device)
+    for k, cuts in enumerate([[1] * 31, [2] * 15 + [1], [5, 3, 2, 7, 1, 1, 4, 8], [29, 2],
+                              [3] + [1] * 28, [4, 4, 4, 4, 4, 4, 4, 3], [7, 7, 7, 7, 3]]):
+        _close(_feed(eng, f"r{k}", toks, cuts), want, what=f"cuts {cuts}")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_long_decode(model, device):
+    cfg, w, path = model
+    toks = _tokens(70, cfg["vocab"], 4)
+    want = oracle.forward(cfg, w, toks)
+    eng = _engine(path, device)
+    _close(_feed(eng, "a", toks, [5] + [1] * 65), want)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_mixed_batch_and_reuse_of_blocks_and_slots(model, device):
+    """Unequal requests in one step, portions beside single tokens, requests
+    that leave and hand their blocks and state slots to later ones."""
+    cfg, w, path = model
+    lens = {"a": 26, "b": 9, "c": 17, "d": 30, "e": 12, "f": 21}
+    toks = {k: _tokens(n, cfg["vocab"], 10 + i) for i, (k, n) in enumerate(lens.items())}
+    want = {k: oracle.forward(cfg, w, t) for k, t in toks.items()}
+    # all six need 32 blocks of 4 tokens and six slots; the pool has 22 blocks
+    # and 4 slots: the later requests run where finished ones were
+    eng = _engine(path, device, blocks=22, slots=4)
+    plan = [
+        [("a", 7), ("b", 2)],
+        [("a", 1), ("b", 5), ("c", 17)],
+        [("a", 9), ("b", 1), ("d", 3)],
+        [("a", 1), ("b", 1), ("d", 2)],
+        [("a", 2), ("d", 1), ("e", 12)],
+        [("a", 6), ("d", 24), ("f", 1)],
+        [("f", 2)],
+        [("f", 18)],
+    ]
+    at = {k: 0 for k in lens}
+    got = {k: [] for k in lens}
+    free_before = eng.block_manager.num_free_blocks
+    for step in plan:
+        entries, end = [], []
+        for k, n in step:
+            entries.append((k, toks[k][at[k]:at[k] + n], list(range(n))))
+            at[k] += n
+            if at[k] == lens[k]:
+                end.append(k)
+        out = eng.replay_step(entries, end).double().cpu()
+        row = 0
+        for k, n in step:
+            got[k].append(out[row:row + n])
+            row += n
+    assert at == lens
+    assert eng.block_manager.num_free_blocks == free_before
+    for k in lens:
+        _close(torch.cat(got[k]), want[k], what=k)
+
+
+def test_a_request_may_sit_out_steps(model):
+    """A request left out of a step goes on later from the state it left."""
+    cfg, w, path = model
+    ta, tb = _tokens(14, cfg["vocab"], 40), _tokens(11, cfg["vocab"], 41)
+    eng = _engine(path, "cpu")
+    ga, gb = [], []
+    ga.append(eng.replay_step([("a", ta[:6], list(range(6)))], []))
+    gb.append(eng.replay_step([("b", tb[:4], list(range(4)))], []))
+    gb.append(eng.replay_step([("b", tb[4:5], [0])], []))
+    out = eng.replay_step([("a", ta[6:7], [0]), ("b", tb[5:], list(range(6)))], ["b"])
+    ga.append(out[:1])
+    gb.append(out[1:])
+    ga.append(eng.replay_step([("a", ta[7:], list(range(7)))], ["a"]))
+    _close(torch.cat(ga).double(), oracle.forward(cfg, w, ta), what="a")
+    _close(torch.cat(gb).double(), oracle.forward(cfg, w, tb), what="b")
+
+
+VARIANTS = {
+    "no_ff_one_head_one_group": (
+        [("parallel", par(left_spec(1, 1, 8, 8, conv=1, size=3, keep=0, rot=8),
+                          right_spec(1, 4, 4, 1.0)), None),
+         ("attention", pooled_spec(1, 1, 4, 4, size=2, pool=2), None)], 1, 1),
+    "pooled_only": (
+        [("attention", pooled_spec(6, 3, 4, 2, size=3, pool=5), dense(6)),
+         ("attention", pooled_spec(2, 2, 12, 5, size=50, pool=8), dense(31)),
+         ("attention", pooled_spec(5, 1, 3, 7, size=1, pool=1), None)], 4, 5),
+    "parallel_only": (
+        [("parallel", par(left_spec(6, 2, 4, 6, conv=4, size=6, keep=4, rot=2),
+                          right_spec(5, 2, 6, 8.0)), dense(7)),
+         ("parallel", par(left_spec(2, 2, 12, 2, conv=2, size=2, keep=1, base=1000.0, rot=12),
+                          right_spec(1, 7, 9, 3.0)), dense(8))], 10, 9),
+}
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("variant", sorted(VARIANTS))
+def test_other_shapes(tmp_path, device, variant):
+    layers, groups, rank = VARIANTS[variant]
+    cfg = make_config(layers, width=20, vocab=31, groups=groups, eps=1e-4)
+    w = oracle.random_weights(cfg, seed=5, rank=rank)
+    oracle.write_model(str(tmp_path / "v"), cfg, w)
+    toks = _tokens(22, cfg["vocab"], 6)
+    want = oracle.forward(cfg, w, toks)
+    eng = _engine(str(tmp_path / "v"), device, block_size=8)
+    _close(_feed(eng, "a", toks, [22]), want, what="whole")
+    _close(_feed(eng, "b", toks, [3, 2, 9, 1, 1, 6]), want, what="portions")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_bf16_stays_near_oracle(model, device):
+    cfg, w, path = model
+    toks = _tokens(25, cfg["vocab"], 7)
+    want = oracle.forward(cfg, w, toks)
+    eng = _engine(path, device, dtype="bfloat16")
+    _close(_feed(eng, "a", toks, [11, 1, 1, 12]), want, "bfloat16")
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_matrix_core_shapes(tmp_path, dtype):
+    """Head sizes the matrix-core attention kernels take, long enough for
+    several key tiles, edges inside tiles."""
+    layers = [("parallel", par(left_spec(4, 2, 128, 128, conv=3, size=50, keep=20, rot=128,
+                                         base=1000.0), right_spec(2, 64, 64, 8.0)), dense(96)),
+              ("attention", pooled_spec(2, 1, 128, 128, size=40, pool=8), dense(96)),
+              ("parallel", par(left_spec(2, 1, 64, 64, conv=2, size=37, keep=70, rot=32),
+                               right_spec(1, 128, 128, 16.0)), None),
+              ("attention", pooled_spec(4, 2, 64, 64, size=33, pool=24), None)]
+    cfg = make_config(layers, width=64, vocab=40, groups=4)
+    w = oracle.random_weights(cfg, seed=8, rank=16)
+    oracle.write_model(str(tmp_path / "m"), cfg, w)
+    toks = _tokens(190, cfg["vocab"], 9)
+    want = oracle.forward(cfg, w, toks)
+    eng = _engine(str(tmp_path / "m"), "cuda", dtype=dtype, blocks=60, block_size=16)
+    _close(_feed(eng, "a", toks, [190]), want, dtype, "whole")
+    _close(_feed(eng, "b", toks, [70, 3, 60, 2] + [1] * 55), want, dtype, "portions")
+
+
+@pytest.mark.gpu
+def test_captured_decode_steps_match_eager(model):
+    cfg, w, path = model
+    prompts = {k: _tokens(n, cfg["vocab"], 20 + i) for i, (k, n) in
+               enumerate({"a": 9, "b": 4, "c": 13}.items())}
+
+    def generate(eager):
+        eng = _engine(path, "cuda", eager=eager)
+        for k, t in prompts.items():
+            eng.add_request(k, None, list(t), SamplingParams(temperature=0.0, max_tokens=12))
+        out = {}
+        while eng.has_unfinished():
+            for o in eng.step():
+                if o.finished:
+                    out[o.request_id] = list(o.outputs[0].token_ids)
+        return out, eng
+
+    eager, _ = generate(True)
+    graphs, eng = generate(False)
+    assert eng.worker.graph_runner is not None and eng.worker.graph_runner.graphs
+    assert eager == graphs
+
+
+# -- generation through the engine's own entry point --------------------------
+
+
+def _check_greedy(cfg, w, prompt, got, steps, stop=None):
+    seq = list(prompt)
+    for j in range(steps):
+        logits = oracle.forward(cfg, w, seq)[-1]
+        top2 = torch.topk(logits, 2).values
+        if float(top2[0] - top2[1]) < 1e-3:      # a close call proves nothing
+            break
+        seq.append(int(torch.argmax(logits)))
+        assert got[j] == seq[-1], f"token {j}"
+        if seq[-1] == stop:
+            break
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_greedy_generation_matches_oracle(model, device):
+    cfg, w, path = model
+    prompts = {"a": _tokens(7, cfg["vocab"], 30), "b": _tokens(15, cfg["vocab"], 31),
+               "c": _tokens(2, cfg["vocab"], 32)}
+    steps = 10
+    eng = _engine(path, device)
+    for k, t in prompts.items():
+        eng.add_request(k, None, list(t), SamplingParams(temperature=0.0, max_tokens=steps))
+    got = {}
+    while eng.has_unfinished():
+        for o in eng.step():
+            if o.finished:
+                got[o.request_id] = list(o.outputs[0].token_ids)
+    for k, t in prompts.items():
+        _check_greedy(cfg, w, t, got[k], steps)
+
+
+def test_registry_and_cache_layout(model):
+    cfg, w, path = model
+    mc = ModelConfig.from_model_arg(path, dtype="float32")
+    assert mc.architecture == "balenex" and mc.num_layers == 4 and mc.vocab_size == 50
+    from vllm_tgis_adapter_amd.models import get_model, native_extensions
+
+    assert native_extensions(mc) == ["_C_seq"]
+    m = get_model(mc)
+    assert m.uses_seq_state and m.layers[1].mix.right.rank == 5     # from the tensor's shape
+    shapes = [[tuple(c.shape) for c in cs] for cs in m.allocate_caches(3, 4, 2, "cpu")]
+    # keys, values, pooled keys and values (blocks of 3: two may end in four tokens)
+    assert shapes[0] == [(3, 4, 2, 8), (3, 4, 2, 6), (3, 2, 2, 8), (3, 2, 2, 6)]
+    # keys, values, convolution rows, recurrent state
+    assert shapes[1] == [(3, 4, 2, 8), (3, 4, 2, 12), (2, 2, 72), (2, 3, 10, 6)]
+    assert shapes[2] == [(3, 4, 3, 6), (3, 4, 3, 10), (3, 1, 3, 6), (3, 1, 3, 10)]
+    assert m.state_bytes_per_slot() == 4 * (2 * 72 + 3 * 10 * 6 + 1 * 22 + 2 * 4 * 4)
+    assert m.cache_bytes_per_block(4) == 4 * (
+        4 * 28 + 2 * 28 + 4 * 40 + 4 * 48 + 1 * 48 + 4 * 10)
+
+
+def test_config_errors():
+    from vllm_tgis_adapter_amd.models.balenex import build_ff, model_config_from_json
+
+    with pytest.raises(ValueError):
+        model_config_from_json("x", make_config([("rwkv", {}, None)]))
+    with pytest.raises(ValueError):
+        model_config_from_json("x", make_config(groups=7))
+    with pytest.raises(ValueError):
+        build_ff({"kind": "moe"}, 8, torch.float32)
+    with pytest.raises(ValueError):
+        blocks.SpanAttention(8, heads=2, kv_heads=1, dim=4, vdim=4, scale=1.0, eps=EPS, window=4,
+                             keep_first=1, pool=2)
+
+
+def test_served_from_command_line_flags(tmp_path):
+    """A model directory given as --model goes through the server's flag
+    parsing into the async engine and streams greedy tokens equal to the
+    oracle's, concurrent requests included."""
+    import asyncio
+
+    from vllm_tgis_adapter_amd.__main__ import parse_args
+    from vllm_tgis_adapter_amd.engine.async_engine import AsyncLLMEngine
+    from vllm_tgis_adapter_amd.tgis_utils.args import engine_config_from_args
+
+    cfg = make_config(vocab=300)    # room for the byte-level test tokenizer
+    w = oracle.random_weights(cfg, seed=5)
+    oracle.write_model(str(tmp_path / "served"), cfg, w)
+    args = parse_args(["--model", str(tmp_path / "served"), "--dtype", "float32",
+                       "--max-num-seqs", "2", "--num-gpu-blocks", "64", "--block-size", "8",
+                       "--device", "cpu"])
+    engine = AsyncLLMEngine(engine_config_from_args(args))
+    prompts = {"x": _tokens(12, 300, 61), "y": _tokens(5, 300, 62), "z": _tokens(9, 300, 63)}
+
+    async def one(rid):
+        last = None
+        async for out in engine.generate(
+                {"prompt_token_ids": prompts[rid]},
+                SamplingParams(temperature=0.0, max_tokens=5), request_id=rid):
+            last = out
+        return rid, list(last.outputs[0].token_ids)
+
+    async def main():
+        return dict(await asyncio.gather(*[one(r) for r in prompts]))
+
+    try:
+        got = asyncio.run(main())
+    finally:
+        engine.shutdown()
+    for rid, p in prompts.items():
+        _check_greedy(cfg, w, p, got[rid], 5, stop=engine.engine.eos_token_id)
