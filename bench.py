@@ -45,7 +45,7 @@ def parse_args():
     p.add_argument("--arch-sizes", type=str, default="s,m",
                    help="arch mode: comma list of sizes (s, m)")
     p.add_argument("--arch-models", type=str, default="dolodra,llama",
-                   help="arch mode: which models to run (dolodra, kezunex, relerax, gumozen, "
+                   help="arch mode: which models to run (dolodra, kezunex, relerax, gumozen, balenex, "
                         "llama)")
     p.add_argument("--model", type=str, default="llama-3-8b")
     p.add_argument("--batch", type=int, default=512)
@@ -647,6 +647,41 @@ def _gumozen_model_config(name: str, sz: dict, dtype: str):
     return mc
 
 
+# Balenex at the same widths: eight layers [parallel, attention, attention,
+# parallel] x 2, every one with the llama's feed-forward.  Both attention kinds
+# have the llama's heads of 128: beside the recurrence with a window of 512 that
+# also keeps the first 64 tokens, alone with a window of 256 and older tokens in
+# pooled blocks of 16.  The recurrence has width / 128 heads of 128 x 128.
+BALENEX_SIZES = {
+    "s": dict(groups=2, taps=3, window=512, keep=64, pool_window=256, pool=16),
+    "m": dict(groups=4, taps=3, window=512, keep=64, pool_window=256, pool=16),
+    "t": dict(groups=2, taps=3, window=12, keep=4, pool_window=9, pool=4),
+}
+
+
+def _balenex_model_config(name: str, sz: dict, dtype: str):
+    from vllm_tgis_adapter_amd.engine.config import _DTYPES
+    from vllm_tgis_adapter_amd.models.balenex import model_config_from_json
+
+    bx = BALENEX_SIZES[name]
+    hd = sz["width"] // sz["heads"]
+    att = {"heads": sz["heads"], "kv_heads": sz["llama_kv_heads"], "dim": hd, "vdim": hd,
+           "scale": hd ** -0.5}
+    pair = {"left": dict(att, conv=bx["taps"], rot={"base": 10000.0, "dims": hd},
+                         mask={"size": bx["window"], "keep_first": bx["keep"]}),
+            "right": {"heads": sz["heads"], "dim": hd, "vdim": hd, "tau": 16.0}}
+    pooled = dict(att, mask={"size": bx["pool_window"], "pool": bx["pool"]})
+    kinds = [("parallel", pair), ("attention", pooled), ("attention", pooled),
+             ("parallel", pair)]
+    layers = [{"type": kinds[i % 4][0], "mixer": kinds[i % 4][1],
+               "mlp": {"kind": "dense", "ff": sz["llama_inter"]}} for i in range(sz["layers"])]
+    hf = {"architecture": "Balenex", "vocab": sz["vocab"], "width": sz["width"],
+          "layers": layers, "norm": {"eps": 1e-6, "groups": bx["groups"]}}
+    mc = model_config_from_json("balenex-synthetic", hf)
+    mc.dtype = _DTYPES[dtype]
+    return mc
+
+
 def _arch_measure(mc, args, device: str, batch: int, prompt_len: int, steps: int,
                   warmup: int) -> dict:
     from vllm_tgis_adapter_amd.engine import EngineConfig, LLMEngine, SamplingParams
@@ -713,7 +748,7 @@ def run_arch(args, device: str) -> None:
         steps = args.steps if device == "cuda" else 4
         warm = args.warmup if device == "cuda" else 1
         models = [("dolodra", dolo), ("kezunex", None), ("relerax", None), ("gumozen", None),
-                  ("llama", llama)]
+                  ("balenex", None), ("llama", llama)]
         for label, mc in models:
             if label not in args.arch_models.split(","):
                 continue
@@ -723,6 +758,8 @@ def run_arch(args, device: str) -> None:
                 mc = _relerax_model_config(name, sz, args.dtype)
             if label == "gumozen":
                 mc = _gumozen_model_config(name, sz, args.dtype)
+            if label == "balenex":
+                mc = _balenex_model_config(name, sz, args.dtype)
             r = _arch_measure(mc, args, device, batch, plen, steps, warm)
             r.update(size=name, model=label, batch=batch, prompt_len=plen)
             out.append(r)

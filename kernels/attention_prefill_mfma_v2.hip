@@ -466,22 +466,25 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
     const int q_local = tile_base + wave * 32 + qrow;
     if (q_local >= q_len) continue;
     OT* out_row = out + ((long)(q_start + q_local) * nheads + head) * HEAD_DIM;
+    float o[DT];
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) o[dt] = acc_o[dt][r] * l_inv;
     if (PX != PX_NONE && sp.back != nullptr) {
       const float2* tab = sp.back + (long)(q_start + q_local) * (HEAD_DIM / 2);
 #pragma unroll
       for (int dt = 0; dt < DT / 2; ++dt) {
         const float2 cs = tab[dt * 32 + col];
-        const float a = acc_o[dt][r], b = acc_o[dt + DT / 2][r];
-        acc_o[dt][r] = a * cs.x + b * cs.y;
-        acc_o[dt + DT / 2][r] = b * cs.x - a * cs.y;
+        const float a = o[dt], b = o[dt + DT / 2];
+        o[dt] = a * cs.x + b * cs.y;
+        o[dt + DT / 2] = b * cs.x - a * cs.y;
       }
     }
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
       if constexpr (CH)
-        out_row[dt * 32 + col] = acc_o[dt][r] * l_inv;
+        out_row[dt * 32 + col] = o[dt];
       else
-        out_row[dt * 32 + col] = __float2bfloat16(acc_o[dt][r] * l_inv);
+        out_row[dt * 32 + col] = __float2bfloat16(o[dt]);
     }
   }
 }

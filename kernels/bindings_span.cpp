@@ -33,6 +33,15 @@ void launch_gla_scan(float*, const T*, long, const T*, long, const T*, long, con
                      long, const float*, const float*, float, float, float*, const int*,
                      const int*, const int*, int, int, int, int, int, int, float*, int,
                      hipStream_t);
+int gla_fused_columns(int dim, int vdim);
+template <typename T>
+void launch_gla_fused(T*, const T*, long, const T*, long, const T*, long, const T*, long,
+                      const T*, long, const float*, const float*, float, float,
+                      const float*, float, float*, const int*, const int*, const int*, int,
+                      int, int, int, int, int, hipStream_t);
+template <typename T>
+void launch_gated_group_norm(T*, const float*, const T*, long, const float*, float, int, int,
+                             int, int, hipStream_t);
 
 namespace {
 
@@ -338,6 +347,59 @@ void gla_scan(torch::Tensor o, torch::Tensor q, torch::Tensor k, torch::Tensor v
   });
 }
 
+// the scan followed by the per-head norm, its weight and silu(gate): one kernel
+// where the shape fits, three otherwise
+void gla_gated(torch::Tensor out, torch::Tensor q, torch::Tensor k, torch::Tensor v,
+               torch::Tensor g, torch::Tensor a1, torch::Tensor a2, torch::Tensor a2_bias,
+               double inv_tau, double q_scale, torch::Tensor norm, double eps,
+               torch::Tensor state, torch::Tensor loc, torch::Tensor seq_lens,
+               torch::Tensor slots, bool general) {
+  const auto dt = q.scalar_type();
+  check_heads_view(q, dt, "q");
+  check_heads_view(k, dt, "k");
+  check_heads_view(v, dt, "v");
+  const int rows = q.size(0), heads = q.size(1), dim = q.size(2), vdim = v.size(2);
+  TORCH_CHECK(g.is_cuda() && g.dim() == 2 && g.size(0) == rows && g.stride(1) == 1 &&
+              g.size(1) == (long)heads * vdim && g.scalar_type() == dt,
+              "the gate is [rows, heads * vdim]");
+  check_f32(norm, (long)heads * vdim, "norm");
+  check_type(out, dt, "out");
+  TORCH_CHECK(out.numel() == (long)rows * heads * vdim);
+  const int nseq = check_seqs(loc, seq_lens, slots);
+  if (rows == 0 || nseq == 0) return;
+  const int64_t rank = a1.dim() == 2 ? a1.size(1) : 0;
+  bool fits = !general && gla_fused_columns(dim, vdim) > 0 && rank <= 64 && aligned16(state);
+  for (const torch::Tensor* t : {&q, &k, &v})
+    fits = fits && t->stride(0) % 8 == 0 && aligned16(*t);
+  if (!fits) {
+    auto o = torch::empty({(long)rows, (long)heads * vdim}, state.options());
+    gla_scan(o, q, k, v, a1, a2, a2_bias, inv_tau, q_scale, state, loc, seq_lens, slots);
+    DISPATCH_F32_BF16(dt, {
+      launch_gated_group_norm<scalar_t>(ptr<scalar_t>(out), ptr<float>(o), ptr<scalar_t>(g),
+                                        (long)g.stride(0), ptr<float>(norm), (float)eps,
+                                        rows, heads * vdim, heads, 2, stream());
+    });
+    return;
+  }
+  TORCH_CHECK(k.sizes() == q.sizes() && v.size(0) == rows && v.size(1) == heads);
+  TORCH_CHECK(a1.is_cuda() && a1.size(0) == rows && a1.stride(1) == 1 && rank >= 1 &&
+              a1.scalar_type() == dt, "a1 is [rows, rank]");
+  check_f32(a2, (long)rank * heads * dim, "a2");
+  check_f32(a2_bias, (long)heads * dim, "a2_bias");
+  check_f32(state, -1, "state");
+  TORCH_CHECK(state.dim() == 4 && state.size(1) == heads && state.size(2) == vdim &&
+              state.size(3) == dim, "state must be [slots, heads, vdim, dim]");
+  DISPATCH_F32_BF16(dt, {
+    launch_gla_fused<scalar_t>(
+        ptr<scalar_t>(out), ptr<scalar_t>(q), (long)q.stride(0), ptr<scalar_t>(k),
+        (long)k.stride(0), ptr<scalar_t>(v), (long)v.stride(0), ptr<scalar_t>(g),
+        (long)g.stride(0), ptr<scalar_t>(a1), (long)a1.stride(0), ptr<float>(a2),
+        ptr<float>(a2_bias), (float)inv_tau, (float)q_scale, ptr<float>(norm), (float)eps,
+        ptr<float>(state), ptr<int>(loc), ptr<int>(seq_lens), ptr<int>(slots), nseq, heads,
+        dim, vdim, (int)rank, rows, stream());
+  });
+}
+
 void silu_mul_bias(torch::Tensor out, torch::Tensor gu, OptTensor bias) {
   TORCH_CHECK(gu.is_cuda() && gu.is_contiguous() && gu.dim() == 2 && gu.size(1) % 2 == 0);
   const long rows = gu.size(0);
@@ -361,5 +423,6 @@ void register_span_ops(pybind11::module& m) {
   m.def("pool_cache_write", &pool_cache_write);
   m.def("span_attention", &span_attention);
   m.def("gla_scan", &gla_scan);
+  m.def("gla_gated", &gla_gated);
   m.def("silu_mul_bias", &silu_mul_bias);
 }

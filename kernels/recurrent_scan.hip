@@ -344,6 +344,15 @@ __global__ __launch_bounds__(256) void hgrn2_gates_kernel(
   gq[row * 2 * hd + hd + c] = qv * sigmoid_f(qv);
 }
 
+// exp(logsigmoid(z) * inv_tau) on the hardware's exp2 / log2: log1p through
+// log(u), u = 1 + e, with what the rounding of u lost added back
+DEVINLINE float gla_decay_of(float z, float inv_tau) {
+  const float e = __expf(-fabsf(z));
+  const float u = 1.0f + e;
+  const float l = __logf(u) + (e - (u - 1.0f)) * __builtin_amdgcn_rcpf(u);
+  return __expf((fminf(z, 0.f) - l) * inv_tau);
+}
+
 // GLA pre-pass: decay [T, channels] f32 = exp(logsigmoid(a1 . a2[:, c] + b) / tau).
 // One thread per channel and GLA_ROWS rows; the rows' inner projections are
 // broadcast from LDS, a channel's column of a2 [rank, channels] is read once.
@@ -376,7 +385,392 @@ __global__ __launch_bounds__(256) void gla_decay_kernel(
   }
 #pragma unroll
   for (int r = 0; r < GLA_ROWS; ++r)
-    if (r < n) decay[(long)(r0 + r) * channels + c] = expf(logsigmoid_f(z[r]) * inv_tau);
+    if (r < n) decay[(long)(r0 + r) * channels + c] = gla_decay_of(z[r], inv_tau);
+}
+
+// GLA in one kernel where a workgroup can own all value columns of a head: per
+// chunk of GLA_ROWS rows the projected rows go through registers (loaded while
+// the previous chunk is computed) into LDS as f32, the decays are computed
+// there from the inner projections, the recurrence runs on them, and the
+// chunk's outputs, kept in LDS where the values were, are normed per head,
+// gated with silu and rounded once.  Key-channel rows in LDS are laid out so
+// that the NSP lanes of a column read neighbouring 16-byte pieces.
+struct GlaArgs {
+  const void* q; const void* k; const void* v; const void* g; const void* a1;
+  long q_st, k_st, v_st, g_st, a1_st;
+  const float* a2; const float* a2_bias; const float* norm;
+  float inv_tau, q_scale, eps;
+  void* out;                       // [T, heads * vdim]
+  float* state;
+  const int* loc; const int* seq_lens; const int* slots;
+  int heads, dim, vdim, rank;
+};
+
+template <typename T> struct RowPiece;    // eight elements as stored
+template <> struct RowPiece<__hip_bfloat16> {
+  uint4 u;
+  DEVINLINE float at(int i) const {
+    const unsigned w[4] = {u.x, u.y, u.z, u.w};
+    return __uint_as_float(i & 1 ? w[i / 2] & 0xffff0000u : w[i / 2] << 16);
+  }
+};
+template <> struct RowPiece<float> {
+  float f[8];
+  DEVINLINE float at(int i) const { return f[i]; }
+};
+
+template <typename T, int NSP, int VPT>
+__global__ __launch_bounds__(256) void gla_fused_kernel(GlaArgs a) {
+  constexpr int R = GLA_ROWS;
+  constexpr int DP = NSP * NPT;                 // key channels, padded
+  constexpr int NV = 256 / NSP * VPT;           // value columns, padded
+  constexpr int KU = (R * DP / 8 + 255) / 256;  // pieces of a chunk per thread
+  constexpr int VU = (R * NV / 8 + 255) / 256;
+  constexpr int GV = (NV + 63) / 64;
+  constexpr int CH = DP < 256 ? DP : 256;       // channels side by side in the decay step
+  constexpr int SETS = 256 / CH, RPS = R / SETS;
+  constexpr int GR = R / 4;               // rows per wave in the norm step
+  extern __shared__ float smem[];
+  float* dec_s = smem;              // [R][DP], interleaved
+  float* k_s = dec_s + R * DP;
+  float* q_s = k_s + R * DP;
+  float* v_s = q_s + R * DP;        // [R][NV]; outputs replace the values
+  float* a1_s = v_s + R * NV;       // [R][rank_p]
+  const int rank_p = (a.rank + 15) & ~15;
+
+  const int s = blockIdx.x / a.heads;
+  const int h = blockIdx.x % a.heads;
+  const int tid = threadIdx.x;
+  const int ns = tid % NSP, jg = tid / NSP;
+  const int lane = tid & (WAVE_SIZE - 1), wave = tid / WAVE_SIZE;
+  const int row0 = a.loc[s];
+  const int n = a.loc[s + 1] - row0;
+  if (n <= 0) return;
+  const int slot = a.slots[s];
+  const long out_st = (long)a.heads * a.vdim;
+  T* outp = reinterpret_cast<T*>(a.out) + (long)h * a.vdim;
+  if (slot < 0) {
+    for (int r = 0; r < n; ++r)
+      for (int c = tid; c < a.vdim; c += 256)
+        outp[(row0 + r) * out_st + c] = ScalarOps<T>::from_f32(0.f);
+    return;
+  }
+  const T* kp = reinterpret_cast<const T*>(a.k) + (long)h * a.dim;
+  const T* qp = reinterpret_cast<const T*>(a.q) + (long)h * a.dim;
+  const T* vp = reinterpret_cast<const T*>(a.v) + (long)h * a.vdim;
+  const T* gp = reinterpret_cast<const T*>(a.g) + (long)h * a.vdim;
+  const T* a1p = reinterpret_cast<const T*>(a.a1);
+  const long hd = (long)a.heads * a.dim;
+
+  // state columns of this thread
+  const int n0 = ns * NPT;
+  float S[VPT][NPT];
+  float* sbase = a.state + ((long)slot * a.heads + h) * a.vdim * a.dim;
+  const bool carry = a.seq_lens[s] - n > 0;
+#pragma unroll
+  for (int c = 0; c < VPT; ++c) {
+    const int j = jg * VPT + c;
+    if (carry && j < a.vdim) {
+      load_slice<float>(sbase + (long)j * a.dim, n0, a.dim, true, S[c]);
+    } else {
+#pragma unroll
+      for (int i = 0; i < NPT; ++i) S[c][i] = 0.f;
+    }
+  }
+
+  RowPiece<T> rk[KU], rq[KU], rv[VU];
+  float ra1 = 0.f;
+  auto fetch = [&](int r0) {
+    const int nr = min(R, n - r0);
+#pragma unroll
+    for (int u = 0; u < KU; ++u) {
+      const int idx = tid + u * 256, r = idx / (DP / 8), c = idx % (DP / 8) * 8;
+      rk[u] = rq[u] = RowPiece<T>{};
+      if (r < nr && c < a.dim) {
+        const long row = row0 + r0 + r;
+        rk[u] = *reinterpret_cast<const RowPiece<T>*>(kp + row * a.k_st + c);
+        rq[u] = *reinterpret_cast<const RowPiece<T>*>(qp + row * a.q_st + c);
+      }
+    }
+#pragma unroll
+    for (int u = 0; u < VU; ++u) {
+      const int idx = tid + u * 256, r = idx / (NV / 8), c = idx % (NV / 8) * 8;
+      rv[u] = RowPiece<T>{};
+      if (r < nr && c < a.vdim)
+        rv[u] = *reinterpret_cast<const RowPiece<T>*>(vp + (row0 + r0 + r) * a.v_st + c);
+    }
+    const int r = tid / rank_p, i = tid % rank_p;
+    ra1 = r < nr && i < a.rank
+              ? ScalarOps<T>::to_f32(a1p[(row0 + r0 + r) * a.a1_st + i]) : 0.f;
+  };
+
+  fetch(0);
+  for (int r0 = 0; r0 < n; r0 += R) {
+    const int nr = min(R, n - r0);
+    // ---- this chunk into LDS ------------------------------------------------
+#pragma unroll
+    for (int u = 0; u < KU; ++u) {
+      const int idx = tid + u * 256, r = idx / (DP / 8), c = idx % (DP / 8) * 8;
+      if (r < R) {
+        const int at = r * DP + (c % NPT) / 4 * (NSP * 4) + c / NPT * 4;
+#pragma unroll
+        for (int half = 0; half < 2; ++half) {
+          const int e = half * 4;
+          *reinterpret_cast<float4*>(k_s + at + half * NSP * 4) =
+              make_float4(rk[u].at(e), rk[u].at(e + 1), rk[u].at(e + 2), rk[u].at(e + 3));
+          *reinterpret_cast<float4*>(q_s + at + half * NSP * 4) =
+              make_float4(rq[u].at(e) * a.q_scale, rq[u].at(e + 1) * a.q_scale,
+                          rq[u].at(e + 2) * a.q_scale, rq[u].at(e + 3) * a.q_scale);
+        }
+      }
+    }
+#pragma unroll
+    for (int u = 0; u < VU; ++u) {
+      const int idx = tid + u * 256, r = idx / (NV / 8), c = idx % (NV / 8) * 8;
+      if (r < R) {
+#pragma unroll
+        for (int e = 0; e < 8; e += 4)
+          *reinterpret_cast<float4*>(v_s + r * NV + c + e) =
+              make_float4(rv[u].at(e), rv[u].at(e + 1), rv[u].at(e + 2), rv[u].at(e + 3));
+      }
+    }
+    if (tid < R * rank_p) a1_s[tid] = ra1;
+    for (int idx = tid + 256; idx < R * rank_p; idx += 256) {
+      const int r = idx / rank_p, i = idx % rank_p;
+      a1_s[idx] = r < nr && i < a.rank
+                      ? ScalarOps<T>::to_f32(a1p[(row0 + r0 + r) * a.a1_st + i]) : 0.f;
+    }
+    __syncthreads();
+    if (r0 + R < n) fetch(r0 + R);
+    // the gates of this chunk, needed after the recurrence: rows wave, wave + 4, ..
+    float gv[GR][GV];
+#pragma unroll
+    for (int i = 0; i < GR; ++i)
+#pragma unroll
+      for (int j = 0; j < GV; ++j) {
+        const int r = wave + 4 * i, c = lane + 64 * j;
+        gv[i][j] = r < nr && c < a.vdim
+                       ? ScalarOps<T>::to_f32(gp[(row0 + r0 + r) * a.g_st + c]) : 0.f;
+      }
+    // ---- decays: a thread has one channel of RPS rows ------------------------
+#pragma unroll
+    for (int cb = 0; cb < DP; cb += CH) {
+      const int c = cb + tid % CH, rb = tid / CH * RPS;
+      if (c < a.dim && rb < nr) {
+        float z[RPS];
+        const float* w2 = a.a2 + (long)h * a.dim + c;
+        const float bias = a.a2_bias[(long)h * a.dim + c];
+#pragma unroll
+        for (int r = 0; r < RPS; ++r) z[r] = bias;
+        for (int i0 = 0; i0 < a.rank; i0 += 16) {
+          float w[16];
+#pragma unroll
+          for (int i = 0; i < 16; ++i) w[i] = i0 + i < a.rank ? w2[(i0 + i) * hd] : 0.f;
+#pragma unroll
+          for (int r = 0; r < RPS; ++r)
+#pragma unroll
+            for (int i = 0; i < 16; i += 4) {
+              const float4 x =
+                  *reinterpret_cast<const float4*>(a1_s + (rb + r) * rank_p + i0 + i);
+              z[r] += (x.x * w[i] + x.y * w[i + 1]) + (x.z * w[i + 2] + x.w * w[i + 3]);
+            }
+        }
+        float* d = dec_s + rb * DP + (c % NPT) / 4 * (NSP * 4) + c / NPT * 4 + c % 4;
+#pragma unroll
+        for (int r = 0; r < RPS; ++r) d[r * DP] = gla_decay_of(z[r], a.inv_tau);
+      } else if (c >= a.dim) {
+        float* d = dec_s + rb * DP + (c % NPT) / 4 * (NSP * 4) + c / NPT * 4 + c % 4;
+#pragma unroll
+        for (int r = 0; r < RPS; ++r) d[r * DP] = 0.f;   // padding channels stay zero
+      }
+    }
+    __syncthreads();
+    // ---- the recurrence --------------------------------------------------------
+    for (int r = 0; r < nr; ++r) {
+      float vj[VPT], dot[VPT];
+#pragma unroll
+      for (int c = 0; c < VPT; ++c) {
+        vj[c] = v_s[r * NV + jg * VPT + c];
+        dot[c] = 0.f;
+      }
+#pragma unroll
+      for (int i4 = 0; i4 < NPT / 4; ++i4) {
+        const int at = r * DP + i4 * (NSP * 4) + ns * 4;
+        const float4 d4 = *reinterpret_cast<const float4*>(dec_s + at);
+        const float4 k4 = *reinterpret_cast<const float4*>(k_s + at);
+        const float4 q4 = *reinterpret_cast<const float4*>(q_s + at);
+        const float dd[4] = {d4.x, d4.y, d4.z, d4.w};
+        const float kk[4] = {k4.x, k4.y, k4.z, k4.w};
+        const float qq[4] = {q4.x, q4.y, q4.z, q4.w};
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+#pragma unroll
+          for (int c = 0; c < VPT; ++c) {
+            float& st = S[c][i4 * 4 + e];
+            st = dd[e] * st + kk[e] * vj[c];
+            dot[c] += st * qq[e];
+          }
+      }
+#pragma unroll
+      for (int c = 0; c < VPT; ++c) dot[c] = lanes_sum<NSP>(dot[c]);
+      // only the lanes of this column group read these values, all before now
+      if (ns == 0) {
+#pragma unroll
+        for (int c = 0; c < VPT; ++c) v_s[r * NV + jg * VPT + c] = dot[c];
+      }
+    }
+    __syncthreads();
+    // ---- norm and gate ----------------------------------------------------------
+#pragma unroll
+    for (int i = 0; i < GR; ++i) {
+      const int r = wave + 4 * i;
+      if (r >= nr) continue;                 // uniform over the wave
+      float y[GV];
+      float ss = 0.f;
+#pragma unroll
+      for (int j = 0; j < GV; ++j) {
+        const int c = lane + 64 * j;
+        y[j] = c < a.vdim ? v_s[r * NV + c] : 0.f;
+        ss += y[j] * y[j];
+      }
+      ss = wave_reduce_sum(ss);
+      const float inv = 1.0f / sqrtf(ss / a.vdim + a.eps);
+#pragma unroll
+      for (int j = 0; j < GV; ++j) {
+        const int c = lane + 64 * j;
+        if (c < a.vdim)
+          outp[(row0 + r0 + r) * out_st + c] = ScalarOps<T>::from_f32(
+              y[j] * inv * a.norm[(long)h * a.vdim + c] * gv[i][j] * sigmoid_f(gv[i][j]));
+      }
+    }
+    __syncthreads();   // the next chunk overwrites LDS
+  }
+
+#pragma unroll
+  for (int c = 0; c < VPT; ++c) {
+    const int j = jg * VPT + c;
+    if (j >= a.vdim) continue;
+    float* srow = sbase + (long)j * a.dim;
+#pragma unroll
+    for (int i = 0; i < NPT; i += 4)
+      if (n0 + i < a.dim)      // dim is a multiple of 8
+        *reinterpret_cast<float4*>(srow + n0 + i) =
+            make_float4(S[c][i], S[c][i + 1], S[c][i + 2], S[c][i + 3]);
+  }
+}
+
+// GLA for steps in which the sequences bring single rows: the state is the
+// traffic, so it is streamed column by column (LW lanes per column, a lane
+// holding eight of its elements as two 16-byte pieces) with the row's decays,
+// keys and queries in registers; few registers and many resident waves keep
+// the loads in flight.  Correct for
+// any number of rows: each row reads back what the one before stored.
+template <typename T, int LW>
+__global__ __launch_bounds__(256) void gla_row_kernel(GlaArgs a) {
+  constexpr int COLS = 256 / LW;    // columns side by side
+  constexpr int FLY = 2;            // column groups in flight
+  extern __shared__ float smem[];
+  float* dec_s = smem;              // [LW * 8]
+  float* y_s = dec_s + LW * 8;      // [vdim]
+  float* v_s = y_s + a.vdim;        // [vdim]
+  float* a1_s = v_s + a.vdim;       // [rank]
+  __shared__ float red[8];
+  const int s = blockIdx.x / a.heads;
+  const int h = blockIdx.x % a.heads;
+  const int tid = threadIdx.x, l = tid % LW, jg = tid / LW;
+  const int row0 = a.loc[s];
+  const int n = a.loc[s + 1] - row0;
+  if (n <= 0) return;
+  const int slot = a.slots[s];
+  const long out_st = (long)a.heads * a.vdim;
+  T* outp = reinterpret_cast<T*>(a.out) + (long)h * a.vdim;
+  if (slot < 0) {
+    for (int r = 0; r < n; ++r)
+      for (int c = tid; c < a.vdim; c += 256)
+        outp[(row0 + r) * out_st + c] = ScalarOps<T>::from_f32(0.f);
+    return;
+  }
+  float* sbase = a.state + ((long)slot * a.heads + h) * a.vdim * a.dim;
+  const int p0 = l * 4, p1 = (LW + l) * 4;      // the lane's two pieces of a column
+  const bool in0 = p0 < a.dim, in1 = p1 < a.dim;
+  const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
+  bool carry = a.seq_lens[s] - n > 0;
+  for (int r = 0; r < n; ++r) {
+    const long row = row0 + r;
+    const T* kp = reinterpret_cast<const T*>(a.k) + row * a.k_st + (long)h * a.dim;
+    const T* qp = reinterpret_cast<const T*>(a.q) + row * a.q_st + (long)h * a.dim;
+    const T* vp = reinterpret_cast<const T*>(a.v) + row * a.v_st + (long)h * a.vdim;
+    const T* gp = reinterpret_cast<const T*>(a.g) + row * a.g_st + (long)h * a.vdim;
+    const T* a1p = reinterpret_cast<const T*>(a.a1) + row * a.a1_st;
+    float k[8], q[8], d[8];
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      const int c = (i < 4 ? p0 : p1 - 4) + i;
+      const bool in = i < 4 ? in0 : in1;
+      k[i] = in ? ScalarOps<T>::to_f32(kp[c]) : 0.f;
+      q[i] = in ? ScalarOps<T>::to_f32(qp[c]) * a.q_scale : 0.f;
+    }
+    for (int i = tid; i < a.rank; i += 256) a1_s[i] = ScalarOps<T>::to_f32(a1p[i]);
+    // through LDS: a load inside the column loop would wait for the columns ahead
+    for (int c = tid; c < a.vdim; c += 256) v_s[c] = ScalarOps<T>::to_f32(vp[c]);
+    __syncthreads();
+    for (int c = tid; c < LW * 8; c += 256) {
+      float dv = 0.f;
+      if (c < a.dim) {
+        const float* w2 = a.a2 + (long)h * a.dim + c;
+        const long hd = (long)a.heads * a.dim;
+        float z = a.a2_bias[(long)h * a.dim + c];
+#pragma unroll 8
+        for (int i = 0; i < a.rank; ++i) z += a1_s[i] * w2[i * hd];
+        dv = gla_decay_of(z, a.inv_tau);
+      }
+      dec_s[c] = dv;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < 8; ++i) d[i] = dec_s[(i < 4 ? p0 : p1 - 4) + i];
+    for (int j0 = jg; j0 < a.vdim; j0 += FLY * COLS) {
+      float4 cur[FLY][2];
+#pragma unroll
+      for (int f = 0; f < FLY; ++f) {
+        const int j = j0 + f * COLS;
+        const float* p = sbase + (long)j * a.dim;
+        cur[f][0] = carry && in0 && j < a.vdim ? *reinterpret_cast<const float4*>(p + p0) : zero;
+        cur[f][1] = carry && in1 && j < a.vdim ? *reinterpret_cast<const float4*>(p + p1) : zero;
+      }
+#pragma unroll
+      for (int f = 0; f < FLY; ++f) {
+        const int j = j0 + f * COLS;
+        const bool live = j < a.vdim;
+        const float v = live ? v_s[j] : 0.f;
+        float x[8] = {cur[f][0].x, cur[f][0].y, cur[f][0].z, cur[f][0].w,
+                      cur[f][1].x, cur[f][1].y, cur[f][1].z, cur[f][1].w};
+        float dot = 0.f;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+          x[i] = d[i] * x[i] + k[i] * v;
+          dot += x[i] * q[i];
+        }
+        float* p = sbase + (long)j * a.dim;
+        if (live && in0) *reinterpret_cast<float4*>(p + p0) = make_float4(x[0], x[1], x[2], x[3]);
+        if (live && in1) *reinterpret_cast<float4*>(p + p1) = make_float4(x[4], x[5], x[6], x[7]);
+        dot = lanes_sum<LW>(dot);
+        if (live && l == 0) y_s[j] = dot;
+      }
+    }
+    __syncthreads();
+    float ss = 0.f;
+    for (int c = tid; c < a.vdim; c += 256) ss += y_s[c] * y_s[c];
+    ss = block_reduce_sum(ss, red);
+    const float inv = 1.0f / sqrtf(ss / a.vdim + a.eps);
+    for (int c = tid; c < a.vdim; c += 256) {
+      const float g = ScalarOps<T>::to_f32(gp[c]);
+      outp[row * out_st + c] = ScalarOps<T>::from_f32(
+          y_s[c] * inv * a.norm[(long)h * a.vdim + c] * g * sigmoid_f(g));
+    }
+    __syncthreads();   // LDS is rewritten by the next row
+    carry = true;
+  }
 }
 
 template <typename T, int KIND>
@@ -547,6 +941,57 @@ void launch_gla_scan(float* o, const T* q, long q_st, const T* k, long k_st, con
   launch_matrix_scan<T, KIND_GLA>(a, nseq, stream);
 }
 
+// value columns per thread of the one-kernel form, 0 when the shape does not fit
+int gla_fused_columns(int dim, int vdim) {
+  if (dim % 8 || vdim % 8 || dim > 256) return 0;
+  const int nsp = dim <= 32 ? 2 : dim <= 64 ? 4 : dim <= 128 ? 8 : 16;
+  for (int vpt = 1; vpt <= 4; vpt *= 2)
+    if (256 / nsp * vpt >= vdim) return vpt;
+  return 0;
+}
+
+template <typename T>
+void launch_gla_fused(T* out, const T* q, long q_st, const T* k, long k_st, const T* v,
+                      long v_st, const T* g, long g_st, const T* a1, long a1_st,
+                      const float* a2, const float* a2_bias, float inv_tau, float q_scale,
+                      const float* norm, float eps, float* state, const int* loc,
+                      const int* seq_lens, const int* slots, int nseq, int heads, int dim,
+                      int vdim, int rank, int rows, hipStream_t stream) {
+  GlaArgs a;
+  a.q = q; a.k = k; a.v = v; a.g = g; a.a1 = a1;
+  a.q_st = q_st; a.k_st = k_st; a.v_st = v_st; a.g_st = g_st; a.a1_st = a1_st;
+  a.a2 = a2; a.a2_bias = a2_bias; a.norm = norm;
+  a.inv_tau = inv_tau; a.q_scale = q_scale; a.eps = eps;
+  a.out = out; a.state = state;
+  a.loc = loc; a.seq_lens = seq_lens; a.slots = slots;
+  a.heads = heads; a.dim = dim; a.vdim = vdim; a.rank = rank;
+  const int vpt = gla_fused_columns(dim, vdim);
+  const int rank_p = (rank + 15) & ~15;
+  if (rows <= nseq) {   // a handful of rows per sequence at most: stream the state
+    const int lw = dim <= 32 ? 4 : dim <= 64 ? 8 : dim <= 128 ? 16 : 32;
+    const size_t smem = sizeof(float) * (lw * 8 + 2 * vdim + rank);
+    if (lw == 4) gla_row_kernel<T, 4><<<nseq * heads, 256, smem, stream>>>(a);
+    else if (lw == 8) gla_row_kernel<T, 8><<<nseq * heads, 256, smem, stream>>>(a);
+    else if (lw == 16) gla_row_kernel<T, 16><<<nseq * heads, 256, smem, stream>>>(a);
+    else gla_row_kernel<T, 32><<<nseq * heads, 256, smem, stream>>>(a);
+    return;
+  }
+#define GLA_LAUNCH(N, V)                                                               \
+  gla_fused_kernel<T, N, V><<<nseq * heads, 256,                                       \
+                              sizeof(float) * GLA_ROWS *                               \
+                                  (3 * N * NPT + 256 / N * V + rank_p), stream>>>(a)
+#define GLA_CASE(N)                                                                    \
+  if (vpt == 1) GLA_LAUNCH(N, 1);                                                      \
+  else if (vpt == 2) GLA_LAUNCH(N, 2);                                                 \
+  else GLA_LAUNCH(N, 4)
+  if (dim <= 32) { GLA_CASE(2); }
+  else if (dim <= 64) { GLA_CASE(4); }
+  else if (dim <= 128) { GLA_CASE(8); }
+  else { GLA_CASE(16); }
+#undef GLA_CASE
+#undef GLA_LAUNCH
+}
+
 template <typename T>
 void launch_rglru_scan(T* out, const T* u, const T* r_pre, const T* i_pre,
                        const float* r_bias, const float* i_bias, const float* lam,
@@ -581,6 +1026,12 @@ void launch_rglru_scan(T* out, const T* u, const T* r_pre, const T* i_pre,
                                    const float*, float, float, float*,          \
                                    const int*, const int*, const int*, int, int, \
                                    int, int, int, int, float*, int, hipStream_t); \
+  template void launch_gla_fused<T>(T*, const T*, long, const T*, long,         \
+                                    const T*, long, const T*, long, const T*,   \
+                                    long, const float*, const float*, float,    \
+                                    float, const float*, float, float*,         \
+                                    const int*, const int*, const int*, int,    \
+                                    int, int, int, int, int, hipStream_t);      \
   template void launch_rglru_scan<T>(T*, const T*, const T*, const T*,          \
                                      const float*, const float*, const float*,  \
                                      float, const T*, float*, const int*,       \

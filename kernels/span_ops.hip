@@ -56,6 +56,27 @@ DEVINLINE void ld8<__hip_bfloat16>(const __hip_bfloat16* p, float* f) {
     f[2 * i + 1] = __uint_as_float(u[i] & 0xffff0000u);
   }
 }
+// eight elements as they are stored
+template <typename T> struct Raw8;
+template <> struct Raw8<__hip_bfloat16> { uint4 u; };
+template <> struct Raw8<float> { float4 a, b; };
+template <typename T>
+DEVINLINE Raw8<T> ldraw(const T* p) { return *reinterpret_cast<const Raw8<T>*>(p); }
+template <typename T>
+DEVINLINE void straw(T* p, const Raw8<T>& r) { *reinterpret_cast<Raw8<T>*>(p) = r; }
+DEVINLINE void unpack8(const Raw8<float>& r, float* f) {
+  f[0] = r.a.x; f[1] = r.a.y; f[2] = r.a.z; f[3] = r.a.w;
+  f[4] = r.b.x; f[5] = r.b.y; f[6] = r.b.z; f[7] = r.b.w;
+}
+DEVINLINE void unpack8(const Raw8<__hip_bfloat16>& r, float* f) {
+  const unsigned u[4] = {r.u.x, r.u.y, r.u.z, r.u.w};
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    f[2 * i] = __uint_as_float(u[i] << 16);
+    f[2 * i + 1] = __uint_as_float(u[i] & 0xffff0000u);
+  }
+}
+
 template <typename T>
 DEVINLINE void st8(T* p, const float* f) {
   st4<T>(p, F4{{f[0], f[1], f[2], f[3]}});
@@ -91,12 +112,18 @@ __global__ __launch_bounds__(1024) void stream_add_group_norm_reg_kernel(
   const int t = (wave - g * wpg) * WAVE_SIZE + lane;
   const int step = wpg * WAVE_SIZE;
   const int c0 = g * gsize;
-  F4 xv[NV];
+  F4 xv[NV], wo[NV], wn[NV];
   auto col = [&](int i) { return (t + i * step) * 4; };
+  // everything a reduction does not decide is loaded ahead of it
 #pragma unroll
-  for (int i = 0; i < NV; ++i)
-    if (col(i) < gsize) xv[i] = ld4<float>(x + row * width + c0 + col(i));
-    else xv[i] = F4{{0.f, 0.f, 0.f, 0.f}};
+  for (int i = 0; i < NV; ++i) {
+    xv[i] = wo[i] = wn[i] = F4{{0.f, 0.f, 0.f, 0.f}};
+    if (col(i) < gsize) {
+      xv[i] = ld4<float>(x + row * width + c0 + col(i));
+      if (w_out != nullptr) wo[i] = ld4<float>(w_out + c0 + col(i));
+      if (next_w != nullptr) wn[i] = ld4<float>(next_w + c0 + col(i));
+    }
+  }
   auto group_sum = [&](float s, float* r) {
     s = wave_reduce_sum(s);
     if (lane == 0) r[wave] = s;
@@ -166,9 +193,8 @@ __global__ __launch_bounds__(1024) void stream_add_group_norm_reg_kernel(
 #pragma unroll
     for (int i = 0; i < NV; ++i)
       if (col(i) < gsize) {
-        const F4 w = ld4<float>(w_out + c0 + col(i));
 #pragma unroll
-        for (int k = 0; k < 4; ++k) xv[i].v[k] += y[i].v[k] * inv * w.v[k];
+        for (int k = 0; k < 4; ++k) xv[i].v[k] += y[i].v[k] * inv * wo[i].v[k];
         st4<float>(x + row * width + c0 + col(i), xv[i]);
       }
   }
@@ -182,10 +208,9 @@ __global__ __launch_bounds__(1024) void stream_add_group_norm_reg_kernel(
 #pragma unroll
   for (int i = 0; i < NV; ++i)
     if (col(i) < gsize) {
-      const F4 w = ld4<float>(next_w + c0 + col(i));
       F4 o;
 #pragma unroll
-      for (int k = 0; k < 4; ++k) o.v[k] = xv[i].v[k] * inv * w.v[k];
+      for (int k = 0; k < 4; ++k) o.v[k] = xv[i].v[k] * inv * wn[i].v[k];
       st4<T>(next_out + row * width + c0 + col(i), o);
     }
 }
@@ -398,26 +423,30 @@ __global__ __launch_bounds__(256) void attn_inputs_kernel(AttnIn<T> p) {
 
 // 16-byte accesses: eight lanes per head, a lane owning chunks of eight
 // consecutive channels (for a rotated pair also the partner chunk).  A
-// workgroup walks `tb` consecutive rows per head, so that bias and convolution
-// weights are read once for all of them and earlier rows stay in registers.
-// PC pair chunks and TC unrotated chunks per lane at most.
+// workgroup walks up to AI_ROWS consecutive rows per head, so that bias and convolution
+// weights are read once for all of them and earlier rows stay in registers; the
+// next row is loaded while the current one is computed.  PC pair chunks and TC unrotated chunks per lane at most.
+constexpr int AI_ROWS = 16;
+
 template <typename T, int TAPS, int PC, int TC>
 __global__ __launch_bounds__(256) void attn_inputs_vec_kernel(AttnIn<T> p, int tb) {
   constexpr int NC = 2 * PC + TC;
   constexpr int HIST = TAPS > 1 ? TAPS - 1 : 1;
   constexpr int NW = TAPS > 0 ? TAPS : 1;
-  __shared__ int s_row0[8], s_start[8], s_slot[8];
+  __shared__ int s_row0[AI_ROWS], s_start[AI_ROWS], s_slot[AI_ROWS];
+  __shared__ long s_cache[AI_ROWS];
   const int t0 = blockIdx.x * tb;
   const int n = min(tb, p.rows - t0);
-  if (TAPS > 0) {
-    if (threadIdx.x < n) {
+  if (threadIdx.x < n) {
+    s_cache[threadIdx.x] = p.slot_mapping[t0 + threadIdx.x];
+    if (TAPS > 0) {
       const int s = seq_of_row(p.loc, p.nseq, t0 + threadIdx.x);
       s_row0[threadIdx.x] = p.loc[s];
       s_start[threadIdx.x] = p.lens[s] - (p.loc[s + 1] - p.loc[s]);
       s_slot[threadIdx.x] = p.slots[s];
     }
-    __syncthreads();
   }
+  __syncthreads();
   const int sub = threadIdx.x & 7;
   const int total = p.heads + 2 * p.kv_heads;
   for (int hh = blockIdx.y * 32 + threadIdx.x / 8; hh < total; hh += gridDim.y * 32) {
@@ -439,12 +468,14 @@ __global__ __launch_bounds__(256) void attn_inputs_vec_kernel(AttnIn<T> p, int t
       }
     }
     const int chan = unit_of(p, hh, 0, 0).chan;
-    float bias[NC][8], w[NC][NW][8], hist[NC][HIST][8];
+    float bias[NC][8], wn[NC][8], w[NC][NW][8], hist[NC][HIST][8];
+    const float* norm_w = unit_of(p, hh, 0, 0).w;
 #pragma unroll
     for (int i = 0; i < NC; ++i) {
 #pragma unroll
-      for (int k = 0; k < 8; ++k) bias[i][k] = 0.f;
+      for (int k = 0; k < 8; ++k) { bias[i][k] = 0.f; wn[i][k] = 1.f; }
       if (off[i] >= 0) {
+        if (norm_w != nullptr) ld8<float>(norm_w + off[i], wn[i]);
         if (p.bias != nullptr) ld8<float>(p.bias + chan + off[i], bias[i]);
         if (TAPS > 0) {
 #pragma unroll
@@ -453,9 +484,35 @@ __global__ __launch_bounds__(256) void attn_inputs_vec_kernel(AttnIn<T> p, int t
         }
       }
     }
+    // the next row and its angles, both ahead of this row's stores: loads and
+    // stores retire in order, so a later load would wait for the stores too
+    Raw8<T> next[NC];
+    float next_cs[PC > 0 ? PC : 1][16];
+    auto fetch = [&](long row) {
+      const float2* tab = unit_of(p, hh, row, 0).tab;
+#pragma unroll
+      for (int i = 0; i < NC; ++i)
+        if (off[i] >= 0) next[i] = ldraw<T>(p.proj + row * p.st + chan + off[i]);
+#pragma unroll
+      for (int j = 0; j < PC; ++j)
+        if (off[2 * j] >= 0) {
+          ld8<float>(reinterpret_cast<const float*>(tab + off[2 * j]), next_cs[j]);
+          ld8<float>(reinterpret_cast<const float*>(tab + off[2 * j] + 4), next_cs[j] + 8);
+        }
+    };
+    fetch(t0);
     for (int tt = 0; tt < n; ++tt) {
       const long row = t0 + tt;
-      const long slot = p.slot_mapping[row];
+      const long slot = s_cache[tt];
+      Raw8<T> raw[NC];
+      float cs[PC > 0 ? PC : 1][16];
+#pragma unroll
+      for (int i = 0; i < NC; ++i) raw[i] = next[i];
+#pragma unroll
+      for (int j = 0; j < PC; ++j)
+#pragma unroll
+        for (int k = 0; k < 16; ++k) cs[j][k] = next_cs[j][k];
+      if (tt + 1 < n) fetch(row + 1);
       const Unit<T> u = unit_of(p, hh, row, slot);
       int row0 = 0, start = 0, pos = 0, state_slot = -1;
       T* state = nullptr;
@@ -493,8 +550,7 @@ __global__ __launch_bounds__(256) void attn_inputs_vec_kernel(AttnIn<T> p, int t
       for (int i = 0; i < NC; ++i) {
         if (off[i] < 0) continue;
         float cur[8];
-        const T* src = p.proj + row * p.st + chan + off[i];
-        ld8<T>(src, cur);
+        unpack8(raw[i], cur);
 #pragma unroll
         for (int k = 0; k < 8; ++k) {
           cur[k] += bias[i][k];
@@ -508,17 +564,11 @@ __global__ __launch_bounds__(256) void attn_inputs_vec_kernel(AttnIn<T> p, int t
         }
         if (TAPS > 1) {
           if (p.update_state && state_slot >= 0) {
-            constexpr int V = 16 / sizeof(T);   // elements per 16 bytes
             T* sc = state + chan + off[i];
 #pragma unroll
-            for (int e = 0; e < 8; e += V) {
-#pragma unroll
-              for (int j = 0; j < TAPS - 2; ++j)
-                *reinterpret_cast<uint4*>(sc + (long)j * p.channels + e) =
-                    *reinterpret_cast<const uint4*>(sc + (long)(j + 1) * p.channels + e);
-              *reinterpret_cast<uint4*>(sc + (long)(TAPS - 2) * p.channels + e) =
-                  *reinterpret_cast<const uint4*>(src + e);
-            }
+            for (int j = 0; j < TAPS - 2; ++j)
+              straw<T>(sc + (long)j * p.channels, ldraw<T>(sc + (long)(j + 1) * p.channels));
+            straw<T>(sc + (long)(TAPS - 2) * p.channels, raw[i]);
           }
 #pragma unroll
           for (int j = 0; j < TAPS - 2; ++j)
@@ -534,26 +584,17 @@ __global__ __launch_bounds__(256) void attn_inputs_vec_kernel(AttnIn<T> p, int t
 #pragma unroll
       for (int i = 0; i < NC; ++i) {
         if (off[i] < 0) continue;
-        if (u.w != nullptr) {
-          float wt[8];
-          ld8<float>(u.w + off[i], wt);
 #pragma unroll
-          for (int k = 0; k < 8; ++k) y[i][k] *= inv * wt[k];
-        } else {
-#pragma unroll
-          for (int k = 0; k < 8; ++k) y[i][k] *= inv;
-        }
+        for (int k = 0; k < 8; ++k) y[i][k] *= inv * wn[i][k];
       }
 #pragma unroll
       for (int j = 0; j < PC; ++j) {
         if (off[2 * j] < 0) continue;
-        float oa[8], ob[8], cs[16];
-        ld8<float>(reinterpret_cast<const float*>(u.tab + off[2 * j]), cs);
-        ld8<float>(reinterpret_cast<const float*>(u.tab + off[2 * j] + 4), cs + 8);
+        float oa[8], ob[8];
 #pragma unroll
         for (int k = 0; k < 8; ++k) {
-          oa[k] = y[2 * j][k] * cs[2 * k] - y[2 * j + 1][k] * cs[2 * k + 1];
-          ob[k] = y[2 * j + 1][k] * cs[2 * k] + y[2 * j][k] * cs[2 * k + 1];
+          oa[k] = y[2 * j][k] * cs[j][2 * k] - y[2 * j + 1][k] * cs[j][2 * k + 1];
+          ob[k] = y[2 * j + 1][k] * cs[j][2 * k] + y[2 * j][k] * cs[j][2 * k + 1];
         }
         st8<T>(u.dst + off[2 * j], oa);
         st8<T>(u.dst + off[2 * j + 1], ob);
@@ -566,60 +607,74 @@ __global__ __launch_bounds__(256) void attn_inputs_vec_kernel(AttnIn<T> p, int t
 }
 
 // ---------------------------------------------------------------------------
-// pool_cache_write: one workgroup per new row; the row that completes a block
-// writes the means of the block's cached keys and values to the place of that
-// block inside the cache block that holds its last token.
+// pool_cache_write: one workgroup per `chunk` new rows (<= 256).  Rows that
+// complete a block are found first, one row per thread; for each of them the
+// workgroup writes the means of the block's cached keys and values to the place
+// of that block inside the cache block that holds its last token.
 // ---------------------------------------------------------------------------
 template <typename T>
 __global__ __launch_bounds__(256) void pool_cache_write_kernel(
     const T* __restrict__ k_cache, const T* __restrict__ v_cache, T* __restrict__ k_pool,
     T* __restrict__ v_pool, int pool, int per_block, const int* __restrict__ block_tables,
     int bt_stride, const int* __restrict__ qsl, const int* __restrict__ seq_lens, int nseq,
-    int block_size, int kn, int vn, int vec) {
-  int seq = blockIdx.x, end;
-  if (qsl != nullptr) {
-    seq = seq_of_row(qsl, nseq, blockIdx.x);
-    end = seq_lens[seq] - (qsl[seq + 1] - (int)blockIdx.x) + 1;   // row's position + 1
-  } else {
-    end = seq_lens[seq];
+    int rows, int chunk, int block_size, int kn, int vn, int vec) {
+  __shared__ int done_seq[256], done_end[256], count;
+  if (threadIdx.x == 0) count = 0;
+  __syncthreads();
+  const int row = blockIdx.x * chunk + threadIdx.x;
+  if (threadIdx.x < chunk && row < rows) {
+    int seq = row, end;
+    if (qsl != nullptr) {
+      seq = seq_of_row(qsl, nseq, row);
+      end = seq_lens[seq] - (qsl[seq + 1] - row) + 1;   // row's position + 1
+    } else {
+      end = seq_lens[seq];
+    }
+    if (end > 0 && end % pool == 0) {
+      const int i = atomicAdd(&count, 1);
+      done_seq[i] = seq;
+      done_end[i] = end;
+    }
   }
-  if (end <= 0 || end % pool != 0) return;
-  const int b = end / pool - 1;
-  const int page = (end - 1) / block_size;
-  const int* bt = block_tables + (long)seq * bt_stride;
-  const long dst = (long)bt[page] * per_block + (b - page * block_size / pool);
+  __syncthreads();
+  const int found = count;
   const float inv = 1.0f / pool;
-  const int first = end - pool;
-  auto tok = [&](int j) { return (long)bt[j / block_size] * block_size + j % block_size; };
-  if (vec) {   // eight elements per thread
-    for (int c = threadIdx.x * 8; c < kn + vn; c += blockDim.x * 8) {
+  for (int i = 0; i < found; ++i) {
+    const int end = done_end[i], first = end - pool, b = end / pool - 1;
+    const int page = (end - 1) / block_size;
+    const int* bt = block_tables + (long)done_seq[i] * bt_stride;
+    const long dst = (long)bt[page] * per_block + (b - page * block_size / pool);
+    auto tok = [&](int j) { return (long)bt[j / block_size] * block_size + j % block_size; };
+    if (vec) {   // eight elements per thread
+      for (int c = threadIdx.x * 8; c < kn + vn; c += blockDim.x * 8) {
+        const bool isk = c < kn;
+        const T* src = isk ? k_cache + c : v_cache + (c - kn);
+        const long n = isk ? kn : vn;
+        float s[8];
+#pragma unroll
+        for (int u = 0; u < 8; ++u) s[u] = 0.f;
+#pragma unroll 8
+        for (int j = first; j < end; ++j) {
+          float f[8];
+          ld8<T>(src + tok(j) * n, f);
+#pragma unroll
+          for (int u = 0; u < 8; ++u) s[u] += f[u];
+        }
+#pragma unroll
+        for (int u = 0; u < 8; ++u) s[u] *= inv;
+        st8<T>(isk ? k_pool + dst * kn + c : v_pool + dst * vn + (c - kn), s);
+      }
+      continue;
+    }
+    for (int c = threadIdx.x; c < kn + vn; c += blockDim.x) {
       const bool isk = c < kn;
       const T* src = isk ? k_cache + c : v_cache + (c - kn);
       const long n = isk ? kn : vn;
-      float s[8];
-#pragma unroll
-      for (int u = 0; u < 8; ++u) s[u] = 0.f;
-#pragma unroll 4
-      for (int j = first; j < end; ++j) {
-        float f[8];
-        ld8<T>(src + tok(j) * n, f);
-#pragma unroll
-        for (int u = 0; u < 8; ++u) s[u] += f[u];
-      }
-#pragma unroll
-      for (int u = 0; u < 8; ++u) s[u] *= inv;
-      st8<T>(isk ? k_pool + dst * kn + c : v_pool + dst * vn + (c - kn), s);
+      float s = 0.f;
+      for (int j = first; j < end; ++j) s += ScalarOps<T>::to_f32(src[tok(j) * n]);
+      *(isk ? k_pool + dst * kn + c : v_pool + dst * vn + (c - kn)) =
+          ScalarOps<T>::from_f32(s * inv);
     }
-    return;
-  }
-  for (int c = threadIdx.x; c < kn + vn; c += blockDim.x) {
-    const bool isk = c < kn;
-    const T* src = isk ? k_cache + c : v_cache + (c - kn);
-    const long n = isk ? kn : vn;
-    float s = 0.f;
-    for (int j = first; j < end; ++j) s += ScalarOps<T>::to_f32(src[tok(j) * n]);
-    *(isk ? k_pool + dst * kn + c : v_pool + dst * vn + (c - kn)) =
-        ScalarOps<T>::from_f32(s * inv);
   }
 }
 
@@ -735,10 +790,9 @@ void launch_attn_inputs(T* q_out, const T* proj, long st, const float* bias,
   const int tmax = dim - rot > vdim - vrot ? dim - rot : vdim - vrot;
   vec = vec && pmax <= 128 && tmax <= 128;
   if (vec) {
-    const int tb = rows >= 2048 ? 8 : 1;
+    const int tb = rows >= 4096 ? AI_ROWS : rows >= 2048 ? 8 : 1;
     const int total = heads + 2 * kv_heads;
-    // enough workgroups for few rows too
-    const dim3 grid((rows + tb - 1) / tb, rows < 512 ? (total + 31) / 32 : 1);
+    const dim3 grid((rows + tb - 1) / tb, (total + 31) / 32);
 #define AI_LAUNCH(TP)                                                                   \
     if (tmax == 0) attn_inputs_vec_kernel<T, TP, 1, 0><<<grid, 256, 0, s>>>(p, tb);     \
     else if (pmax == 0) attn_inputs_vec_kernel<T, TP, 0, 2><<<grid, 256, 0, s>>>(p, tb); \
@@ -767,9 +821,11 @@ void launch_pool_cache_write(const T* k_cache, const T* v_cache, T* k_pool, T* v
                              int block_size, int kn, int vn, hipStream_t s) {
   const int vec = kn % 8 == 0 && vn % 8 == 0 && al16(k_cache) && al16(v_cache) &&
                   al16(k_pool) && al16(v_pool);
-  pool_cache_write_kernel<T><<<rows, 256, 0, s>>>(k_cache, v_cache, k_pool, v_pool, pool,
-                                                  per_block, block_tables, bt_stride, qsl,
-                                                  seq_lens, nseq, block_size, kn, vn, vec);
+  // about one completed block per workgroup
+  const int chunk = qsl == nullptr ? 1 : (pool < 256 ? pool : 256);
+  pool_cache_write_kernel<T><<<(rows + chunk - 1) / chunk, 256, 0, s>>>(
+      k_cache, v_cache, k_pool, v_pool, pool, per_block, block_tables, bt_stride, qsl,
+      seq_lens, nseq, rows, chunk, block_size, kn, vn, vec);
 }
 
 template <typename T>

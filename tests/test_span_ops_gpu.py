@@ -141,12 +141,13 @@ def test_attn_inputs_cache_write(dtype, taps, heads, kv_heads, dim, vdim, rot, v
                     _close(gg, ww, dtype, f"{what} case {case}")
 
 
-def test_attn_inputs_many_rows_in_one_workgroup():
-    """Rows enough for the kernel to walk eight of them per workgroup, with
-    sequences that begin and end inside such a run."""
+@pytest.mark.parametrize("long", [1100, 3300])
+def test_attn_inputs_many_rows_in_one_workgroup(long):
+    """Rows enough for the kernel to walk eight or sixteen of them per
+    workgroup, with sequences that begin and end inside such a run."""
     g = torch.Generator().manual_seed(1)
-    rows = [5, 1, 900, 2, 3, 1100, 70]
-    lens = [5, 4, 900, 9, 3, 1103, 70]
+    rows = [5, 1, 900, 2, 3, long, 70]
+    lens = [5, 4, 900, 9, 3, long + 3, 70]
     slots = [0, 3, 1, 2, 5, 4, 6]
     heads, kvh, dim, taps, bs = 2, 1, 32, 3, 16
     t, ch = sum(rows), (2 + 1 + 1) * 32
@@ -292,6 +293,40 @@ def test_gla_scan(dtype, heads, dim, vdim, rank, case):
     want, got = run("cpu", ref.gla_scan), run(DEV, ops.gla_scan)
     _close(got[0], want[0], torch.float32, "outputs")
     _close(got[1], want[1], torch.float32, "state")
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("heads,dim,vdim,rank", [
+    (3, 6, 10, 5),                                          # scan and norm apart
+    (2, 64, 64, 16), (1, 128, 128, 16), (2, 48, 64, 16), (1, 256, 24, 40), (4, 16, 304, 3),
+    (2, 32, 8, 1), (2, 40, 200, 64), (1, 136, 64, 17), (1, 96, 120, 70),
+])
+@pytest.mark.parametrize("case", range(len(SEQS)))
+def test_gla_gated(dtype, heads, dim, vdim, rank, case):
+    rows, lens, slots = SEQS[case]
+    g = torch.Generator().manual_seed(case)
+    t, a, vw = sum(rows), heads * dim, heads * vdim
+    loc = _i32([0] + torch.tensor(rows).cumsum(0).tolist())
+    proj = torch.randn(t, (2 * a + 2 * vw + rank + 15) // 8 * 8, generator=g).to(dtype)
+    a2 = torch.randn(rank, a, generator=g) / math.sqrt(rank)
+    bias = torch.randn(a, generator=g)
+    norm = torch.rand(vw, generator=g) + 0.5
+    state = torch.randn(4, heads, vdim, dim, generator=g)
+    b, c = 2 * a + vw, 2 * a + 2 * vw
+
+    def run(dev, **kw):
+        p, st = proj.to(dev), state.clone().to(dev)
+        out = ops.gla_gated(p[:, :a].view(t, heads, dim), p[:, a:2 * a].view(t, heads, dim),
+                            p[:, 2 * a:b].view(t, heads, vdim), p[:, b:c], p[:, c:c + rank],
+                            a2.to(dev), bias.to(dev), 1.0 / 7.0, dim ** -0.5, norm.to(dev), 1e-5,
+                            st, loc.to(dev), _i32(lens).to(dev), _i32(slots).to(dev), **kw)
+        return out, st
+
+    want = run("cpu")
+    for general in (False, True):
+        got = run(DEV, general=general)
+        _close(got[0], want[0], dtype, f"outputs general={general}")
+        _close(got[1], want[1], torch.float32, f"state general={general}")
 
 
 @pytest.mark.parametrize("dtype", DTYPES)

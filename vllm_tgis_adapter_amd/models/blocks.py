@@ -1347,13 +1347,11 @@ class GLAMixer(_Mixer):
         a = nh * d
         b = 2 * a + nh * dv
         c = b + nh * dv
-        o = ops.gla_scan(
+        return ops.gla_gated(
             proj[:, :a].view(t, nh, d), proj[:, a:2 * a].view(t, nh, d),
-            proj[:, 2 * a:b].view(t, nh, dv), proj[:, c:c + self.rank], self.a2_t,
-            self.a2_bias, 1.0 / self.tau, d ** -0.5, cache[0], meta.seq_start_loc,
-            meta.seq_lens, meta.state_slots)
-        return ops.gated_group_norm(o, proj[:, b:c], self.norm, nh, self.eps,
-                                    gate_first=False, out_dtype=self.dtype, silu_after=True)
+            proj[:, 2 * a:b].view(t, nh, dv), proj[:, b:c], proj[:, c:c + self.rank], self.a2_t,
+            self.a2_bias, 1.0 / self.tau, d ** -0.5, self.norm, self.eps, cache[0],
+            meta.seq_start_loc, meta.seq_lens, meta.state_slots)
 
 
 class BiasedGatedMLP(nn.Module):

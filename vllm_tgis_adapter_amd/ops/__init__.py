@@ -1386,6 +1386,22 @@ def gla_scan(q, k, v, a1, a2_t, a2_bias, inv_tau: float, q_scale: float, state,
                               seq_start_loc.cpu(), seq_lens.cpu(), state_slots.cpu())
 
 
+def gla_gated(q, k, v, gate, a1, a2_t, a2_bias, inv_tau: float, q_scale: float, norm, eps: float,
+              state, seq_start_loc, seq_lens, state_slots, general: bool = False) -> torch.Tensor:
+    """gla_scan, then an RMS norm of every head's output over vdim times
+    ``norm`` [H * vdim] f32 times silu(gate), gate [T, H * vdim] -> [T, H * vdim]
+    in the compute dtype.  One kernel where a workgroup can own a head's value
+    columns (sizes in multiples of 8, rank up to 64) unless ``general``."""
+    if q.numel() and _native_seq(q):
+        out = torch.empty(gate.shape, dtype=q.dtype, device=q.device)
+        _S.gla_gated(out, q, k, v, gate, a1, a2_t, a2_bias, float(inv_tau), float(q_scale), norm,
+                     float(eps), state, seq_start_loc, seq_lens, state_slots, bool(general))
+        return out
+    o = reference.gla_scan(q, k, v, a1, a2_t, a2_bias, inv_tau, q_scale, state,
+                           seq_start_loc.cpu(), seq_lens.cpu(), state_slots.cpu())
+    return reference.gated_group_norm(o, gate, norm, q.shape[1], eps, False, q.dtype, True)
+
+
 def silu_mul_bias(gu: torch.Tensor, bias: torch.Tensor | None = None) -> torch.Tensor:
     """gu [T, 2 ff] (gate columns, then up columns) -> silu(gate + b) * (up + b)
     [T, ff], bias [2 ff] f32."""
