@@ -435,7 +435,9 @@ __global__ __launch_bounds__(256) void attn_inputs_vec_kernel(AttnIn<T> p, int t
   constexpr int NW = TAPS > 0 ? TAPS : 1;
   __shared__ int s_row0[AI_ROWS], s_start[AI_ROWS], s_slot[AI_ROWS];
   __shared__ long s_cache[AI_ROWS];
-  const int t0 = blockIdx.x * tb;
+  // last rows first: a step's single-row sequences lie there and, each with
+  // earlier rows of its own to fetch, take longest
+  const int t0 = (gridDim.x - 1 - blockIdx.x) * tb;
   const int n = min(tb, p.rows - t0);
   if (threadIdx.x < n) {
     s_cache[threadIdx.x] = p.slot_mapping[t0 + threadIdx.x];
@@ -488,8 +490,26 @@ __global__ __launch_bounds__(256) void attn_inputs_vec_kernel(AttnIn<T> p, int t
     // stores retire in order, so a later load would wait for the stores too
     Raw8<T> next[NC];
     float next_cs[PC > 0 ? PC : 1][16];
-    auto fetch = [&](long row) {
+    // ... and the rows ahead of it where they are not the ones just computed
+    Raw8<T> before[NC][HIST];
+    auto fetch = [&](int tt) {
+      const long row = t0 + tt;
       const float2* tab = unit_of(p, hh, row, 0).tab;
+      if (TAPS > 1 && (tt == 0 || row == s_row0[tt])) {
+        const int row0 = s_row0[tt], start = s_start[tt], state_slot = s_slot[tt];
+        const int pos = start + (int)row - row0;
+        const T* state = p.conv_state + (long)max(state_slot, 0) * (TAPS - 1) * p.channels;
+#pragma unroll
+        for (int j = 0; j < TAPS - 1; ++j) {
+          const int pj = pos - (TAPS - 1) + j;
+          if (pj < 0 || (pj < start && state_slot < 0)) continue;
+          const T* src = pj >= start ? p.proj + (long)(row0 + pj - start) * p.st
+                                     : state + (long)(pj - start + TAPS - 1) * p.channels;
+#pragma unroll
+          for (int i = 0; i < NC; ++i)
+            if (off[i] >= 0) before[i][j] = ldraw<T>(src + chan + off[i]);
+        }
+      }
 #pragma unroll
       for (int i = 0; i < NC; ++i)
         if (off[i] >= 0) next[i] = ldraw<T>(p.proj + row * p.st + chan + off[i]);
@@ -500,7 +520,7 @@ __global__ __launch_bounds__(256) void attn_inputs_vec_kernel(AttnIn<T> p, int t
           ld8<float>(reinterpret_cast<const float*>(tab + off[2 * j] + 4), next_cs[j] + 8);
         }
     };
-    fetch(t0);
+    fetch(0);
     for (int tt = 0; tt < n; ++tt) {
       const long row = t0 + tt;
       const long slot = s_cache[tt];
@@ -512,38 +532,30 @@ __global__ __launch_bounds__(256) void attn_inputs_vec_kernel(AttnIn<T> p, int t
       for (int j = 0; j < PC; ++j)
 #pragma unroll
         for (int k = 0; k < 16; ++k) cs[j][k] = next_cs[j][k];
-      if (tt + 1 < n) fetch(row + 1);
-      const Unit<T> u = unit_of(p, hh, row, slot);
-      int row0 = 0, start = 0, pos = 0, state_slot = -1;
+      int state_slot = -1;
       T* state = nullptr;
-      if (TAPS > 0) {
-        row0 = s_row0[tt];
-        start = s_start[tt];
+      if (TAPS > 1) {
         state_slot = s_slot[tt];
-        pos = start + (int)row - row0;
         state = p.conv_state + (long)max(state_slot, 0) * (TAPS - 1) * p.channels;
-        if (TAPS > 1 && (tt == 0 || row == row0)) {   // earlier rows from elsewhere
+        if (tt == 0 || row == s_row0[tt]) {
+          const int start = s_start[tt], pos = start + (int)row - s_row0[tt];
 #pragma unroll
           for (int j = 0; j < TAPS - 1; ++j) {
             const int pj = pos - (TAPS - 1) + j;
+            const bool none = pj < 0 || (pj < start && state_slot < 0);
 #pragma unroll
             for (int i = 0; i < NC; ++i) {
               if (off[i] < 0) continue;
-              if (pj < 0 || (pj < start && state_slot < 0)) {
+              float f[8];
+              unpack8(before[i][j], f);
 #pragma unroll
-                for (int k = 0; k < 8; ++k) hist[i][j][k] = 0.f;
-                continue;
-              }
-              const T* src = pj >= start
-                  ? p.proj + (long)(row0 + pj - start) * p.st
-                  : state + (long)(pj - start + TAPS - 1) * p.channels;
-              ld8<T>(src + chan + off[i], hist[i][j]);
-#pragma unroll
-              for (int k = 0; k < 8; ++k) hist[i][j][k] += bias[i][k];
+              for (int k = 0; k < 8; ++k) hist[i][j][k] = none ? 0.f : f[k] + bias[i][k];
             }
           }
         }
       }
+      if (tt + 1 < n) fetch(tt + 1);
+      const Unit<T> u = unit_of(p, hh, row, slot);
       float y[NC][8];
       float ss = 0.f;
 #pragma unroll

@@ -380,7 +380,7 @@ def _expected_height(window, keep, pool, ctx, at):
     return 0.0
 
 
-MASKS = [(6, 2, 0), (6, 0, 3), (8, 9, 0), (1, 1, 0), (1, 0, 1), (5, 0, 16), (16, 0, 4), (40, 20, 0),
+MASKS = [(6, 2, 0), (6, 0, 3), (8, 9, 0), (1, 1, 0), (1, 0, 1), (5, 0, 16), (16, 0, 4), (41, 19, 0),
          (9, 0, 7)]
 
 
