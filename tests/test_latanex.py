@@ -1,0 +1,660 @@
+"""Latanex through the engine against the plain oracle (tests/latanex_oracle.py).
+
+Every test builds its own small configuration with random weights.  CPU runs
+use the reference ops, GPU runs (marked) the HIP kernels; both go through the
+engine's request, cache-block and state-slot bookkeeping.
+"""
+
+from __future__ import annotations
+
+import math
+
+import pytest
+import torch
+
+import latanex_oracle as oracle
+from test_balenex import _close, _engine, _feed, _run_block, _tokens
+from vllm_tgis_adapter_amd import ops
+from vllm_tgis_adapter_amd.engine import ModelConfig, SamplingParams
+from vllm_tgis_adapter_amd.models import blocks
+
+CPU = pytest.param("cpu", id="cpu")
+GPU = pytest.param("cuda", id="gpu", marks=pytest.mark.gpu)
+DEVICES = [CPU, GPU]
+F64 = torch.float64
+EPS = 1e-5
+
+
+def att_spec(heads=4, kv_heads=2, dim=8, vdim=12, size=7, cap=3.0, v_mix=True, gain=1.3):
+    return {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim,
+            "scale": gain / math.sqrt(dim), "softcap": cap, "mask": {"size": size},
+            "v_mix": v_mix}
+
+
+def delta_spec(heads=6, kv_heads=2, dim=8, vdim=10, conv=3):
+    return {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "conv": conv}
+
+
+def dense(ff=20):
+    return {"kind": "dense", "ff": ff}
+
+
+def routed(experts=12, top=3, count=4, keep=2, ff=9, limit=0.8, scale=1.7, shared=(14, 1.5)):
+    f = {"kind": "moe", "expert": {"ff": ff, "limit": limit},
+         "router": {"experts": experts, "top": top, "scale": scale,
+                    "groups": {"count": count, "keep": keep}}}
+    if shared:
+        f["shared"] = {"ff": shared[0], "limit": shared[1]}
+    return f
+
+
+def make_config(layers=None, width=30, vocab=50, eps=EPS, embed=1.5, logit=0.7):
+    if layers is None:
+        # values are mixed from the second attention on; sizes differ by layer
+        layers = [("attention", att_spec(v_mix=False), dense()),
+                  ("attention", att_spec(size=5), routed()),
+                  ("delta", delta_spec(), routed(8, 2, 2, 1, shared=None)),
+                  ("attention", att_spec(2, 2, 6, 12, size=9, cap=20.0), None),
+                  ("delta", delta_spec(3, 3, 6, 4, conv=4), dense(14)),
+                  ("attention", att_spec(6, 2, 10, 12, size=4), routed(6, 2, 1, 1, ff=5))]
+    return {"architecture": "Latanex", "vocab": vocab, "width": width, "norm": {"eps": eps},
+            "embedding": {"scale": embed}, "logit_scale": logit,
+            "layers": [{"type": t, "mixer": m, "mlp": f} for t, m, f in layers]}
+
+
+@pytest.fixture(scope="module")
+def model(tmp_path_factory):
+    cfg = make_config()
+    w = oracle.random_weights(cfg, seed=1)
+    path = str(tmp_path_factory.mktemp("latanex") / "m")
+    oracle.write_model(path, cfg, w)
+    return cfg, w, path
+
+
+# -- each mechanism alone, as the framework's block, in portions --------------
+
+CUTS = [[23], [1] * 23, [2] * 11 + [1], [7, 1, 1, 3, 2, 9], [21, 2]]
+
+
+def _tensors(shapes, seed):
+    g = torch.Generator().manual_seed(seed)
+    return {n: oracle.random_tensor(n, s, g) for n, s in shapes.items()}
+
+
+def _f64(w):
+    return {k: v.double() for k, v in w.items()}
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("mixes", [False, True])
+@pytest.mark.parametrize("spec", [
+    att_spec(),
+    att_spec(3, 3, 6, 6, size=1, cap=0.5),         # a window of one
+    att_spec(4, 1, 10, 4, size=40, cap=50.0),      # nothing leaves the window
+    att_spec(1, 1, 16, 32, size=3, cap=5.0),       # one head
+    att_spec(6, 2, 24, 16, size=8, cap=1.0, gain=6.0),   # scores far above the cap
+])
+def test_attention_alone(device, spec, mixes):
+    width = 24
+    g = torch.Generator().manual_seed(4)
+    h = torch.randn(23, width, generator=g)
+    w = _tensors(oracle.mixer_shapes("attention", spec, width), 5)
+    ng, dv = spec["kv_heads"], spec["vdim"]
+    first = torch.randn(23, ng, dv, generator=g) if mixes else None
+    want, _ = oracle.attention(h.double(), _f64(w), spec, EPS,
+                               None if first is None else first.double().view(23, -1))
+    mod = blocks.CappedAttention(
+        width, heads=spec["heads"], kv_heads=ng, dim=spec["dim"], vdim=dv, scale=spec["scale"],
+        eps=EPS, window=spec["mask"]["size"], softcap=spec["softcap"], mixes_values=mixes,
+        dtype=torch.float32)
+    mod.load(w)
+    mod = mod.to(device)
+    shapes = mod.cache_shapes(4)
+    if mixes:
+        shapes = shapes + [shapes[1]]
+
+    def call(sl, pos, cache, m):
+        if mixes:     # what the earlier layer cached for these tokens
+            cache[2].view(-1, ng, dv)[m.slot_mapping] = first[sl].to(device)
+        return mod(h[sl].to(device), pos, cache, m)
+
+    for cuts in CUTS:
+        _close(_run_block(call, shapes, 23, device, cuts), want, what=f"cuts {cuts}")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("spec", [
+    delta_spec(), delta_spec(1, 1, 4, 4, conv=1), delta_spec(4, 4, 16, 8, conv=2),
+    delta_spec(3, 1, 5, 7, conv=4),             # sizes off the vector kernels
+    delta_spec(4, 2, 64, 24, conv=3), delta_spec(2, 1, 40, 136, conv=6)])
+def test_delta_alone(device, spec):
+    width = 24
+    g = torch.Generator().manual_seed(6)
+    h = torch.randn(23, width, generator=g)
+    w = _tensors(oracle.mixer_shapes("delta", spec, width), 7)
+    want = oracle.delta(h.double(), _f64(w), spec, EPS)
+    mod = blocks.DeltaMixer(width, heads=spec["heads"], kv_heads=spec["kv_heads"],
+                            dim=spec["dim"], vdim=spec["vdim"], taps=spec["conv"], eps=EPS,
+                            dtype=torch.float32)
+    mod.load(w)
+    mod = mod.to(device)
+    for cuts in CUTS:
+        got = _run_block(lambda sl, pos, cache, m: mod(h[sl].to(device), pos, cache, m),
+                         mod.cache_shapes(4), 23, device, cuts)
+        _close(got, want, what=f"cuts {cuts}")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_tanh_norm_alone(device):
+    g = torch.Generator().manual_seed(10)
+    d = lambda t: t.to(device)
+    for width in (24, 30, 64, 1030):
+        x, a, b = (torch.randn(9, width, generator=g) for _ in range(3))
+        a *= torch.logspace(-5, 1.3, width)      # tiny arguments as well as saturated ones
+        n1 = (0.7, torch.randn(width, generator=g), torch.randn(width, generator=g))
+        n2 = (1.9, torch.randn(width, generator=g), torch.randn(width, generator=g))
+        f = lambda y, n: oracle.tanh_norm(y, n[0], n[1].double(), n[2].double())
+        dn = lambda n: (n[0], d(n[1]), d(n[2]))
+        for two in (False, True):
+            y = a.double() + (b.double() if two else 0.0)
+            want = x.double() + f(y, n1)
+            xs = d(x.clone())
+            nxt = ops.stream_add_tanh_norm(xs, d(a), dn(n1), b=d(b) if two else None,
+                                           next_norm=dn(n2), out_dtype=torch.float32)
+            assert float((xs.double().cpu() - want).abs().max()) < 2e-6
+            assert float((nxt.double().cpu() - f(want, n2)).abs().max()) < 4e-6
+        nxt = ops.stream_add_tanh_norm(d(x), None, None, next_norm=dn(n2),
+                                       out_dtype=torch.float32)
+        assert float((nxt.double().cpu() - f(x.double(), n2)).abs().max()) < 4e-6
+
+
+def test_tanh_norm_keeps_no_statistics():
+    """Scaling one element leaves the others as they are."""
+    x = torch.randn(1, 16, generator=torch.Generator().manual_seed(0))
+    n = (0.9, torch.ones(16), torch.zeros(16))
+    a = ops.stream_add_tanh_norm(x.clone(), None, None, next_norm=n, out_dtype=torch.float32)
+    x[0, 3] *= 1000.0
+    b = ops.stream_add_tanh_norm(x.clone(), None, None, next_norm=n, out_dtype=torch.float32)
+    keep = [i for i in range(16) if i != 3]
+    assert torch.equal(a[0, keep], b[0, keep]) and abs(float(b[0, 3])) == 1.0
+
+
+FFS = [dense(26), routed(), routed(8, 2, 2, 1, ff=7, limit=0.3, shared=None),
+       routed(6, 4, 1, 1, ff=5, scale=1.0, shared=(4, 0.2)),
+       routed(16, 2, 8, 1, ff=3, shared=(11, 3.0)),      # groups of two
+       routed(5, 3, 5, 4, ff=6, limit=2.0),              # groups of one
+       routed(70, 6, 7, 3, ff=4)]                        # more experts than lanes of a wave
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("f", FFS, ids=range(len(FFS)))
+def test_feed_forward_alone(device, f):
+    from vllm_tgis_adapter_amd.models.latanex import SharedAndRouted, build_ff
+
+    g = torch.Generator().manual_seed(11)
+    width = 18
+    w = _tensors(oracle.ff_shapes(f, width), 12)
+    h = torch.randn(11, width, generator=g)
+    mod = build_ff(f, width, torch.float32)
+    if isinstance(mod, SharedAndRouted):
+        mod.load(w)
+    else:
+        mod.load(w["gate"], w["up"], w["down"])
+    y = mod.to(device)(h.to(device))
+    if isinstance(y, tuple):
+        y = y[0] if y[1] is None else y[0] + y[1]
+    _close(y.double().cpu(), oracle.feed_forward(h.double(), _f64(w), f))
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_routing_by_hand(device):
+    """Two groups of three.  Group 1 holds the best single choice score but
+    group 0 the better pair; all choice scores but one are negative; the weights
+    are the scores without the correction."""
+    z = torch.tensor([[0.0, 0.1, -9.0, 1.0, -9.0, -9.0]])
+    corr = torch.tensor([-0.6, -0.6, -0.9, 0.0, -1.5, -1.5])
+    s = torch.sigmoid(z)[0]
+    choice = s + corr
+    assert choice[3] == choice.max() and choice[:2].max() < 0
+    dense_w, ids, w = (t.cpu() for t in ops.moe_route_sigmoid(
+        z.to(device), 2, corr.to(device), 2, 1, True, 2.5))
+    # pairs: (-0.1, -0.075) against (0.73, -1.5)
+    assert sorted(ids[0].tolist()) == [0, 1]
+    total = float(s[0] + s[1])
+    for e in (0, 1):
+        assert abs(float(dense_w[0, e]) - 2.5 * float(s[e]) / total) < 1e-6
+    assert float(dense_w[0, 2:].abs().max()) == 0.0
+    assert abs(float(w.sum()) - 2.5) < 1e-5
+    # a closed group stays closed although every open score left is negative
+    _, ids, _ = ops.moe_route_sigmoid(z.to(device), 3, corr.to(device), 2, 1, True, 1.0)
+    assert sorted(ids[0].tolist()) == [0, 1, 2]
+    # with both groups open the best one wins
+    _, ids, _ = ops.moe_route_sigmoid(z.to(device), 1, corr.to(device), 2, 2, True, 1.0)
+    assert ids[0].tolist() == [3]
+
+
+def test_clamped_gate_by_hand():
+    """The gate is cut from above only, the other factor on both sides and then
+    shifted by one."""
+    gu = torch.tensor([[5.0, -7.0, 0.5, 9.0, -9.0, 0.25]])
+    got = ops.clamped_glu(gu, 2.0)[0]
+    for i, (g, u) in enumerate([(2.0, 2.0), (-7.0, -2.0), (0.5, 0.25)]):
+        want = g / (1.0 + math.exp(-1.702 * g)) * (u + 1.0)
+        assert abs(float(got[i]) - want) < 1e-6
+
+
+def test_delta_rule_replaces_what_a_key_held():
+    """Writing twice under one key with beta 1 and no decay leaves the second
+    value alone, not the sum; the read-out sees the current token's write."""
+    one = torch.tensor([[1.0, 0.0]])
+    k = torch.cat([one, one, one])
+    v = torch.tensor([[3.0], [5.0], [-2.0]])
+    big = torch.full((3, 1), 40.0)               # sigmoid = 1
+    i32 = lambda x: torch.tensor(x, dtype=torch.int32)
+    state = torch.zeros(1, 1, 1, 2)
+    o = ops.delta_scan(k.view(3, 1, 2), k.view(3, 1, 2), v.view(3, 1, 1), big, -big,
+                       torch.zeros(1), torch.zeros(1), state, i32([0, 3]), i32([3]), i32([0]))
+    assert float((o[:, 0] * math.sqrt(2.0) - v[:, 0]).abs().max()) < 1e-4
+    assert abs(float(state[0, 0, 0, 0]) + 2.0) < 1e-4
+
+
+# -- what a query sees: keys far away, at page borders, just inside and outside --
+
+
+def _spike(window, ctx, at, n_new, device, bs=4, dim=8, dtype=torch.float32, cap=30.0,
+           sinks=(-50.0, 9.0)):
+    """Two heads over one key head; every key is small noise but the one at
+    ``at``, which the last query points at; its value is all 100.  The heads
+    differ in their sinks: one without weight, one about as heavy as the spike.
+    Returns the last query's output through the op and from the definition."""
+    g = torch.Generator().manual_seed(ctx * 31 + at)
+    k = torch.randn(ctx, 1, dim, generator=g) * 0.05
+    v = torch.randn(ctx, 1, dim, generator=g) * 0.05
+    q = torch.randn(n_new, 2, dim, generator=g) * 0.05
+    direction = torch.ones(dim) / math.sqrt(dim)
+    k[at, 0] = 3.0 * direction
+    v[at, 0] = 100.0
+    q[-1] = 3.0 * direction
+    k, v, q = k.to(dtype), v.to(dtype), q.to(dtype)
+    sinks = torch.tensor(sinks)
+    nb = (ctx + bs - 1) // bs
+    table = list(range(nb - 1, -1, -1))
+    kc = torch.zeros(nb, bs, 1, dim, dtype=dtype)
+    vc = torch.zeros(nb, bs, 1, dim, dtype=dtype)
+    for p in range(ctx):
+        kc[table[p // bs], p % bs] = k[p]
+        vc[table[p // bs], p % bs] = v[p]
+    dev = lambda t: t.to(device)
+    i32 = lambda x: torch.tensor(x, dtype=torch.int32, device=device)
+    out = torch.empty(n_new, 2, dim, dtype=dtype, device=device)
+    kw = dict(out=out, window=window, sinks=dev(sinks), softcap=cap)
+    if n_new > 1:
+        ops.gqa_attention_prefill(dev(q), dev(kc), dev(vc), i32([table]), i32([0, n_new]),
+                                  i32([ctx]), 1.0, n_new, **kw)
+    else:
+        ops.gqa_attention_decode(dev(q), dev(kc), dev(vc), i32([table]), i32([ctx]), 1.0, **kw)
+    seen = oracle.keys_window(ctx - 1, window or ctx)
+    pair = lambda t: t[seen, 0].double().unsqueeze(0).expand(2, -1, -1)
+    want = oracle.attend(q[-1].double(), pair(k), pair(v), 1.0, cap, sinks.double())
+    return out[-1].double().cpu(), want
+
+
+def _edges(window, ctx):
+    first = max(0, ctx - window)
+    places = {0, 1, ctx - 1, first, first - 1, first + 1, 3, 4, 7, 8, 15, 16}
+    return sorted(p for p in places if 0 <= p < ctx)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("n_new", [1, 2, 7])
+@pytest.mark.parametrize("window", [1, 2, 6, 16, 41, 0])
+def test_edges_and_far_keys(device, n_new, window):
+    for ctx in (7, 30, 64, 150):
+        for at in _edges(window or ctx, ctx):
+            got, want = _spike(window, ctx, at, min(n_new, ctx), device)
+            inside = ctx - 1 - at < (window or ctx)
+            # the spike decides the first head's output exactly when it is seen;
+            # the second head's sink takes about half of it
+            assert (float(want[0].mean()) > 95.0) == inside, (ctx, at)
+            assert not inside or 20.0 < float(want[1].mean()) < 80.0
+            assert float((got - want).abs().max()) < 2e-3, f"ctx {ctx} spike at {at}"
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("dim", [64, 128])
+@pytest.mark.parametrize("cap", [30.0, 200.0])      # with and without a running maximum
+@pytest.mark.parametrize("n_new", [1, 5, 300])
+@pytest.mark.parametrize("window", [1, 33, 64, 100, 257, 0])
+def test_edges_and_far_keys_on_matrix_cores(dim, n_new, window, cap):
+    """The same on the bf16 matrix-core kernels (portions: head size 128)."""
+    for ctx in (130, 700):
+        for at in _edges(window or ctx, ctx) + [63, 64, 127, 128]:
+            if at >= ctx:
+                continue
+            got, want = _spike(window, ctx, at, min(n_new, ctx), "cuda", bs=16, dim=dim,
+                               dtype=torch.bfloat16, cap=cap)
+            assert float((got - want).abs().max()) < 0.6, f"ctx {ctx} spike at {at}"
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_cap_acts_before_the_softmax_and_not_on_the_sink(device):
+    """Two keys with scores far above the cap weigh almost the same; a sink at
+    the cap's height takes a third."""
+    cap = 4.0
+    k = torch.tensor([[40.0], [400.0]]).view(1, 2, 1, 1)
+    v = torch.tensor([[0.0], [9.0]]).view(1, 2, 1, 1)
+    i32 = lambda x: torch.tensor(x, dtype=torch.int32, device=device)
+    out = torch.empty(1, 1, 1, device=device)
+    for sink, want in ((-100.0, 4.5), (4.0, 3.0), (50.0, 0.0)):
+        ops.gqa_attention_decode(torch.ones(1, 1, 1, device=device), k.to(device), v.to(device),
+                                 i32([[0]]), i32([2]), 1.0, out=out, softcap=cap,
+                                 sinks=torch.tensor([sink], device=device))
+        assert abs(float(out) - want) < 1e-3
+
+
+# -- the whole model through the engine ----------------------------------------
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_whole_prompt_and_layers_match_oracle(model, device):
+    cfg, w, path = model
+    toks = _tokens(27, cfg["vocab"], 2)
+    layers = []
+    want = oracle.forward(cfg, w, toks, layers)
+    eng = _engine(path, device)
+    probe = eng.worker.model.stream_probe = []
+    got = _feed(eng, "a", toks, [len(toks)])
+    _close(got, want, what="logits")
+    assert len(probe) == len(layers)
+    for i, (a, b) in enumerate(zip(probe, layers)):
+        _close(a.double().cpu(), b, what=f"stream after layer {i}")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_decode_and_portions_equal_whole(model, device):
+    cfg, w, path = model
+    toks = _tokens(31, cfg["vocab"], 3)
+    want = oracle.forward(cfg, w, toks)
+    eng = _engine(path, device)
+    for k, cuts in enumerate([[1] * 31, [2] * 15 + [1], [5, 3, 2, 7, 1, 1, 4, 8], [29, 2],
+                              [3] + [1] * 28, [4, 4, 4, 4, 4, 4, 4, 3], [7, 7, 7, 7, 3]]):
+        _close(_feed(eng, f"r{k}", toks, cuts), want, what=f"cuts {cuts}")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_long_decode(model, device):
+    cfg, w, path = model
+    toks = _tokens(70, cfg["vocab"], 4)
+    want = oracle.forward(cfg, w, toks)
+    eng = _engine(path, device)
+    _close(_feed(eng, "a", toks, [5] + [1] * 65), want)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_mixed_batch_and_reuse_of_blocks_and_slots(model, device):
+    """Unequal requests in one step, portions beside single tokens, requests
+    that leave and hand their blocks and state slots to later ones."""
+    cfg, w, path = model
+    lens = {"a": 26, "b": 9, "c": 17, "d": 30, "e": 12, "f": 21}
+    toks = {k: _tokens(n, cfg["vocab"], 10 + i) for i, (k, n) in enumerate(lens.items())}
+    want = {k: oracle.forward(cfg, w, t) for k, t in toks.items()}
+    # all six need 32 blocks of 4 tokens and six slots; the pool has 22 blocks
+    # and 4 slots: the later requests run where finished ones were
+    eng = _engine(path, device, blocks=22, slots=4)
+    plan = [
+        [("a", 7), ("b", 2)],
+        [("a", 1), ("b", 5), ("c", 17)],
+        [("a", 9), ("b", 1), ("d", 3)],
+        [("a", 1), ("b", 1), ("d", 2)],
+        [("a", 2), ("d", 1), ("e", 12)],
+        [("a", 6), ("d", 24), ("f", 1)],
+        [("f", 2)],
+        [("f", 18)],
+    ]
+    at = {k: 0 for k in lens}
+    got = {k: [] for k in lens}
+    free_before = eng.block_manager.num_free_blocks
+    for step in plan:
+        entries, end = [], []
+        for k, n in step:
+            entries.append((k, toks[k][at[k]:at[k] + n], list(range(n))))
+            at[k] += n
+            if at[k] == lens[k]:
+                end.append(k)
+        out = eng.replay_step(entries, end).double().cpu()
+        row = 0
+        for k, n in step:
+            got[k].append(out[row:row + n])
+            row += n
+    assert at == lens
+    assert eng.block_manager.num_free_blocks == free_before
+    for k in lens:
+        _close(torch.cat(got[k]), want[k], what=k)
+
+
+def test_a_request_may_sit_out_steps(model):
+    """A request left out of a step goes on later from the state it left."""
+    cfg, w, path = model
+    ta, tb = _tokens(14, cfg["vocab"], 40), _tokens(11, cfg["vocab"], 41)
+    eng = _engine(path, "cpu")
+    ga, gb = [], []
+    ga.append(eng.replay_step([("a", ta[:6], list(range(6)))], []))
+    gb.append(eng.replay_step([("b", tb[:4], list(range(4)))], []))
+    gb.append(eng.replay_step([("b", tb[4:5], [0])], []))
+    out = eng.replay_step([("a", ta[6:7], [0]), ("b", tb[5:], list(range(6)))], ["b"])
+    ga.append(out[:1])
+    gb.append(out[1:])
+    ga.append(eng.replay_step([("a", ta[7:], list(range(7)))], ["a"]))
+    _close(torch.cat(ga).double(), oracle.forward(cfg, w, ta), what="a")
+    _close(torch.cat(gb).double(), oracle.forward(cfg, w, tb), what="b")
+
+
+VARIANTS = {
+    "one_head_everywhere": [
+        ("attention", att_spec(1, 1, 8, 8, size=3), None),
+        ("delta", delta_spec(1, 1, 4, 4, conv=1), None)],
+    "delta_only": [
+        ("delta", delta_spec(4, 1, 16, 8, conv=2), routed(4, 1, 1, 1, shared=None)),
+        ("delta", delta_spec(2, 2, 3, 5, conv=4), dense(7))],
+    "attention_only": [
+        ("attention", att_spec(6, 3, 4, 2, size=2, cap=0.7), routed(9, 2, 3, 2)),
+        ("attention", att_spec(3, 3, 12, 2, size=50), dense(31)),
+        ("attention", att_spec(3, 3, 5, 2, size=1), None)],
+    # the layer whose values are mixed in lies behind others that do not mix
+    "late_first_values": [
+        ("delta", delta_spec(), None),
+        ("attention", att_spec(2, 1, 6, 9, v_mix=False), dense(5)),
+        ("attention", att_spec(4, 2, 6, 3, size=6), dense(9)),
+        ("delta", delta_spec(2, 1, 8, 8), dense(4)),
+        ("attention", att_spec(2, 1, 6, 9, v_mix=False), None),
+        ("attention", att_spec(2, 2, 4, 3, size=30), dense(6)),
+        ("attention", att_spec(8, 2, 7, 3, size=2), None)],
+}
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("variant", sorted(VARIANTS))
+def test_other_shapes(tmp_path, device, variant):
+    cfg = make_config(VARIANTS[variant], width=20, vocab=31, eps=1e-4, embed=0.6, logit=3.0)
+    w = oracle.random_weights(cfg, seed=5)
+    oracle.write_model(str(tmp_path / "v"), cfg, w)
+    toks = _tokens(22, cfg["vocab"], 6)
+    want = oracle.forward(cfg, w, toks)
+    eng = _engine(str(tmp_path / "v"), device, block_size=8)
+    _close(_feed(eng, "a", toks, [22]), want, what="whole")
+    _close(_feed(eng, "b", toks, [3, 2, 9, 1, 1, 6]), want, what="portions")
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_bf16_stays_near_oracle(model, device):
+    cfg, w, path = model
+    toks = _tokens(25, cfg["vocab"], 7)
+    want = oracle.forward(cfg, w, toks)
+    eng = _engine(path, device, dtype="bfloat16")
+    got = _feed(eng, "a", toks, [11, 1, 1, 12])
+    # a close call of a router may fall the other way in bf16
+    err = (got - want).abs().amax(1)
+    assert float(err.median()) < 0.05 * float(want.abs().max())
+    assert int((err > 0.05 * float(want.abs().max())).sum()) <= 3
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_matrix_core_shapes(tmp_path, dtype):
+    """Head sizes the matrix-core attention kernels take and experts the grouped
+    product takes, long enough for several key tiles, edges inside tiles."""
+    layers = [("attention", att_spec(4, 2, 128, 128, size=50, cap=20.0), dense(256)),
+              ("delta", delta_spec(4, 2, 64, 128, conv=4),
+               routed(8, 2, 4, 2, ff=128, shared=(256, 1.0))),
+              ("attention", att_spec(4, 2, 64, 128, size=37, cap=90.0), None),
+              ("attention", att_spec(2, 2, 128, 128, size=300, cap=5.0), dense(128)),
+              ("attention", att_spec(8, 1, 64, 64, size=33, v_mix=False), None),
+              ("delta", delta_spec(2, 2, 128, 32, conv=2), None)]
+    cfg = make_config(layers, width=128, vocab=40)
+    w = oracle.random_weights(cfg, seed=8)
+    oracle.write_model(str(tmp_path / "m"), cfg, w)
+    toks = _tokens(190, cfg["vocab"], 9)
+    want = oracle.forward(cfg, w, toks)
+    eng = _engine(str(tmp_path / "m"), "cuda", dtype=dtype, blocks=60, block_size=16)
+    for rid, cuts in (("a", [190]), ("b", [70, 3, 60, 2] + [1] * 55)):
+        got = _feed(eng, rid, toks, cuts)
+        if dtype == "float32":
+            _close(got, want, dtype, rid)
+        else:
+            err = (got - want).abs().amax(1) / float(want.abs().max())
+            assert float(err.median()) < 0.05 and int((err > 0.08).sum()) <= 12, rid
+
+
+@pytest.mark.gpu
+def test_captured_decode_steps_match_eager(model):
+    cfg, w, path = model
+    prompts = {k: _tokens(n, cfg["vocab"], 20 + i) for i, (k, n) in
+               enumerate({"a": 9, "b": 4, "c": 13}.items())}
+
+    def generate(eager):
+        eng = _engine(path, "cuda", eager=eager)
+        for k, t in prompts.items():
+            eng.add_request(k, None, list(t), SamplingParams(temperature=0.0, max_tokens=12))
+        out = {}
+        while eng.has_unfinished():
+            for o in eng.step():
+                if o.finished:
+                    out[o.request_id] = list(o.outputs[0].token_ids)
+        return out, eng
+
+    eager, _ = generate(True)
+    graphs, eng = generate(False)
+    assert eng.worker.graph_runner is not None and eng.worker.graph_runner.graphs
+    assert eager == graphs
+
+
+# -- generation through the engine's own entry point --------------------------
+
+
+def _check_greedy(cfg, w, prompt, got, steps, stop=None):
+    seq = list(prompt)
+    for j in range(steps):
+        logits = oracle.forward(cfg, w, seq)[-1]
+        top2 = torch.topk(logits, 2).values
+        if float(top2[0] - top2[1]) < 1e-3:      # a close call proves nothing
+            break
+        seq.append(int(torch.argmax(logits)))
+        assert got[j] == seq[-1], f"token {j}"
+        if seq[-1] == stop:
+            break
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_greedy_generation_matches_oracle(model, device):
+    cfg, w, path = model
+    prompts = {"a": _tokens(7, cfg["vocab"], 30), "b": _tokens(15, cfg["vocab"], 31),
+               "c": _tokens(2, cfg["vocab"], 32)}
+    steps = 10
+    eng = _engine(path, device)
+    for k, t in prompts.items():
+        eng.add_request(k, None, list(t), SamplingParams(temperature=0.0, max_tokens=steps))
+    got = {}
+    while eng.has_unfinished():
+        for o in eng.step():
+            if o.finished:
+                got[o.request_id] = list(o.outputs[0].token_ids)
+    for k, t in prompts.items():
+        _check_greedy(cfg, w, t, got[k], steps)
+
+
+def test_registry_and_cache_layout(model):
+    cfg, w, path = model
+    mc = ModelConfig.from_model_arg(path, dtype="float32")
+    assert mc.architecture == "latanex" and mc.num_layers == 6 and mc.vocab_size == 50
+    from vllm_tgis_adapter_amd.models import get_model, native_extensions
+
+    assert native_extensions(mc) == ["_C_seq"]
+    m = get_model(mc)
+    assert m.uses_seq_state and m.first_values == 1
+    caches = m.allocate_caches(3, 4, 2, "cpu")
+    shapes = [[tuple(c.shape) for c in cs] for cs in caches]
+    assert shapes[0] == [(3, 4, 2, 8), (3, 4, 2, 12)]
+    assert shapes[1] == [(3, 4, 2, 8), (3, 4, 2, 12)]
+    # convolution rows of [q | k | v], recurrent state
+    assert shapes[2] == [(2, 2, 92), (2, 6, 10, 8)]
+    # own keys and values, then the first mixing layer's values
+    assert shapes[3] == [(3, 4, 2, 6), (3, 4, 2, 12), (3, 4, 2, 12)]
+    assert caches[3][2] is caches[1][1] and caches[5][2] is caches[1][1]
+    assert m.state_bytes_per_slot() == 4 * (2 * 92 + 6 * 10 * 8 + 3 * 48 + 3 * 4 * 6)
+    assert m.cache_bytes_per_block(4) == 4 * 4 * 2 * ((8 + 12) * 2 + (6 + 12) + (10 + 12))
+
+
+def test_config_errors():
+    from vllm_tgis_adapter_amd.models.latanex import build_ff, model_config_from_json
+
+    with pytest.raises(ValueError):
+        model_config_from_json("x", make_config([("rwkv", {}, None)]))
+    with pytest.raises(ValueError):     # values of another shape cannot be mixed
+        model_config_from_json("x", make_config([("attention", att_spec(), None),
+                                                 ("attention", att_spec(vdim=6), None)]))
+    with pytest.raises(ValueError):
+        build_ff({"kind": "sparse"}, 8, torch.float32)
+    with pytest.raises(ValueError):     # more chosen experts than one group holds
+        build_ff(routed(8, 5, 2, 1), 8, torch.float32)
+    with pytest.raises(ValueError):
+        build_ff(routed(9, 2, 2, 1), 8, torch.float32)
+    with pytest.raises(ValueError):
+        blocks.DeltaMixer(8, heads=3, kv_heads=2, dim=4, vdim=4, taps=2, eps=EPS)
+
+
+def test_served_from_command_line_flags(tmp_path):
+    """A model directory given as --model goes through the server's flag
+    parsing into the async engine and streams greedy tokens equal to the
+    oracle's, concurrent requests included."""
+    import asyncio
+
+    from vllm_tgis_adapter_amd.__main__ import parse_args
+    from vllm_tgis_adapter_amd.engine.async_engine import AsyncLLMEngine
+    from vllm_tgis_adapter_amd.tgis_utils.args import engine_config_from_args
+
+    cfg = make_config(vocab=300)    # room for the byte-level test tokenizer
+    w = oracle.random_weights(cfg, seed=5)
+    oracle.write_model(str(tmp_path / "served"), cfg, w)
+    args = parse_args(["--model", str(tmp_path / "served"), "--dtype", "float32",
+                       "--max-num-seqs", "2", "--num-gpu-blocks", "64", "--block-size", "8",
+                       "--device", "cpu"])
+    engine = AsyncLLMEngine(engine_config_from_args(args))
+    prompts = {"x": _tokens(12, 300, 61), "y": _tokens(5, 300, 62), "z": _tokens(9, 300, 63)}
+
+    async def one(rid):
+        last = None
+        async for out in engine.generate(
+                {"prompt_token_ids": prompts[rid]},
+                SamplingParams(temperature=0.0, max_tokens=5), request_id=rid):
+            last = out
+        return rid, list(last.outputs[0].token_ids)
+
+    async def main():
+        return dict(await asyncio.gather(*[one(r) for r in prompts]))
+
+    try:
+        got = asyncio.run(main())
+    finally:
+        engine.shutdown()
+    for rid, p in prompts.items():
+        _check_greedy(cfg, w, p, got[rid], 5, stop=engine.engine.eos_token_id)

@@ -38,6 +38,10 @@ def get_model(cfg: ModelConfig):
         from .balenex import BalenexForCausalLM
 
         return BalenexForCausalLM(cfg)
+    if cfg.architecture == "latanex":
+        from .latanex import LatanexForCausalLM
+
+        return LatanexForCausalLM(cfg)
     raise ValueError(f"Unsupported architecture: {cfg.architecture}")
 
 
@@ -63,4 +67,8 @@ def native_extensions(cfg: ModelConfig) -> list[str]:
         from .balenex import native_extensions as bx
 
         return bx(cfg)
+    if cfg.architecture == "latanex":
+        from .latanex import native_extensions as lx
+
+        return lx(cfg)
     return ["_C"]

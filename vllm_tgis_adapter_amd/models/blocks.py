@@ -14,7 +14,8 @@ that another design can assemble them differently:
 - ``TokenSideInput``    gated per-layer token embedding added to the stream
                         through its own RMS norm
 - ``StreamLayerNorm``   bias-free layer norm of the f32 stream
-- ``GatedDenseMLP``     down(act(gate(h)) * up(h)) with the tanh-form GELU
+- ``GatedDenseMLP``     down(act(gate(h)) * up(h)) with the tanh-form GELU or
+                        silu, or a clamped gate
 - ``QKNormAttention``   grouped-query softmax attention over the paged cache,
                         per-head RMS norm on queries and keys, no rotation, an
                         optional position-dependent query temperature; the
@@ -43,8 +44,10 @@ that another design can assemble them differently:
                         sigmoid gate
 - ``HGRN2Mixer``        gated linear recurrence whose forget gate (with a
                         per-channel lower bound) also sets what is written
-- ``GatedRoutedExperts`` sigmoid router, top-k of small gated (silu) experts
-                        whose input is multiplied by the routing weight
+- ``GatedRoutedExperts`` sigmoid router (optionally with a choice correction,
+                        groups of experts, renormalised weights), top-k of small
+                        gated experts (silu, or a clamped gate) whose input or
+                        output is multiplied by the routing weight
 - ``stepped_rotary_frequencies``  rotation frequencies divided by a factor
                         for long wavelengths, kept for short ones, blended
                         linearly in between
@@ -58,6 +61,13 @@ that another design can assemble them differently:
                         data-dependent decay per key channel from a low-rank
                         projection
 - ``BiasedGatedMLP``    down(silu(gate h + b) * (up h + b)) + b
+- ``StreamTanhNorm``    tanh(alpha x) * w + b, a norm without statistics
+- ``CappedAttention``   grouped-query attention over a sliding window with
+                        soft-capped scores, a learned sink per head, query/key
+                        norm over the whole projection and values mixed with
+                        those of an earlier layer
+- ``DeltaMixer``        gated delta rule: a matrix state per head that is decayed
+                        and corrected towards each token's value
 
 The recurrent mixers keep their state (f32) and the last inputs of their short
 convolutions in per-sequence slots; a sequence that starts in a step starts
@@ -365,13 +375,18 @@ class StreamLayerNorm(nn.Module):
 
 
 class GatedDenseMLP(nn.Module):
-    """down(gelu_tanh(gate h) * (up h)); gate and up are one merged product."""
+    """down(act(gate h, up h)); gate and up are one merged product.  ``act``:
+    "gelu_tanh" or "silu" of the gate times up, or "clamped", with ``limit``:
+    g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = up within +-limit."""
 
-    def __init__(self, width: int, ff: int, dtype: torch.dtype):
+    def __init__(self, width: int, ff: int, dtype: torch.dtype, act: str = "gelu_tanh",
+                 limit: float = 0.0):
         super().__init__()
         if get_tp_world_size() != 1:
             raise ValueError("GatedDenseMLP is not sharded; run it with one rank")
-        self.ff = ff
+        if act not in ("gelu_tanh", "silu", "clamped"):
+            raise ValueError(f"unknown activation {act!r}")
+        self.ff, self.act, self.limit = ff, act, limit
         self.gate_up = _randn_param((2 * ff, width), dtype)
         self.down = _randn_param((width, ff), dtype)
 
@@ -382,7 +397,12 @@ class GatedDenseMLP(nn.Module):
 
     def forward(self, h: torch.Tensor) -> torch.Tensor:
         gu = ops.linear(h, self.gate_up)
-        a = ops.gelu_tanh(gu[:, :self.ff], mul=gu[:, self.ff:])
+        if self.act == "clamped":
+            a = ops.clamped_glu(gu, self.limit)
+        elif self.act == "silu":
+            a = ops.silu_mul_bias(gu)
+        else:
+            a = ops.gelu_tanh(gu[:, :self.ff], mul=gu[:, self.ff:])
         return ops.linear(a, self.down)
 
 
@@ -1095,31 +1115,44 @@ class HGRN2Mixer(_Mixer):
 
 
 class GatedRoutedExperts(nn.Module):
-    """Mixture of ``experts`` small feed-forwards down(silu(gate x) * (up x))
-    without biases.  Router: z = W_r h in f32, s = sigmoid(z); the ``top``
-    largest s are chosen and weigh their experts as they are (no
-    renormalising).  The weight multiplies the expert's *input*: y = sum
-    expert(s_e h).
+    """Mixture of ``experts`` small gated feed-forwards without biases.  Router:
+    z = W_r h in f32, s = sigmoid(z); choice scores are s (``correction``: plus
+    one learned number per expert); with ``groups`` = (count, keep) only experts
+    of the ``keep`` best groups of neighbours stay open (best by the sum of a
+    group's two largest choice scores); the ``top`` largest are chosen.  Their
+    weights are s as it is, or (``renormalise``) divided by their sum, times
+    ``weight_scale``.  Expert: down(silu(gate x) * (up x)), whose *input* is
+    multiplied by the weight, y = sum expert(s_e h); or, with ``limit``, the
+    clamped gate of GatedDenseMLP, weighted at the output, y = sum s_e expert(h).
 
-    Without biases gate (s h) = s (gate h), so the weight is applied to the
-    projected rows.  Two ways to run the experts, chosen by shape:
+    A weight at the input goes through gate (s h) = s (gate h) to the projected
+    rows; one at the output multiplies the activation or the combined rows.
+    Two ways to run the experts, chosen by shape:
 
     - stacked: one product with every expert's [gate ; up] rows stacked
-      [E * 2 ff, width], silu(s g) * (s u) with s = 0 for unchosen experts (they
+      [E * 2 ff, width], the activation with weight 0 for unchosen experts (they
       vanish exactly), one product with the down-projections stacked along the
       contraction axis.  Any size, f32 or bf16, shape-static.
-    - grouped: token-expert pairs grouped by expert, their rows multiplied by
-      s, one grouped gated product and one grouped down-projection over the
-      expert segments (bf16, sizes in multiples of 128), gather-sum."""
+    - grouped: token-expert pairs grouped by expert (their rows multiplied by s
+      if the weight is the input's), one grouped gated product and one grouped
+      down-projection over the expert segments (bf16, sizes in multiples of
+      128), gather-sum."""
 
     def __init__(self, width: int, *, experts: int, top: int, ff: int,
-                 dtype: torch.dtype, grouped: Optional[bool] = None):
+                 dtype: torch.dtype, grouped: Optional[bool] = None, correction: bool = False,
+                 groups: tuple = (1, 1), renormalise: bool = False, weight_scale: float = 1.0,
+                 limit: Optional[float] = None):
         super().__init__()
         if get_tp_world_size() != 1:
             raise ValueError("GatedRoutedExperts is not sharded; run it with one rank")
-        if not 1 <= top <= experts:
-            raise ValueError("top must lie between 1 and the number of experts")
+        count, keep = groups
+        if experts % count or not 1 <= keep <= count:
+            raise ValueError("groups must be equal, and some of them kept")
+        if not 1 <= top <= keep * (experts // count):
+            raise ValueError("top must lie between 1 and the number of open experts")
         self.width, self.experts, self.top, self.ff = width, experts, top, ff
+        self.groups, self.renormalise, self.weight_scale = (count, keep), renormalise, weight_scale
+        self.limit = limit
         self.dtype = dtype
         fits = dtype == torch.bfloat16 and ff % 128 == 0 and width % 128 == 0
         self.grouped = (fits and experts > 2 * top) if grouped is None else bool(grouped)
@@ -1128,6 +1161,7 @@ class GatedRoutedExperts(nn.Module):
         self.router = nn.Parameter(
             torch.empty(experts, width, dtype=torch.float32).normal_(0.0, width ** -0.5),
             requires_grad=False)
+        self.correction = _f32_param(experts) if correction else None
         # per expert: ff gate rows, then ff up rows
         self.gate_up = _randn_param((experts, 2 * ff, width), dtype, std=width ** -0.5)
         if self.grouped:
@@ -1135,8 +1169,10 @@ class GatedRoutedExperts(nn.Module):
         else:
             self.down = _randn_param((width, experts * ff), dtype, std=ff ** -0.5)
 
-    def load(self, router, gates: list, ups: list, downs: list) -> None:
+    def load(self, router, gates: list, ups: list, downs: list, correction=None) -> None:
         self.router.data.copy_(router.float())
+        if self.correction is not None:
+            self.correction.data.copy_(correction.float())
         ff = self.ff
         for e, (g, u, d) in enumerate(zip(gates, ups, downs)):
             self.gate_up.data[e, :ff].copy_(g.to(self.dtype))
@@ -1146,20 +1182,29 @@ class GatedRoutedExperts(nn.Module):
             else:
                 self.down.data[:, e * ff:(e + 1) * ff].copy_(d.to(self.dtype))
 
+    def route(self, z: torch.Tensor):
+        return ops.moe_route_sigmoid(z, self.top, self.correction, *self.groups,
+                                     self.renormalise, self.weight_scale)
+
     def forward(self, h: torch.Tensor, router_in: Optional[torch.Tensor] = None) -> torch.Tensor:
         """``router_in``: the f32 rows h was rounded from, when the caller has
         them; the router then reads those instead of the rounded copy."""
-        z = torch.nn.functional.linear(h.float() if router_in is None else router_in,
-                                       self.router)
-        dense, ids, w = ops.moe_route_sigmoid(z, self.top)
+        dense, ids, w = self.route(
+            ops.router_logits(h if router_in is None else router_in, self.router))
         ne = self.experts
         if not self.grouped:
             gu = ops.linear(h, self.gate_up.view(ne * 2 * self.ff, self.width))
-            return ops.linear(ops.silu_mul_scaled(gu, dense), self.down)
-        xs, pos, seg = ops.moe_sort(ids, ne, h, row_scale=w)
-        a = ops.moe_gemm(xs, self.gate_up, seg, gated=True)
-        ye = ops.moe_gemm(a, self.down, seg, gated=False)
-        return ops.moe_combine(ye, pos, ids, torch.ones_like(w), ne)
+            a = (ops.silu_mul_scaled(gu, dense) if self.limit is None
+                 else ops.clamped_glu(gu, self.limit, dense))
+            return ops.linear(a, self.down)
+        if self.limit is None:
+            xs, pos, seg = ops.moe_sort(ids, ne, h, row_scale=w)
+            a = ops.moe_gemm(xs, self.gate_up, seg, gated=True)
+            w = torch.ones_like(w)
+        else:
+            xs, pos, seg = ops.moe_sort(ids, ne, h)
+            a = ops.moe_gemm(xs, self.gate_up, seg, gated=True, act="clamped", limit=self.limit)
+        return ops.moe_combine(ops.moe_gemm(a, self.down, seg, gated=False), pos, ids, w, ne)
 
 
 # ---------------------------------------------------------------------------
@@ -1381,3 +1426,170 @@ class BiasedGatedMLP(nn.Module):
     def forward(self, h: torch.Tensor) -> torch.Tensor:
         return ops.linear(ops.silu_mul_bias(ops.linear(h, self.gate_up), self.gate_up_bias),
                           self.down)
+
+
+# ---------------------------------------------------------------------------
+# Norms without statistics, soft-capped windowed attention with sinks per head
+# and mixed values, the gated delta rule.
+# ---------------------------------------------------------------------------
+
+
+class StreamTanhNorm(nn.Module):
+    """tanh(alpha x) * w + b, alpha one number: a norm that computes no mean or
+    variance.  Applied by the residual kernel, which takes ``triple()``."""
+
+    def __init__(self, width: int, alpha: float = 0.5):
+        super().__init__()
+        self.alpha = alpha
+        self.weight = _f32_param(width, fill=1.0)
+        self.bias = _f32_param(width)
+
+    def load(self, weight, alpha, bias) -> None:
+        self.weight.data.copy_(weight.float())
+        self.bias.data.copy_(bias.float())
+        self.alpha = float(alpha)
+
+    def triple(self):
+        return (self.alpha, self.weight, self.bias)
+
+
+class CappedAttention(_Mixer):
+    """Causal grouped-query softmax attention without positions.
+
+    Projected rows: [q | k | v], plus biases.  q and k are RMS-normed over the
+    whole projection (one mean over all heads, a weight per row).  score =
+    q . k * scale, then ``softcap`` * tanh(score / softcap) (0: no cap); a query
+    at position i sees keys j with 0 <= i - j < ``window`` (0: every j <= i); the
+    softmax denominator of head h also holds exp(sink_h).  ``mixes_values``: v
+    <- (1 - lam) v + lam v_first before it is cached, v_first being the cached
+    values of an earlier layer for the same token, whose value cache follows
+    this layer's own tensors in ``cache``."""
+
+    def __init__(self, width: int, *, heads: int, kv_heads: int, dim: int, vdim: int,
+                 scale: float, eps: float, window: int = 0, softcap: float = 0.0,
+                 mixes_values: bool = False, own_in: bool = True,
+                 dtype: torch.dtype = torch.bfloat16):
+        super().__init__()
+        if heads % kv_heads:
+            raise ValueError("heads must be a multiple of kv_heads")
+        if window < 0 or softcap < 0:
+            raise ValueError("window and softcap must not be negative")
+        self.heads, self.kv_heads, self.dim, self.vdim = heads, kv_heads, dim, vdim
+        self.scale, self.eps, self.window, self.softcap = scale, eps, window, softcap
+        self.mixes_values = mixes_values
+        self.v_mix = 0.5
+        self.in_rows = heads * dim + kv_heads * (dim + vdim)
+        self.out_rows = heads * vdim
+        self._alloc(width, own_in, dtype)
+        self.qkv_bias = _f32_param(self.in_rows)
+        self.q_norm = _f32_param(heads * dim, fill=1.0)
+        self.k_norm = _f32_param(kv_heads * dim, fill=1.0)
+        self.sinks = _f32_param(heads)
+
+    def load_in(self, weight, bias, t) -> None:
+        off = 0
+        for name in ("q", "k", "v"):
+            n = t[name].shape[0]
+            weight[off:off + n].copy_(t[name].to(weight.dtype))
+            self.qkv_bias.data[off:off + n].copy_(t[name + ".b"].float())
+            off += n
+        if off != self.in_rows:
+            raise ValueError("projection tensors do not add up to the mixer's rows")
+
+    def load_rest(self, t) -> None:
+        self.q_norm.data.copy_(t["q.norm"].float())
+        self.k_norm.data.copy_(t["k.norm"].float())
+        self.sinks.data.copy_(t["sink"].float())
+        if self.mixes_values:
+            self.v_mix = float(t["vmix"])
+
+    def cache_shapes(self, block_size: int) -> list:
+        return [("paged", (block_size, self.kv_heads, self.dim), self.dtype),
+                ("paged", (block_size, self.kv_heads, self.vdim), self.dtype)]
+
+    def mix(self, proj, positions, cache, meta: AttnMetadata) -> torch.Tensor:
+        t, nh, dv = proj.shape[0], self.heads, self.vdim
+        k_cache, v_cache = cache[0], cache[1]
+        q = ops.wide_norm_cache_write(
+            proj, self.qkv_bias, nh, self.kv_heads, self.dim, dv, self.eps, self.q_norm,
+            self.k_norm, cache[2] if self.mixes_values else None, self.v_mix, k_cache, v_cache,
+            meta.slot_mapping)
+        out = torch.empty((t, nh, dv), dtype=proj.dtype, device=proj.device)
+        npt = meta.num_prefill_tokens
+        kw = dict(window=self.window, sinks=self.sinks, softcap=self.softcap)
+        if npt:
+            ops.gqa_attention_prefill(
+                q[:npt], k_cache, v_cache, meta.prefill_block_tables,
+                meta.prefill_query_start_loc, meta.prefill_seq_lens, self.scale,
+                meta.max_prefill_query_len, out=out[:npt], **kw)
+        if meta.num_decode_seqs:
+            ops.gqa_attention_decode(
+                q[npt:], k_cache, v_cache, meta.decode_block_tables, meta.decode_seq_lens,
+                self.scale, out=out[npt:], **kw)
+        return out.view(t, nh * dv)
+
+
+class DeltaMixer(_Mixer):
+    """Gated delta rule.  q, k (kv_heads x dim) and v (heads x vdim) pass a short
+    causal convolution per channel and silu; q and k become unit vectors per
+    head, q times dim^-1/2; beta = sigmoid(W_b h), decay g = exp(-exp(A_log)
+    softplus(W_a h + dt_bias)) per head.  S <- g S, u = beta (v - S^T k), S <- S +
+    k u^T, o = S^T q; head h uses query / key head h / (heads / kv_heads).  Each
+    head's o is RMS-normed over vdim with one weight for all heads, times
+    silu(W_g h).  Projected rows: [q | k | v | g | b | a], zero rows up to a
+    multiple of 8."""
+
+    def __init__(self, width: int, *, heads: int, kv_heads: int, dim: int, vdim: int, taps: int,
+                 eps: float, own_in: bool = True, dtype: torch.dtype = torch.bfloat16):
+        super().__init__()
+        if heads % kv_heads or taps < 1:
+            raise ValueError("heads must be a multiple of kv_heads, taps at least 1")
+        self.heads, self.kv_heads, self.dim, self.vdim = heads, kv_heads, dim, vdim
+        self.taps, self.eps = taps, eps
+        self.channels = 2 * kv_heads * dim + heads * vdim
+        rows = self.channels + heads * vdim + 2 * heads
+        self.pad_rows = -rows % 8
+        self.in_rows = rows + self.pad_rows
+        self.out_rows = heads * vdim
+        self._alloc(width, own_in, dtype)
+        w = torch.empty(self.channels, taps, dtype=torch.float32).normal_(0.0, 0.2)
+        w[:, -1] += 0.7
+        self.conv_weight = nn.Parameter(w, requires_grad=False)
+        self.dt_bias = nn.Parameter(torch.empty(heads).uniform_(-4.6, -2.2), requires_grad=False)
+        self.a_log = nn.Parameter(torch.empty(heads).uniform_(0.0, 2.77), requires_grad=False)
+        self.norm = _f32_param(heads * vdim, fill=1.0)   # the head weight, repeated
+
+    def load_in(self, weight, bias, t) -> None:
+        off = 0
+        for name in ("q", "k", "v", "g", "b", "a"):
+            n = t[name].shape[0]
+            weight[off:off + n].copy_(t[name].to(weight.dtype))
+            if name in ("q", "k", "v"):
+                self.conv_weight.data[off:off + n].copy_(t[name + ".conv"].float())
+            off += n
+        if off != self.in_rows - self.pad_rows:
+            raise ValueError("projection tensors do not add up to the mixer's rows")
+        weight[off:].zero_()
+
+    def load_rest(self, t) -> None:
+        self.a_log.data.copy_(t["A_log"].float())
+        self.dt_bias.data.copy_(t["dt_bias"].float())
+        self.norm.data.copy_(t["norm"].float().repeat(self.heads))
+
+    def cache_shapes(self, block_size: int) -> list:
+        return [("slot", (self.taps - 1, self.channels), self.dtype),
+                ("slot", (self.heads, self.vdim, self.dim), torch.float32)]
+
+    def mix(self, proj, positions, cache, meta: AttnMetadata) -> torch.Tensor:
+        conv_state, state = cache
+        t, nh, ng, d, dv = proj.shape[0], self.heads, self.kv_heads, self.dim, self.vdim
+        a, c = ng * d, self.channels
+        e = c + nh * dv
+        qkv = ops.causal_conv_state(
+            proj[:, :c], self.conv_weight, conv_state, meta.seq_start_loc, meta.seq_lens,
+            meta.state_slots, add_input=False, act="silu")
+        return ops.delta_gated(
+            qkv[:, :a].view(t, ng, d), qkv[:, a:2 * a].view(t, ng, d),
+            qkv[:, 2 * a:].view(t, nh, dv), proj[:, e:e + nh], proj[:, e + nh:e + 2 * nh],
+            self.a_log, self.dt_bias, proj[:, c:e], self.norm, self.eps, state,
+            meta.seq_start_loc, meta.seq_lens, meta.state_slots)

@@ -379,17 +379,23 @@ def moe_gemm(
     seg_off: torch.Tensor,  # [E+1] int32 device row offsets
     gated: bool,
     act: str | None = None,
+    limit: float = 0.0,
 ) -> torch.Tensor:
-    """Grouped GEMM over expert segments (E16); gated fuses SiLU(g)*u; a plain
-    product may be followed by ``act`` ("relu2": the squared relu).  Rows past
-    the last segment are left unwritten."""
-    if act not in (None, "relu2") or (gated and act):
+    """Grouped GEMM over expert segments (E16); gated fuses SiLU(g)*u, or with
+    act "clamped" the clamped gate (see clamped_glu); a plain product may be
+    followed by "relu2", the squared relu.  Rows past the last segment are left
+    unwritten."""
+    if act not in ((None, "clamped") if gated else (None, "relu2")):
         raise ValueError(f"unknown activation {act!r}")
     n = w.shape[1] // 2 if gated else w.shape[1]
     if x.device.type != "cuda" or _FORCE_REFERENCE:
-        return reference.moe_gemm(x, w, seg_off.cpu(), gated, act)
-    ext = _C if _C is not None else (_S if _native_seq(x) else None)
+        return reference.moe_gemm(x, w, seg_off.cpu(), gated, act, limit)
     out = torch.empty((x.shape[0], n), dtype=x.dtype, device=x.device)
+    if act == "clamped":
+        _native_seq(x)
+        _S.moe_gemm_clamped(out, x, w, seg_off, float(limit))
+        return out
+    ext = _C if _C is not None else (_S if _native_seq(x) else None)
     ext.moe_gemm(out, x, w, seg_off, 1 if gated else (2 if act == "relu2" else 0))
     return out
 
@@ -791,16 +797,56 @@ def attention_uses_matrix_cores(dtype: torch.dtype, heads: int, kv_heads: int,
             and heads % kv_heads == 0 and 1 <= heads // kv_heads <= 8)
 
 
+def capped_attention_uses_matrix_cores(dtype: torch.dtype, heads: int, kv_heads: int,
+                                       dim: int, vdim: int) -> bool:
+    """Shapes the capped (score cap, sinks per head) variants of the MFMA
+    kernels take (prompt portions need size 128, single queries 64 or 128)."""
+    return (dtype == torch.bfloat16 and dim == vdim and dim in (64, 128)
+            and heads % kv_heads == 0 and 1 <= heads // kv_heads <= 8)
+
+
+def _capped_matrix_core_fits(q, k_cache, v_cache, out, single: bool) -> bool:
+    if _attn_ext() is None or _FORCE_REFERENCE:
+        return False
+    return (capped_attention_uses_matrix_cores(q.dtype, q.shape[1], k_cache.shape[2],
+                                               q.shape[2], v_cache.shape[3])
+            and (single or q.shape[2] == 128) and q.is_contiguous() and out.is_contiguous())
+
+
+def _repeat_sink(sink: float | None, q: torch.Tensor) -> torch.Tensor | None:
+    if sink is None:
+        return None
+    return torch.full((q.shape[1],), float(sink), dtype=torch.float32, device=q.device)
+
+
 def gqa_attention_prefill(q, k_cache, v_cache, block_tables, query_start_loc,
                           seq_lens, scale, max_query_len, out: torch.Tensor,
-                          window: int = 0, sink: float | None = None) -> torch.Tensor:
+                          window: int = 0, sink: float | None = None,
+                          sinks: torch.Tensor | None = None, softcap: float = 0.0,
+                          general: bool = False) -> torch.Tensor:
     """Causal grouped-query softmax attention of query chunks (the tail rows
     of each sequence) over the paged cache; q [T, H, dim], out [T, H, vdim].
     ``window`` > 0: position i sees j with 0 <= i - j < window.  ``sink``: the
-    softmax denominator also holds exp(sink), a key without a value.
+    softmax denominator also holds exp(sink), a key without a value (``sinks``
+    [H] f32: one per head).  ``softcap`` > 0: scores become softcap *
+    tanh(score / softcap); the sink is not capped.
     bf16 shapes the MFMA kernels take run there, everything else (f32, other
-    sizes, value size unlike the key size) on the any-shape kernel."""
+    sizes, value size unlike the key size) on the any-shape kernel (``general``:
+    always, for capped scores or sinks per head)."""
+    if sinks is not None and sink is not None:
+        raise ValueError("one sink for all heads or one per head, not both")
     if q.numel() and _native_seq(q):
+        if sinks is not None or softcap > 0:
+            if sinks is None:
+                sinks = _repeat_sink(sink, q)
+            if not general and _capped_matrix_core_fits(q, k_cache, v_cache, out, single=False):
+                _attn_ext().capped_attention_prefill(
+                    out, q, k_cache, v_cache, block_tables, query_start_loc, seq_lens,
+                    float(scale), int(max_query_len), int(window), sinks, float(softcap))
+            else:
+                _S.capped_attention(out, q, k_cache, v_cache, block_tables, query_start_loc,
+                                    seq_lens, float(scale), int(window), sinks, float(softcap))
+            return out
         if window > 0 or sink is not None:
             if _windowed_matrix_core_fits(q, k_cache, v_cache, single=False):
                 dst = out if out.is_contiguous() else torch.empty_like(q)
@@ -830,16 +876,30 @@ def gqa_attention_prefill(q, k_cache, v_cache, block_tables, query_start_loc,
         return out
     out.copy_(reference.paged_attention(
         q, k_cache, v_cache, block_tables.cpu(), query_start_loc.cpu(),
-        seq_lens.cpu(), scale, window, sink))
+        seq_lens.cpu(), scale, window, sink if sinks is None else sinks, softcap))
     return out
 
 
 def gqa_attention_decode(q, k_cache, v_cache, block_tables, seq_lens, scale,
                          out: torch.Tensor, window: int = 0,
-                         sink: float | None = None) -> torch.Tensor:
+                         sink: float | None = None, sinks: torch.Tensor | None = None,
+                         softcap: float = 0.0, general: bool = False) -> torch.Tensor:
     """Same attention for one new query per sequence (seq_len 0 = padding row,
     zeros)."""
+    if sinks is not None and sink is not None:
+        raise ValueError("one sink for all heads or one per head, not both")
     if q.numel() and _native_seq(q):
+        if sinks is not None or softcap > 0:
+            if sinks is None:
+                sinks = _repeat_sink(sink, q)
+            if not general and _capped_matrix_core_fits(q, k_cache, v_cache, out, single=True):
+                _attn_ext().capped_attention_decode(
+                    out, q, k_cache, v_cache, block_tables, seq_lens, float(scale),
+                    int(window), sinks, float(softcap))
+            else:
+                _S.capped_attention(out, q, k_cache, v_cache, block_tables, None, seq_lens,
+                                    float(scale), int(window), sinks, float(softcap))
+            return out
         if window > 0 or sink is not None:
             if _windowed_matrix_core_fits(q, k_cache, v_cache, single=True):
                 dst = out if out.is_contiguous() else torch.empty_like(q)
@@ -870,7 +930,7 @@ def gqa_attention_decode(q, k_cache, v_cache, block_tables, seq_lens, scale,
     qsl = torch.arange(n + 1, dtype=torch.int32)
     out.copy_(reference.paged_attention(
         q, k_cache, v_cache, block_tables.cpu(), qsl, seq_lens.cpu(), scale,
-        window, sink))
+        window, sink if sinks is None else sinks, softcap))
     return out
 
 
@@ -1187,19 +1247,28 @@ def group_rms_norm(y: torch.Tensor, weight: torch.Tensor, groups: int, eps: floa
     return reference.group_rms_norm(y, weight, groups, eps, out_dtype)
 
 
-def moe_route_sigmoid(logits: torch.Tensor, top: int):
-    """Sigmoid router: the ``top`` largest sigmoid(logits) per row, weighted by
-    those scores as they are.  Returns (dense [T, E] f32, ids [T, top] int32,
-    weights [T, top] f32)."""
+def moe_route_sigmoid(logits: torch.Tensor, top: int, correction: torch.Tensor | None = None,
+                      groups: int = 1, keep: int = 1, renormalise: bool = False,
+                      scale: float = 1.0):
+    """Sigmoid router: the ``top`` largest sigmoid(logits) (+ correction [E])
+    per row, among the ``keep`` best of ``groups`` equal runs of experts (best by
+    the sum of a group's two largest choice scores), weighted by their scores
+    without the correction (divided by their sum when ``renormalise``), times
+    ``scale``.  Returns (dense [T, E] f32, ids [T, top] int32, weights [T, top]
+    f32)."""
+    n = logits.shape[1]
+    if n % groups or not 1 <= keep <= groups or top > keep * (n // groups):
+        raise ValueError("the kept groups must be equal and hold the chosen experts")
     if logits.numel() and _native_seq(logits):
-        t, n = logits.shape
+        t = logits.shape[0]
         dev = logits.device
         dense = torch.empty((t, n), dtype=torch.float32, device=dev)
         ids = torch.empty((t, top), dtype=torch.int32, device=dev)
         w = torch.empty((t, top), dtype=torch.float32, device=dev)
-        _S.moe_route_sigmoid(dense, ids, w, logits)
+        _S.moe_route_sigmoid(dense, ids, w, logits, correction, int(groups), int(keep),
+                             bool(renormalise), float(scale))
         return dense, ids, w
-    return reference.moe_route_sigmoid(logits, top)
+    return reference.moe_route_sigmoid(logits, top, correction, groups, keep, renormalise, scale)
 
 
 def silu_mul_scaled(gu: torch.Tensor, col_scale: torch.Tensor) -> torch.Tensor:
@@ -1410,3 +1479,110 @@ def silu_mul_bias(gu: torch.Tensor, bias: torch.Tensor | None = None) -> torch.T
         _S.silu_mul_bias(out, gu, bias)
         return out
     return reference.silu_mul_bias(gu, bias)
+
+
+# ---------------------------------------------------------------------------
+# Tanh norms around both ends of a sublayer, query/key norm over the whole
+# projection with value mixing, the gated delta rule, clamped gates, f32 router
+# products.  Same extension as the stream ops.
+# ---------------------------------------------------------------------------
+
+
+def stream_add_tanh_norm(x: torch.Tensor, a: torch.Tensor | None, norm, *,
+                         b: torch.Tensor | None = None, next_norm=None,
+                         out_dtype: torch.dtype = torch.bfloat16) -> torch.Tensor | None:
+    """x (f32 [T, W], in place) += F(a + b), F(y) = tanh(alpha y) * w + bias with
+    ``norm`` = (alpha, w [W] f32, bias [W] f32); b is optional, nothing is added
+    when ``a`` is None.  With ``next_norm`` (the same triple) F of the updated
+    stream is returned in ``out_dtype`` for the sublayer that reads it next."""
+    if x.numel() and _native_seq(x):
+        out = torch.empty(x.shape, dtype=out_dtype, device=x.device) if next_norm else None
+        al, w, bias = norm if a is not None else (0.0, None, None)
+        nal, nw, nbias = next_norm if next_norm else (0.0, None, None)
+        _S.stream_add_tanh_norm(x, a, b, float(al), w, bias, float(nal), nw, nbias, out)
+        return out
+    return reference.stream_add_tanh_norm(x, a, b, norm, next_norm, out_dtype)
+
+
+def wide_norm_cache_write(proj: torch.Tensor, bias, heads: int, kv_heads: int, dim: int,
+                          vdim: int, eps: float, q_weight, k_weight, v_first, v_mix: float,
+                          k_cache, v_cache, slot_mapping) -> torch.Tensor:
+    """From projected rows [q | k | v] (proj [T, C], rows may be strided) to the
+    attention's inputs, one pass: + bias [C] f32; RMS norm of all of q and of
+    all of k (one mean over every head; weights [heads * dim], [kv_heads * dim]
+    f32); with ``v_first`` (the value cache of an earlier layer, same slots) v
+    becomes (1 - v_mix) v + v_mix v_first[token]; keys and values stored in the
+    paged cache.  Returns the queries [T, heads, dim]."""
+    if proj.numel() and _native_seq(proj):
+        out = torch.empty((proj.shape[0], heads, dim), dtype=proj.dtype, device=proj.device)
+        _S.wide_norm_cache_write(out, proj, bias, int(kv_heads), int(vdim), float(eps), q_weight,
+                                 k_weight, v_first, float(v_mix), k_cache, v_cache, slot_mapping)
+        return out
+    return reference.wide_norm_cache_write(proj, bias, heads, kv_heads, dim, vdim, eps, q_weight,
+                                           k_weight, v_first, v_mix, k_cache, v_cache,
+                                           slot_mapping)
+
+
+def delta_scan(q, k, v, b_pre, a_pre, a_log, dt_bias, state, seq_start_loc, seq_lens,
+               state_slots) -> torch.Tensor:
+    """Gated delta rule over each sequence's new rows.  q, k [T, G, dim], v [T,
+    H, vdim] (views into wider rows are fine; head h uses query / key head
+    h / (H / G)), b_pre, a_pre [T, H]; per head, all f32: q, k to unit length
+    (q also times dim^-1/2), beta = sigmoid(b_pre), g = exp(-exp(a_log)
+    softplus(a_pre + dt_bias)); S <- g S, u = beta (v - S^T k), S <- S + k u^T,
+    o = S^T q.  State [slots, H, vdim, dim] f32, advanced in place.  Returns o
+    [T, H * vdim] f32."""
+    if q.numel() and _native_seq(q):
+        o = torch.empty((q.shape[0], v.shape[1] * v.shape[2]), dtype=torch.float32,
+                        device=q.device)
+        _S.delta_scan(o, q, k, v, b_pre, a_pre, a_log, dt_bias, state, seq_start_loc, seq_lens,
+                      state_slots)
+        return o
+    return reference.delta_scan(q, k, v, b_pre, a_pre, a_log, dt_bias, state,
+                                seq_start_loc.cpu(), seq_lens.cpu(), state_slots.cpu())
+
+
+def delta_gated(q, k, v, b_pre, a_pre, a_log, dt_bias, gate, norm, eps: float, state,
+                seq_start_loc, seq_lens, state_slots, general: bool = False) -> torch.Tensor:
+    """delta_scan, then an RMS norm of every head's output over vdim times
+    ``norm`` [H * vdim] f32 times silu(gate), gate [T, H * vdim] -> [T, H * vdim]
+    in the compute dtype.  One kernel where a workgroup can own a head's value
+    columns (sizes in multiples of 8) unless ``general``."""
+    if q.numel() and _native_seq(q):
+        out = torch.empty(gate.shape, dtype=q.dtype, device=q.device)
+        _S.delta_gated(out, q, k, v, b_pre, a_pre, a_log, dt_bias, gate, norm, float(eps), state,
+                       seq_start_loc, seq_lens, state_slots, bool(general))
+        return out
+    o = delta_scan(q, k, v, b_pre, a_pre, a_log, dt_bias, state, seq_start_loc, seq_lens,
+                   state_slots)
+    return reference.gated_group_norm(o, gate, norm, v.shape[1], eps, False, q.dtype, True)
+
+
+def clamped_glu(gu: torch.Tensor, limit: float,
+                col_scale: torch.Tensor | None = None) -> torch.Tensor:
+    """gu [T, E * 2 ff] (per expert its gate columns, then its up columns; E = 1
+    without ``col_scale``) -> [T, E * ff]: g sigmoid(1.702 g) (u + 1) with g =
+    min(gate, limit), u = up clamped to +-limit, times col_scale[t, expert] f32."""
+    if gu.numel() and _native_seq(gu):
+        out = torch.empty((gu.shape[0], gu.shape[1] // 2), dtype=gu.dtype, device=gu.device)
+        _S.clamped_glu(out, gu, float(limit), col_scale)
+        return out
+    return reference.clamped_glu(gu, limit, col_scale)
+
+
+def router_logits(h: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
+    """h [T, W] (compute dtype or f32) times weight [E, W] f32, all in f32."""
+    if h.numel() and _native_seq(h):
+        out = torch.empty((h.shape[0], weight.shape[0]), dtype=torch.float32, device=h.device)
+        _S.router_logits(out, h, weight)
+        return out
+    return reference.router_logits(h, weight)
+
+
+def scale_logits(logits: torch.Tensor, scale: float) -> torch.Tensor:
+    """f32 logits * scale."""
+    if logits.numel() and _native_seq(logits):
+        out = torch.empty(logits.shape, dtype=torch.float32, device=logits.device)
+        _S.scale_logits(out, logits.contiguous(), float(scale))
+        return out
+    return reference.scale_logits(logits, scale)

@@ -115,12 +115,15 @@ def paged_attention(
     seq_lens: torch.Tensor,         # [num_seqs] total context per seq (cpu)
     scale: float,
     window: int = 0,
-    sink: float | None = None,
+    sink: "float | torch.Tensor | None" = None,
+    softcap: float = 0.0,
 ) -> torch.Tensor:
     """Causal paged attention over queries that are the *tail* of each
     sequence (covers prefill chunks and single-token decode uniformly).
     ``window`` > 0: a query at position i sees keys j with 0 <= i - j < window.
-    ``sink``: the softmax denominator also holds exp(sink) (no key, no value)."""
+    ``sink``: the softmax denominator also holds exp(sink) (no key, no value;
+    one number, or one per head).  ``softcap`` > 0: scores become
+    softcap * tanh(score / softcap) before the softmax."""
     num_heads = q.shape[1]
     num_kv_heads = k_cache.shape[2]
     group = num_heads // num_kv_heads
@@ -141,6 +144,8 @@ def paged_attention(
         kf = k.float().repeat_interleave(group, dim=1)  # [S, H, d]
         vf = v.float().repeat_interleave(group, dim=1)
         scores = torch.einsum("qhd,shd->hqs", qf, kf) * scale
+        if softcap > 0:
+            scores = softcap * torch.tanh(scores / softcap)
         # causal: query position j (global seq_len - q_len + j) sees keys <= it
         kpos = torch.arange(seq_len, device=q.device)
         qpos = torch.arange(seq_len - q_len, seq_len, device=q.device)
@@ -151,9 +156,10 @@ def paged_attention(
         if sink is None:
             probs = torch.softmax(scores, dim=-1)
         else:
-            m = scores.max(dim=-1, keepdim=True).values.clamp(min=float(sink))
+            b = torch.as_tensor(sink, dtype=torch.float32, device=q.device).reshape(-1, 1, 1)
+            m = torch.maximum(scores.max(dim=-1, keepdim=True).values, b)
             probs = torch.exp(scores - m)
-            probs = probs / (probs.sum(dim=-1, keepdim=True) + torch.exp(float(sink) - m))
+            probs = probs / (probs.sum(dim=-1, keepdim=True) + torch.exp(b - m))
         out[s:e] = torch.einsum("hqs,shd->qhd", probs, vf).to(q.dtype)
     return out
 
@@ -703,11 +709,20 @@ def moe_combine(ye: torch.Tensor, pos: torch.Tensor, ids: torch.Tensor,
     return (rows * w.unsqueeze(-1)).sum(dim=1).to(ye.dtype)
 
 
+def clamped_gate(g: torch.Tensor, u: torch.Tensor, limit: float) -> torch.Tensor:
+    """f32: g' sigmoid(1.702 g') (u' + 1) with g' = min(g, limit) and u' = u
+    clamped to +-limit."""
+    g = torch.clamp(g.float(), max=limit)
+    u = torch.clamp(u.float(), min=-limit, max=limit)
+    return g * torch.sigmoid(1.702 * g) * (u + 1.0)
+
+
 def moe_gemm(x: torch.Tensor, w: torch.Tensor, seg_off: torch.Tensor, gated: bool,
-             act: str | None = None) -> torch.Tensor:
+             act: str | None = None, limit: float = 0.0) -> torch.Tensor:
     """Rows seg_off[e] .. seg_off[e+1] of x times expert e's weight w[e]
-    ([2N, K] gated: silu(first half) * second half; else [N, K], optionally
-    followed by the squared relu).  Rows past the last segment are zeros."""
+    ([2N, K] gated: silu(first half) * second half, or with act "clamped"
+    clamped_gate of the halves; else [N, K], optionally followed by the squared
+    relu).  Rows past the last segment are zeros."""
     n = w.shape[1] // 2 if gated else w.shape[1]
     out = torch.zeros((x.shape[0], n), dtype=x.dtype, device=x.device)
     off = seg_off.tolist()
@@ -716,7 +731,9 @@ def moe_gemm(x: torch.Tensor, w: torch.Tensor, seg_off: torch.Tensor, gated: boo
         if b <= a:
             continue
         y = x[a:b].float() @ w[e].float().T
-        if gated:
+        if gated and act == "clamped":
+            y = clamped_gate(y[:, :n], y[:, n:], limit)
+        elif gated:
             y = torch.nn.functional.silu(y[:, :n]) * y[:, n:]
         elif act == "relu2":
             y = torch.clamp(y, min=0.0) ** 2
@@ -879,13 +896,31 @@ def group_rms_norm(y: torch.Tensor, weight: torch.Tensor, groups: int, eps: floa
     return (yg.reshape(t, c) * weight.float()).to(out_dtype)
 
 
-def moe_route_sigmoid(logits: torch.Tensor, top: int):
-    """s = sigmoid(logits) [T, E] f32; the ``top`` largest are chosen (ties:
-    the lower index); weights = their s as they are.  Returns (dense [T, E]
-    f32: weight or 0, ids [T, top] int32, weights [T, top] f32)."""
+def moe_route_sigmoid(logits: torch.Tensor, top: int, correction: torch.Tensor | None = None,
+                      groups: int = 1, keep: int = 1, renormalise: bool = False,
+                      scale: float = 1.0):
+    """s = sigmoid(logits) [T, E] f32.  Choice scores are s (+ correction [E]);
+    with ``groups`` > 1 equal runs of neighbouring experts only the ``keep``
+    groups with the largest sum of their two best choice scores stay open.  The
+    ``top`` largest open choice scores are chosen (ties: the lower index);
+    weights = their s, divided by their sum (+ 1e-20) when ``renormalise``,
+    times ``scale``.  Returns (dense [T, E] f32: weight or 0, ids [T, top]
+    int32, weights [T, top] f32)."""
     s = torch.sigmoid(logits.float())
-    order = torch.sort(s, dim=-1, descending=True, stable=True).indices[:, :top]
+    choice = s if correction is None else s + correction.float()
+    if groups > 1:
+        t, e = s.shape
+        g = choice.view(t, groups, e // groups)
+        score = torch.topk(g, min(2, e // groups), dim=-1).values.sum(-1)
+        best = torch.sort(score, dim=-1, descending=True, stable=True).indices[:, :keep]
+        is_open = torch.zeros((t, groups), dtype=torch.bool, device=s.device)
+        is_open.scatter_(1, best, True)
+        choice = g.masked_fill(~is_open.unsqueeze(-1), float("-inf")).reshape(t, e)
+    order = torch.sort(choice, dim=-1, descending=True, stable=True).indices[:, :top]
     w = torch.gather(s, 1, order)
+    if renormalise:
+        w = w / (w.sum(dim=-1, keepdim=True) + 1e-20)
+    w = w * scale
     return torch.zeros_like(s).scatter_(1, order, w), order.to(torch.int32), w
 
 
@@ -1097,3 +1132,95 @@ def silu_mul_bias(gu: torch.Tensor, bias: torch.Tensor | None) -> torch.Tensor:
         z = z + bias.float()
     g, u = z.chunk(2, dim=-1)
     return (g * torch.sigmoid(g) * u).to(gu.dtype)
+
+
+# ---------------------------------------------------------------------------
+# Tanh norms around both ends of a sublayer, query/key norm over the whole
+# projection with value mixing, the gated delta rule, clamped gates, f32 router
+# products.
+# ---------------------------------------------------------------------------
+
+
+def stream_add_tanh_norm(x: torch.Tensor, a: torch.Tensor | None, b: torch.Tensor | None,
+                         norm, next_norm, out_dtype: torch.dtype) -> torch.Tensor | None:
+    """See ops.stream_add_tanh_norm."""
+    def f(y, n):
+        alpha, w, bias = n
+        return torch.tanh(alpha * y) * w.float() + bias.float()
+
+    if a is not None:
+        y = a.float() if b is None else a.float() + b.float()
+        x += f(y, norm)
+    return None if next_norm is None else f(x, next_norm).to(out_dtype)
+
+
+def wide_norm_cache_write(proj, bias, heads, kv_heads, dim, vdim, eps, q_weight, k_weight,
+                          v_first, v_mix, k_cache, v_cache, slot_mapping) -> torch.Tensor:
+    """See ops.wide_norm_cache_write."""
+    t = proj.shape[0]
+    z = proj.float() if bias is None else proj.float() + bias.float()
+    a, b = heads * dim, heads * dim + kv_heads * dim
+
+    def norm(y, w):
+        return y * torch.rsqrt(y.pow(2).mean(dim=-1, keepdim=True) + eps) * w.float()
+
+    q, k = norm(z[:, :a], q_weight), norm(z[:, a:b], k_weight)
+    v = z[:, b:b + kv_heads * vdim].reshape(t, kv_heads, vdim)
+    ok = slot_mapping >= 0
+    sm = slot_mapping[ok]
+    bs = k_cache.shape[1]
+    blk = torch.div(sm, bs, rounding_mode="floor")
+    v = v[ok]
+    if v_first is not None:
+        v = (1.0 - v_mix) * v + v_mix * v_first[blk, sm % bs].float()
+    k_cache[blk, sm % bs] = k.view(t, kv_heads, dim)[ok].to(k_cache.dtype)
+    v_cache[blk, sm % bs] = v.to(v_cache.dtype)
+    return q.to(proj.dtype).view(t, heads, dim).contiguous()
+
+
+def delta_scan(q, k, v, b_pre, a_pre, a_log, dt_bias, state, seq_start_loc, seq_lens,
+               state_slots) -> torch.Tensor:
+    """See ops.delta_scan."""
+    t, ng, d = q.shape
+    nh, dv = v.shape[1], v.shape[2]
+
+    def unit(y):
+        y = y.float()
+        return y * torch.rsqrt(y.pow(2).sum(dim=-1, keepdim=True) + 1e-6)
+
+    qf = (unit(q) * d ** -0.5).repeat_interleave(nh // ng, dim=1)
+    kf = unit(k).repeat_interleave(nh // ng, dim=1)
+    vf = v.float()
+    beta = torch.sigmoid(b_pre.float())
+    g = torch.exp(-torch.exp(a_log.float()) * _softplus(a_pre.float() + dt_bias.float()))
+    out = torch.zeros((t, nh, dv), dtype=torch.float32, device=q.device)
+    for lo, hi, start, slot in _seq_iter(seq_start_loc, seq_lens, state_slots):
+        if slot < 0:
+            continue
+        s = state[slot].clone() if start > 0 else torch.zeros_like(state[slot])   # [H, vdim, dim]
+        for i in range(lo, hi):
+            s = g[i].view(nh, 1, 1) * s
+            u = beta[i].unsqueeze(1) * (vf[i] - (s * kf[i].unsqueeze(1)).sum(-1))
+            s = s + u.unsqueeze(2) * kf[i].unsqueeze(1)
+            out[i] = (s * qf[i].unsqueeze(1)).sum(-1)
+        state[slot] = s
+    return out.view(t, nh * dv)
+
+
+def clamped_glu(gu: torch.Tensor, limit: float, col_scale: torch.Tensor | None) -> torch.Tensor:
+    """See ops.clamped_glu."""
+    t = gu.shape[0]
+    e = 1 if col_scale is None else col_scale.shape[1]
+    z = gu.view(t, e, 2, -1)
+    y = clamped_gate(z[:, :, 0], z[:, :, 1], limit)
+    if col_scale is not None:
+        y = y * col_scale.float().unsqueeze(-1)
+    return y.to(gu.dtype).reshape(t, -1)
+
+
+def router_logits(h: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
+    return torch.nn.functional.linear(h.float(), weight)
+
+
+def scale_logits(logits: torch.Tensor, scale: float) -> torch.Tensor:
+    return logits.float() * scale
