@@ -53,14 +53,19 @@ DEVINLINE bf16x8_t load_kv8<unsigned char>(const unsigned char* p) {
 // tokens.  PX_POOL: one pooled key and value per block of `pool` positions that
 // ends at or before seq_len - 1 - window; pooled block b is kept in the cache
 // block that holds its last token (per_block places each).
+// CAP (capped variant, on top of WS): scores become softcap tanh(score / softcap)
+// (softcap 0: as they are).  Up to kFixedMaxCap the cap bounds them well enough
+// that the exponentials are taken without a running maximum.
 enum { PX_NONE = 0, PX_KEEP = 1, PX_POOL = 2 };
+constexpr float kFixedMaxCap = 60.f;
 struct SpanKeys {
   int keep, pool, per_block;
   const __hip_bfloat16* k_pool;
   const __hip_bfloat16* v_pool;
 };
 
-template <int HEAD_DIM, typename CT, bool WS, bool CH = false, int PX = PX_NONE>
+template <int HEAD_DIM, typename CT, bool WS, bool CH = false, int PX = PX_NONE,
+          bool CAP = false>
 __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
     float* __restrict__ part_acc,   // [nseq, nheads, P, HEAD_DIM] f32
     float* __restrict__ part_ml,    // [nseq, nheads, P, 2] f32 (m, l)
@@ -78,7 +83,10 @@ __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
     const int window,
     const int chunk = 0,
     const int v_heads = 0,
-    const SpanKeys sp = SpanKeys{}) {
+    const SpanKeys sp = SpanKeys{},
+    const float softcap = 0.f) {
+  static_assert(!CAP || (WS && !CH && PX == PX_NONE),
+                "the capped variant builds on the window variant");
   static_assert(!CH || WS, "the chunk variant builds on the window variant");
   static_assert(PX == PX_NONE || (WS && !CH), "prefixes build on the window variant");
   constexpr int KCH = HEAD_DIM / 16;  // k-chunks for the QK^T mfma
@@ -138,6 +146,11 @@ __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
   f32x16_t acc_o[DT];
 #pragma unroll
   for (int dt = 0; dt < DT; ++dt) acc_o[dt] = f32x16_t{};
+
+  const bool capped = CAP && softcap > 0.f;
+  const bool fixed_max = capped && softcap <= kFixedMaxCap;
+  const float cap_in = capped ? scale / softcap : 0.f;
+  if (fixed_max) m_state = 0.f;
 
   constexpr int VPASS = KVT * HEAD_DIM / 8 / 64;  // V staging passes per wave
 
@@ -214,36 +227,41 @@ __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
 #pragma unroll
     for (int r = 0; r < 16; ++r) {
       const int kv_pos = kv_base + (r & 3) + 8 * (r >> 2) + 4 * half;
-      float sv = acc_s[r] * scale;
+      float sv = capped ? softcap * tanh_f32(acc_s[r] * cap_in) : acc_s[r] * scale;
       if (kv_pos >= limit || (WS && !prefix && kv_pos < first_pos)) sv = -FLT_MAX;
       s_val[r] = sv;
       local_max = fmaxf(local_max, sv);
     }
-    const float tile_max = fmaxf(local_max, __shfl_xor(local_max, 32, 64));
-    const float m_new = fmaxf(m_state, tile_max);
-    const float rescale = __expf(m_state - m_new);
-    m_state = m_new;
+    float rescale = 1.f;
+    if (!(CAP && fixed_max)) {
+      const float tile_max = fmaxf(local_max, __shfl_xor(local_max, 32, 64));
+      const float m_new = fmaxf(m_state, tile_max);
+      rescale = __expf(m_state - m_new);
+      m_state = m_new;
+    }
 
     float p[16];
     float local_sum = 0.f;
 #pragma unroll
     for (int r = 0; r < 16; ++r) {
-      p[r] = s_val[r] == -FLT_MAX ? 0.f : __expf(s_val[r] - m_new);
+      p[r] = s_val[r] == -FLT_MAX ? 0.f : __expf(s_val[r] - m_state);
       local_sum += p[r];
     }
     l_state = l_state * rescale + local_sum + __shfl_xor(local_sum, 32, 64);
 
     // rescale factors redistributed to the PV accumulator's q rows
-    float f_reg[16];
+    if (!(CAP && fixed_max)) {
+      float f_reg[16];
 #pragma unroll
-    for (int r = 0; r < 16; ++r) {
-      const int qrow = (r & 3) + 8 * (r >> 2) + 4 * half;
-      f_reg[r] = __shfl(rescale, qrow, 64);
-    }
+      for (int r = 0; r < 16; ++r) {
+        const int qrow = (r & 3) + 8 * (r >> 2) + 4 * half;
+        f_reg[r] = __shfl(rescale, qrow, 64);
+      }
 #pragma unroll
-    for (int dt = 0; dt < DT; ++dt) {
+      for (int dt = 0; dt < DT; ++dt) {
 #pragma unroll
-      for (int r = 0; r < 16; ++r) acc_o[dt][r] *= f_reg[r];
+        for (int r = 0; r < 16; ++r) acc_o[dt][r] *= f_reg[r];
+      }
     }
 
     // ---- pack P to bf16 A-fragments (cvt_pk + permlane32_swap) -----------
@@ -317,6 +335,7 @@ __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
 // Reduce the P partials of each (seq, head) row: out = sum_p f_p acc_p / sum_p f_p l_p
 // back (cos, sin per row and pair, or null): dims m and m + HEAD_DIM/2 are turned
 // back by the row's angles before the rounding.
+// sinks: one sink per head instead of `sink` (or null).
 template <int HEAD_DIM, typename OT = __hip_bfloat16, bool BACK = false>
 __global__ void decode_merge_kernel(
     OT* __restrict__ out,                  // [nseq, nheads, HD]
@@ -325,11 +344,13 @@ __global__ void decode_merge_kernel(
     const int nheads,
     const int P,
     const int has_sink,
-    const float sink,
-    const float2* __restrict__ back = nullptr) {
+    float sink,
+    const float2* __restrict__ back = nullptr,
+    const float* __restrict__ sinks = nullptr) {
   const int seq = blockIdx.x;
   const int head = blockIdx.y;
   const int d = threadIdx.x;
+  if (sinks != nullptr) sink = sinks[head];
   const long row = (long)seq * nheads + head;
   const float* ml = part_ml + row * P * 2;
   const float* acc = part_acc + row * P * HEAD_DIM + d;
@@ -394,14 +415,14 @@ static void launch_decode_ct(__hip_bfloat16* out, float* part_acc,
                            stream, part_acc, part_ml, q, kc, vc, bt, sl, scale,
                            nheads, kvh, group, block_size, max_blocks, window);
         hipLaunchKernelGGL((decode_merge_kernel<64>), mgrid, dim3(64), 0, stream,
-                           out, part_acc, part_ml, nheads, P, has_sink, sink, nullptr);
+                           out, part_acc, part_ml, nheads, P, has_sink, sink, nullptr, nullptr);
         break;
       case 128:
         hipLaunchKernelGGL((paged_decode_mfma_kernel<128, CT, true>), grid, block, 0,
                            stream, part_acc, part_ml, q, kc, vc, bt, sl, scale,
                            nheads, kvh, group, block_size, max_blocks, window);
         hipLaunchKernelGGL((decode_merge_kernel<128>), mgrid, dim3(128), 0, stream,
-                           out, part_acc, part_ml, nheads, P, has_sink, sink, nullptr);
+                           out, part_acc, part_ml, nheads, P, has_sink, sink, nullptr, nullptr);
         break;
       default:
         abort();
@@ -414,14 +435,14 @@ static void launch_decode_ct(__hip_bfloat16* out, float* part_acc,
                          stream, part_acc, part_ml, q, kc, vc, bt, sl, scale,
                          nheads, kvh, group, block_size, max_blocks, 0);
       hipLaunchKernelGGL((decode_merge_kernel<64>), mgrid, dim3(64), 0, stream,
-                         out, part_acc, part_ml, nheads, P, 0, 0.f, nullptr);
+                         out, part_acc, part_ml, nheads, P, 0, 0.f, nullptr, nullptr);
       break;
     case 128:
       hipLaunchKernelGGL((paged_decode_mfma_kernel<128, CT, false>), grid, block, 0,
                          stream, part_acc, part_ml, q, kc, vc, bt, sl, scale,
                          nheads, kvh, group, block_size, max_blocks, 0);
       hipLaunchKernelGGL((decode_merge_kernel<128>), mgrid, dim3(128), 0, stream,
-                         out, part_acc, part_ml, nheads, P, 0, 0.f, nullptr);
+                         out, part_acc, part_ml, nheads, P, 0, 0.f, nullptr, nullptr);
       break;
     default:
       abort();
@@ -486,7 +507,7 @@ void launch_paged_decode_mfma_chunk(float* out, float* part_acc, float* part_ml,
           0, stream, part_acc, part_ml, q, kc, vc, bt, sl, scale, nheads, kvh, group,
           block_size, max_blocks, 0, chunk, v_heads);
       hipLaunchKernelGGL((decode_merge_kernel<64, float>), mgrid, dim3(64), 0, stream,
-                         out, part_acc, part_ml, nheads, P, 0, 0.f, nullptr);
+                         out, part_acc, part_ml, nheads, P, 0, 0.f, nullptr, nullptr);
       break;
     case 128:
       hipLaunchKernelGGL(
@@ -494,7 +515,7 @@ void launch_paged_decode_mfma_chunk(float* out, float* part_acc, float* part_ml,
           dim3(256), 0, stream, part_acc, part_ml, q, kc, vc, bt, sl, scale, nheads,
           kvh, group, block_size, max_blocks, 0, chunk, v_heads);
       hipLaunchKernelGGL((decode_merge_kernel<128, float>), mgrid, dim3(128), 0,
-                         stream, out, part_acc, part_ml, nheads, P, 0, 0.f, nullptr);
+                         stream, out, part_acc, part_ml, nheads, P, 0, 0.f, nullptr, nullptr);
       break;
     default:
       abort();
@@ -522,10 +543,10 @@ static void launch_decode_span(__hip_bfloat16* out, float* part_acc, float* part
                        scale, nheads, kvh, group, block_size, max_blocks, window, 0, 0, sp);
   if (back != nullptr)
     hipLaunchKernelGGL((decode_merge_kernel<HD, __hip_bfloat16, true>), mgrid, dim3(HD), 0,
-                       stream, out, part_acc, part_ml, nheads, P, 0, 0.f, back);
+                       stream, out, part_acc, part_ml, nheads, P, 0, 0.f, back, nullptr);
   else
     hipLaunchKernelGGL((decode_merge_kernel<HD>), mgrid, dim3(HD), 0, stream, out, part_acc,
-                       part_ml, nheads, P, 0, 0.f, nullptr);
+                       part_ml, nheads, P, 0, 0.f, nullptr, nullptr);
 }
 
 void launch_paged_decode_mfma_span(__hip_bfloat16* out, float* part_acc, float* part_ml,
@@ -546,6 +567,41 @@ void launch_paged_decode_mfma_span(__hip_bfloat16* out, float* part_acc, float* 
   else if (head_dim == 128)
     launch_decode_span<128>(out, part_acc, part_ml, q, kc, vc, bt, sl, scale, nseq, nheads,
                             kvh, block_size, max_blocks, npart, window, sp, b2, stream);
+  else
+    abort();
+}
+
+// soft-capped scores, window, sinks per head or none (bf16 cache)
+template <int HD>
+static void launch_decode_capped(__hip_bfloat16* out, float* part_acc, float* part_ml,
+                                 const __hip_bfloat16* q, const __hip_bfloat16* kc,
+                                 const __hip_bfloat16* vc, const int* bt, const int* sl,
+                                 float scale, int nseq, int nheads, int kvh, int block_size,
+                                 int max_blocks, int npart, int window, const float* sinks,
+                                 float softcap, hipStream_t stream) {
+  const dim3 grid(nseq, kvh, npart), mgrid(nseq, nheads);
+  hipLaunchKernelGGL(
+      (paged_decode_mfma_kernel<HD, __hip_bfloat16, true, false, PX_NONE, true>), grid,
+      dim3(256), 0, stream, part_acc, part_ml, q, kc, vc, bt, sl, scale, nheads, kvh,
+      nheads / kvh, block_size, max_blocks, window, 0, 0, SpanKeys{}, softcap);
+  hipLaunchKernelGGL((decode_merge_kernel<HD>), mgrid, dim3(HD), 0, stream, out, part_acc,
+                     part_ml, nheads, npart * NWAVES, sinks != nullptr ? 1 : 0, 0.f, nullptr,
+                     sinks);
+}
+
+void launch_paged_decode_mfma_capped(__hip_bfloat16* out, float* part_acc, float* part_ml,
+                                     const __hip_bfloat16* q, const __hip_bfloat16* kc,
+                                     const __hip_bfloat16* vc, const int* bt, const int* sl,
+                                     float scale, int nseq, int nheads, int kvh, int head_dim,
+                                     int block_size, int max_blocks, int npart, int window,
+                                     const float* sinks, float softcap, hipStream_t stream) {
+  if (head_dim == 64)
+    launch_decode_capped<64>(out, part_acc, part_ml, q, kc, vc, bt, sl, scale, nseq, nheads,
+                             kvh, block_size, max_blocks, npart, window, sinks, softcap, stream);
+  else if (head_dim == 128)
+    launch_decode_capped<128>(out, part_acc, part_ml, q, kc, vc, bt, sl, scale, nseq, nheads,
+                              kvh, block_size, max_blocks, npart, window, sinks, softcap,
+                              stream);
   else
     abort();
 }

@@ -74,7 +74,17 @@ __device__ inline float cross_half_sum(float v) {
 // cache block that holds its last token (per_block places each).  back (cos,
 // sin per query row and pair): the output's dims m and m + HEAD_DIM/2 are turned
 // back by the row's angles before they are rounded.
+// CAP (capped variant, on top of WS): scores become softcap tanh(score / softcap)
+// before the softmax (softcap 0: as they are), and the sink is one per head.  A
+// cap also bounds the scores: up to kFixedMaxCap the exponentials are taken as
+// they are, without a running maximum or a rescale (e^60 and its inverse times
+// any count of keys stay inside f32 and bf16).
 enum { PX_NONE = 0, PX_KEEP = 1, PX_POOL = 2 };
+constexpr float kFixedMaxCap = 60.f;
+struct Capped {
+  float softcap;
+  const float* sinks;   // [nheads] or null
+};
 struct SpanTiles {
   int keep, pool, per_block;
   const __hip_bfloat16* k_pool;
@@ -83,7 +93,7 @@ struct SpanTiles {
 };
 
 template <int HEAD_DIM, typename CT, int NW, bool WS, bool CH = false,
-          typename OT = __hip_bfloat16, int PX = PX_NONE>
+          typename OT = __hip_bfloat16, int PX = PX_NONE, bool CAP = false>
 __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v2_kernel(
     OT* __restrict__ out,                        // [total_q, nheads, HD]
     const __hip_bfloat16* __restrict__ q,        // [total_q, nheads, HD]
@@ -102,7 +112,10 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
     const float sink,
     const int chunk = 0,
     const int v_heads = 0,
-    const SpanTiles sp = SpanTiles{}) {
+    const SpanTiles sp = SpanTiles{},
+    const Capped cap = Capped{}) {
+  static_assert(!CAP || (WS && !CH && PX == PX_NONE),
+                "the capped variant builds on the window variant");
   static_assert(HEAD_DIM == 128, "v2 is specialised for HD=128");
   static_assert(PX == PX_NONE || (WS && !CH), "prefixes build on the window variant");
   static_assert(!CH || WS, "the chunk variant builds on the window variant");
@@ -251,7 +264,12 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
   stage_load(tile_pos(0), PX != PX_NONE && pre_tiles > 0);
   stage_write(0);
 
-  const float sc2 = scale * LOG2E;  // fold softmax scale into exp2 domain
+  // fold softmax scale into exp2 domain; capped scores are already there
+  const bool capped = CAP && cap.softcap > 0.f;
+  const bool fixed_max = capped && cap.softcap <= kFixedMaxCap;
+  const float sc2 = capped ? 1.f : scale * LOG2E;
+  const float cap_in = capped ? scale / cap.softcap : 0.f, cap_out = cap.softcap * LOG2E;
+  if (fixed_max) m2_state = 0.f;
 
   for (int it = 0; it < num_tiles; ++it) {
     const int kv_base = tile_pos(it);
@@ -291,6 +309,29 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
     // ---- async stage: issue next tile's HBM loads now ------------------
     const bool more = it + 1 < num_tiles;
     if (more) stage_load(tile_pos(it + 1), PX != PX_NONE && it + 1 < pre_tiles);
+
+    if (CAP && capped && wave_active) {
+      // the tile's largest argument decides whether the polynomial alone will do
+      float big = 0.f;
+#pragma unroll
+      for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+        for (int r = 0; r < 16; ++r) {
+          acc_s[kb][r] *= cap_in;
+          big = fmaxf(big, fabsf(acc_s[kb][r]));
+        }
+      if (__all(big < kTanhSmall)) {
+#pragma unroll
+        for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+          for (int r = 0; r < 16; ++r) acc_s[kb][r] = cap_out * tanh_small(acc_s[kb][r]);
+      } else {
+#pragma unroll
+        for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+          for (int r = 0; r < 16; ++r) acc_s[kb][r] = cap_out * tanh_f32(acc_s[kb][r]);
+      }
+    }
 
     if (wave_active) {
       // ---- online softmax; the running max m2_state lives in the RAW
@@ -332,13 +373,13 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
             local_max = fmaxf(local_max, v);
           }
       }
-      const float tile_max = cross_half_max(local_max);
+      const float tile_max = CAP && fixed_max ? 0.f : cross_half_max(local_max);
 
       // defer-max (T13): skip the O/l rescale while the running max holds.
       // The decision is wave-uniform and taken BEFORE any of this tile's P
       // enters O or l, so everything at the old scale rescales exactly once.
       const float thr = DEFER_MAX_THR / sc2;
-      const bool need_rescale = !__all(
+      const bool need_rescale = !(CAP && fixed_max) && !__all(
           m2_state != -FLT_MAX && tile_max <= m2_state + thr);
       float m2_new = m2_state;
       if (need_rescale) {
@@ -449,11 +490,12 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
   // column and carries ALL 32 q rows for it; q-row validity is per row
   // (q_local check below), not per lane.
   float l_fin = l_state, o_scale = 1.f;
+  const float sink_h = CAP && cap.sinks != nullptr ? cap.sinks[head] : sink;
   if (WS && has_sink) {
     // the sink joins the denominator; both terms relative to the larger of
     // the running max and the sink (log2 domain)
     const float a2 = m2_state == -FLT_MAX ? -FLT_MAX : m2_state * sc2;
-    const float s2 = sink * LOG2E;
+    const float s2 = sink_h * LOG2E;
     const float mf = fmaxf(a2, s2);
     o_scale = a2 == -FLT_MAX ? 0.f : exp2f(a2 - mf);
     l_fin = l_state * o_scale + exp2f(s2 - mf);
@@ -504,7 +546,7 @@ static void launch_prefill_v2_ct(
     hipLaunchKernelGGL((paged_prefill_mfma_v2_kernel<128, CT, 8, true>),
                        dim3(nseq, nheads, qtiles), dim3(512), 0, stream, out,
                        q, kc, vc, bt, qsl, sl, scale, nheads, kvh, block_size,
-                       max_blocks, window, has_sink, sink);
+                       max_blocks, window, has_sink, sink, 0, 0, SpanTiles{}, Capped{});
     return;
   }
   static const int nw = [] {
@@ -518,13 +560,13 @@ static void launch_prefill_v2_ct(
     hipLaunchKernelGGL((paged_prefill_mfma_v2_kernel<128, CT, 8, false>),
                        dim3(nseq, nheads, qtiles), dim3(512), 0, stream, out,
                        q, kc, vc, bt, qsl, sl, scale, nheads, kvh, block_size,
-                       max_blocks, 0, 0, 0.f);
+                       max_blocks, 0, 0, 0.f, 0, 0, SpanTiles{}, Capped{});
   } else {
     const int qtiles = (max_query_len + 127) / 128;
     hipLaunchKernelGGL((paged_prefill_mfma_v2_kernel<128, CT, 4, false>),
                        dim3(nseq, nheads, qtiles), dim3(256), 0, stream, out,
                        q, kc, vc, bt, qsl, sl, scale, nheads, kvh, block_size,
-                       max_blocks, 0, 0, 0.f);
+                       max_blocks, 0, 0, 0.f, 0, 0, SpanTiles{}, Capped{});
   }
 }
 
@@ -572,7 +614,8 @@ void launch_paged_prefill_mfma_v2_chunk(
   hipLaunchKernelGGL(
       (paged_prefill_mfma_v2_kernel<128, __hip_bfloat16, 8, true, true, float>),
       dim3(nseq, nheads, qtiles), dim3(512), 0, stream, out, q, kc, vc, bt, qsl,
-      sl, scale, nheads, kvh, block_size, max_blocks, 0, 0, 0.f, chunk, v_heads);
+      sl, scale, nheads, kvh, block_size, max_blocks, 0, 0, 0.f, chunk, v_heads,
+      SpanTiles{}, Capped{});
 }
 
 // window plus a prefix of first tokens or pooled blocks (bf16 cache, HD = 128)
@@ -591,10 +634,28 @@ void launch_paged_prefill_mfma_v2_span(
     hipLaunchKernelGGL((paged_prefill_mfma_v2_kernel<128, __hip_bfloat16, 8, true, false,
                                                      __hip_bfloat16, PX_POOL>),
                        grid, dim3(512), 0, stream, out, q, kc, vc, bt, qsl, sl, scale,
-                       nheads, kvh, block_size, max_blocks, window, 0, 0.f, 0, 0, sp);
+                       nheads, kvh, block_size, max_blocks, window, 0, 0.f, 0, 0, sp,
+                       Capped{});
   else
     hipLaunchKernelGGL((paged_prefill_mfma_v2_kernel<128, __hip_bfloat16, 8, true, false,
                                                      __hip_bfloat16, PX_KEEP>),
                        grid, dim3(512), 0, stream, out, q, kc, vc, bt, qsl, sl, scale,
-                       nheads, kvh, block_size, max_blocks, window, 0, 0.f, 0, 0, sp);
+                       nheads, kvh, block_size, max_blocks, window, 0, 0.f, 0, 0, sp,
+                       Capped{});
+}
+
+// soft-capped scores, window, sinks per head or none (bf16 cache, HD = 128)
+void launch_paged_prefill_mfma_v2_capped(
+    __hip_bfloat16* out, const __hip_bfloat16* q, const __hip_bfloat16* kc,
+    const __hip_bfloat16* vc, const int* bt, const int* qsl, const int* sl, float scale,
+    int nseq, int nheads, int kvh, int block_size, int max_blocks, int max_query_len,
+    int window, const float* sinks, float softcap, hipStream_t stream) {
+  const dim3 grid(nseq, nheads, (max_query_len + 255) / 256);
+  Capped cap;
+  cap.softcap = softcap; cap.sinks = sinks;
+  hipLaunchKernelGGL((paged_prefill_mfma_v2_kernel<128, __hip_bfloat16, 8, true, false,
+                                                   __hip_bfloat16, PX_NONE, true>),
+                     grid, dim3(512), 0, stream, out, q, kc, vc, bt, qsl, sl, scale, nheads,
+                     kvh, block_size, max_blocks, window, sinks != nullptr ? 1 : 0, 0.f, 0, 0,
+                     SpanTiles{}, cap);
 }

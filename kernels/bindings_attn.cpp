@@ -26,6 +26,15 @@ void launch_paged_prefill_mfma(__hip_bfloat16*, const __hip_bfloat16*,
                                const __hip_bfloat16*, const __hip_bfloat16*,
                                const int*, const int*, const int*, float, int,
                                int, int, int, int, int, int, hipStream_t);
+void launch_paged_prefill_mfma_v2_capped(__hip_bfloat16*, const __hip_bfloat16*,
+                                         const __hip_bfloat16*, const __hip_bfloat16*,
+                                         const int*, const int*, const int*, float, int, int,
+                                         int, int, int, int, int, const float*, float,
+                                         hipStream_t);
+void launch_paged_decode_mfma_capped(__hip_bfloat16*, float*, float*, const __hip_bfloat16*,
+                                     const __hip_bfloat16*, const __hip_bfloat16*, const int*,
+                                     const int*, float, int, int, int, int, int, int, int, int,
+                                     const float*, float, hipStream_t);
 int decode_mfma_num_partitions(int nseq, int kvh, int max_context);
 void launch_paged_decode_mfma_fp8(__hip_bfloat16*, float*, float*,
                                   const __hip_bfloat16*, const unsigned char*,
@@ -328,6 +337,71 @@ void windowed_attention_decode(torch::Tensor out, torch::Tensor q,
       has_sink ? 1 : 0, (float)sink, current_stream());
 }
 
+// Capped variants: scores softcap * tanh(score / softcap) (0: as they are), sinks
+// per head or none; window, sizes and types as for the window variants.
+void check_sinks(const c10::optional<torch::Tensor>& sinks, int64_t heads, double softcap) {
+  TORCH_CHECK(softcap >= 0.0, "softcap");
+  if (!sinks.has_value()) return;
+  const auto& t = sinks.value();
+  TORCH_CHECK(t.is_cuda() && t.is_contiguous() && t.scalar_type() == at::ScalarType::Float &&
+              t.numel() == heads, "one f32 sink per head");
+}
+
+void capped_attention_prefill(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
+                              torch::Tensor v_cache, torch::Tensor block_tables,
+                              torch::Tensor query_start_loc, torch::Tensor seq_lens,
+                              double scale, int64_t max_query_len, int64_t window,
+                              c10::optional<torch::Tensor> sinks, double softcap) {
+  check_windowed(out, q, k_cache, v_cache, block_tables, seq_lens, window);
+  check_sinks(sinks, q.size(1), softcap);
+  TORCH_CHECK(q.size(2) == 128, "prompt portions need key size 128");
+  const int nseq = seq_lens.numel();
+  TORCH_CHECK(query_start_loc.is_cuda() && query_start_loc.is_contiguous() &&
+              query_start_loc.scalar_type() == at::ScalarType::Int &&
+              query_start_loc.numel() == nseq + 1 && max_query_len >= 1);
+  if (q.size(0) == 0 || nseq == 0) return;
+  launch_paged_prefill_mfma_v2_capped(
+      reinterpret_cast<__hip_bfloat16*>(out.data_ptr()),
+      reinterpret_cast<const __hip_bfloat16*>(q.data_ptr()),
+      reinterpret_cast<const __hip_bfloat16*>(k_cache.data_ptr()),
+      reinterpret_cast<const __hip_bfloat16*>(v_cache.data_ptr()),
+      block_tables.data_ptr<int>(), query_start_loc.data_ptr<int>(),
+      seq_lens.data_ptr<int>(), (float)scale, nseq, (int)q.size(1), (int)k_cache.size(2),
+      (int)k_cache.size(1), (int)block_tables.size(1), (int)max_query_len, (int)window,
+      sinks.has_value() ? sinks.value().data_ptr<float>() : nullptr, (float)softcap,
+      current_stream());
+}
+
+void capped_attention_decode(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache,
+                             torch::Tensor v_cache, torch::Tensor block_tables,
+                             torch::Tensor seq_lens, double scale, int64_t window,
+                             c10::optional<torch::Tensor> sinks, double softcap) {
+  check_windowed(out, q, k_cache, v_cache, block_tables, seq_lens, window);
+  check_sinks(sinks, q.size(1), softcap);
+  const int nseq = q.size(0), nheads = q.size(1), head_dim = q.size(2);
+  TORCH_CHECK(head_dim == 64 || head_dim == 128, "key size 64 or 128");
+  TORCH_CHECK(seq_lens.numel() == nseq, "one query row per sequence expected");
+  if (nseq == 0) return;
+  const int kvh = k_cache.size(2), block_size = k_cache.size(1);
+  const int max_blocks = block_tables.size(1);
+  int span = max_blocks * block_size;
+  if (window > 0 && window + 32 < span) span = (int)window + 32;
+  const int npart = decode_mfma_num_partitions(nseq, kvh, span);
+  const int P = npart * 4;
+  auto opts = q.options().dtype(at::ScalarType::Float);
+  auto part_acc = at::empty({nseq, nheads, P, head_dim}, opts);
+  auto part_ml = at::empty({nseq, nheads, P, 2}, opts);
+  launch_paged_decode_mfma_capped(
+      reinterpret_cast<__hip_bfloat16*>(out.data_ptr()), part_acc.data_ptr<float>(),
+      part_ml.data_ptr<float>(), reinterpret_cast<const __hip_bfloat16*>(q.data_ptr()),
+      reinterpret_cast<const __hip_bfloat16*>(k_cache.data_ptr()),
+      reinterpret_cast<const __hip_bfloat16*>(v_cache.data_ptr()),
+      block_tables.data_ptr<int>(), seq_lens.data_ptr<int>(), (float)scale, nseq, nheads, kvh,
+      head_dim, block_size, max_blocks, npart, (int)window,
+      sinks.has_value() ? sinks.value().data_ptr<float>() : nullptr, (float)softcap,
+      current_stream());
+}
+
 // Chunk variants of the bf16 MFMA kernels: position i sees keys j <= i with
 // floor(j / chunk) = floor(i / chunk) (0: all j <= i); the value cache may hold
 // fewer heads than the key cache (key head g reads value head g mod Gv); the
@@ -520,6 +594,10 @@ void register_attention_ops(pybind11::module& m) {
         "paged chunk-masked decode attention, f32 out (CDNA4)");
   m.def("windowed_attention_prefill", &windowed_attention_prefill,
         "paged windowed prefill attention with a softmax sink (CDNA4)");
+  m.def("capped_attention_prefill", &capped_attention_prefill,
+        "paged windowed prefill attention, soft-capped scores, sinks per head (CDNA4)");
+  m.def("capped_attention_decode", &capped_attention_decode,
+        "paged windowed decode attention, soft-capped scores, sinks per head (CDNA4)");
   m.def("windowed_attention_decode", &windowed_attention_decode,
         "paged windowed decode attention with a softmax sink (CDNA4)");
   m.def("paged_attention_decode", &paged_attention_decode,

@@ -23,8 +23,8 @@ template <typename T>
 void launch_relu2(T*, const T*, long, const T*, const float*, int, int, int,
                   hipStream_t);
 int moe_route_max_experts();
-void launch_moe_route(float*, float*, int*, float*, const float*, const float*,
-                      int, int, int, int, int, hipStream_t);
+void launch_moe_route(float*, float*, int*, float*, const float*, const float*, int, int,
+                      int, int, int, int, int, int, float, hipStream_t);
 template <typename T>
 void launch_moe_combine(T*, const T*, const int*, const int*, const float*, int,
                         int, int, int, hipStream_t);
@@ -35,6 +35,8 @@ void launch_moe_sort(T*, int*, int*, int*, const T*, long, const int*, int, int,
 void launch_moe_gemm(__hip_bfloat16*, const __hip_bfloat16*,
                      const __hip_bfloat16*, const int*, int, int, int, int, int,
                      hipStream_t);
+void launch_moe_gemm_clamped(__hip_bfloat16*, const __hip_bfloat16*, const __hip_bfloat16*,
+                             const int*, int, int, int, int, float, hipStream_t);
 
 namespace {
 
@@ -238,12 +240,14 @@ void moe_route(torch::Tensor dense, torch::Tensor ident, torch::Tensor ids,
   if (tokens == 0) return;
   launch_moe_route(ptr<float>(dense), ptr<float>(ident), ptr<int>(ids), ptr<float>(wts),
                    ptr<float>(logits), ptr<float>(correction), tokens, n, (int)num_real,
-                   top, 0, stream());
+                   top, 0, 1, 1, 1, 1.0f, stream());
 }
 
-// sigmoid scores, the top ones as they are (no correction, no renormalising)
+// sigmoid scores, optional correction of the choice, groups of experts of which
+// the best are kept, weights as they are or divided by their sum, times scale
 void moe_route_sigmoid(torch::Tensor dense, torch::Tensor ids, torch::Tensor wts,
-                       torch::Tensor logits) {
+                       torch::Tensor logits, c10::optional<torch::Tensor> correction,
+                       int64_t groups, int64_t keep, bool renormalise, double scale) {
   check_f32(logits, "logits");
   check_f32(dense, "dense");
   check_f32(wts, "weights");
@@ -254,9 +258,16 @@ void moe_route_sigmoid(torch::Tensor dense, torch::Tensor ids, torch::Tensor wts
   TORCH_CHECK(top >= 1 && top <= n && ids.size(0) == tokens && wts.dim() == 2 &&
               wts.size(0) == tokens && wts.size(1) == top &&
               dense.numel() == (long)tokens * n);
+  if (correction.has_value()) {
+    check_f32(correction.value(), "correction");
+    TORCH_CHECK(correction.value().numel() == n, "one correction per expert");
+  }
+  TORCH_CHECK(groups >= 1 && groups <= 64 && n % groups == 0 && keep >= 1 && keep <= groups &&
+              top <= keep * (n / groups), "expert groups (at most 64)");
   if (tokens == 0) return;
   launch_moe_route(ptr<float>(dense), nullptr, ptr<int>(ids), ptr<float>(wts),
-                   ptr<float>(logits), nullptr, tokens, n, n, top, 1, stream());
+                   ptr<float>(logits), optr<float>(correction), tokens, n, n, top, 1,
+                   (int)groups, (int)keep, renormalise ? 1 : 0, (float)scale, stream());
 }
 
 void moe_combine(torch::Tensor out, torch::Tensor ye, torch::Tensor pos,
@@ -329,6 +340,23 @@ void moe_gemm(torch::Tensor y, torch::Tensor x, torch::Tensor w,
                   stream());
 }
 
+// clamped gate of the halves, see common.h
+void moe_gemm_clamped(torch::Tensor y, torch::Tensor x, torch::Tensor w,
+                      torch::Tensor seg_off, double limit) {
+  TORCH_CHECK(x.is_cuda() && x.dim() == 2 && w.dim() == 3 && y.dim() == 2);
+  const int T = x.size(0), K = x.size(1), E = w.size(0), N = w.size(1) / 2;
+  for (const auto* t : {&x, &w, &y})
+    TORCH_CHECK(t->scalar_type() == at::ScalarType::BFloat16 && t->is_contiguous(),
+                "contiguous bf16 tensors");
+  check_i32(seg_off, "seg_off");
+  TORCH_CHECK(seg_off.numel() == E + 1 && w.size(1) == 2L * N && w.size(2) == K &&
+              N % 128 == 0 && K % 64 == 0 && y.size(0) == T && y.size(1) == N);
+  if (T == 0) return;
+  launch_moe_gemm_clamped(ptr<__hip_bfloat16>(y), ptr<__hip_bfloat16>(x),
+                          ptr<__hip_bfloat16>(w), ptr<int>(seg_off), E, N, K, T, (float)limit,
+                          stream());
+}
+
 }  // namespace
 
 void register_par_ops(pybind11::module& m) {
@@ -341,4 +369,5 @@ void register_par_ops(pybind11::module& m) {
   m.def("moe_combine", &moe_combine);
   m.def("moe_sort", &moe_sort);
   m.def("moe_gemm", &moe_gemm);
+  m.def("moe_gemm_clamped", &moe_gemm_clamped);
 }

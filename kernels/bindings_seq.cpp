@@ -47,6 +47,8 @@ void register_mix_ops(pybind11::module& m);
 // span_ops.hip, the window-plus-prefix attention and the gated linear attention
 // scan (bindings_span.cpp)
 void register_span_ops(pybind11::module& m);
+// tanh norms, wide query/key norm, delta rule, clamped gates (bindings_row.cpp)
+void register_row_ops(pybind11::module& m);
 namespace {
 
 hipStream_t stream() { return at::hip::getCurrentHIPStream().stream(); }
@@ -302,4 +304,5 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   register_par_ops(m);
   register_mix_ops(m);
   register_span_ops(m);
+  register_row_ops(m);
 }

@@ -18,9 +18,11 @@ Several extensions, so that a model only builds the ones it uses
             rotation + cache write, gates, expert routing, the grouped expert
             product, token shift, chunk-masked differential attention pieces,
             grouped norms around sublayers, attention inputs in one pass,
-            attention over a window plus a prefix, gated linear attention
+            attention over a window plus a prefix, gated linear attention,
+            tanh norms, query/key norm over the whole projection, the gated
+            delta rule, clamped gates, f32 router products
             + bindings_seq.cpp, bindings_rec.cpp, bindings_par.cpp,
-            bindings_mix.cpp, bindings_span.cpp
+            bindings_mix.cpp, bindings_span.cpp, bindings_row.cpp
 ``_C_lat``  windowed latent attention with sinks + bindings_lat.cpp
 """
 
@@ -40,7 +42,7 @@ ARCH = os.environ.get("PYTORCH_ROCM_ARCH", "gfx950")
 
 _SEQ_SOURCES = ["stream_ops.hip", "canon_conv.hip", "layer_norm_stream.hip",
                 "paged_attention_any.hip", "recurrent_scan.hip", "gated_block.hip",
-                "mix_ops.hip", "span_ops.hip"]
+                "mix_ops.hip", "span_ops.hip", "row_ops.hip", "delta_scan.hip"]
 # kernels without torch types that more than one extension links
 _SHARED_SOURCES = ["moe_gemm.hip"]
 _LAT_SOURCES = ["latent_attention.hip", "latent_attention_mfma.hip"]
@@ -61,7 +63,7 @@ EXTENSIONS = {
         sources=lambda: [KERNELS / n for n in _SEQ_SOURCES + _SHARED_SOURCES]
         + [KERNELS / "bindings_seq.cpp", KERNELS / "bindings_rec.cpp",
            KERNELS / "bindings_par.cpp", KERNELS / "bindings_mix.cpp",
-           KERNELS / "bindings_span.cpp"],
+           KERNELS / "bindings_span.cpp", KERNELS / "bindings_row.cpp"],
     ),
     "_C_lat": dict(
         sources=lambda: [KERNELS / n for n in _LAT_SOURCES] + [KERNELS / "bindings_lat.cpp"],
@@ -80,9 +82,10 @@ def build_ext(name: str, verbose: bool = True, force: bool = False) -> Path:
 
     sources = EXTENSIONS[name]["sources"]()
     out = ext_path(name)
-    common_h = KERNELS / "common.h"
+    headers = sorted(KERNELS.glob("*.h"))
+    newest_header = max(p.stat().st_mtime for p in headers)
     if out.exists() and not force:
-        newest_src = max(p.stat().st_mtime for p in sources + [common_h])
+        newest_src = max(p.stat().st_mtime for p in sources + headers)
         if out.stat().st_mtime > newest_src:
             if verbose:
                 print(f"[kernels/build] {out} up to date")
@@ -124,7 +127,7 @@ def build_ext(name: str, verbose: bool = True, force: bool = False) -> Path:
         assert src.name in module_sources or "TORCH_EXTENSION_NAME" not in src.read_text()
         objects.append(obj)
         if obj.exists() and not force and obj.stat().st_mtime > max(
-            src.stat().st_mtime, common_h.stat().st_mtime
+            src.stat().st_mtime, newest_header
         ):
             continue
         jobs.append(["hipcc", "-c", str(src), "-o", str(obj)] + common_flags)

@@ -141,6 +141,39 @@ DEVINLINE float block_reduce_sum(float x, float* lds_scratch) {
   return lds_scratch[0];
 }
 
+// ---------------------------------------------------------------------------
+// tanh to f32 accuracy on the hardware's exp2 and reciprocal.  Near zero the
+// quotient cancels, so small arguments take the odd Taylor polynomial (the
+// first dropped term is 1e-8 of the result at the switch).
+// ---------------------------------------------------------------------------
+
+constexpr float kTanhSmall = 0.35f;
+
+DEVINLINE float tanh_small(float x) {
+  const float z = x * x;
+  float p = __builtin_fmaf(z, -0.0088632355f, 0.0218694885f);
+  p = __builtin_fmaf(z, p, -0.0539682540f);
+  p = __builtin_fmaf(z, p, 0.1333333333f);
+  p = __builtin_fmaf(z, p, -0.3333333333f);
+  return __builtin_fmaf(x * z, p, x);
+}
+
+DEVINLINE float tanh_large(float x) {
+  const float e = __builtin_amdgcn_exp2f(-2.8853900818f * fabsf(x));   // exp(-2|x|)
+  return copysignf((1.0f - e) * __builtin_amdgcn_rcpf(1.0f + e), x);
+}
+
+DEVINLINE float tanh_f32(float x) {
+  return fabsf(x) < kTanhSmall ? tanh_small(x) : tanh_large(x);
+}
+
+// g' sigmoid(1.702 g') (u' + 1), g' = min(g, limit), u' = u within +-limit
+DEVINLINE float clamped_gate(float g, float u, float limit) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g / (1.0f + __expf(-1.702f * g)) * (u + 1.0f);
+}
+
 #define DISPATCH_BY_DTYPE(TORCH_DTYPE, FN)                                   \
   switch (TORCH_DTYPE) {                                                     \
     case at::ScalarType::BFloat16: {                                         \

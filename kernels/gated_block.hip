@@ -347,9 +347,11 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
     float* __restrict__ dense, float* __restrict__ ident, int* __restrict__ ids,
     float* __restrict__ wts, const float* __restrict__ logits,
     const float* __restrict__ correction, int tokens, int n, int num_real,
-    int top, int sigmoid) {
-  // sigmoid: scores are sigmoid(logit) instead of the softmax, there is no
-  // correction (nullptr), no identity output and no renormalising
+    int top, int sigmoid, int groups, int keep, int renorm, float scale) {
+  // sigmoid: scores are sigmoid(logit) instead of the softmax, the correction is
+  // optional and there is no identity output.  groups > 1: only the experts of
+  // the `keep` groups of neighbours with the largest sum of their two best choice
+  // scores stay open.  renorm: weights are divided by their sum; then times scale.
   const int lane = threadIdx.x & (WAVE_SIZE - 1);
   const long t = blockIdx.x * (long)(blockDim.x / WAVE_SIZE) + threadIdx.x / WAVE_SIZE;
   if (t >= tokens) return;
@@ -369,7 +371,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
     for (int i = 0; i < RT_MAX; ++i) {
       const int e = lane + i * WAVE_SIZE;
       s[i] = (e < n) ? 1.0f / (1.0f + expf(-s[i])) : 0.f;
-      ch[i] = (e < n) ? s[i] : -INFINITY;
+      ch[i] = (e < n) ? s[i] + (correction != nullptr ? correction[e] : 0.f) : -INFINITY;
     }
   } else {
     m = wave_reduce_max(m);
@@ -386,6 +388,46 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
       const int e = lane + i * WAVE_SIZE;
       s[i] = s[i] / den;
       ch[i] = (e < n) ? s[i] + correction[e] : -INFINITY;
+    }
+  }
+  if (groups > 1) {
+    // lane g ends up with group g's score (at most 64 groups)
+    const int size = n / groups;
+    float score = -INFINITY;
+    for (int g = 0; g < groups; ++g) {
+      float b1 = -INFINITY, b2 = -INFINITY;   // this lane's two best in the group
+#pragma unroll
+      for (int i = 0; i < RT_MAX; ++i) {
+        const int e = lane + i * WAVE_SIZE;
+        if (e >= g * size && e < (g + 1) * size) {
+          b2 = fmaxf(b2, fminf(b1, ch[i]));
+          b1 = fmaxf(b1, ch[i]);
+        }
+      }
+#pragma unroll
+      for (int off = 32; off > 0; off >>= 1) {
+        const float o1 = __shfl_xor(b1, off, WAVE_SIZE), o2 = __shfl_xor(b2, off, WAVE_SIZE);
+        b2 = fmaxf(fmaxf(b2, o2), fminf(b1, o1));
+        b1 = fmaxf(b1, o1);
+      }
+      if (lane == g) score = size > 1 ? b1 + b2 : b1;
+    }
+    unsigned long long open = 0;
+    for (int k = 0; k < keep; ++k) {
+      float best = (open >> lane) & 1 ? -INFINITY : score;
+      int at = lane < groups && !((open >> lane) & 1) ? lane : 0x7fffffff;
+#pragma unroll
+      for (int off = 32; off > 0; off >>= 1) {
+        const float ob = __shfl_xor(best, off, WAVE_SIZE);
+        const int oa = __shfl_xor(at, off, WAVE_SIZE);
+        if (ob > best || (ob == best && oa < at)) { best = ob; at = oa; }
+      }
+      if (at < groups) open |= 1ull << at;
+    }
+#pragma unroll
+    for (int i = 0; i < RT_MAX; ++i) {
+      const int e = lane + i * WAVE_SIZE;
+      if (e < n && !((open >> (e / size)) & 1)) ch[i] = -INFINITY;
     }
   }
   float total = 0.f, id_sum = 0.f;
@@ -427,16 +469,17 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
       wts[t * top + k] = sv;
     }
   }
-  const float inv = sigmoid ? 1.0f : 1.0f / (total + 1e-20f);
+  const float inv = (renorm ? 1.0f / (total + 1e-20f) : 1.0f) * scale;
 #pragma unroll
   for (int i = 0; i < RT_MAX; ++i) {
     const int e = lane + i * WAVE_SIZE;
     if (e < num_real) dense[t * num_real + e] = taken[i] ? s[i] * inv : 0.f;
   }
   // lane 0 wrote wts[t, :] itself, so it may rescale them in place
-  if (lane == 0 && !sigmoid) {
-    for (int k = 0; k < top; ++k) wts[t * top + k] *= inv;
-    ident[t] = id_sum * inv;
+  if (lane == 0) {
+    if (renorm || scale != 1.0f)
+      for (int k = 0; k < top; ++k) wts[t * top + k] *= inv;
+    if (!sigmoid) ident[t] = id_sum * inv;
   }
 }
 
@@ -678,10 +721,12 @@ int moe_route_max_experts() { return RT_MAX * WAVE_SIZE; }
 
 void launch_moe_route(float* dense, float* ident, int* ids, float* wts,
                       const float* logits, const float* correction, int tokens,
-                      int n, int num_real, int top, int sigmoid, hipStream_t s) {
+                      int n, int num_real, int top, int sigmoid, int groups, int keep,
+                      int renorm, float scale, hipStream_t s) {
   const int waves = 256 / WAVE_SIZE;
   moe_route_kernel<<<(tokens + waves - 1) / waves, 256, 0, s>>>(
-      dense, ident, ids, wts, logits, correction, tokens, n, num_real, top, sigmoid);
+      dense, ident, ids, wts, logits, correction, tokens, n, num_real, top, sigmoid, groups,
+      keep, renorm, scale);
 }
 
 template <typename T>

@@ -6,6 +6,7 @@
 //   h[r, :]  = silu(x[r]·Wg_e^T) * (x[r]·Wu_e^T)   (gated, w13 = [E, 2I, H])
 //   y[r, :]  = h[r]·W2_e^T                          (plain, w2  = [E, H, I])
 //   a[r, :]  = relu(x[r]·Wu_e^T)^2                  (squared relu, w = [E, I, H])
+//   h[r, :]  = clamped gate of x[r]·Wg_e^T, x[r]·Wu_e^T (see common.h; as gated)
 // where e = the expert owning sorted row r (seg_off[e] <= r < seg_off[e+1]).
 //
 // Geometry per kernel: grid (N/128, E * MBLK); each workgroup owns one
@@ -27,7 +28,7 @@ DEVINLINE int mg_swz(int row, int byte_in_row) {
   return row * (MG_KB * 2) + (byte_in_row ^ ((row & 7) << 4));
 }
 
-// MODE 0: plain, 1: gated (silu(g) * u), 2: squared relu
+// MODE 0: plain, 1: gated (silu(g) * u), 2: squared relu, 3: clamped gate
 template <int MODE>
 __global__ __launch_bounds__(256, 2) void moe_gemm_kernel(
     __hip_bfloat16* __restrict__ y,        // [T, N_out] (N_out = I or H)
@@ -37,8 +38,9 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_kernel(
     const int E,
     const int N,   // output width (I for gated, H for plain)
     const int K,
-    const int MBLK) {
-  constexpr bool GATED = MODE == 1;
+    const int MBLK,
+    const float limit = 0.f) {
+  constexpr bool GATED = MODE == 1 || MODE == 3;
   const int n_blk = blockIdx.x;
   const int e = blockIdx.y / MBLK;
   const int mb = blockIdx.y % MBLK;
@@ -159,7 +161,9 @@ __global__ __launch_bounds__(256, 2) void moe_gemm_kernel(
         const int m = mh * 64 + mt * 32 + (r & 3) + 8 * (r >> 2) + 4 * half;
         if (m >= M) continue;
         float v = acc_g[mt][nt][r];
-        if (GATED) {
+        if (MODE == 3) {
+          v = clamped_gate(v, acc_u[mt][nt][r], limit);
+        } else if (GATED) {
           const float act = v / (1.f + __expf(-v));
           v = act * acc_u[mt][nt][r];
         } else if (MODE == 2) {
@@ -180,11 +184,19 @@ void launch_moe_gemm(__hip_bfloat16* y, const __hip_bfloat16* x,
   dim3 block(256);
   if (mode == 1)
     hipLaunchKernelGGL(moe_gemm_kernel<1>, grid, block, 0, stream, y, x, w,
-                       seg_off, E, N, K, mblk);
+                       seg_off, E, N, K, mblk, 0.f);
   else if (mode == 2)
     hipLaunchKernelGGL(moe_gemm_kernel<2>, grid, block, 0, stream, y, x, w,
-                       seg_off, E, N, K, mblk);
+                       seg_off, E, N, K, mblk, 0.f);
   else
     hipLaunchKernelGGL(moe_gemm_kernel<0>, grid, block, 0, stream, y, x, w,
-                       seg_off, E, N, K, mblk);
+                       seg_off, E, N, K, mblk, 0.f);
+}
+
+void launch_moe_gemm_clamped(__hip_bfloat16* y, const __hip_bfloat16* x,
+                             const __hip_bfloat16* w, const int* seg_off, int E, int N,
+                             int K, int T, float limit, hipStream_t stream) {
+  const int mblk = (T + 127) / 128;
+  hipLaunchKernelGGL(moe_gemm_kernel<3>, dim3(N / 128, E * mblk), dim3(256), 0, stream, y,
+                     x, w, seg_off, E, N, K, mblk, limit);
 }

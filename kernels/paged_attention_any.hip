@@ -16,6 +16,7 @@
 // tokens, or one pooled key and value for every block of `pool` positions that
 // ends at or before i - window (block b is kept in the cache block that holds
 // its last token), and its output may be turned back by its position's angles.
+// With a soft cap c scores become c tanh(score / c); sinks may be one per head.
 // Prefix and window form one list of keys that is walked in order.  One workgroup per (query row, head).  Per tile of 256 keys:
 //   phase 1  thread j scores key j (q, already multiplied by the score scale,
 //            broadcast from LDS; the key row read with 16-byte loads), block
@@ -76,7 +77,8 @@ __global__ __launch_bounds__(PA_THREADS) void paged_attention_any_kernel(
     const int* __restrict__ qsl, const int* __restrict__ seq_lens, int nseq,
     float scale, int heads, int kv_heads, int dim, int vdim, int block_size,
     int vp /* pow2 >= min(vdim, 256) */, int vec_ok, int window, int has_sink,
-    float sink, int chunk, int v_heads, SpanPrefix<T> sp) {
+    float sink, int chunk, int v_heads, SpanPrefix<T> sp, float softcap,
+    const float* __restrict__ sinks) {
   extern __shared__ float smem[];
   float* q_s = smem;                               // [dim]
   float* p_s = q_s + ((dim + 1) & ~1);             // [256]
@@ -158,7 +160,7 @@ __global__ __launch_bounds__(PA_THREADS) void paged_attention_any_kernel(
       } else {
         for (int k = 0; k < dim; ++k) a += q_s[k] * ScalarOps<T>::to_f32(kr[k]);
       }
-      s = a;
+      s = softcap > 0.f ? softcap * tanh_f32(a / softcap) : a;
     }
     const float m_tile = pa_reduce_max(s, red);
     const float m_new = fmaxf(m_run, m_tile);
@@ -186,6 +188,7 @@ __global__ __launch_bounds__(PA_THREADS) void paged_attention_any_kernel(
   }
 
   float inv = 1.0f / l_run;
+  if (sinks != nullptr) sink = sinks[h];
   if (has_sink) {
     const float m_fin = fmaxf(m_run, sink);
     const float rescale = expf(m_run - m_fin);
@@ -236,7 +239,8 @@ static void launch_any(O* out, long o_st, const T* q, long q_st, const T* k_cach
                        int rows, int heads, int kv_heads, int dim, int vdim,
                        int block_size, int vec_ok, int window, int has_sink,
                        float sink, int chunk, int v_heads, hipStream_t stream,
-                       SpanPrefix<T> sp = SpanPrefix<T>{}) {
+                       SpanPrefix<T> sp = SpanPrefix<T>{}, float softcap = 0.f,
+                       const float* sinks = nullptr) {
   int vp = 1;
   while (vp < vdim && vp < PA_THREADS) vp <<= 1;
   const size_t smem = sizeof(float) * (((dim + 1) & ~1) + PA_THREADS + 16 +
@@ -246,7 +250,7 @@ static void launch_any(O* out, long o_st, const T* q, long q_st, const T* k_cach
   paged_attention_any_kernel<T, O, SPAN><<<grid, PA_THREADS, smem, stream>>>(
       out, o_st, q, q_st, k_cache, v_cache, block_tables, bt_stride, qsl,
       seq_lens, nseq, scale, heads, kv_heads, dim, vdim, block_size, vp, vec_ok,
-      window, has_sink, sink, chunk, v_heads, sp);
+      window, has_sink, sink, chunk, v_heads, sp, softcap, sinks);
 }
 
 template <typename T>
@@ -261,6 +265,20 @@ void launch_paged_attention_any(T* out, long o_st, const T* q, long q_st,
   launch_any<T, T>(out, o_st, q, q_st, k_cache, v_cache, block_tables, bt_stride, qsl,
                    seq_lens, nseq, scale, rows, heads, kv_heads, dim, vdim,
                    block_size, vec_ok, window, has_sink, sink, 0, kv_heads, stream);
+}
+
+// soft-capped scores, sinks per head (null: none)
+template <typename T>
+void launch_capped_attention(T* out, long o_st, const T* q, long q_st, const T* k_cache,
+                             const T* v_cache, const int* block_tables, int bt_stride,
+                             const int* qsl, const int* seq_lens, int nseq, float scale,
+                             int rows, int heads, int kv_heads, int dim, int vdim,
+                             int block_size, int vec_ok, int window, const float* sinks,
+                             float softcap, hipStream_t stream) {
+  launch_any<T, T>(out, o_st, q, q_st, k_cache, v_cache, block_tables, bt_stride, qsl,
+                   seq_lens, nseq, scale, rows, heads, kv_heads, dim, vdim, block_size, vec_ok,
+                   window, sinks != nullptr, 0.f, 0, kv_heads, stream, SpanPrefix<T>{}, softcap,
+                   sinks);
 }
 
 // chunk-masked variant with f32 output and a value cache of v_heads heads
@@ -320,3 +338,11 @@ template void launch_chunk_attention<__hip_bfloat16>(
     float*, long, const __hip_bfloat16*, long, const __hip_bfloat16*,
     const __hip_bfloat16*, const int*, int, const int*, const int*, int, float,
     int, int, int, int, int, int, int, int, int, hipStream_t);
+template void launch_capped_attention<float>(
+    float*, long, const float*, long, const float*, const float*, const int*, int,
+    const int*, const int*, int, float, int, int, int, int, int, int, int, int,
+    const float*, float, hipStream_t);
+template void launch_capped_attention<__hip_bfloat16>(
+    __hip_bfloat16*, long, const __hip_bfloat16*, long, const __hip_bfloat16*,
+    const __hip_bfloat16*, const int*, int, const int*, const int*, int, float, int, int,
+    int, int, int, int, int, int, const float*, float, hipStream_t);

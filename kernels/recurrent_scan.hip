@@ -22,6 +22,11 @@
 //               g = l + (1 - l) sigmoid(f + b) with a lower bound l per
 //               channel, y = S silu(q); a pointwise kernel ahead of the scan
 //               writes g and silu(q) in f32 once per (row, head, channel)
+//   KIND_DELTA  gated delta rule, alpha = g per head: u_t[j] = beta_t (v_t[j] -
+//               g_t S_(t-1)[j, :] . k_t), S_t[j, :] = g_t S_(t-1)[j, :] + u_t[j] k_t,
+//               y = g_t S_(t-1) . q_t + (k_t . q_t) u_t (the read-out sees the write);
+//               unit keys and scaled unit queries come in f32 from a pre-pass
+//               together with g, beta and k . q per (row, head)
 //   KIND_GLA    a decay per key channel: S_t[j, i] = alpha_t[i] S_(t-1)[j, i] +
 //               k_t[i] v_t[j], y = S q * q_scale; alpha = sigmoid(z)^(1/tau) with z
 //               from a low-rank product, written by a pre-pass in f32 once per
@@ -41,59 +46,13 @@
 // rglru_scan: elementwise linear recurrence, one thread per (sequence,
 // channel), gates and decay computed in f32 on the fly.
 
-#include "common.h"
+#include "scan_common.h"
 
 #include <type_traits>
 
 namespace {
 
-constexpr int NPT = 16;   // state values per thread along N
-enum { KIND_SSD = 0, KIND_MLSTM = 1, KIND_HGRN2 = 2, KIND_GLA = 3 };
-
-DEVINLINE float softplus_f(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
-DEVINLINE float logsigmoid_f(float x) { return fminf(x, 0.f) - log1pf(expf(-fabsf(x))); }
-DEVINLINE float sigmoid_f(float x) { return 1.0f / (1.0f + expf(-x)); }
-
-// Sum over NSP adjacent lanes (NSP a power of two, groups aligned), result in
-// every lane.  Up to 16 lanes the partner values come through DPP modifiers on
-// the adds (quad permutes, then the half-row and row mirrors — each mirror
-// pairs a lane with one from the other, already uniform, half), which costs no
-// LDS-crossbar round trip; wider groups finish with two shuffles.
-template <int CTRL>
-DEVINLINE float dpp_move(float v) {
-  return __int_as_float(
-      __builtin_amdgcn_update_dpp(0, __float_as_int(v), CTRL, 0xf, 0xf, true));
-}
-template <int NSP>
-DEVINLINE float lanes_sum(float x) {
-  if (NSP >= 2) x += dpp_move<0xB1>(x);    // quad_perm [1,0,3,2]
-  if (NSP >= 4) x += dpp_move<0x4E>(x);    // quad_perm [2,3,0,1]
-  if (NSP >= 8) x += dpp_move<0x141>(x);   // row_half_mirror
-  if (NSP >= 16) x += dpp_move<0x140>(x);  // row_mirror
-  if (NSP >= 32) x += __shfl_xor(x, 16, WAVE_SIZE);
-  if (NSP >= 64) x += __shfl_xor(x, 32, WAVE_SIZE);
-  return x;
-}
-
-// 16 consecutive values p[n0 .. n0+16) of a row of length n_total as f32,
-// zeros past the end
-template <typename T>
-DEVINLINE void load_slice(const T* __restrict__ p, int n0, int n_total, bool vec,
-                          float* dst) {
-  if (vec && n0 + NPT <= n_total) {
-    constexpr int V = Vec16<T>::kElems;
-#pragma unroll
-    for (int i = 0; i < NPT; i += V) {
-      const Vec16<T> v = load16(p + n0 + i);
-#pragma unroll
-      for (int u = 0; u < V; ++u) dst[i + u] = ScalarOps<T>::to_f32(v.data[u]);
-    }
-  } else {
-#pragma unroll
-    for (int i = 0; i < NPT; ++i)
-      dst[i] = (n0 + i < n_total) ? ScalarOps<T>::to_f32(p[n0 + i]) : 0.f;
-  }
-}
+enum { KIND_SSD = 0, KIND_MLSTM = 1, KIND_HGRN2 = 2, KIND_GLA = 3, KIND_DELTA = 4 };
 
 struct ScanArgs {
   // rows
@@ -209,8 +168,10 @@ __global__ __launch_bounds__(256) void matrix_scan_kernel(ScanArgs a) {
 
   const float c2 = KIND == KIND_SSD ? a.p2[h] : 0.f;   // D
   const float4* gp = a.gates + h;
-  // HGRN2 reads its gate and activated query from the f32 rows of the pre-pass
-  using KQ = typename std::conditional<KIND == KIND_HGRN2, float, T>::type;
+  // HGRN2 reads its gate and activated query, the delta rule its unit keys and
+  // queries from the f32 rows of a pre-pass
+  using KQ =
+      typename std::conditional<KIND == KIND_HGRN2 || KIND == KIND_DELTA, float, T>::type;
   const KQ* qp = reinterpret_cast<const KQ*>(a.q) + (long)grp * a.nk;
   const KQ* kp = reinterpret_cast<const KQ*>(a.k) + (long)grp * a.nk;
   const T* vp = reinterpret_cast<const T*>(a.v) + (long)h * a.vdim;
@@ -239,6 +200,24 @@ __global__ __launch_bounds__(256) void matrix_scan_kernel(ScanArgs a) {
     const bool more = r + 1 < n;       // uniform over the workgroup
     if (more) load_row(row + 1, kn, qn, vn, dn, gn);
     const float alpha = gt.x, beta = gt.y;
+    if constexpr (KIND == KIND_DELTA) {
+      float dk[VPT], dq[VPT], u[VPT];
+#pragma unroll
+      for (int c = 0; c < VPT; ++c) {
+        dk[c] = dq[c] = 0.f;
+#pragma unroll
+        for (int i = 0; i < NPT; ++i) {
+          dk[c] += S[c][i] * kk[i];
+          dq[c] += S[c][i] * qq[i];
+        }
+        u[c] = beta * (vj[c] - alpha * lanes_sum<NSP>(dk[c]));
+        const float yv = alpha * lanes_sum<NSP>(dq[c]) + gt.z * u[c];
+        if (ns == 0 && jbase + c < a.vdim)
+          a.y[row * a.y_st + (long)h * a.vdim + jbase + c] = yv;
+#pragma unroll
+        for (int i = 0; i < NPT; ++i) S[c][i] = alpha * S[c][i] + u[c] * kk[i];
+      }
+    } else {
     float dot[VPT], ndot = 0.f;
 #pragma unroll
     for (int c = 0; c < VPT; ++c) dot[c] = 0.f;
@@ -268,6 +247,7 @@ __global__ __launch_bounds__(256) void matrix_scan_kernel(ScanArgs a) {
                        : KIND == KIND_GLA ? d * a.q_scale : d + c2 * vj[c];
       if (ns == 0 && jbase + c < a.vdim)
         a.y[row * a.y_st + (long)h * a.vdim + jbase + c] = yv;
+    }
     }
     if (more) {
 #pragma unroll
@@ -344,6 +324,42 @@ __global__ __launch_bounds__(256) void hgrn2_gates_kernel(
   gq[row * 2 * hd + hd + c] = qv * sigmoid_f(qv);
 }
 
+// Delta-rule pre-pass, one workgroup per row: kq [T, 2, G * dim] f32 = (k / |k|,
+// q / |q| * q_scale) per head of the short-convolved rows, gates (g, beta,
+// k . q, -) per head of the values.
+template <typename T>
+__global__ __launch_bounds__(256) void delta_inputs_kernel(
+    float* __restrict__ kq, float4* __restrict__ gates, const T* __restrict__ q, long q_st,
+    const T* __restrict__ k, long k_st, const T* __restrict__ b_pre, long b_st,
+    const T* __restrict__ a_pre, long a_st, const float* __restrict__ a_log,
+    const float* __restrict__ dt_bias, float q_scale, int heads, int groups, int dim) {
+  extern __shared__ float both[];   // [groups] k . q
+  const long row = blockIdx.x;
+  const int lane = threadIdx.x & (WAVE_SIZE - 1), wave = threadIdx.x / WAVE_SIZE;
+  const int gd = groups * dim;
+  for (int g = wave; g < groups; g += 256 / WAVE_SIZE) {
+    float sk = 0.f, sq = 0.f, kqs = 0.f;
+    for (int c = lane; c < dim; c += WAVE_SIZE) {
+      const float kv = ScalarOps<T>::to_f32(k[row * k_st + g * dim + c]);
+      const float qv = ScalarOps<T>::to_f32(q[row * q_st + g * dim + c]);
+      sk += kv * kv; sq += qv * qv; kqs += kv * qv;
+    }
+    sk = wave_reduce_sum(sk); sq = wave_reduce_sum(sq); kqs = wave_reduce_sum(kqs);
+    const float ik = 1.0f / sqrtf(sk + kUnitEps), iq = q_scale / sqrtf(sq + kUnitEps);
+    for (int c = lane; c < dim; c += WAVE_SIZE) {
+      kq[row * 2 * gd + g * dim + c] = ScalarOps<T>::to_f32(k[row * k_st + g * dim + c]) * ik;
+      kq[row * 2 * gd + gd + g * dim + c] =
+          ScalarOps<T>::to_f32(q[row * q_st + g * dim + c]) * iq;
+    }
+    if (lane == 0) both[g] = kqs * ik * iq;
+  }
+  __syncthreads();
+  for (int h = threadIdx.x; h < heads; h += 256)
+    gates[row * heads + h] = make_float4(
+        delta_decay(ScalarOps<T>::to_f32(a_pre[row * a_st + h]), a_log[h], dt_bias[h]),
+        sigmoid_f(ScalarOps<T>::to_f32(b_pre[row * b_st + h])), both[h / (heads / groups)], 0.f);
+}
+
 // exp(logsigmoid(z) * inv_tau) on the hardware's exp2 / log2: log1p through
 // log(u), u = 1 + e, with what the rounding of u lost added back
 DEVINLINE float gla_decay_of(float z, float inv_tau) {
@@ -404,19 +420,6 @@ struct GlaArgs {
   float* state;
   const int* loc; const int* seq_lens; const int* slots;
   int heads, dim, vdim, rank;
-};
-
-template <typename T> struct RowPiece;    // eight elements as stored
-template <> struct RowPiece<__hip_bfloat16> {
-  uint4 u;
-  DEVINLINE float at(int i) const {
-    const unsigned w[4] = {u.x, u.y, u.z, u.w};
-    return __uint_as_float(i & 1 ? w[i / 2] & 0xffff0000u : w[i / 2] << 16);
-  }
-};
-template <> struct RowPiece<float> {
-  float f[8];
-  DEVINLINE float at(int i) const { return f[i]; }
 };
 
 template <typename T, int NSP, int VPT>
@@ -941,6 +944,30 @@ void launch_gla_scan(float* o, const T* q, long q_st, const T* k, long k_st, con
   launch_matrix_scan<T, KIND_GLA>(a, nseq, stream);
 }
 
+template <typename T>
+void launch_delta_scan(float* o, const T* q, long q_st, const T* k, long k_st, const T* v,
+                       long v_st, const T* b_pre, long b_st, const T* a_pre, long a_st,
+                       const float* a_log, const float* dt_bias, float q_scale, float* state,
+                       const int* loc, const int* seq_lens, const int* slots, int nseq,
+                       int heads, int groups, int dim, int vdim, int vec_ok, float* kq,
+                       float* gates, int rows, hipStream_t stream) {
+  const int gd = groups * dim;
+  ScanArgs a{};
+  a.gates = reinterpret_cast<float4*>(gates); a.rows = rows;
+  delta_inputs_kernel<T><<<rows, 256, sizeof(float) * groups, stream>>>(
+      kq, a.gates, q, q_st, k, k_st, b_pre, b_st, a_pre, a_st, a_log, dt_bias, q_scale, heads,
+      groups, dim);
+  a.k = kq;      a.k_st = 2L * gd;
+  a.q = kq + gd; a.q_st = 2L * gd;
+  a.v = v;       a.v_st = v_st;
+  a.y = o; a.y_st = (long)heads * vdim;
+  a.s_state = state;
+  a.loc = loc; a.seq_lens = seq_lens; a.slots = slots;
+  a.heads = heads; a.vdim = vdim; a.nk = dim; a.per_group = heads / groups;
+  a.vec_ok = vec_ok;
+  launch_matrix_scan<T, KIND_DELTA>(a, nseq, stream);
+}
+
 // value columns per thread of the one-kernel form, 0 when the shape does not fit
 int gla_fused_columns(int dim, int vdim) {
   if (dim % 8 || vdim % 8 || dim > 256) return 0;
@@ -1026,6 +1053,12 @@ void launch_rglru_scan(T* out, const T* u, const T* r_pre, const T* i_pre,
                                    const float*, float, float, float*,          \
                                    const int*, const int*, const int*, int, int, \
                                    int, int, int, int, float*, int, hipStream_t); \
+  template void launch_delta_scan<T>(float*, const T*, long, const T*, long,    \
+                                     const T*, long, const T*, long, const T*,  \
+                                     long, const float*, const float*, float,   \
+                                     float*, const int*, const int*, const int*, \
+                                     int, int, int, int, int, int, float*,      \
+                                     float*, int, hipStream_t);                 \
   template void launch_gla_fused<T>(T*, const T*, long, const T*, long,         \
                                     const T*, long, const T*, long, const T*,   \
                                     long, const float*, const float*, float,    \
