@@ -45,8 +45,8 @@ def parse_args():
     p.add_argument("--arch-sizes", type=str, default="s,m",
                    help="arch mode: comma list of sizes (s, m)")
     p.add_argument("--arch-models", type=str, default="dolodra,llama",
-                   help="arch mode: which models to run (dolodra, kezunex, relerax, gumozen, balenex, "
-                        "llama)")
+                   help="arch mode: which models to run (dolodra, kezunex, relerax, gumozen, "
+                        "balenex, latanex, llama)")
     p.add_argument("--model", type=str, default="llama-3-8b")
     p.add_argument("--batch", type=int, default=512)
     p.add_argument("--prompt-len", type=int, default=512)
@@ -682,6 +682,43 @@ def _balenex_model_config(name: str, sz: dict, dtype: str):
     return mc
 
 
+# Latanex at the same widths: eight layers [attention, delta, attention, attention]
+# x 2.  The attention has the llama's heads of 128 with a window of 512 and capped
+# scores, the delta rule width / 128 value heads of 128 over half as many key heads.
+# Every second layer has the llama's feed-forward, the others route: the chosen
+# experts and the shared one add up to the llama's feed-forward.
+LATANEX_SIZES = {
+    "s": dict(experts=16, top=3, groups=4, keep=2, expert_ff=1408, window=512),
+    "m": dict(experts=16, top=3, groups=4, keep=2, expert_ff=3584, window=512),
+    "t": dict(experts=8, top=2, groups=2, keep=1, expert_ff=32, window=12),
+}
+
+
+def _latanex_model_config(name: str, sz: dict, dtype: str):
+    from vllm_tgis_adapter_amd.engine.config import _DTYPES
+    from vllm_tgis_adapter_amd.models.latanex import model_config_from_json
+
+    lx = LATANEX_SIZES[name]
+    hd = sz["width"] // sz["heads"]
+    attn = {"heads": sz["heads"], "kv_heads": sz["llama_kv_heads"], "dim": hd, "vdim": hd,
+            "scale": hd ** -0.5, "softcap": 50.0, "mask": {"size": lx["window"]}, "v_mix": True}
+    delta = {"heads": sz["heads"], "kv_heads": sz["heads"] // 2, "dim": hd, "vdim": hd, "conv": 4}
+    dense = {"kind": "dense", "ff": sz["llama_inter"]}
+    moe = {"kind": "moe", "expert": {"ff": lx["expert_ff"], "limit": 7.0},
+           "router": {"experts": lx["experts"], "top": lx["top"], "scale": 2.5,
+                      "groups": {"count": lx["groups"], "keep": lx["keep"]}},
+           "shared": {"ff": lx["expert_ff"], "limit": 7.0}}
+    layers = [{"type": "delta" if i % 4 == 1 else "attention",
+               "mixer": delta if i % 4 == 1 else attn,
+               "mlp": moe if i % 2 else dense} for i in range(sz["layers"])]
+    hf = {"architecture": "Latanex", "vocab": sz["vocab"], "width": sz["width"],
+          "layers": layers, "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0},
+          "logit_scale": 1.0}
+    mc = model_config_from_json("latanex-synthetic", hf)
+    mc.dtype = _DTYPES[dtype]
+    return mc
+
+
 def _arch_measure(mc, args, device: str, batch: int, prompt_len: int, steps: int,
                   warmup: int) -> dict:
     from vllm_tgis_adapter_amd.engine import EngineConfig, LLMEngine, SamplingParams
@@ -748,7 +785,7 @@ def run_arch(args, device: str) -> None:
         steps = args.steps if device == "cuda" else 4
         warm = args.warmup if device == "cuda" else 1
         models = [("dolodra", dolo), ("kezunex", None), ("relerax", None), ("gumozen", None),
-                  ("balenex", None), ("llama", llama)]
+                  ("balenex", None), ("latanex", None), ("llama", llama)]
         for label, mc in models:
             if label not in args.arch_models.split(","):
                 continue
@@ -760,6 +797,8 @@ def run_arch(args, device: str) -> None:
                 mc = _gumozen_model_config(name, sz, args.dtype)
             if label == "balenex":
                 mc = _balenex_model_config(name, sz, args.dtype)
+            if label == "latanex":
+                mc = _latanex_model_config(name, sz, args.dtype)
             r = _arch_measure(mc, args, device, batch, plen, steps, warm)
             r.update(size=name, model=label, batch=batch, prompt_len=plen)
             out.append(r)
