@@ -224,10 +224,26 @@ __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
     // ---- online softmax (stats per q col = this lane's col) --------------
     float s_val[16];
     float local_max = -FLT_MAX;
+    if (CAP && capped) {
+      // the tile's largest argument decides whether the polynomial alone will do
+      float big = 0.f;
+#pragma unroll
+      for (int r = 0; r < 16; ++r) {
+        acc_s[r] *= cap_in;
+        big = fmaxf(big, fabsf(acc_s[r]));
+      }
+      if (__all(big < kTanhSmall)) {
+#pragma unroll
+        for (int r = 0; r < 16; ++r) acc_s[r] = tanh_small(acc_s[r]);
+      } else {
+#pragma unroll
+        for (int r = 0; r < 16; ++r) acc_s[r] = tanh_f32(acc_s[r]);
+      }
+    }
 #pragma unroll
     for (int r = 0; r < 16; ++r) {
       const int kv_pos = kv_base + (r & 3) + 8 * (r >> 2) + 4 * half;
-      float sv = capped ? softcap * tanh_f32(acc_s[r] * cap_in) : acc_s[r] * scale;
+      float sv = acc_s[r] * (CAP && capped ? softcap : scale);
       if (kv_pos >= limit || (WS && !prefix && kv_pos < first_pos)) sv = -FLT_MAX;
       s_val[r] = sv;
       local_max = fmaxf(local_max, sv);

@@ -34,7 +34,7 @@ void launch_latent_kv_write(const T*, const float*, float, const long*,
 template <typename T>
 void launch_causal_conv_state(T*, const T*, const float*, T*, const int*,
                               const int*, const int*, int, int, int, int, int,
-                              long, const float*, int, hipStream_t);
+                              long, const float*, int, int, hipStream_t);
 // layer norms of the stream, attention of any shape, recurrences
 // (bindings_rec.cpp)
 void register_rec_ops(pybind11::module& m);
@@ -257,7 +257,7 @@ void causal_conv_state(torch::Tensor out, torch::Tensor h, torch::Tensor weight,
                        torch::Tensor state, torch::Tensor loc,
                        torch::Tensor seq_lens, torch::Tensor slots,
                        bool add_input, c10::optional<torch::Tensor> bias,
-                       int64_t act) {
+                       int64_t act, bool has_portions) {
   TORCH_CHECK(h.is_cuda() && h.dim() == 2 && h.stride(1) == 1 &&
               out.is_contiguous() && out.scalar_type() == h.scalar_type() &&
               out.numel() == h.numel());
@@ -275,6 +275,7 @@ void causal_conv_state(torch::Tensor out, torch::Tensor h, torch::Tensor weight,
   const int nseq = seq_lens.numel();
   TORCH_CHECK(weight.size(0) == width && loc.numel() == nseq + 1 &&
               slots.numel() == nseq && taps >= 1);
+  TORCH_CHECK(has_portions || h.size(0) == nseq, "one row per sequence expected");
   TORCH_CHECK(state.is_contiguous() && state.scalar_type() == h.scalar_type() &&
               state.dim() == 3 && state.size(1) == taps - 1 &&
               (taps == 1 || state.size(2) == width), "conv state shape");
@@ -284,7 +285,7 @@ void causal_conv_state(torch::Tensor out, torch::Tensor h, torch::Tensor weight,
         ptr<scalar_t>(state), ptr<int>(loc), ptr<int>(seq_lens), ptr<int>(slots),
         (int)h.size(0), nseq, width, taps, add_input ? 1 : 0, (long)h.stride(0),
         bias.has_value() ? ptr<float>(bias.value()) : nullptr, (int)act,
-        stream());
+        has_portions ? 0 : 1, stream());
   });
 }
 

@@ -15,8 +15,13 @@
 // is shorter than taps-1, from old state row j + n — each thread walks j
 // upwards, so it reads row j + n before that row is overwritten.
 //
-// One thread per (row, 4 channels) — or one channel when the width is not a
-// multiple of 4: consecutive threads take consecutive channels,
+// Two kernels.  The row-walking one: a thread owns 8 channels and walks up to
+// CW_ROWS consecutive rows with their weights and the last taps-1 inputs in
+// registers, so every input is read once, the next row's while this one is
+// computed; where every sequence of the step brings a single row it also
+// advances the state itself (nobody else reads that sequence's rows).  The other
+// takes any tap count and width: one thread per (row, 4 channels) — or one channel when the width is not a
+// multiple of 4.  Consecutive threads take consecutive channels,
 // every load and store is coalesced; accumulation is f32.
 
 #include "common.h"
@@ -44,6 +49,43 @@ DEVINLINE void store_ch(T* p, const float* v) {
 #pragma unroll
   for (int k = 0; k < CH; ++k) p[k] = ScalarOps<T>::from_f32(v[k]);
 }
+
+// eight channels as they are stored
+template <typename T> struct Vec8;
+template <> struct Vec8<__hip_bfloat16> {
+  uint4 u;
+  static DEVINLINE Vec8 load(const __hip_bfloat16* p) {
+    return Vec8{*reinterpret_cast<const uint4*>(p)};
+  }
+  DEVINLINE void unpack(float* f) const {
+    const unsigned t[4] = {u.x, u.y, u.z, u.w};
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      f[2 * i] = __uint_as_float(t[i] << 16);
+      f[2 * i + 1] = __uint_as_float(t[i] & 0xffff0000u);
+    }
+  }
+  static DEVINLINE void store(__hip_bfloat16* p, const float* f) {
+    union { __hip_bfloat16 h[8]; uint4 u; } o;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) o.h[i] = __float2bfloat16(f[i]);
+    *reinterpret_cast<uint4*>(p) = o.u;
+  }
+};
+template <> struct Vec8<float> {
+  float4 a, b;
+  static DEVINLINE Vec8 load(const float* p) {
+    return Vec8{reinterpret_cast<const float4*>(p)[0], reinterpret_cast<const float4*>(p)[1]};
+  }
+  DEVINLINE void unpack(float* f) const {
+    f[0] = a.x; f[1] = a.y; f[2] = a.z; f[3] = a.w;
+    f[4] = b.x; f[5] = b.y; f[6] = b.z; f[7] = b.w;
+  }
+  static DEVINLINE void store(float* p, const float* f) {
+    reinterpret_cast<float4*>(p)[0] = make_float4(f[0], f[1], f[2], f[3]);
+    reinterpret_cast<float4*>(p)[1] = make_float4(f[4], f[5], f[6], f[7]);
+  }
+};
 
 DEVINLINE int find_seq(const int* __restrict__ loc, int nseq, int row) {
   int lo = 0, hi = nseq;  // largest s with loc[s] <= row
@@ -125,6 +167,71 @@ __global__ void causal_conv_kernel(T* __restrict__ out, const T* __restrict__ h,
   store_ch<T, CH>(out + o, acc);
 }
 
+constexpr int CW_ROWS = 16;
+
+template <typename T, int TAPS, int ROWS>
+__global__ __launch_bounds__(256) void causal_conv_walk_kernel(
+    T* __restrict__ out, const T* __restrict__ h, const float* __restrict__ w,
+    T* __restrict__ state, const int* __restrict__ loc, const int* __restrict__ seq_lens,
+    const int* __restrict__ slots, int nseq, int rows, int width, int add_input, long in_st,
+    const float* __restrict__ bias, int act, int single_rows) {
+  const int c = (blockIdx.y * 256 + threadIdx.x) * 8;
+  if (c >= width) return;
+  const int r0 = blockIdx.x * ROWS, r1 = min(r0 + ROWS, rows);
+  Vec8<T> nxt = Vec8<T>::load(h + (long)r0 * in_st + c);
+  float wv[TAPS][8], bv[8], hist[TAPS][8];   // hist[TAPS - 1]: the current row
+#pragma unroll
+  for (int k = 0; k < 8; ++k) {
+    bv[k] = bias != nullptr ? bias[c + k] : 0.f;
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) wv[j][k] = w[(long)(c + k) * TAPS + j];
+  }
+  int s = find_seq(loc, nseq, r0);
+  bool fresh = true;             // the history registers do not hold this sequence's rows
+  for (int row = r0; row < r1; ++row) {
+    while (s + 1 < nseq && row >= loc[s + 1]) { ++s; fresh = true; }
+    const int slot = slots[s], first = loc[s];
+    const int start = seq_lens[s] - (loc[s + 1] - first);
+    const int p = start + row - first;
+    const Vec8<T> cur = nxt;
+    if (row + 1 < r1) nxt = Vec8<T>::load(h + (long)(row + 1) * in_st + c);
+    if (fresh) {
+#pragma unroll
+      for (int j = 0; j < TAPS - 1; ++j) {
+        const int pj = p - (TAPS - 1) + j;
+#pragma unroll
+        for (int k = 0; k < 8; ++k) hist[j][k] = 0.f;
+        if (pj >= start)
+          Vec8<T>::load(h + (long)(first + pj - start) * in_st + c).unpack(hist[j]);
+        else if (pj >= 0 && slot >= 0)
+          Vec8<T>::load(state + ((long)slot * (TAPS - 1) + pj - start + TAPS - 1) * width + c)
+              .unpack(hist[j]);
+      }
+      fresh = false;
+    }
+    cur.unpack(hist[TAPS - 1]);
+    float acc[8];
+#pragma unroll
+    for (int k = 0; k < 8; ++k) {
+      acc[k] = bv[k] + (add_input ? hist[TAPS - 1][k] : 0.f);
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) acc[k] += wv[j][k] * hist[j][k];
+      if (act == 1) acc[k] = acc[k] / (1.0f + __expf(-acc[k]));
+      if (slot < 0) acc[k] = 0.f;           // padding row of a captured bucket
+    }
+    Vec8<T>::store(out + (long)row * width + c, acc);
+    if (single_rows && slot >= 0) {
+      T* st = state + (long)slot * (TAPS - 1) * width + c;
+#pragma unroll
+      for (int j = 0; j < TAPS - 1; ++j) Vec8<T>::store(st + (long)j * width, hist[j + 1]);
+    }
+#pragma unroll
+    for (int j = 0; j + 1 < TAPS; ++j)
+#pragma unroll
+      for (int k = 0; k < 8; ++k) hist[j][k] = hist[j + 1][k];
+  }
+}
+
 template <typename T>
 __global__ void conv_state_update_kernel(T* __restrict__ state,
                                          const T* __restrict__ h,
@@ -169,8 +276,31 @@ void launch_causal_conv_state(T* out, const T* h, const float* w, T* state,
                               const int* loc, const int* seq_lens,
                               const int* slots, int rows, int nseq, int width,
                               int taps, int add_input, long in_st,
-                              const float* bias, int act, hipStream_t stream) {
+                              const float* bias, int act, int single_rows,
+                              hipStream_t stream) {
   const int block = 256;
+  const bool walk = taps >= 2 && taps <= 4 && width % 8 == 0 && in_st % 8 == 0 &&
+                    reinterpret_cast<uintptr_t>(h) % 16 == 0 &&
+                    reinterpret_cast<uintptr_t>(out) % 16 == 0 &&
+                    reinterpret_cast<uintptr_t>(state) % 16 == 0;
+  if (walk) {
+    const int gy = (width / 8 + block - 1) / block;
+#define WALK_LAUNCH(TP, R)                                                         \
+    causal_conv_walk_kernel<T, TP, R><<<dim3((rows + R - 1) / R, gy), block, 0, stream>>>( \
+        out, h, w, state, loc, seq_lens, slots, nseq, rows, width, add_input, in_st, bias, act, \
+        single_rows)
+#define WALK_CASE(TP)                                                              \
+    if (single_rows || rows < 1024) WALK_LAUNCH(TP, 1); else WALK_LAUNCH(TP, CW_ROWS)
+    if (taps == 2) { WALK_CASE(2); }
+    else if (taps == 3) { WALK_CASE(3); }
+    else { WALK_CASE(4); }
+#undef WALK_CASE
+#undef WALK_LAUNCH
+    if (!single_rows)
+      launch_conv_state_update<T>(state, h, loc, seq_lens, slots, nseq, width, taps, in_st,
+                                  stream);
+    return;
+  }
   const bool vec = width % 4 == 0 && in_st % 4 == 0 &&
                    (bias == nullptr || reinterpret_cast<uintptr_t>(bias) % 16 == 0) &&
                    reinterpret_cast<uintptr_t>(h) % (4 * sizeof(T)) == 0 &&
@@ -203,12 +333,12 @@ void launch_causal_conv_state(T* out, const T* h, const float* w, T* state,
 template void launch_causal_conv_state<float>(float*, const float*, const float*,
                                               float*, const int*, const int*,
                                               const int*, int, int, int, int,
-                                              int, long, const float*, int,
+                                              int, long, const float*, int, int,
                                               hipStream_t);
 template void launch_causal_conv_state<__hip_bfloat16>(
     __hip_bfloat16*, const __hip_bfloat16*, const float*, __hip_bfloat16*,
     const int*, const int*, const int*, int, int, int, int, int, long,
-    const float*, int, hipStream_t);
+    const float*, int, int, hipStream_t);
 template void launch_conv_state_update<float>(float*, const float*, const int*,
                                               const int*, const int*, int, int, int,
                                               long, hipStream_t);

@@ -291,7 +291,7 @@ __global__ void clamped_glu_kernel(T* __restrict__ out, const T* __restrict__ gu
 // instruction j is element 8 s + j on both sides.
 // ---------------------------------------------------------------------------
 typedef __attribute__((ext_vector_type(4))) float f32x4_t;
-constexpr int RL_WAVES = 8;
+constexpr int RL_WAVES = 16;
 
 template <typename T>
 __global__ __launch_bounds__(RL_WAVES * 64) void router_logits_kernel(
@@ -305,14 +305,25 @@ __global__ __launch_bounds__(RL_WAVES * 64) void router_logits_kernel(
   const T* hp = h + (long)min(row, rows - 1) * h_st + s * 8;
   const float* wp = w + (long)min(e, experts - 1) * width + s * 8;
   f32x4_t acc{};
-#pragma unroll 2
-  for (int c = wave * 32; c < width; c += RL_WAVES * 32) {
-    float a[8], b[8];
-    ld8<T>(hp + c, a);
-    ld8<float>(wp + c, b);
+  // FLY pieces are loaded before the first of them is used
+  constexpr int FLY = 4;
+  for (int c0 = wave * 32; c0 < width; c0 += FLY * RL_WAVES * 32) {
+    float a[FLY][8], b[FLY][8];
 #pragma unroll
-    for (int j = 0; j < 8; ++j)
-      acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[j], b[j], acc, 0, 0, 0);
+    for (int f = 0; f < FLY; ++f) {
+      const int c = c0 + f * RL_WAVES * 32;
+#pragma unroll
+      for (int j = 0; j < 8; ++j) a[f][j] = b[f][j] = 0.f;
+      if (c < width) {               // uniform over the wave
+        ld8<T>(hp + c, a[f]);
+        ld8<float>(wp + c, b[f]);
+      }
+    }
+#pragma unroll
+    for (int f = 0; f < FLY; ++f)
+#pragma unroll
+      for (int j = 0; j < 8; ++j)
+        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[f][j], b[f][j], acc, 0, 0, 0);
   }
   // lane holds out[4 * (lane / 16) + r][lane % 16]
 #pragma unroll
@@ -396,8 +407,11 @@ void launch_wide_norm(T* q_out, const T* proj, long st, const float* bias, const
   const bool vec = nq % 8 == 0 && nk % 8 == 0 && nv % 8 == 0 && st % 8 == 0 && per <= 8 &&
                    al(proj, 16) && al(bias, 16) && al(qw, 16) && al(kw, 16) && al(v_first, 16) &&
                    al(q_out, 16) && al(k_cache, 16) && al(v_cache, 16);
+  static const int wr = getenv("WN_ROWS") ? atoi(getenv("WN_ROWS")) : 4;
 #define WIDE_LAUNCH(NV)                                                                \
-  if (rows < 2048) wide_norm_vec_kernel<T, NV, 1><<<rows, 256, 0, s>>>(p);             \
+  if (rows < 2048 || wr == 1) wide_norm_vec_kernel<T, NV, 1><<<rows, 256, 0, s>>>(p);             \
+  else if (wr == 2) wide_norm_vec_kernel<T, NV, 2><<<(rows + 1) / 2, 256, 0, s>>>(p);             \
+  else if (wr == 8) wide_norm_vec_kernel<T, NV, 8><<<(rows + 7) / 8, 256, 0, s>>>(p);             \
   else wide_norm_vec_kernel<T, NV, 4><<<(rows + 3) / 4, 256, 0, s>>>(p)
   if (!vec) wide_norm_kernel<T><<<rows, 256, 0, s>>>(p);
   else if (per == 1) { WIDE_LAUNCH(1); }

@@ -126,7 +126,7 @@ class ShortConv(nn.Module):
     def forward(self, h: torch.Tensor, state: torch.Tensor, meta: AttnMetadata) -> torch.Tensor:
         return ops.causal_conv_state(
             h, self.weight, state, meta.seq_start_loc, meta.seq_lens,
-            meta.state_slots, add_input=True)
+            meta.state_slots, add_input=True, has_portions=meta.num_prefill_tokens > 0)
 
 
 def scaled_rotary_frequencies(base: float, dims: int,
@@ -561,7 +561,7 @@ class SSDMixer(_Mixer):
         xbc = ops.causal_conv_state(
             proj[:, inner:inner + self.conv_ch], self.conv_weight, conv_state,
             meta.seq_start_loc, meta.seq_lens, meta.state_slots, add_input=False,
-            bias=self.conv_bias, act="silu")
+            bias=self.conv_bias, act="silu", has_portions=meta.num_prefill_tokens > 0)
         y = ops.ssd_scan(xbc, proj[:, inner + self.conv_ch:], self.dt_bias, self.a_log,
                          self.d_skip, ssm_state, meta.seq_start_loc, meta.seq_lens,
                          meta.state_slots, self.heads, self.vdim, self.nstate, self.groups)
@@ -626,7 +626,8 @@ class RGLRUMixer(_Mixer):
         yb = ops.gelu_tanh(proj[:, :w])
         u = ops.causal_conv_state(
             proj[:, w:], self.conv_weight, conv_state, meta.seq_start_loc,
-            meta.seq_lens, meta.state_slots, add_input=False, bias=self.conv_bias)
+            meta.seq_lens, meta.state_slots, add_input=False, bias=self.conv_bias,
+            has_portions=meta.num_prefill_tokens > 0)
         ub = u.view(t, nb, w // nb).transpose(0, 1)              # [blocks, T, bw]
         r_pre = torch.bmm(ub, self.ra_t).transpose(0, 1).reshape(t, w)
         i_pre = torch.bmm(ub, self.ri_t).transpose(0, 1).reshape(t, w)
@@ -1587,7 +1588,8 @@ class DeltaMixer(_Mixer):
         e = c + nh * dv
         qkv = ops.causal_conv_state(
             proj[:, :c], self.conv_weight, conv_state, meta.seq_start_loc, meta.seq_lens,
-            meta.state_slots, add_input=False, act="silu")
+            meta.state_slots, add_input=False, act="silu",
+            has_portions=meta.num_prefill_tokens > 0)
         return ops.delta_gated(
             qkv[:, :a].view(t, ng, d), qkv[:, a:2 * a].view(t, ng, d),
             qkv[:, 2 * a:].view(t, nh, dv), proj[:, e:e + nh], proj[:, e + nh:e + 2 * nh],

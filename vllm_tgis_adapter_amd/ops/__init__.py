@@ -608,18 +608,19 @@ def softcap(logits: torch.Tensor, cap: float) -> torch.Tensor:
 
 def causal_conv_state(h, weight, state, seq_start_loc, seq_lens, state_slots,
                       add_input: bool = True, bias: torch.Tensor | None = None,
-                      act: str | None = None) -> torch.Tensor:
+                      act: str | None = None, has_portions: bool = True) -> torch.Tensor:
     """Depthwise causal convolution over each sequence's new rows with the
     last taps-1 inputs carried in ``state[slot]`` (advanced in place).  ``h``
     may be a column slice of a wider matrix; ``bias`` [W] f32 and ``act``
-    ("silu") are applied to the result."""
+    ("silu") are applied to the result.  ``has_portions`` False promises that
+    every sequence brings one row."""
     if act not in (None, "silu"):
         raise ValueError(f"unknown activation {act!r}")
     if h.numel() and _native_seq(h):
         out = torch.empty(h.shape, dtype=h.dtype, device=h.device)
         _S.causal_conv_state(out, h, weight, state, seq_start_loc, seq_lens,
                              state_slots, bool(add_input), bias,
-                             1 if act == "silu" else 0)
+                             1 if act == "silu" else 0, bool(has_portions))
         return out
     return reference.causal_conv_state(
         h, weight, state, seq_start_loc.cpu(), seq_lens.cpu(), state_slots.cpu(),
