@@ -53,10 +53,11 @@ DEVINLINE bf16x8_t load_kv8<unsigned char>(const unsigned char* p) {
 // tokens.  PX_POOL: one pooled key and value per block of `pool` positions that
 // ends at or before seq_len - 1 - window; pooled block b is kept in the cache
 // block that holds its last token (per_block places each).
-// CAP (capped variant, on top of WS): scores become softcap tanh(score / softcap)
-// (softcap 0: as they are).  Up to kFixedMaxCap the cap bounds them well enough
-// that the exponentials are taken without a running maximum.
+// CAP (capped variants, on top of WS): scores become softcap tanh(score / softcap)
+// (softcap 0: as they are).  CAP_FIXED: up to kFixedMaxCap the cap bounds them well
+// enough that the exponentials are taken without a running maximum.
 enum { PX_NONE = 0, PX_KEEP = 1, PX_POOL = 2 };
+enum { CAP_NONE = 0, CAP_RUN = 1, CAP_FIXED = 2 };
 constexpr float kFixedMaxCap = 60.f;
 struct SpanKeys {
   int keep, pool, per_block;
@@ -65,7 +66,7 @@ struct SpanKeys {
 };
 
 template <int HEAD_DIM, typename CT, bool WS, bool CH = false, int PX = PX_NONE,
-          bool CAP = false>
+          int CAP = CAP_NONE>
 __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
     float* __restrict__ part_acc,   // [nseq, nheads, P, HEAD_DIM] f32
     float* __restrict__ part_ml,    // [nseq, nheads, P, 2] f32 (m, l)
@@ -85,7 +86,7 @@ __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
     const int v_heads = 0,
     const SpanKeys sp = SpanKeys{},
     const float softcap = 0.f) {
-  static_assert(!CAP || (WS && !CH && PX == PX_NONE),
+  static_assert(CAP == CAP_NONE || (WS && !CH && PX == PX_NONE),
                 "the capped variant builds on the window variant");
   static_assert(!CH || WS, "the chunk variant builds on the window variant");
   static_assert(PX == PX_NONE || (WS && !CH), "prefixes build on the window variant");
@@ -147,10 +148,9 @@ __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
 #pragma unroll
   for (int dt = 0; dt < DT; ++dt) acc_o[dt] = f32x16_t{};
 
-  const bool capped = CAP && softcap > 0.f;
-  const bool fixed_max = capped && softcap <= kFixedMaxCap;
+  const bool capped = CAP == CAP_FIXED || (CAP == CAP_RUN && softcap > 0.f);
   const float cap_in = capped ? scale / softcap : 0.f;
-  if (fixed_max) m_state = 0.f;
+  if (CAP == CAP_FIXED) m_state = 0.f;
 
   constexpr int VPASS = KVT * HEAD_DIM / 8 / 64;  // V staging passes per wave
 
@@ -224,7 +224,7 @@ __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
     // ---- online softmax (stats per q col = this lane's col) --------------
     float s_val[16];
     float local_max = -FLT_MAX;
-    if (CAP && capped) {
+    if (CAP != CAP_NONE && capped) {
       // the tile's largest argument decides whether the polynomial alone will do
       float big = 0.f;
 #pragma unroll
@@ -243,13 +243,13 @@ __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
 #pragma unroll
     for (int r = 0; r < 16; ++r) {
       const int kv_pos = kv_base + (r & 3) + 8 * (r >> 2) + 4 * half;
-      float sv = acc_s[r] * (CAP && capped ? softcap : scale);
+      float sv = acc_s[r] * (CAP != CAP_NONE && capped ? softcap : scale);
       if (kv_pos >= limit || (WS && !prefix && kv_pos < first_pos)) sv = -FLT_MAX;
       s_val[r] = sv;
       local_max = fmaxf(local_max, sv);
     }
     float rescale = 1.f;
-    if (!(CAP && fixed_max)) {
+    if constexpr (CAP != CAP_FIXED) {
       const float tile_max = fmaxf(local_max, __shfl_xor(local_max, 32, 64));
       const float m_new = fmaxf(m_state, tile_max);
       rescale = __expf(m_state - m_new);
@@ -266,7 +266,7 @@ __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
     l_state = l_state * rescale + local_sum + __shfl_xor(local_sum, 32, 64);
 
     // rescale factors redistributed to the PV accumulator's q rows
-    if (!(CAP && fixed_max)) {
+    if constexpr (CAP != CAP_FIXED) {
       float f_reg[16];
 #pragma unroll
       for (int r = 0; r < 16; ++r) {
@@ -588,7 +588,7 @@ void launch_paged_decode_mfma_span(__hip_bfloat16* out, float* part_acc, float* 
 }
 
 // soft-capped scores, window, sinks per head or none (bf16 cache)
-template <int HD>
+template <int HD, int CAP>
 static void launch_decode_capped(__hip_bfloat16* out, float* part_acc, float* part_ml,
                                  const __hip_bfloat16* q, const __hip_bfloat16* kc,
                                  const __hip_bfloat16* vc, const int* bt, const int* sl,
@@ -597,7 +597,7 @@ static void launch_decode_capped(__hip_bfloat16* out, float* part_acc, float* pa
                                  float softcap, hipStream_t stream) {
   const dim3 grid(nseq, kvh, npart), mgrid(nseq, nheads);
   hipLaunchKernelGGL(
-      (paged_decode_mfma_kernel<HD, __hip_bfloat16, true, false, PX_NONE, true>), grid,
+      (paged_decode_mfma_kernel<HD, __hip_bfloat16, true, false, PX_NONE, CAP>), grid,
       dim3(256), 0, stream, part_acc, part_ml, q, kc, vc, bt, sl, scale, nheads, kvh,
       nheads / kvh, block_size, max_blocks, window, 0, 0, SpanKeys{}, softcap);
   hipLaunchKernelGGL((decode_merge_kernel<HD>), mgrid, dim3(HD), 0, stream, out, part_acc,
@@ -611,13 +611,14 @@ void launch_paged_decode_mfma_capped(__hip_bfloat16* out, float* part_acc, float
                                      float scale, int nseq, int nheads, int kvh, int head_dim,
                                      int block_size, int max_blocks, int npart, int window,
                                      const float* sinks, float softcap, hipStream_t stream) {
-  if (head_dim == 64)
-    launch_decode_capped<64>(out, part_acc, part_ml, q, kc, vc, bt, sl, scale, nseq, nheads,
-                             kvh, block_size, max_blocks, npart, window, sinks, softcap, stream);
-  else if (head_dim == 128)
-    launch_decode_capped<128>(out, part_acc, part_ml, q, kc, vc, bt, sl, scale, nseq, nheads,
-                              kvh, block_size, max_blocks, npart, window, sinks, softcap,
-                              stream);
-  else
-    abort();
+  const bool fixed = softcap > 0.f && softcap <= kFixedMaxCap;
+  auto go = [&](auto launch) {
+    launch(out, part_acc, part_ml, q, kc, vc, bt, sl, scale, nseq, nheads, kvh, block_size,
+           max_blocks, npart, window, sinks, softcap, stream);
+  };
+  if (head_dim == 64 && fixed) go(launch_decode_capped<64, CAP_FIXED>);
+  else if (head_dim == 64) go(launch_decode_capped<64, CAP_RUN>);
+  else if (head_dim == 128 && fixed) go(launch_decode_capped<128, CAP_FIXED>);
+  else if (head_dim == 128) go(launch_decode_capped<128, CAP_RUN>);
+  else abort();
 }

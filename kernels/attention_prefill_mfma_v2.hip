@@ -74,12 +74,13 @@ __device__ inline float cross_half_sum(float v) {
 // cache block that holds its last token (per_block places each).  back (cos,
 // sin per query row and pair): the output's dims m and m + HEAD_DIM/2 are turned
 // back by the row's angles before they are rounded.
-// CAP (capped variant, on top of WS): scores become softcap tanh(score / softcap)
-// before the softmax (softcap 0: as they are), and the sink is one per head.  A
-// cap also bounds the scores: up to kFixedMaxCap the exponentials are taken as
-// they are, without a running maximum or a rescale (e^60 and its inverse times
-// any count of keys stay inside f32 and bf16).
+// CAP (capped variants, on top of WS): the sink is one per head, and scores
+// become softcap tanh(score / softcap) before the softmax (softcap 0: as they are).
+// CAP_FIXED: a cap also bounds the scores; up to kFixedMaxCap the exponentials are
+// taken as they are, without a running maximum or a rescale (e^60 and its inverse
+// times any count of keys stay inside f32 and bf16).
 enum { PX_NONE = 0, PX_KEEP = 1, PX_POOL = 2 };
+enum { CAP_NONE = 0, CAP_RUN = 1, CAP_FIXED = 2 };
 constexpr float kFixedMaxCap = 60.f;
 struct Capped {
   float softcap;
@@ -92,8 +93,47 @@ struct SpanTiles {
   const float2* back;
 };
 
+// raw products -> softcap tanh(product scale / softcap) in the log2 domain.  The
+// tile's largest argument x decides between a short odd polynomial (its first
+// dropped term is 5e-8 of the result), a long one (tanh_small's), and
+// 1 - 2 / (1 + e^2x), whose error is absolute, 1e-7 of the cap.
+DEVINLINE void cap_scores(f32x16_t* s, float scale, float softcap) {
+  const float in = scale / softcap, out = softcap * LOG2E;
+  float big = 0.f;
+#pragma unroll
+  for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+    for (int r = 0; r < 16; ++r) big = fmaxf(big, fabsf(s[kb][r]));
+  big *= in;
+  if (__all(big < 0.1f)) {
+    const float c0 = out * in, c1 = c0 * in * in * -0.3333333333f;
+    const float c2 = c0 * in * in * in * in * 0.1333333333f;
+#pragma unroll
+    for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+      for (int r = 0; r < 16; ++r) {
+        const float z = s[kb][r] * s[kb][r];
+        s[kb][r] *= __builtin_fmaf(z, __builtin_fmaf(z, c2, c1), c0);
+      }
+  } else if (__all(big < kTanhSmall)) {
+#pragma unroll
+    for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+      for (int r = 0; r < 16; ++r) s[kb][r] = out * tanh_small(s[kb][r] * in);
+  } else {
+    const float in2 = 2.8853900818f * in, out2 = -2.f * out;
+#pragma unroll
+    for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+      for (int r = 0; r < 16; ++r) {
+        const float e = __builtin_amdgcn_exp2f(s[kb][r] * in2);
+        s[kb][r] = __builtin_fmaf(out2, __builtin_amdgcn_rcpf(1.f + e), out);
+      }
+  }
+}
+
 template <int HEAD_DIM, typename CT, int NW, bool WS, bool CH = false,
-          typename OT = __hip_bfloat16, int PX = PX_NONE, bool CAP = false>
+          typename OT = __hip_bfloat16, int PX = PX_NONE, int CAP = CAP_NONE>
 __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v2_kernel(
     OT* __restrict__ out,                        // [total_q, nheads, HD]
     const __hip_bfloat16* __restrict__ q,        // [total_q, nheads, HD]
@@ -114,7 +154,7 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
     const int v_heads = 0,
     const SpanTiles sp = SpanTiles{},
     const Capped cap = Capped{}) {
-  static_assert(!CAP || (WS && !CH && PX == PX_NONE),
+  static_assert(CAP == CAP_NONE || (WS && !CH && PX == PX_NONE),
                 "the capped variant builds on the window variant");
   static_assert(HEAD_DIM == 128, "v2 is specialised for HD=128");
   static_assert(PX == PX_NONE || (WS && !CH), "prefixes build on the window variant");
@@ -265,11 +305,9 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
   stage_write(0);
 
   // fold softmax scale into exp2 domain; capped scores are already there
-  const bool capped = CAP && cap.softcap > 0.f;
-  const bool fixed_max = capped && cap.softcap <= kFixedMaxCap;
+  const bool capped = CAP == CAP_FIXED || (CAP == CAP_RUN && cap.softcap > 0.f);
   const float sc2 = capped ? 1.f : scale * LOG2E;
-  const float cap_in = capped ? scale / cap.softcap : 0.f, cap_out = cap.softcap * LOG2E;
-  if (fixed_max) m2_state = 0.f;
+  if (CAP == CAP_FIXED) m2_state = 0.f;
 
   for (int it = 0; it < num_tiles; ++it) {
     const int kv_base = tile_pos(it);
@@ -310,28 +348,7 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
     const bool more = it + 1 < num_tiles;
     if (more) stage_load(tile_pos(it + 1), PX != PX_NONE && it + 1 < pre_tiles);
 
-    if (CAP && capped && wave_active) {
-      // the tile's largest argument decides whether the polynomial alone will do
-      float big = 0.f;
-#pragma unroll
-      for (int kb = 0; kb < 2; ++kb)
-#pragma unroll
-        for (int r = 0; r < 16; ++r) {
-          acc_s[kb][r] *= cap_in;
-          big = fmaxf(big, fabsf(acc_s[kb][r]));
-        }
-      if (__all(big < kTanhSmall)) {
-#pragma unroll
-        for (int kb = 0; kb < 2; ++kb)
-#pragma unroll
-          for (int r = 0; r < 16; ++r) acc_s[kb][r] = cap_out * tanh_small(acc_s[kb][r]);
-      } else {
-#pragma unroll
-        for (int kb = 0; kb < 2; ++kb)
-#pragma unroll
-          for (int r = 0; r < 16; ++r) acc_s[kb][r] = cap_out * tanh_f32(acc_s[kb][r]);
-      }
-    }
+    if (CAP != CAP_NONE && capped && wave_active) cap_scores(acc_s, scale, cap.softcap);
 
     if (wave_active) {
       // ---- online softmax; the running max m2_state lives in the RAW
@@ -349,11 +366,13 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
                          kv_base >= (wave_q_pos_min + 31) / chunk * chunk));
       float local_max = -FLT_MAX;
       if (full_tile) {
+        if constexpr (CAP != CAP_FIXED) {
 #pragma unroll
-        for (int kb = 0; kb < 2; ++kb)
+          for (int kb = 0; kb < 2; ++kb)
 #pragma unroll
-          for (int r = 0; r < 16; ++r)
-            local_max = fmaxf(local_max, acc_s[kb][r]);
+            for (int r = 0; r < 16; ++r)
+              local_max = fmaxf(local_max, acc_s[kb][r]);
+        }
       } else {
 #pragma unroll
         for (int kb = 0; kb < 2; ++kb)
@@ -370,16 +389,16 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
                              (CH && kv_pos < q_lo);
             if (!q_valid || hidden) v = -FLT_MAX;
             acc_s[kb][r] = v;
-            local_max = fmaxf(local_max, v);
+            if constexpr (CAP != CAP_FIXED) local_max = fmaxf(local_max, v);
           }
       }
-      const float tile_max = CAP && fixed_max ? 0.f : cross_half_max(local_max);
+      const float tile_max = CAP == CAP_FIXED ? 0.f : cross_half_max(local_max);
 
       // defer-max (T13): skip the O/l rescale while the running max holds.
       // The decision is wave-uniform and taken BEFORE any of this tile's P
       // enters O or l, so everything at the old scale rescales exactly once.
       const float thr = DEFER_MAX_THR / sc2;
-      const bool need_rescale = !(CAP && fixed_max) && !__all(
+      const bool need_rescale = CAP != CAP_FIXED && !__all(
           m2_state != -FLT_MAX && tile_max <= m2_state + thr);
       float m2_new = m2_state;
       if (need_rescale) {
@@ -409,7 +428,7 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
 #pragma unroll
         for (int r = 0; r < 16; ++r) {
           const float v = __builtin_amdgcn_exp2f(
-              __builtin_fmaf(acc_s[kb][r], sc2, bias));
+              CAP == CAP_FIXED ? acc_s[kb][r] : __builtin_fmaf(acc_s[kb][r], sc2, bias));
           p[kb * 16 + r] = v;
           local_sum += v;
         }
@@ -490,7 +509,7 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
   // column and carries ALL 32 q rows for it; q-row validity is per row
   // (q_local check below), not per lane.
   float l_fin = l_state, o_scale = 1.f;
-  const float sink_h = CAP && cap.sinks != nullptr ? cap.sinks[head] : sink;
+  const float sink_h = CAP != CAP_NONE && cap.sinks != nullptr ? cap.sinks[head] : sink;
   if (WS && has_sink) {
     // the sink joins the denominator; both terms relative to the larger of
     // the running max and the sink (log2 domain)
@@ -645,17 +664,31 @@ void launch_paged_prefill_mfma_v2_span(
 }
 
 // soft-capped scores, window, sinks per head or none (bf16 cache, HD = 128)
+template <int CAP>
+static void launch_prefill_capped(
+    __hip_bfloat16* out, const __hip_bfloat16* q, const __hip_bfloat16* kc,
+    const __hip_bfloat16* vc, const int* bt, const int* qsl, const int* sl, float scale,
+    int nseq, int nheads, int kvh, int block_size, int max_blocks, int max_query_len,
+    int window, const Capped& cap, hipStream_t stream) {
+  const dim3 grid(nseq, nheads, (max_query_len + 255) / 256);
+  hipLaunchKernelGGL((paged_prefill_mfma_v2_kernel<128, __hip_bfloat16, 8, true, false,
+                                                   __hip_bfloat16, PX_NONE, CAP>),
+                     grid, dim3(512), 0, stream, out, q, kc, vc, bt, qsl, sl, scale, nheads,
+                     kvh, block_size, max_blocks, window, cap.sinks != nullptr ? 1 : 0, 0.f, 0,
+                     0, SpanTiles{}, cap);
+}
+
 void launch_paged_prefill_mfma_v2_capped(
     __hip_bfloat16* out, const __hip_bfloat16* q, const __hip_bfloat16* kc,
     const __hip_bfloat16* vc, const int* bt, const int* qsl, const int* sl, float scale,
     int nseq, int nheads, int kvh, int block_size, int max_blocks, int max_query_len,
     int window, const float* sinks, float softcap, hipStream_t stream) {
-  const dim3 grid(nseq, nheads, (max_query_len + 255) / 256);
   Capped cap;
   cap.softcap = softcap; cap.sinks = sinks;
-  hipLaunchKernelGGL((paged_prefill_mfma_v2_kernel<128, __hip_bfloat16, 8, true, false,
-                                                   __hip_bfloat16, PX_NONE, true>),
-                     grid, dim3(512), 0, stream, out, q, kc, vc, bt, qsl, sl, scale, nheads,
-                     kvh, block_size, max_blocks, window, sinks != nullptr ? 1 : 0, 0.f, 0, 0,
-                     SpanTiles{}, cap);
+  if (softcap > 0.f && softcap <= kFixedMaxCap)
+    launch_prefill_capped<CAP_FIXED>(out, q, kc, vc, bt, qsl, sl, scale, nseq, nheads, kvh,
+                                     block_size, max_blocks, max_query_len, window, cap, stream);
+  else
+    launch_prefill_capped<CAP_RUN>(out, q, kc, vc, bt, qsl, sl, scale, nseq, nheads, kvh,
+                                   block_size, max_blocks, max_query_len, window, cap, stream);
 }

@@ -29,6 +29,7 @@ template <typename T>
 void launch_moe_combine(T*, const T*, const int*, const int*, const float*, int,
                         int, int, int, hipStream_t);
 int moe_sort_max_experts();
+int moe_sort_small_pairs();
 template <typename T>
 void launch_moe_sort(T*, int*, int*, int*, const T*, long, const int*, int, int,
                      int, int, const float*, hipStream_t);
@@ -290,18 +291,22 @@ void moe_combine(torch::Tensor out, torch::Tensor ye, torch::Tensor pos,
 }
 
 void moe_sort(torch::Tensor xs, torch::Tensor pos, torch::Tensor seg,
-              torch::Tensor scratch, torch::Tensor h, torch::Tensor ids,
+              c10::optional<torch::Tensor> scratch, torch::Tensor h, torch::Tensor ids,
               int64_t num_real, c10::optional<torch::Tensor> row_scale) {
   check_i32(ids, "ids");
   check_i32(pos, "pos");
   check_i32(seg, "seg");
-  check_i32(scratch, "scratch");
   TORCH_CHECK(h.is_cuda() && h.dim() == 2 && h.stride(1) == 1 && ids.dim() == 2 &&
               ids.size(0) == h.size(0));
   const int tokens = h.size(0), width = h.size(1), top = ids.size(1);
   TORCH_CHECK(num_real >= 1 && num_real <= moe_sort_max_experts(), "number of experts");
-  TORCH_CHECK(pos.sizes() == ids.sizes() && seg.numel() == num_real + 1 &&
-              scratch.numel() == 2 * num_real);
+  TORCH_CHECK(pos.sizes() == ids.sizes() && seg.numel() == num_real + 1);
+  if (scratch.has_value()) {
+    check_i32(scratch.value(), "scratch");
+    TORCH_CHECK(scratch.value().numel() == 2 * num_real);
+  } else {
+    TORCH_CHECK(ids.numel() <= moe_sort_small_pairs(), "scratch missing");
+  }
   TORCH_CHECK(xs.is_contiguous() && xs.dim() == 2 && xs.size(0) == (long)tokens * top &&
               xs.size(1) == width && xs.scalar_type() == h.scalar_type());
   if (row_scale.has_value()) {
@@ -311,7 +316,7 @@ void moe_sort(torch::Tensor xs, torch::Tensor pos, torch::Tensor seg,
   if (tokens == 0) return;
   DISPATCH_F32_BF16(h.scalar_type(), {
     launch_moe_sort<scalar_t>(ptr<scalar_t>(xs), ptr<int>(pos), ptr<int>(seg),
-                              ptr<int>(scratch), ptr<scalar_t>(h), (long)h.stride(0),
+                              optr<int>(scratch), ptr<scalar_t>(h), (long)h.stride(0),
                               ptr<int>(ids), tokens, top, (int)num_real, width,
                               optr<float>(row_scale), stream());
   });
@@ -368,6 +373,7 @@ void register_par_ops(pybind11::module& m) {
   m.def("moe_route_sigmoid", &moe_route_sigmoid);
   m.def("moe_combine", &moe_combine);
   m.def("moe_sort", &moe_sort);
+  m.def("moe_sort_small_pairs", &moe_sort_small_pairs);
   m.def("moe_gemm", &moe_gemm);
   m.def("moe_gemm_clamped", &moe_gemm_clamped);
 }

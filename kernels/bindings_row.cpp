@@ -16,8 +16,11 @@ void launch_wide_norm(T*, const T*, long, const float*, const float*, const floa
                       float, T*, T*, const long*, int, int, int, int, float, hipStream_t);
 template <typename T>
 void launch_clamped_glu(T*, const T*, float, const float*, int, long, hipStream_t);
-template <typename T>
-void launch_router_logits(float*, const T*, long, const float*, int, int, int, hipStream_t);
+template <typename T, typename W>
+void launch_router_logits(float*, const T*, long, const W*, int, int, int, hipStream_t);
+template <typename T, typename W>
+void launch_route_experts(float*, int*, float*, const T*, long, const W*, const float*, int,
+                          int, int, int, int, int, int, float, hipStream_t);
 template <typename T>
 void launch_scale_logits(float*, const T*, float, long, hipStream_t);
 template <typename T>
@@ -331,16 +334,57 @@ void clamped_glu(torch::Tensor out, torch::Tensor gu, double limit, OptTensor co
   });
 }
 
+// router weights are f32 or bf16 whatever the rows are
+template <typename F>
+void with_router(const torch::Tensor& w, F launch) {
+  if (w.scalar_type() == at::ScalarType::Float) launch(ptr<const float>(w));
+  else launch(ptr<const __hip_bfloat16>(w));
+}
+
 void router_logits(torch::Tensor out, torch::Tensor h, torch::Tensor w) {
   TORCH_CHECK(h.is_cuda() && h.dim() == 2 && h.stride(1) == 1 && w.dim() == 2 &&
               w.size(1) == h.size(1), "rows and router width");
-  check_f32(w, -1, "router");
+  TORCH_CHECK(w.is_cuda() && w.is_contiguous() &&
+              (w.scalar_type() == at::ScalarType::Float ||
+               w.scalar_type() == at::ScalarType::BFloat16), "router: f32 or bf16 weights");
   const int rows = h.size(0), width = h.size(1), experts = w.size(0);
   check_f32(out, (long)rows * experts, "out");
   if (rows == 0 || experts == 0) return;
   DISPATCH_F32_BF16(h.scalar_type(), {
-    launch_router_logits<scalar_t>(ptr<float>(out), ptr<scalar_t>(h), (long)h.stride(0),
-                                   ptr<float>(w), rows, experts, width, stream());
+    with_router(w, [&](auto* wp) {
+      launch_router_logits(ptr<float>(out), ptr<scalar_t>(h), (long)h.stride(0), wp, rows,
+                           experts, width, stream());
+    });
+  });
+}
+
+void route_experts(torch::Tensor dense, torch::Tensor ids, torch::Tensor wts, torch::Tensor h,
+                   torch::Tensor w, OptTensor correction, int64_t groups, int64_t keep,
+                   bool renormalise, double scale) {
+  TORCH_CHECK(h.is_cuda() && h.dim() == 2 && h.stride(1) == 1 && w.dim() == 2 &&
+              w.size(1) == h.size(1), "rows and router width");
+  TORCH_CHECK(w.is_cuda() && w.is_contiguous() &&
+              (w.scalar_type() == at::ScalarType::Float ||
+               w.scalar_type() == at::ScalarType::BFloat16), "router: f32 or bf16 weights");
+  const int rows = h.size(0), width = h.size(1), experts = w.size(0);
+  TORCH_CHECK(experts >= 1 && experts <= 64 && width % 32 == 0 && h.stride(0) % 8 == 0 &&
+              aligned16(h) && aligned16(w), "shape off the fused router");
+  check_f32(correction, experts, "correction");
+  check_f32(dense, (long)rows * experts, "dense");
+  check_f32(wts, -1, "weights");
+  check_type(ids, at::ScalarType::Int, "ids");
+  TORCH_CHECK(ids.dim() == 2 && ids.size(0) == rows && wts.sizes() == ids.sizes());
+  const int top = ids.size(1);
+  TORCH_CHECK(groups >= 1 && experts % groups == 0 && keep >= 1 && keep <= groups && top >= 1 &&
+              top <= keep * (experts / groups), "expert groups");
+  if (rows == 0) return;
+  DISPATCH_F32_BF16(h.scalar_type(), {
+    with_router(w, [&](auto* wp) {
+      launch_route_experts(ptr<float>(dense), ptr<int>(ids), ptr<float>(wts), ptr<scalar_t>(h),
+                           (long)h.stride(0), wp, optr<float>(correction), rows, experts, width,
+                           top, (int)groups, (int)keep, renormalise ? 1 : 0, (float)scale,
+                           stream());
+    });
   });
 }
 
@@ -364,5 +408,6 @@ void register_row_ops(pybind11::module& m) {
   m.def("delta_gated", &delta_gated);
   m.def("clamped_glu", &clamped_glu);
   m.def("router_logits", &router_logits);
+  m.def("route_experts", &route_experts);
   m.def("scale_logits", &scale_logits);
 }

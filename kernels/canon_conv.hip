@@ -17,7 +17,7 @@
 //
 // Two kernels.  The row-walking one: a thread owns 8 channels and walks up to
 // CW_ROWS consecutive rows with their weights and the last taps-1 inputs in
-// registers, so every input is read once, the next row's while this one is
+// registers, so every input is read once, the next rows' while these are
 // computed; where every sequence of the step brings a single row it also
 // advances the state itself (nobody else reads that sequence's rows).  The other
 // takes any tap count and width: one thread per (row, 4 channels) — or one channel when the width is not a
@@ -177,8 +177,15 @@ __global__ __launch_bounds__(256) void causal_conv_walk_kernel(
     const float* __restrict__ bias, int act, int single_rows) {
   const int c = (blockIdx.y * 256 + threadIdx.x) * 8;
   if (c >= width) return;
+  constexpr int AHEAD = ROWS < 4 ? ROWS : 4;   // rows loaded ahead of the ones computed
   const int r0 = blockIdx.x * ROWS, r1 = min(r0 + ROWS, rows);
-  Vec8<T> nxt = Vec8<T>::load(h + (long)r0 * in_st + c);
+  Vec8<T> nxt[AHEAD];
+  auto fetch = [&](int row) {
+#pragma unroll
+    for (int u = 0; u < AHEAD; ++u)
+      if (row + u < r1) nxt[u] = Vec8<T>::load(h + (long)(row + u) * in_st + c);
+  };
+  fetch(r0);
   float wv[TAPS][8], bv[8], hist[TAPS][8];   // hist[TAPS - 1]: the current row
 #pragma unroll
   for (int k = 0; k < 8; ++k) {
@@ -188,13 +195,19 @@ __global__ __launch_bounds__(256) void causal_conv_walk_kernel(
   }
   int s = find_seq(loc, nseq, r0);
   bool fresh = true;             // the history registers do not hold this sequence's rows
-  for (int row = r0; row < r1; ++row) {
+  for (int g0 = r0; g0 < r1; g0 += AHEAD) {
+  Vec8<T> now[AHEAD];
+#pragma unroll
+  for (int u = 0; u < AHEAD; ++u) now[u] = nxt[u];
+  if (g0 + AHEAD < r1) fetch(g0 + AHEAD);
+#pragma unroll
+  for (int u = 0; u < AHEAD; ++u) {
+    const int row = g0 + u;
+    if (row >= r1) break;
     while (s + 1 < nseq && row >= loc[s + 1]) { ++s; fresh = true; }
     const int slot = slots[s], first = loc[s];
     const int start = seq_lens[s] - (loc[s + 1] - first);
     const int p = start + row - first;
-    const Vec8<T> cur = nxt;
-    if (row + 1 < r1) nxt = Vec8<T>::load(h + (long)(row + 1) * in_st + c);
     if (fresh) {
 #pragma unroll
       for (int j = 0; j < TAPS - 1; ++j) {
@@ -209,7 +222,7 @@ __global__ __launch_bounds__(256) void causal_conv_walk_kernel(
       }
       fresh = false;
     }
-    cur.unpack(hist[TAPS - 1]);
+    now[u].unpack(hist[TAPS - 1]);
     float acc[8];
 #pragma unroll
     for (int k = 0; k < 8; ++k) {
@@ -229,6 +242,7 @@ __global__ __launch_bounds__(256) void causal_conv_walk_kernel(
     for (int j = 0; j + 1 < TAPS; ++j)
 #pragma unroll
       for (int k = 0; k < 8; ++k) hist[j][k] = hist[j + 1][k];
+  }
   }
 }
 

@@ -18,7 +18,7 @@
 // All memory-bound; norm statistics, angles, sigmoids, router arithmetic and
 // the stream are f32 whatever the storage type.
 
-#include "common.h"
+#include "moe_route.h"
 
 namespace {
 
@@ -340,147 +340,14 @@ __global__ void relu2_kernel(T* __restrict__ out, const T* __restrict__ x,
   }
 }
 
-// One wave per token; lane l owns experts l, l + 64, ... (at most RT_MAX each).
-constexpr int RT_MAX = 8;
-
+// one wave per token
 __global__ __launch_bounds__(256) void moe_route_kernel(
     float* __restrict__ dense, float* __restrict__ ident, int* __restrict__ ids,
-    float* __restrict__ wts, const float* __restrict__ logits,
-    const float* __restrict__ correction, int tokens, int n, int num_real,
-    int top, int sigmoid, int groups, int keep, int renorm, float scale) {
-  // sigmoid: scores are sigmoid(logit) instead of the softmax, the correction is
-  // optional and there is no identity output.  groups > 1: only the experts of
-  // the `keep` groups of neighbours with the largest sum of their two best choice
-  // scores stay open.  renorm: weights are divided by their sum; then times scale.
-  const int lane = threadIdx.x & (WAVE_SIZE - 1);
+    float* __restrict__ wts, const float* __restrict__ logits, int tokens, RouteRule rule) {
   const long t = blockIdx.x * (long)(blockDim.x / WAVE_SIZE) + threadIdx.x / WAVE_SIZE;
   if (t >= tokens) return;
-  const float* z = logits + t * n;
-  float s[RT_MAX], ch[RT_MAX];
-  bool taken[RT_MAX];
-  float m = -INFINITY;
-#pragma unroll
-  for (int i = 0; i < RT_MAX; ++i) {
-    const int e = lane + i * WAVE_SIZE;
-    s[i] = (e < n) ? z[e] : -INFINITY;
-    taken[i] = false;
-    m = fmaxf(m, s[i]);
-  }
-  if (sigmoid) {
-#pragma unroll
-    for (int i = 0; i < RT_MAX; ++i) {
-      const int e = lane + i * WAVE_SIZE;
-      s[i] = (e < n) ? 1.0f / (1.0f + expf(-s[i])) : 0.f;
-      ch[i] = (e < n) ? s[i] + (correction != nullptr ? correction[e] : 0.f) : -INFINITY;
-    }
-  } else {
-    m = wave_reduce_max(m);
-    float den = 0.f;
-#pragma unroll
-    for (int i = 0; i < RT_MAX; ++i) {
-      const int e = lane + i * WAVE_SIZE;
-      s[i] = (e < n) ? expf(s[i] - m) : 0.f;
-      den += s[i];
-    }
-    den = wave_reduce_sum(den);
-#pragma unroll
-    for (int i = 0; i < RT_MAX; ++i) {
-      const int e = lane + i * WAVE_SIZE;
-      s[i] = s[i] / den;
-      ch[i] = (e < n) ? s[i] + correction[e] : -INFINITY;
-    }
-  }
-  if (groups > 1) {
-    // lane g ends up with group g's score (at most 64 groups)
-    const int size = n / groups;
-    float score = -INFINITY;
-    for (int g = 0; g < groups; ++g) {
-      float b1 = -INFINITY, b2 = -INFINITY;   // this lane's two best in the group
-#pragma unroll
-      for (int i = 0; i < RT_MAX; ++i) {
-        const int e = lane + i * WAVE_SIZE;
-        if (e >= g * size && e < (g + 1) * size) {
-          b2 = fmaxf(b2, fminf(b1, ch[i]));
-          b1 = fmaxf(b1, ch[i]);
-        }
-      }
-#pragma unroll
-      for (int off = 32; off > 0; off >>= 1) {
-        const float o1 = __shfl_xor(b1, off, WAVE_SIZE), o2 = __shfl_xor(b2, off, WAVE_SIZE);
-        b2 = fmaxf(fmaxf(b2, o2), fminf(b1, o1));
-        b1 = fmaxf(b1, o1);
-      }
-      if (lane == g) score = size > 1 ? b1 + b2 : b1;
-    }
-    unsigned long long open = 0;
-    for (int k = 0; k < keep; ++k) {
-      float best = (open >> lane) & 1 ? -INFINITY : score;
-      int at = lane < groups && !((open >> lane) & 1) ? lane : 0x7fffffff;
-#pragma unroll
-      for (int off = 32; off > 0; off >>= 1) {
-        const float ob = __shfl_xor(best, off, WAVE_SIZE);
-        const int oa = __shfl_xor(at, off, WAVE_SIZE);
-        if (ob > best || (ob == best && oa < at)) { best = ob; at = oa; }
-      }
-      if (at < groups) open |= 1ull << at;
-    }
-#pragma unroll
-    for (int i = 0; i < RT_MAX; ++i) {
-      const int e = lane + i * WAVE_SIZE;
-      if (e < n && !((open >> (e / size)) & 1)) ch[i] = -INFINITY;
-    }
-  }
-  float total = 0.f, id_sum = 0.f;
-  for (int k = 0; k < top; ++k) {
-    // the largest remaining choice score; ties go to the lower index
-    float best = -INFINITY;
-    int best_e = 0x7fffffff;
-#pragma unroll
-    for (int i = 0; i < RT_MAX; ++i) {
-      const int e = lane + i * WAVE_SIZE;
-      if (e < n && !taken[i] && (ch[i] > best || (ch[i] == best && e < best_e))) {
-        best = ch[i];
-        best_e = e;
-      }
-    }
-#pragma unroll
-    for (int off = 32; off > 0; off >>= 1) {
-      const float ob = __shfl_xor(best, off, WAVE_SIZE);
-      const int oe = __shfl_xor(best_e, off, WAVE_SIZE);
-      if (ob > best || (ob == best && oe < best_e)) {
-        best = ob;
-        best_e = oe;
-      }
-    }
-    // the owner marks it and tells everyone its softmax score
-    float sv = 0.f;
-#pragma unroll
-    for (int i = 0; i < RT_MAX; ++i) {
-      if (lane + i * WAVE_SIZE == best_e) {
-        taken[i] = true;
-        sv = s[i];
-      }
-    }
-    sv = wave_reduce_sum(sv);
-    total += sv;
-    if (best_e >= num_real) id_sum += sv;
-    if (lane == 0) {
-      ids[t * top + k] = best_e;
-      wts[t * top + k] = sv;
-    }
-  }
-  const float inv = (renorm ? 1.0f / (total + 1e-20f) : 1.0f) * scale;
-#pragma unroll
-  for (int i = 0; i < RT_MAX; ++i) {
-    const int e = lane + i * WAVE_SIZE;
-    if (e < num_real) dense[t * num_real + e] = taken[i] ? s[i] * inv : 0.f;
-  }
-  // lane 0 wrote wts[t, :] itself, so it may rescale them in place
-  if (lane == 0) {
-    if (renorm || scale != 1.0f)
-      for (int k = 0; k < top; ++k) wts[t * top + k] *= inv;
-    if (!sigmoid) ident[t] = id_sum * inv;
-  }
+  moe_route_token(logits + t * rule.n, rule, dense == nullptr ? nullptr : dense + t * rule.num_real,
+                  ident == nullptr ? nullptr : ident + t, ids + t * rule.top, wts + t * rule.top);
 }
 
 // out[t, :] = sum_k [ids[t,k] < num_real] w[t,k] * ye[pos[t,k], :]
@@ -572,6 +439,51 @@ __global__ __launch_bounds__(256) void moe_place_kernel(
   }
 }
 
+// counts, offsets and rows of at most MS_SMALL pairs in one workgroup
+constexpr int MS_SMALL = 4096;
+
+__global__ __launch_bounds__(1024) void moe_place_small_kernel(
+    int* __restrict__ pos, int* __restrict__ seg, const int* __restrict__ ids, int npairs,
+    int num_real) {
+  constexpr int PER = MS_SMALL / 1024;
+  __shared__ int hist[MS_MAX], start[MS_MAX];
+  for (int e = threadIdx.x; e < num_real; e += 1024) hist[e] = 0;
+  __syncthreads();
+  int e[PER], local[PER];
+#pragma unroll
+  for (int u = 0; u < PER; ++u) {
+    const int i = threadIdx.x + u * 1024;
+    e[u] = i < npairs ? ids[i] : num_real;
+    local[u] = e[u] < num_real ? atomicAdd(&hist[e[u]], 1) : 0;
+  }
+  __syncthreads();
+  if (threadIdx.x < WAVE_SIZE) {   // exclusive sums, a wave over 64 experts at a time
+    int run = 0;
+    for (int e0 = 0; e0 < num_real; e0 += WAVE_SIZE) {
+      const int x = e0 + threadIdx.x;
+      const int own = x < num_real ? hist[x] : 0;
+      int sum = own;
+#pragma unroll
+      for (int off = 1; off < WAVE_SIZE; off <<= 1) {
+        const int o = __shfl_up(sum, off, WAVE_SIZE);
+        if ((int)threadIdx.x >= off) sum += o;
+      }
+      if (x < num_real) {
+        start[x] = run + sum - own;
+        seg[x] = start[x];
+      }
+      run += __shfl(sum, WAVE_SIZE - 1, WAVE_SIZE);
+    }
+    if (threadIdx.x == 0) seg[num_real] = run;
+  }
+  __syncthreads();
+#pragma unroll
+  for (int u = 0; u < PER; ++u) {
+    const int i = threadIdx.x + u * 1024;
+    if (i < npairs) pos[i] = e[u] < num_real ? start[e[u]] + local[u] : 0;
+  }
+}
+
 // one workgroup per token: its row goes to the rows of its real experts
 template <typename T>
 __global__ __launch_bounds__(256) void moe_gather_kernel(
@@ -619,17 +531,24 @@ __global__ __launch_bounds__(256) void moe_gather_kernel(
 // ---------------------------------------------------------------------------
 
 int moe_sort_max_experts() { return MS_MAX; }
+// up to this many pairs moe_sort needs no zeroed scratch
+int moe_sort_small_pairs() { return MS_SMALL; }
 
-// counts_cursor: 2 * num_real zeros (counts, then the per-expert cursors)
+// counts_cursor: 2 * num_real zeros (counts, then the per-expert cursors), or
+// null for at most moe_sort_small_pairs() pairs
 template <typename T>
 void launch_moe_sort(T* xs, int* pos, int* seg, int* counts_cursor, const T* h,
                      long h_st, const int* ids, int tokens, int top, int num_real,
                      int width, const float* row_scale, hipStream_t s) {
   const int npairs = tokens * top;
   const int blocks = grid_for(npairs, 256) > 1024 ? 1024 : grid_for(npairs, 256);
-  moe_count_kernel<<<blocks, 256, 0, s>>>(counts_cursor, ids, npairs, num_real);
-  moe_place_kernel<<<blocks, 256, 0, s>>>(pos, seg, counts_cursor + num_real,
-                                           counts_cursor, ids, npairs, num_real);
+  if (counts_cursor == nullptr) {
+    moe_place_small_kernel<<<1, 1024, 0, s>>>(pos, seg, ids, npairs, num_real);
+  } else {
+    moe_count_kernel<<<blocks, 256, 0, s>>>(counts_cursor, ids, npairs, num_real);
+    moe_place_kernel<<<blocks, 256, 0, s>>>(pos, seg, counts_cursor + num_real,
+                                             counts_cursor, ids, npairs, num_real);
+  }
   constexpr int V = Vec16<T>::kElems;
   const int vec = width % V == 0 && h_st % V == 0 && al(xs, 16) && al(h, 16);
   moe_gather_kernel<T><<<tokens, 256, 0, s>>>(xs, h, h_st, pos, ids, top, num_real,
@@ -725,8 +644,8 @@ void launch_moe_route(float* dense, float* ident, int* ids, float* wts,
                       int renorm, float scale, hipStream_t s) {
   const int waves = 256 / WAVE_SIZE;
   moe_route_kernel<<<(tokens + waves - 1) / waves, 256, 0, s>>>(
-      dense, ident, ids, wts, logits, correction, tokens, n, num_real, top, sigmoid, groups,
-      keep, renorm, scale);
+      dense, ident, ids, wts, logits, tokens,
+      RouteRule{correction, n, num_real, top, sigmoid, groups, keep, renorm, scale});
 }
 
 template <typename T>

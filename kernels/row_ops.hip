@@ -8,13 +8,14 @@
 //                         an earlier layer's cached values, paged cache write
 //   clamped_glu           g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = up
 //                         clamped to +-limit, times a weight per expert
-//   router_logits         rows times a small f32 matrix, in f32 on the matrix cores
+//   router_logits         rows times a small f32 matrix, in f32 on the matrix cores;
+//                         route_experts: and the choice of experts from them
 //   scale_logits          f32 copy times a constant
 //
 // All memory-bound.  Statistics, tanh, gates, mixing and the stream are f32
 // whatever the storage type; every result is rounded once.
 
-#include "common.h"
+#include "moe_route.h"
 
 namespace {
 
@@ -284,72 +285,126 @@ __global__ void clamped_glu_kernel(T* __restrict__ out, const T* __restrict__ gu
 
 // ---------------------------------------------------------------------------
 // router_logits: out [T, E] = h [T, W] . w [E, W]^T in f32.  A workgroup has 16
-// rows and 16 experts; its waves split the width in interleaved pieces of 32 and
-// are summed through LDS.  v_mfma_f32_16x16x4_f32 takes one element of row (or
-// expert) lane % 16 per lane and four contraction slots, lane / 16; a lane feeds
-// the eight consecutive elements it loaded to eight instructions, so slot s of
-// instruction j is element 8 s + j on both sides.
+// rows and NT tiles of 16 experts; its waves split the width in interleaved pieces
+// of 32 and are summed through LDS.  A lane loads eight consecutive elements of row
+// (or expert) lane % 16, the eight of slot lane / 16.  bf16 rows and weights go
+// straight to v_mfma_f32_16x16x32_bf16, whose products are exact in f32; with f32 on
+// either side they are fed one by one to v_mfma_f32_16x16x4_f32, slot s of
+// instruction j being element 8 s + j on both sides.
 // ---------------------------------------------------------------------------
 typedef __attribute__((ext_vector_type(4))) float f32x4_t;
+typedef __attribute__((ext_vector_type(8))) short bf16x8_t;
 constexpr int RL_WAVES = 16;
 
-template <typename T>
-__global__ __launch_bounds__(RL_WAVES * 64) void router_logits_kernel(
-    float* __restrict__ out, const T* __restrict__ h, long h_st,
-    const float* __restrict__ w, int rows, int experts, int width) {
-  __shared__ float part[RL_WAVES][256];
+DEVINLINE f32x4_t router_mfma(const Raw8<__hip_bfloat16>& a, const Raw8<__hip_bfloat16>& b,
+                              f32x4_t acc) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a.u),
+                                                 __builtin_bit_cast(bf16x8_t, b.u), acc, 0, 0, 0);
+}
+template <typename A, typename B>
+DEVINLINE f32x4_t router_mfma(const Raw8<A>& a, const Raw8<B>& b, f32x4_t acc) {
+  float x[8], y[8];
+  unpack8(a, x);
+  unpack8(b, y);
+#pragma unroll
+  for (int j = 0; j < 8; ++j) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(x[j], y[j], acc, 0, 0, 0);
+  return acc;
+}
+
+// z_s [16][NT * 16]: the logits of rows row0 .. row0 + 15, experts e0 ..
+template <typename T, typename W, int NT>
+DEVINLINE void router_tile(float* z_s, float* part, const T* __restrict__ h, long h_st,
+                           const W* __restrict__ w, int row0, int e0, int rows, int experts,
+                           int width) {
+  // pieces loaded ahead of the products
+  constexpr int FLY = (sizeof(T) == 2 && sizeof(W) == 2 ? 8 : 4) / NT;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int i = lane & 15, s = lane >> 4;
-  const int row = blockIdx.x * 16 + i, e = blockIdx.y * 16 + i;
-  // rows and experts past the end are clamped: they compute and never store
-  const T* hp = h + (long)min(row, rows - 1) * h_st + s * 8;
-  const float* wp = w + (long)min(e, experts - 1) * width + s * 8;
-  f32x4_t acc{};
-  // FLY pieces are loaded before the first of them is used
-  constexpr int FLY = 4;
+  // rows and experts past the end are clamped: they compute and are not used
+  const T* hp = h + (long)min(row0 + i, rows - 1) * h_st + s * 8;
+  const W* wp[NT];
+#pragma unroll
+  for (int t = 0; t < NT; ++t)
+    wp[t] = w + (long)min(e0 + t * 16 + i, experts - 1) * width + s * 8;
+  f32x4_t acc[NT];
+#pragma unroll
+  for (int t = 0; t < NT; ++t) acc[t] = f32x4_t{};
   for (int c0 = wave * 32; c0 < width; c0 += FLY * RL_WAVES * 32) {
-    float a[FLY][8], b[FLY][8];
+    Raw8<T> a[FLY];
+    Raw8<W> b[FLY][NT];
 #pragma unroll
     for (int f = 0; f < FLY; ++f) {
       const int c = c0 + f * RL_WAVES * 32;
+      a[f] = Raw8<T>{};
 #pragma unroll
-      for (int j = 0; j < 8; ++j) a[f][j] = b[f][j] = 0.f;
+      for (int t = 0; t < NT; ++t) b[f][t] = Raw8<W>{};
       if (c < width) {               // uniform over the wave
-        ld8<T>(hp + c, a[f]);
-        ld8<float>(wp + c, b[f]);
+        a[f] = ldraw<T>(hp + c);
+#pragma unroll
+        for (int t = 0; t < NT; ++t) b[f][t] = ldraw<W>(wp[t] + c);
       }
     }
 #pragma unroll
     for (int f = 0; f < FLY; ++f)
 #pragma unroll
-      for (int j = 0; j < 8; ++j)
-        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[f][j], b[f][j], acc, 0, 0, 0);
+      for (int t = 0; t < NT; ++t) acc[t] = router_mfma(a[f], b[f][t], acc[t]);
   }
-  // lane holds out[4 * (lane / 16) + r][lane % 16]
+  // lane holds element [4 * (lane / 16) + r][lane % 16] of a tile
 #pragma unroll
-  for (int r = 0; r < 4; ++r) part[wave][(4 * s + r) * 16 + i] = acc[r];
+  for (int t = 0; t < NT; ++t)
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      part[wave * NT * 256 + (4 * s + r) * NT * 16 + t * 16 + i] = acc[t][r];
   __syncthreads();
-  if (threadIdx.x < 256) {
+  for (int x = threadIdx.x; x < NT * 256; x += RL_WAVES * 64) {
     float z = 0.f;
 #pragma unroll
-    for (int k = 0; k < RL_WAVES; ++k) z += part[k][threadIdx.x];
-    const int r = blockIdx.x * 16 + threadIdx.x / 16, x = blockIdx.y * 16 + threadIdx.x % 16;
-    if (r < rows && x < experts) out[(long)r * experts + x] = z;
+    for (int k = 0; k < RL_WAVES; ++k) z += part[k * NT * 256 + x];
+    z_s[x] = z;
+  }
+  __syncthreads();
+}
+
+template <typename T, typename W, int NT>
+__global__ __launch_bounds__(RL_WAVES * 64) void router_logits_kernel(
+    float* __restrict__ out, const T* __restrict__ h, long h_st,
+    const W* __restrict__ w, int rows, int experts, int width) {
+  __shared__ float part[RL_WAVES * NT * 256], z_s[NT * 256];
+  const int row0 = blockIdx.x * 16, e0 = blockIdx.y * NT * 16;
+  router_tile<T, W, NT>(z_s, part, h, h_st, w, row0, e0, rows, experts, width);
+  for (int x = threadIdx.x; x < NT * 256; x += RL_WAVES * 64) {
+    const int r = row0 + x / (NT * 16), e = e0 + x % (NT * 16);
+    if (r < rows && e < experts) out[(long)r * experts + e] = z_s[x];
   }
 }
 
+// a wave per row chooses from the logits in LDS (at most NT * 16 experts)
+template <typename T, typename W, int NT>
+__global__ __launch_bounds__(RL_WAVES * 64) void route_experts_kernel(
+    float* __restrict__ dense, int* __restrict__ ids, float* __restrict__ wts,
+    const T* __restrict__ h, long h_st, const W* __restrict__ w, int rows, int width,
+    RouteRule rule) {
+  __shared__ float part[RL_WAVES * NT * 256], z_s[NT * 256];
+  const int row0 = blockIdx.x * 16, wave = threadIdx.x >> 6;
+  router_tile<T, W, NT>(z_s, part, h, h_st, w, row0, 0, rows, rule.n, width);
+  const long t = row0 + wave;
+  if (t >= rows) return;
+  moe_route_lanes<1>(z_s + wave * NT * 16, rule, dense + t * rule.n, nullptr, ids + t * rule.top,
+                     wts + t * rule.top);
+}
+
 // any width: one wave per (row, expert)
-template <typename T>
+template <typename T, typename W>
 __global__ __launch_bounds__(256) void router_logits_any_kernel(
     float* __restrict__ out, const T* __restrict__ h, long h_st,
-    const float* __restrict__ w, int rows, int experts, int width) {
+    const W* __restrict__ w, int rows, int experts, int width) {
   const long id = blockIdx.x * 4L + threadIdx.x / WAVE_SIZE;
   if (id >= (long)rows * experts) return;
   const long row = id / experts;
   const int e = (int)(id - row * experts);
   float z = 0.f;
   for (int c = threadIdx.x & (WAVE_SIZE - 1); c < width; c += WAVE_SIZE)
-    z += ScalarOps<T>::to_f32(h[row * h_st + c]) * w[(long)e * width + c];
+    z += ScalarOps<T>::to_f32(h[row * h_st + c]) * ScalarOps<W>::to_f32(w[(long)e * width + c]);
   z = wave_reduce_sum(z);
   if ((threadIdx.x & (WAVE_SIZE - 1)) == 0) out[id] = z;
 }
@@ -407,11 +462,8 @@ void launch_wide_norm(T* q_out, const T* proj, long st, const float* bias, const
   const bool vec = nq % 8 == 0 && nk % 8 == 0 && nv % 8 == 0 && st % 8 == 0 && per <= 8 &&
                    al(proj, 16) && al(bias, 16) && al(qw, 16) && al(kw, 16) && al(v_first, 16) &&
                    al(q_out, 16) && al(k_cache, 16) && al(v_cache, 16);
-  static const int wr = getenv("WN_ROWS") ? atoi(getenv("WN_ROWS")) : 4;
 #define WIDE_LAUNCH(NV)                                                                \
-  if (rows < 2048 || wr == 1) wide_norm_vec_kernel<T, NV, 1><<<rows, 256, 0, s>>>(p);             \
-  else if (wr == 2) wide_norm_vec_kernel<T, NV, 2><<<(rows + 1) / 2, 256, 0, s>>>(p);             \
-  else if (wr == 8) wide_norm_vec_kernel<T, NV, 8><<<(rows + 7) / 8, 256, 0, s>>>(p);             \
+  if (rows < 2048) wide_norm_vec_kernel<T, NV, 1><<<rows, 256, 0, s>>>(p);             \
   else wide_norm_vec_kernel<T, NV, 4><<<(rows + 3) / 4, 256, 0, s>>>(p)
   if (!vec) wide_norm_kernel<T><<<rows, 256, 0, s>>>(p);
   else if (per == 1) { WIDE_LAUNCH(1); }
@@ -432,15 +484,36 @@ void launch_clamped_glu(T* out, const T* gu, float limit, const float* col_scale
   else clamped_glu_kernel<T, 1><<<blocks, 256, 0, s>>>(out, gu, limit, col_scale, ff, work);
 }
 
-template <typename T>
-void launch_router_logits(float* out, const T* h, long h_st, const float* w, int rows,
+template <typename T, typename W>
+void launch_router_logits(float* out, const T* h, long h_st, const W* w, int rows,
                           int experts, int width, hipStream_t s) {
-  if (width % 32 == 0 && h_st % 8 == 0 && al(h, 16) && al(w, 16))
-    router_logits_kernel<T><<<dim3((rows + 15) / 16, (experts + 15) / 16), RL_WAVES * 64, 0, s>>>(
+  const int tiles = (experts + 15) / 16;
+#define ROUTER_LAUNCH(NT)                                                              \
+  router_logits_kernel<T, W, NT><<<dim3((rows + 15) / 16, (tiles + NT - 1) / NT),         \
+                                RL_WAVES * 64, 0, s>>>(out, h, h_st, w, rows, experts, width)
+  if (width % 32 || h_st % 8 || !al(h, 16) || !al(w, 16))
+    router_logits_any_kernel<T, W><<<(int)(((long)rows * experts + 3) / 4), 256, 0, s>>>(
         out, h, h_st, w, rows, experts, width);
-  else
-    router_logits_any_kernel<T><<<(int)(((long)rows * experts + 3) / 4), 256, 0, s>>>(
-        out, h, h_st, w, rows, experts, width);
+  else if (tiles == 1) ROUTER_LAUNCH(1);
+  else if (tiles == 2) ROUTER_LAUNCH(2);
+  else ROUTER_LAUNCH(4);
+#undef ROUTER_LAUNCH
+}
+
+// at most 64 experts, width a multiple of 32, 16-byte aligned rows
+template <typename T, typename W>
+void launch_route_experts(float* dense, int* ids, float* wts, const T* h, long h_st,
+                          const W* w, const float* correction, int rows, int experts,
+                          int width, int top, int groups, int keep, int renorm, float scale,
+                          hipStream_t s) {
+  const RouteRule rule{correction, experts, experts, top, 1, groups, keep, renorm, scale};
+#define ROUTE_LAUNCH(NT)                                                               \
+  route_experts_kernel<T, W, NT><<<(rows + 15) / 16, RL_WAVES * 64, 0, s>>>(              \
+      dense, ids, wts, h, h_st, w, rows, width, rule)
+  if (experts <= 16) ROUTE_LAUNCH(1);
+  else if (experts <= 32) ROUTE_LAUNCH(2);
+  else ROUTE_LAUNCH(4);
+#undef ROUTE_LAUNCH
 }
 
 template <typename T>
@@ -459,8 +532,17 @@ void launch_scale_logits(float* out, const T* x, float scale, long n, hipStream_
                                     int, int, int, int, float, hipStream_t);             \
   template void launch_clamped_glu<T>(T*, const T*, float, const float*, int, long,      \
                                       hipStream_t);                                      \
-  template void launch_router_logits<T>(float*, const T*, long, const float*, int, int,  \
-                                        int, hipStream_t);                               \
   template void launch_scale_logits<T>(float*, const T*, float, long, hipStream_t);
 INSTANTIATE(float)
 INSTANTIATE(__hip_bfloat16)
+
+#define INSTANTIATE_ROUTER(T, W)                                                         \
+  template void launch_router_logits<T, W>(float*, const T*, long, const W*, int, int,   \
+                                           int, hipStream_t);                            \
+  template void launch_route_experts<T, W>(float*, int*, float*, const T*, long,         \
+                                           const W*, const float*, int, int, int, int,   \
+                                           int, int, int, float, hipStream_t);
+INSTANTIATE_ROUTER(float, float)
+INSTANTIATE_ROUTER(float, __hip_bfloat16)
+INSTANTIATE_ROUTER(__hip_bfloat16, float)
+INSTANTIATE_ROUTER(__hip_bfloat16, __hip_bfloat16)

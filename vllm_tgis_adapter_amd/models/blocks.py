@@ -1159,9 +1159,8 @@ class GatedRoutedExperts(nn.Module):
         self.grouped = (fits and experts > 2 * top) if grouped is None else bool(grouped)
         if self.grouped and not fits:
             raise ValueError("grouped experts need bf16 and sizes in multiples of 128")
-        self.router = nn.Parameter(
-            torch.empty(experts, width, dtype=torch.float32).normal_(0.0, width ** -0.5),
-            requires_grad=False)
+        # logits are f32 products and sums of weights as the checkpoint stores them
+        self.router = _randn_param((experts, width), dtype, std=width ** -0.5)
         self.correction = _f32_param(experts) if correction else None
         # per expert: ff gate rows, then ff up rows
         self.gate_up = _randn_param((experts, 2 * ff, width), dtype, std=width ** -0.5)
@@ -1171,7 +1170,11 @@ class GatedRoutedExperts(nn.Module):
             self.down = _randn_param((width, experts * ff), dtype, std=ff ** -0.5)
 
     def load(self, router, gates: list, ups: list, downs: list, correction=None) -> None:
-        self.router.data.copy_(router.float())
+        if not torch.equal(router.to(self.dtype).float(), router.float()):
+            # the checkpoint's weights do not fit the compute dtype: keep them in f32
+            self.router = nn.Parameter(torch.empty_like(self.router, dtype=torch.float32),
+                                       requires_grad=False)
+        self.router.data.copy_(router)
         if self.correction is not None:
             self.correction.data.copy_(correction.float())
         ff = self.ff
@@ -1183,15 +1186,12 @@ class GatedRoutedExperts(nn.Module):
             else:
                 self.down.data[:, e * ff:(e + 1) * ff].copy_(d.to(self.dtype))
 
-    def route(self, z: torch.Tensor):
-        return ops.moe_route_sigmoid(z, self.top, self.correction, *self.groups,
-                                     self.renormalise, self.weight_scale)
-
     def forward(self, h: torch.Tensor, router_in: Optional[torch.Tensor] = None) -> torch.Tensor:
         """``router_in``: the f32 rows h was rounded from, when the caller has
         them; the router then reads those instead of the rounded copy."""
-        dense, ids, w = self.route(
-            ops.router_logits(h if router_in is None else router_in, self.router))
+        dense, ids, w = ops.route_experts(
+            h if router_in is None else router_in, self.router, self.top, self.correction,
+            *self.groups, self.renormalise, self.weight_scale)
         ne = self.experts
         if not self.grouped:
             gu = ops.linear(h, self.gate_up.view(ne * 2 * self.ff, self.width))

@@ -1104,7 +1104,8 @@ def moe_sort(ids: torch.Tensor, num_real: int, h: torch.Tensor,
         xs = torch.empty((t * top, h.shape[1]), dtype=h.dtype, device=dev)
         pos = torch.empty((t, top), dtype=torch.int32, device=dev)
         seg = torch.empty((num_real + 1,), dtype=torch.int32, device=dev)
-        scratch = torch.zeros((2 * num_real,), dtype=torch.int32, device=dev)
+        scratch = (None if ids.numel() <= _S.moe_sort_small_pairs() else
+                   torch.zeros((2 * num_real,), dtype=torch.int32, device=dev))
         _S.moe_sort(xs, pos, seg, scratch, h, ids, int(num_real), row_scale)
         return xs, pos, seg
     return reference.moe_sort(ids, num_real, h, row_scale)
@@ -1572,12 +1573,32 @@ def clamped_glu(gu: torch.Tensor, limit: float,
 
 
 def router_logits(h: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
-    """h [T, W] (compute dtype or f32) times weight [E, W] f32, all in f32."""
+    """h [T, W] times weight [E, W] (each f32 or bf16), products and sums in f32."""
     if h.numel() and _native_seq(h):
         out = torch.empty((h.shape[0], weight.shape[0]), dtype=torch.float32, device=h.device)
         _S.router_logits(out, h, weight)
         return out
     return reference.router_logits(h, weight)
+
+
+def route_experts(h: torch.Tensor, weight: torch.Tensor, top: int, correction=None,
+                  groups: int = 1, keep: int = 1, renormalise: bool = False, scale: float = 1.0):
+    """router_logits followed by moe_route_sigmoid, one kernel for up to 64
+    experts and widths in multiples of 32."""
+    e, width = weight.shape
+    if not (h.numel() and _native_seq(h) and e <= 64 and width % 32 == 0
+            and h.stride(0) % 8 == 0):
+        return moe_route_sigmoid(router_logits(h, weight), top, correction, groups, keep,
+                                 renormalise, scale)
+    if e % groups or not 1 <= keep <= groups or top > keep * (e // groups):
+        raise ValueError("the kept groups must be equal and hold the chosen experts")
+    t, dev = h.shape[0], h.device
+    dense = torch.empty((t, e), dtype=torch.float32, device=dev)
+    ids = torch.empty((t, top), dtype=torch.int32, device=dev)
+    w = torch.empty((t, top), dtype=torch.float32, device=dev)
+    _S.route_experts(dense, ids, w, h, weight, correction, int(groups), int(keep),
+                     bool(renormalise), float(scale))
+    return dense, ids, w
 
 
 def scale_logits(logits: torch.Tensor, scale: float) -> torch.Tensor:

@@ -1219,7 +1219,7 @@ def clamped_glu(gu: torch.Tensor, limit: float, col_scale: torch.Tensor | None) 
 
 
 def router_logits(h: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
-    return torch.nn.functional.linear(h.float(), weight)
+    return torch.nn.functional.linear(h.float(), weight.float())
 
 
 def scale_logits(logits: torch.Tensor, scale: float) -> torch.Tensor:
