@@ -66,9 +66,9 @@ struct SpanKeys {
 };
 
 template <int HEAD_DIM, typename CT, bool WS, bool CH = false, int PX = PX_NONE,
-          int CAP = CAP_NONE>
+          int CAP = CAP_NONE, int VD = HEAD_DIM>
 __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
-    float* __restrict__ part_acc,   // [nseq, nheads, P, HEAD_DIM] f32
+    float* __restrict__ part_acc,   // [nseq, nheads, P, VD] f32
     float* __restrict__ part_ml,    // [nseq, nheads, P, 2] f32 (m, l)
     const __hip_bfloat16* __restrict__ q,        // [nseq, nheads, HD]
     const CT* __restrict__ k_cache,  // [nb, bs, kvh, HD] bf16 | e4m3
@@ -91,7 +91,8 @@ __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
   static_assert(!CH || WS, "the chunk variant builds on the window variant");
   static_assert(PX == PX_NONE || (WS && !CH), "prefixes build on the window variant");
   constexpr int KCH = HEAD_DIM / 16;  // k-chunks for the QK^T mfma
-  constexpr int DT = HEAD_DIM / 32;   // 32-col output tiles
+  constexpr int DT = VD / 32;         // 32-col output tiles
+  static_assert(HEAD_DIM % 16 == 0 && (VD == 64 || VD == 128), "head sizes");
 
   const int seq = blockIdx.x;
   const int kv_head = blockIdx.y;
@@ -123,12 +124,12 @@ __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
   const int head0 = kv_head * group;
   const int* btable = block_tables + (long)seq * max_blocks;
   const long kv_row_stride = (long)kvh * HEAD_DIM;
-  const long v_row_stride = CH ? (long)v_heads * HEAD_DIM : kv_row_stride;
+  const long v_row_stride = CH ? (long)v_heads * VD : (long)kvh * VD;
   const int v_head = CH ? kv_head % v_heads : kv_head;
 
   // per-wave V staging tile (linear; the B gather reads rows across lanes)
-  __shared__ __hip_bfloat16 v_lds_all[NWAVES * KVT * HEAD_DIM];
-  __hip_bfloat16* v_lds = v_lds_all + wave * KVT * HEAD_DIM;
+  __shared__ __hip_bfloat16 v_lds_all[NWAVES * KVT * VD];
+  __hip_bfloat16* v_lds = v_lds_all + wave * KVT * VD;
 
   // ---- Q as B fragments: lane holds Q[q=col][ks*16 + half*8 + j] ---------
   bf16x8_t qb[KCH];
@@ -152,7 +153,7 @@ __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
   const float cap_in = capped ? scale / softcap : 0.f;
   if (CAP == CAP_FIXED) m_state = 0.f;
 
-  constexpr int VPASS = KVT * HEAD_DIM / 8 / 64;  // V staging passes per wave
+  constexpr int VPASS = KVT * VD / 8 / 64;  // V staging passes per wave
 
   for (int t = tile_lo + wave; t < tile_hi; t += NWAVES) {
     const bool prefix = PX != PX_NONE && t < pre_tiles;
@@ -194,7 +195,7 @@ __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
     }
     bf16x8_t vv[VPASS];
     {
-      constexpr int LPR = HEAD_DIM / 8;        // lanes per row
+      constexpr int LPR = VD / 8;              // lanes per row
       constexpr int ROWS_PER_PASS = 64 / LPR;  // rows per pass per wave
       const int r_in_pass = lane / LPR;
       const int d8 = (lane % LPR) * 8;
@@ -204,14 +205,14 @@ __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
         const int pos = kv_base + s;
         vv[pass] = bf16x8_t{};
         if (pos < limit) {
-          const long row = row_of(pos) * v_row_stride + (long)v_head * HEAD_DIM + d8;
+          const long row = row_of(pos) * v_row_stride + (long)v_head * VD + d8;
           vv[pass] = load_kv8<CT>(v_src + row);
         }
       }
 #pragma unroll
       for (int pass = 0; pass < VPASS; ++pass) {
         const int s = pass * ROWS_PER_PASS + r_in_pass;
-        *reinterpret_cast<bf16x8_t*>(v_lds + s * HEAD_DIM + d8) = vv[pass];
+        *reinterpret_cast<bf16x8_t*>(v_lds + s * VD + d8) = vv[pass];
       }
     }
 
@@ -320,7 +321,7 @@ __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
 #pragma unroll
         for (int j = 0; j < 8; ++j)
           b[j] = *reinterpret_cast<const short*>(
-              v_lds + (c * 16 + half * 8 + j) * HEAD_DIM + dt * 32 + col);
+              v_lds + (c * 16 + half * 8 + j) * VD + dt * 32 + col);
         acc_o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(pa[0][c], b, acc_o[dt], 0, 0, 0);
         if (WS)
           acc_o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(pa[PASSES - 1][c], b,
@@ -342,7 +343,7 @@ __global__ __launch_bounds__(256, 2) void paged_decode_mfma_kernel(
     const int qrow = (r & 3) + 8 * (r >> 2) + 4 * half;
     if (qrow >= group) continue;
     float* acc_row =
-        part_acc + (((long)seq * nheads + head0 + qrow) * P + pw) * HEAD_DIM;
+        part_acc + (((long)seq * nheads + head0 + qrow) * P + pw) * VD;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) acc_row[dt * 32 + col] = acc_o[dt][r];
   }
@@ -587,8 +588,9 @@ void launch_paged_decode_mfma_span(__hip_bfloat16* out, float* part_acc, float* 
     abort();
 }
 
-// soft-capped scores, window, sinks per head or none (bf16 cache)
-template <int HD, int CAP>
+// soft-capped scores, window, sinks per head or none (bf16 cache); sizes as for
+// prompt portions
+template <int HD, int VD, int CAP>
 static void launch_decode_capped(__hip_bfloat16* out, float* part_acc, float* part_ml,
                                  const __hip_bfloat16* q, const __hip_bfloat16* kc,
                                  const __hip_bfloat16* vc, const int* bt, const int* sl,
@@ -597,10 +599,10 @@ static void launch_decode_capped(__hip_bfloat16* out, float* part_acc, float* pa
                                  float softcap, hipStream_t stream) {
   const dim3 grid(nseq, kvh, npart), mgrid(nseq, nheads);
   hipLaunchKernelGGL(
-      (paged_decode_mfma_kernel<HD, __hip_bfloat16, true, false, PX_NONE, CAP>), grid,
+      (paged_decode_mfma_kernel<HD, __hip_bfloat16, true, false, PX_NONE, CAP, VD>), grid,
       dim3(256), 0, stream, part_acc, part_ml, q, kc, vc, bt, sl, scale, nheads, kvh,
       nheads / kvh, block_size, max_blocks, window, 0, 0, SpanKeys{}, softcap);
-  hipLaunchKernelGGL((decode_merge_kernel<HD>), mgrid, dim3(HD), 0, stream, out, part_acc,
+  hipLaunchKernelGGL((decode_merge_kernel<VD>), mgrid, dim3(VD), 0, stream, out, part_acc,
                      part_ml, nheads, npart * NWAVES, sinks != nullptr ? 1 : 0, 0.f, nullptr,
                      sinks);
 }
@@ -608,7 +610,7 @@ static void launch_decode_capped(__hip_bfloat16* out, float* part_acc, float* pa
 void launch_paged_decode_mfma_capped(__hip_bfloat16* out, float* part_acc, float* part_ml,
                                      const __hip_bfloat16* q, const __hip_bfloat16* kc,
                                      const __hip_bfloat16* vc, const int* bt, const int* sl,
-                                     float scale, int nseq, int nheads, int kvh, int head_dim,
+                                     float scale, int nseq, int nheads, int kvh, int dim, int vdim,
                                      int block_size, int max_blocks, int npart, int window,
                                      const float* sinks, float softcap, hipStream_t stream) {
   const bool fixed = softcap > 0.f && softcap <= kFixedMaxCap;
@@ -616,9 +618,13 @@ void launch_paged_decode_mfma_capped(__hip_bfloat16* out, float* part_acc, float
     launch(out, part_acc, part_ml, q, kc, vc, bt, sl, scale, nseq, nheads, kvh, block_size,
            max_blocks, npart, window, sinks, softcap, stream);
   };
-  if (head_dim == 64 && fixed) go(launch_decode_capped<64, CAP_FIXED>);
-  else if (head_dim == 64) go(launch_decode_capped<64, CAP_RUN>);
-  else if (head_dim == 128 && fixed) go(launch_decode_capped<128, CAP_FIXED>);
-  else if (head_dim == 128) go(launch_decode_capped<128, CAP_RUN>);
-  else abort();
+#define CAPPED_CASE(HD, VD)                                      \
+  if (dim == HD && vdim == VD) {                                 \
+    if (fixed) go(launch_decode_capped<HD, VD, CAP_FIXED>);      \
+    else go(launch_decode_capped<HD, VD, CAP_RUN>);              \
+    return;                                                      \
+  }
+  CAPPED_CASE(64, 64) CAPPED_CASE(96, 64) CAPPED_CASE(128, 128) CAPPED_CASE(192, 128)
+#undef CAPPED_CASE
+  abort();
 }

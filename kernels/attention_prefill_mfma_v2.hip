@@ -133,7 +133,8 @@ DEVINLINE void cap_scores(f32x16_t* s, float scale, float softcap) {
 }
 
 template <int HEAD_DIM, typename CT, int NW, bool WS, bool CH = false,
-          typename OT = __hip_bfloat16, int PX = PX_NONE, int CAP = CAP_NONE>
+          typename OT = __hip_bfloat16, int PX = PX_NONE, int CAP = CAP_NONE,
+          int VD = HEAD_DIM>
 __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v2_kernel(
     OT* __restrict__ out,                        // [total_q, nheads, HD]
     const __hip_bfloat16* __restrict__ q,        // [total_q, nheads, HD]
@@ -156,15 +157,21 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
     const Capped cap = Capped{}) {
   static_assert(CAP == CAP_NONE || (WS && !CH && PX == PX_NONE),
                 "the capped variant builds on the window variant");
-  static_assert(HEAD_DIM == 128, "v2 is specialised for HD=128");
+  static_assert((HEAD_DIM == 128 && VD == 128) || CAP != CAP_NONE,
+                "other head sizes are built for the capped variants only");
+  static_assert(HEAD_DIM % 16 == 0 && HEAD_DIM <= 256 && (VD == 64 || VD == 128), "head sizes");
   static_assert(PX == PX_NONE || (WS && !CH), "prefixes build on the window variant");
   static_assert(!CH || WS, "the chunk variant builds on the window variant");
   constexpr int KCH = HEAD_DIM / 16;  // QK^T k-chunks (8)
-  constexpr int DT = HEAD_DIM / 32;   // 32-col output tiles (4)
+  constexpr int DT = VD / 32;         // 32-col output tiles (4)
+  constexpr int KS = (HEAD_DIM + 127) / 128 * 128;   // K image row stride (elements)
   constexpr int QT = NW * 32;         // q rows per workgroup
   constexpr int NTHREADS = NW * 64;
-  // staging: each thread covers (s, d8) slots; pass count scales with size
-  constexpr int ST_PASS = (KVT2 * (HEAD_DIM / 8)) / NTHREADS;
+  // staging: each thread covers (s, d8) slots of the value row and of the first VD
+  // dims of the key row; pass count scales with size.  XD: key dims past those.
+  constexpr int ST_PASS = (KVT2 * (VD / 8)) / NTHREADS;
+  constexpr int XD = HEAD_DIM - VD;
+  static_assert(XD == 0 || (XD / 8 * KVT2 <= NTHREADS && XD > 0), "key staging");
 
   const int seq = blockIdx.x;
   const int head = blockIdx.y;
@@ -185,12 +192,12 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
 
   const int* btable = block_tables + (long)seq * max_blocks;
   const long kv_row_stride = (long)kvh * HEAD_DIM;
-  const long v_row_stride = CH ? (long)v_heads * HEAD_DIM : kv_row_stride;
+  const long v_row_stride = CH ? (long)v_heads * VD : (long)kvh * VD;
   const int v_head = CH ? kv_head % v_heads : kv_head;
 
-  // K: [64][256B] XOR-swizzled; V: 16 x 1152B subtiles
-  __shared__ __hip_bfloat16 k_lds2[2][KVT2 * HEAD_DIM];
-  __shared__ char v_lds2[2][16 * VSUB_STRIDE];
+  // K: [64][KS] XOR-swizzled inside 256-byte pieces; V: VD / 8 x 1152B subtiles
+  __shared__ __hip_bfloat16 k_lds2[2][KVT2 * KS];
+  __shared__ char v_lds2[2][VD / 8 * VSUB_STRIDE];
 
   // ---- per-wave Q sub-tile as B fragments ------------------------------
   const int q_row_local = tile_base + wave * 32 + col;
@@ -254,12 +261,14 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
                                            : kv_first + (it - pre_tiles) * KVT2;
   };
 
-  // ---- staging map: thread t covers slot (t % ROWS_PER_PASS, t / RPP * 8)
-  // with ROWS_PER_PASS = NTHREADS/16 rows per pass (16 8-elem slots per row)
-  constexpr int RPP = NTHREADS / 16;
+  // ---- staging map: thread t covers slot (t % RPP + pass * RPP, t / RPP * 8) with
+  // RPP = NTHREADS / (VD / 8) rows per pass, and of the other key dims slot
+  // (t % 64, VD + t / 64 * 8)
+  constexpr int RPP = NTHREADS / (VD / 8);
   const int st_s = tid % RPP;
   const int st_d8 = (tid / RPP) * 8;
-  bf16x8_t st_k[ST_PASS], st_v[ST_PASS];
+  const int x_s = tid % KVT2, x_d8 = VD + tid / KVT2 * 8;
+  bf16x8_t st_k[ST_PASS], st_v[ST_PASS], st_x;
   auto stage_load = [&](int kv_base, bool prefix) {
     const int limit = PX != PX_NONE && prefix ? pre_len : kv_limit;
 #pragma unroll
@@ -284,7 +293,16 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
         st_k[pass] = load_kv8_v2<CT>(k_cache + tok * kv_row_stride +
                                      (long)kv_head * HEAD_DIM + st_d8);
         st_v[pass] = load_kv8_v2<CT>(v_cache + tok * v_row_stride +
-                                     (long)v_head * HEAD_DIM + st_d8);
+                                     (long)v_head * VD + st_d8);
+      }
+    }
+    if constexpr (XD > 0) {
+      const int pos = kv_base + x_s;
+      st_x = bf16x8_t{};
+      if (x_d8 < HEAD_DIM && pos < limit) {
+        const int block = btable[pos / block_size];
+        const long tok = (long)block * block_size + pos % block_size;
+        st_x = load_kv8_v2<CT>(k_cache + tok * kv_row_stride + (long)kv_head * HEAD_DIM + x_d8);
       }
     }
   };
@@ -292,12 +310,18 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
 #pragma unroll
     for (int pass = 0; pass < ST_PASS; ++pass) {
       const int s = st_s + pass * RPP;
-      const int k_byte = (s * (HEAD_DIM * 2) + st_d8 * 2) ^ ((s & 15) << 4);
+      const int k_byte = (s * (KS * 2) + st_d8 * 2) ^ ((s & 15) << 4);
       *reinterpret_cast<bf16x8_t*>(
           reinterpret_cast<char*>(k_lds2[buf]) + k_byte) = st_k[pass];
-      const int sub = ((s >> 5) << 3) + (st_d8 >> 4);
+      const int sub = (s >> 5) * (VD / 16) + (st_d8 >> 4);
       const int v_byte = sub * VSUB_STRIDE + (s & 31) * 32 + (st_d8 & 15) * 2;
       *reinterpret_cast<bf16x8_t*>(v_lds2[buf] + v_byte) = st_v[pass];
+    }
+    if constexpr (XD > 0) {
+      if (x_d8 < HEAD_DIM)
+        *reinterpret_cast<bf16x8_t*>(
+            reinterpret_cast<char*>(k_lds2[buf]) +
+            ((x_s * (KS * 2) + x_d8 * 2) ^ ((x_s & 15) << 4))) = st_x;
     }
   };
 
@@ -336,7 +360,7 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
 #pragma unroll
         for (int ks = 0; ks < KCH; ++ks) {
           const int byte =
-              (krow * (HEAD_DIM * 2) + ks * 32 + half * 16) ^ ((krow & 15) << 4);
+              (krow * (KS * 2) + ks * 32 + half * 16) ^ ((krow & 15) << 4);
           bf16x8_t a = *reinterpret_cast<const bf16x8_t*>(k_lds + byte);
           acc_s[kb] =
               __builtin_amdgcn_mfma_f32_32x32x16_bf16(a, qb[ks], acc_s[kb], 0, 0, 0);
@@ -479,7 +503,7 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
         bf16x4_b ra[4], rb[4];
 #pragma unroll
         for (int c = 0; c < 4; ++c) {
-          const int sub = ((c >> 1) << 3) + d0;
+          const int sub = (c >> 1) * (VD / 16) + d0;
           const int r0 = (c & 1) * 16 + (quart >> 1) * 8;
           const char* w =
               v_lds + sub * VSUB_STRIDE + r0 * 32 + (lane & 15) * 8;
@@ -526,7 +550,7 @@ __global__ __launch_bounds__(NW * 64, 512 / (NW * 64)) void paged_prefill_mfma_v
     const float l_inv = __shfl(l_inv_own, qrow, 64);
     const int q_local = tile_base + wave * 32 + qrow;
     if (q_local >= q_len) continue;
-    OT* out_row = out + ((long)(q_start + q_local) * nheads + head) * HEAD_DIM;
+    OT* out_row = out + ((long)(q_start + q_local) * nheads + head) * VD;
     float o[DT];
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) o[dt] = acc_o[dt][r] * l_inv;
@@ -663,16 +687,17 @@ void launch_paged_prefill_mfma_v2_span(
                        Capped{});
 }
 
-// soft-capped scores, window, sinks per head or none (bf16 cache, HD = 128)
-template <int CAP>
+// soft-capped scores, window, sinks per head or none (bf16 cache); key / value
+// sizes 64/64, 96/64, 128/128 and 192/128
+template <int HD, int VD, int CAP>
 static void launch_prefill_capped(
     __hip_bfloat16* out, const __hip_bfloat16* q, const __hip_bfloat16* kc,
     const __hip_bfloat16* vc, const int* bt, const int* qsl, const int* sl, float scale,
     int nseq, int nheads, int kvh, int block_size, int max_blocks, int max_query_len,
     int window, const Capped& cap, hipStream_t stream) {
   const dim3 grid(nseq, nheads, (max_query_len + 255) / 256);
-  hipLaunchKernelGGL((paged_prefill_mfma_v2_kernel<128, __hip_bfloat16, 8, true, false,
-                                                   __hip_bfloat16, PX_NONE, CAP>),
+  hipLaunchKernelGGL((paged_prefill_mfma_v2_kernel<HD, __hip_bfloat16, 8, true, false,
+                                                   __hip_bfloat16, PX_NONE, CAP, VD>),
                      grid, dim3(512), 0, stream, out, q, kc, vc, bt, qsl, sl, scale, nheads,
                      kvh, block_size, max_blocks, window, cap.sinks != nullptr ? 1 : 0, 0.f, 0,
                      0, SpanTiles{}, cap);
@@ -681,14 +706,22 @@ static void launch_prefill_capped(
 void launch_paged_prefill_mfma_v2_capped(
     __hip_bfloat16* out, const __hip_bfloat16* q, const __hip_bfloat16* kc,
     const __hip_bfloat16* vc, const int* bt, const int* qsl, const int* sl, float scale,
-    int nseq, int nheads, int kvh, int block_size, int max_blocks, int max_query_len,
-    int window, const float* sinks, float softcap, hipStream_t stream) {
+    int nseq, int nheads, int kvh, int dim, int vdim, int block_size, int max_blocks,
+    int max_query_len, int window, const float* sinks, float softcap, hipStream_t stream) {
   Capped cap;
   cap.softcap = softcap; cap.sinks = sinks;
-  if (softcap > 0.f && softcap <= kFixedMaxCap)
-    launch_prefill_capped<CAP_FIXED>(out, q, kc, vc, bt, qsl, sl, scale, nseq, nheads, kvh,
-                                     block_size, max_blocks, max_query_len, window, cap, stream);
-  else
-    launch_prefill_capped<CAP_RUN>(out, q, kc, vc, bt, qsl, sl, scale, nseq, nheads, kvh,
-                                   block_size, max_blocks, max_query_len, window, cap, stream);
+  auto go = [&](auto launch) {
+    launch(out, q, kc, vc, bt, qsl, sl, scale, nseq, nheads, kvh, block_size, max_blocks,
+           max_query_len, window, cap, stream);
+  };
+  const bool fixed = softcap > 0.f && softcap <= kFixedMaxCap;
+#define CAPPED_CASE(HD, VD)                                       \
+  if (dim == HD && vdim == VD) {                                  \
+    if (fixed) go(launch_prefill_capped<HD, VD, CAP_FIXED>);      \
+    else go(launch_prefill_capped<HD, VD, CAP_RUN>);              \
+    return;                                                       \
+  }
+  CAPPED_CASE(64, 64) CAPPED_CASE(96, 64) CAPPED_CASE(128, 128) CAPPED_CASE(192, 128)
+#undef CAPPED_CASE
+  abort();
 }

@@ -29,12 +29,12 @@ void launch_paged_prefill_mfma(__hip_bfloat16*, const __hip_bfloat16*,
 void launch_paged_prefill_mfma_v2_capped(__hip_bfloat16*, const __hip_bfloat16*,
                                          const __hip_bfloat16*, const __hip_bfloat16*,
                                          const int*, const int*, const int*, float, int, int,
-                                         int, int, int, int, int, const float*, float,
+                                         int, int, int, int, int, int, int, const float*, float,
                                          hipStream_t);
 void launch_paged_decode_mfma_capped(__hip_bfloat16*, float*, float*, const __hip_bfloat16*,
                                      const __hip_bfloat16*, const __hip_bfloat16*, const int*,
                                      const int*, float, int, int, int, int, int, int, int, int,
-                                     const float*, float, hipStream_t);
+                                     int, const float*, float, hipStream_t);
 int decode_mfma_num_partitions(int nseq, int kvh, int max_context);
 void launch_paged_decode_mfma_fp8(__hip_bfloat16*, float*, float*,
                                   const __hip_bfloat16*, const unsigned char*,
@@ -338,9 +338,30 @@ void windowed_attention_decode(torch::Tensor out, torch::Tensor q,
 }
 
 // Capped variants: scores softcap * tanh(score / softcap) (0: as they are), sinks
-// per head or none; window, sizes and types as for the window variants.
-void check_sinks(const c10::optional<torch::Tensor>& sinks, int64_t heads, double softcap) {
-  TORCH_CHECK(softcap >= 0.0, "softcap");
+// per head or none; window and types as for the window variants, key / value sizes
+// 64/64, 96/64, 128/128 or 192/128.
+void check_capped(const torch::Tensor& out, const torch::Tensor& q,
+                  const torch::Tensor& k_cache, const torch::Tensor& v_cache,
+                  const torch::Tensor& block_tables, const torch::Tensor& seq_lens,
+                  int64_t window, const c10::optional<torch::Tensor>& sinks, double softcap) {
+  TORCH_CHECK(softcap >= 0.0 && window >= 0, "softcap and window");
+  for (const auto* t : {&out, &q, &k_cache, &v_cache})
+    TORCH_CHECK(t->is_cuda() && t->is_contiguous() &&
+                t->scalar_type() == at::ScalarType::BFloat16, "contiguous bf16 tensors");
+  TORCH_CHECK(q.dim() == 3 && out.dim() == 3 && k_cache.dim() == 4 && v_cache.dim() == 4);
+  const int64_t heads = q.size(1), dim = q.size(2), kvh = k_cache.size(2);
+  const int64_t vdim = v_cache.size(3);
+  TORCH_CHECK((dim == 64 && vdim == 64) || (dim == 96 && vdim == 64) ||
+              (dim == 128 && vdim == 128) || (dim == 192 && vdim == 128), "head sizes");
+  TORCH_CHECK(out.size(0) == q.size(0) && out.size(1) == heads && out.size(2) == vdim, "out");
+  TORCH_CHECK(k_cache.size(3) == dim && v_cache.size(0) == k_cache.size(0) &&
+              v_cache.size(1) == k_cache.size(1) && v_cache.size(2) == kvh, "cache shape");
+  TORCH_CHECK(kvh >= 1 && heads % kvh == 0 && heads / kvh <= 8, "at most 8 heads per key head");
+  TORCH_CHECK(seq_lens.is_cuda() && seq_lens.is_contiguous() &&
+              seq_lens.scalar_type() == at::ScalarType::Int);
+  TORCH_CHECK(block_tables.is_cuda() && block_tables.is_contiguous() && block_tables.dim() == 2 &&
+              block_tables.scalar_type() == at::ScalarType::Int &&
+              block_tables.size(0) >= seq_lens.numel(), "block tables");
   if (!sinks.has_value()) return;
   const auto& t = sinks.value();
   TORCH_CHECK(t.is_cuda() && t.is_contiguous() && t.scalar_type() == at::ScalarType::Float &&
@@ -352,9 +373,7 @@ void capped_attention_prefill(torch::Tensor out, torch::Tensor q, torch::Tensor 
                               torch::Tensor query_start_loc, torch::Tensor seq_lens,
                               double scale, int64_t max_query_len, int64_t window,
                               c10::optional<torch::Tensor> sinks, double softcap) {
-  check_windowed(out, q, k_cache, v_cache, block_tables, seq_lens, window);
-  check_sinks(sinks, q.size(1), softcap);
-  TORCH_CHECK(q.size(2) == 128, "prompt portions need key size 128");
+  check_capped(out, q, k_cache, v_cache, block_tables, seq_lens, window, sinks, softcap);
   const int nseq = seq_lens.numel();
   TORCH_CHECK(query_start_loc.is_cuda() && query_start_loc.is_contiguous() &&
               query_start_loc.scalar_type() == at::ScalarType::Int &&
@@ -367,7 +386,7 @@ void capped_attention_prefill(torch::Tensor out, torch::Tensor q, torch::Tensor 
       reinterpret_cast<const __hip_bfloat16*>(v_cache.data_ptr()),
       block_tables.data_ptr<int>(), query_start_loc.data_ptr<int>(),
       seq_lens.data_ptr<int>(), (float)scale, nseq, (int)q.size(1), (int)k_cache.size(2),
-      (int)k_cache.size(1), (int)block_tables.size(1), (int)max_query_len, (int)window,
+      (int)q.size(2), (int)v_cache.size(3), (int)k_cache.size(1), (int)block_tables.size(1), (int)max_query_len, (int)window,
       sinks.has_value() ? sinks.value().data_ptr<float>() : nullptr, (float)softcap,
       current_stream());
 }
@@ -376,10 +395,8 @@ void capped_attention_decode(torch::Tensor out, torch::Tensor q, torch::Tensor k
                              torch::Tensor v_cache, torch::Tensor block_tables,
                              torch::Tensor seq_lens, double scale, int64_t window,
                              c10::optional<torch::Tensor> sinks, double softcap) {
-  check_windowed(out, q, k_cache, v_cache, block_tables, seq_lens, window);
-  check_sinks(sinks, q.size(1), softcap);
-  const int nseq = q.size(0), nheads = q.size(1), head_dim = q.size(2);
-  TORCH_CHECK(head_dim == 64 || head_dim == 128, "key size 64 or 128");
+  check_capped(out, q, k_cache, v_cache, block_tables, seq_lens, window, sinks, softcap);
+  const int nseq = q.size(0), nheads = q.size(1), dim = q.size(2), vdim = v_cache.size(3);
   TORCH_CHECK(seq_lens.numel() == nseq, "one query row per sequence expected");
   if (nseq == 0) return;
   const int kvh = k_cache.size(2), block_size = k_cache.size(1);
@@ -389,7 +406,7 @@ void capped_attention_decode(torch::Tensor out, torch::Tensor q, torch::Tensor k
   const int npart = decode_mfma_num_partitions(nseq, kvh, span);
   const int P = npart * 4;
   auto opts = q.options().dtype(at::ScalarType::Float);
-  auto part_acc = at::empty({nseq, nheads, P, head_dim}, opts);
+  auto part_acc = at::empty({nseq, nheads, P, vdim}, opts);
   auto part_ml = at::empty({nseq, nheads, P, 2}, opts);
   launch_paged_decode_mfma_capped(
       reinterpret_cast<__hip_bfloat16*>(out.data_ptr()), part_acc.data_ptr<float>(),
@@ -397,7 +414,7 @@ void capped_attention_decode(torch::Tensor out, torch::Tensor q, torch::Tensor k
       reinterpret_cast<const __hip_bfloat16*>(k_cache.data_ptr()),
       reinterpret_cast<const __hip_bfloat16*>(v_cache.data_ptr()),
       block_tables.data_ptr<int>(), seq_lens.data_ptr<int>(), (float)scale, nseq, nheads, kvh,
-      head_dim, block_size, max_blocks, npart, (int)window,
+      dim, vdim, block_size, max_blocks, npart, (int)window,
       sinks.has_value() ? sinks.value().data_ptr<float>() : nullptr, (float)softcap,
       current_stream());
 }

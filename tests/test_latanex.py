@@ -261,7 +261,7 @@ def test_delta_rule_replaces_what_a_key_held():
 # -- what a query sees: keys far away, at page borders, just inside and outside --
 
 
-def _spike(window, ctx, at, n_new, device, bs=4, dim=8, dtype=torch.float32, cap=30.0,
+def _spike(window, ctx, at, n_new, device, bs=4, dim=8, vdim=8, dtype=torch.float32, cap=30.0,
            sinks=(-50.0, 9.0)):
     """Two heads over one key head; every key is small noise but the one at
     ``at``, which the last query points at; its value is all 100.  The heads
@@ -269,7 +269,7 @@ def _spike(window, ctx, at, n_new, device, bs=4, dim=8, dtype=torch.float32, cap
     Returns the last query's output through the op and from the definition."""
     g = torch.Generator().manual_seed(ctx * 31 + at)
     k = torch.randn(ctx, 1, dim, generator=g) * 0.05
-    v = torch.randn(ctx, 1, dim, generator=g) * 0.05
+    v = torch.randn(ctx, 1, vdim, generator=g) * 0.05
     q = torch.randn(n_new, 2, dim, generator=g) * 0.05
     direction = torch.ones(dim) / math.sqrt(dim)
     k[at, 0] = 3.0 * direction
@@ -280,13 +280,13 @@ def _spike(window, ctx, at, n_new, device, bs=4, dim=8, dtype=torch.float32, cap
     nb = (ctx + bs - 1) // bs
     table = list(range(nb - 1, -1, -1))
     kc = torch.zeros(nb, bs, 1, dim, dtype=dtype)
-    vc = torch.zeros(nb, bs, 1, dim, dtype=dtype)
+    vc = torch.zeros(nb, bs, 1, vdim, dtype=dtype)
     for p in range(ctx):
         kc[table[p // bs], p % bs] = k[p]
         vc[table[p // bs], p % bs] = v[p]
     dev = lambda t: t.to(device)
     i32 = lambda x: torch.tensor(x, dtype=torch.int32, device=device)
-    out = torch.empty(n_new, 2, dim, dtype=dtype, device=device)
+    out = torch.empty(n_new, 2, vdim, dtype=dtype, device=device)
     kw = dict(out=out, window=window, sinks=dev(sinks), softcap=cap)
     if n_new > 1:
         ops.gqa_attention_prefill(dev(q), dev(kc), dev(vc), i32([table]), i32([0, n_new]),
@@ -321,18 +321,19 @@ def test_edges_and_far_keys(device, n_new, window):
 
 
 @pytest.mark.gpu
-@pytest.mark.parametrize("dim", [64, 128])
+@pytest.mark.parametrize("dim,vdim", [(64, 64), (96, 64), (128, 128), (192, 128)])
 @pytest.mark.parametrize("cap", [30.0, 200.0])      # with and without a running maximum
 @pytest.mark.parametrize("n_new", [1, 5, 300])
 @pytest.mark.parametrize("window", [1, 33, 64, 100, 257, 0])
-def test_edges_and_far_keys_on_matrix_cores(dim, n_new, window, cap):
-    """The same on the bf16 matrix-core kernels (portions: head size 128)."""
+def test_edges_and_far_keys_on_matrix_cores(dim, vdim, n_new, window, cap):
+    """The same on the bf16 matrix-core kernels."""
+    assert ops.capped_attention_uses_matrix_cores(torch.bfloat16, 2, 1, dim, vdim)
     for ctx in (130, 700):
         for at in _edges(window or ctx, ctx) + [63, 64, 127, 128]:
             if at >= ctx:
                 continue
             got, want = _spike(window, ctx, at, min(n_new, ctx), "cuda", bs=16, dim=dim,
-                               dtype=torch.bfloat16, cap=cap)
+                               vdim=vdim, dtype=torch.bfloat16, cap=cap)
             assert float((got - want).abs().max()) < 0.6, f"ctx {ctx} spike at {at}"
 
 
@@ -506,9 +507,10 @@ def test_matrix_core_shapes(tmp_path, dtype):
     layers = [("attention", att_spec(4, 2, 128, 128, size=50, cap=20.0), dense(256)),
               ("delta", delta_spec(4, 2, 64, 128, conv=4),
                routed(8, 2, 4, 2, ff=128, shared=(256, 1.0))),
-              ("attention", att_spec(4, 2, 64, 128, size=37, cap=90.0), None),
+              ("attention", att_spec(4, 2, 192, 128, size=37, cap=90.0), None),
               ("attention", att_spec(2, 2, 128, 128, size=300, cap=5.0), dense(128)),
               ("attention", att_spec(8, 1, 64, 64, size=33, v_mix=False), None),
+              ("attention", att_spec(3, 3, 96, 64, size=70, v_mix=False), None),
               ("delta", delta_spec(2, 2, 128, 32, conv=2), None)]
     cfg = make_config(layers, width=128, vocab=40)
     w = oracle.random_weights(cfg, seed=8)

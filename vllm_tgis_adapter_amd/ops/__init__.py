@@ -801,17 +801,18 @@ def attention_uses_matrix_cores(dtype: torch.dtype, heads: int, kv_heads: int,
 def capped_attention_uses_matrix_cores(dtype: torch.dtype, heads: int, kv_heads: int,
                                        dim: int, vdim: int) -> bool:
     """Shapes the capped (score cap, sinks per head) variants of the MFMA
-    kernels take (prompt portions need size 128, single queries 64 or 128)."""
-    return (dtype == torch.bfloat16 and dim == vdim and dim in (64, 128)
+    kernels take."""
+    return (dtype == torch.bfloat16
+            and (dim, vdim) in ((64, 64), (96, 64), (128, 128), (192, 128))
             and heads % kv_heads == 0 and 1 <= heads // kv_heads <= 8)
 
 
-def _capped_matrix_core_fits(q, k_cache, v_cache, out, single: bool) -> bool:
+def _capped_matrix_core_fits(q, k_cache, v_cache, out) -> bool:
     if _attn_ext() is None or _FORCE_REFERENCE:
         return False
     return (capped_attention_uses_matrix_cores(q.dtype, q.shape[1], k_cache.shape[2],
                                                q.shape[2], v_cache.shape[3])
-            and (single or q.shape[2] == 128) and q.is_contiguous() and out.is_contiguous())
+            and q.is_contiguous() and out.is_contiguous())
 
 
 def _repeat_sink(sink: float | None, q: torch.Tensor) -> torch.Tensor | None:
@@ -840,7 +841,7 @@ def gqa_attention_prefill(q, k_cache, v_cache, block_tables, query_start_loc,
         if sinks is not None or softcap > 0:
             if sinks is None:
                 sinks = _repeat_sink(sink, q)
-            if not general and _capped_matrix_core_fits(q, k_cache, v_cache, out, single=False):
+            if not general and _capped_matrix_core_fits(q, k_cache, v_cache, out):
                 _attn_ext().capped_attention_prefill(
                     out, q, k_cache, v_cache, block_tables, query_start_loc, seq_lens,
                     float(scale), int(max_query_len), int(window), sinks, float(softcap))
@@ -893,7 +894,7 @@ def gqa_attention_decode(q, k_cache, v_cache, block_tables, seq_lens, scale,
         if sinks is not None or softcap > 0:
             if sinks is None:
                 sinks = _repeat_sink(sink, q)
-            if not general and _capped_matrix_core_fits(q, k_cache, v_cache, out, single=True):
+            if not general and _capped_matrix_core_fits(q, k_cache, v_cache, out):
                 _attn_ext().capped_attention_decode(
                     out, q, k_cache, v_cache, block_tables, seq_lens, float(scale),
                     int(window), sinks, float(softcap))
