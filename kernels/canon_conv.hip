@@ -196,53 +196,53 @@ __global__ __launch_bounds__(256) void causal_conv_walk_kernel(
   int s = find_seq(loc, nseq, r0);
   bool fresh = true;             // the history registers do not hold this sequence's rows
   for (int g0 = r0; g0 < r1; g0 += AHEAD) {
-  Vec8<T> now[AHEAD];
+    Vec8<T> now[AHEAD];
 #pragma unroll
-  for (int u = 0; u < AHEAD; ++u) now[u] = nxt[u];
-  if (g0 + AHEAD < r1) fetch(g0 + AHEAD);
+    for (int u = 0; u < AHEAD; ++u) now[u] = nxt[u];
+    if (g0 + AHEAD < r1) fetch(g0 + AHEAD);
 #pragma unroll
-  for (int u = 0; u < AHEAD; ++u) {
-    const int row = g0 + u;
-    if (row >= r1) break;
-    while (s + 1 < nseq && row >= loc[s + 1]) { ++s; fresh = true; }
-    const int slot = slots[s], first = loc[s];
-    const int start = seq_lens[s] - (loc[s + 1] - first);
-    const int p = start + row - first;
-    if (fresh) {
+    for (int u = 0; u < AHEAD; ++u) {
+      const int row = g0 + u;
+      if (row >= r1) break;
+      while (s + 1 < nseq && row >= loc[s + 1]) { ++s; fresh = true; }
+      const int slot = slots[s], first = loc[s];
+      const int start = seq_lens[s] - (loc[s + 1] - first);
+      const int p = start + row - first;
+      if (fresh) {
 #pragma unroll
-      for (int j = 0; j < TAPS - 1; ++j) {
-        const int pj = p - (TAPS - 1) + j;
+        for (int j = 0; j < TAPS - 1; ++j) {
+          const int pj = p - (TAPS - 1) + j;
 #pragma unroll
-        for (int k = 0; k < 8; ++k) hist[j][k] = 0.f;
-        if (pj >= start)
-          Vec8<T>::load(h + (long)(first + pj - start) * in_st + c).unpack(hist[j]);
-        else if (pj >= 0 && slot >= 0)
-          Vec8<T>::load(state + ((long)slot * (TAPS - 1) + pj - start + TAPS - 1) * width + c)
-              .unpack(hist[j]);
+          for (int k = 0; k < 8; ++k) hist[j][k] = 0.f;
+          if (pj >= start)
+            Vec8<T>::load(h + (long)(first + pj - start) * in_st + c).unpack(hist[j]);
+          else if (pj >= 0 && slot >= 0)
+            Vec8<T>::load(state + ((long)slot * (TAPS - 1) + pj - start + TAPS - 1) * width + c)
+                .unpack(hist[j]);
+        }
+        fresh = false;
       }
-      fresh = false;
+      now[u].unpack(hist[TAPS - 1]);
+      float acc[8];
+#pragma unroll
+      for (int k = 0; k < 8; ++k) {
+        acc[k] = bv[k] + (add_input ? hist[TAPS - 1][k] : 0.f);
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j) acc[k] += wv[j][k] * hist[j][k];
+        if (act == 1) acc[k] = acc[k] / (1.0f + __expf(-acc[k]));
+        if (slot < 0) acc[k] = 0.f;           // padding row of a captured bucket
+      }
+      Vec8<T>::store(out + (long)row * width + c, acc);
+      if (single_rows && slot >= 0) {
+        T* st = state + (long)slot * (TAPS - 1) * width + c;
+#pragma unroll
+        for (int j = 0; j < TAPS - 1; ++j) Vec8<T>::store(st + (long)j * width, hist[j + 1]);
+      }
+#pragma unroll
+      for (int j = 0; j + 1 < TAPS; ++j)
+#pragma unroll
+        for (int k = 0; k < 8; ++k) hist[j][k] = hist[j + 1][k];
     }
-    now[u].unpack(hist[TAPS - 1]);
-    float acc[8];
-#pragma unroll
-    for (int k = 0; k < 8; ++k) {
-      acc[k] = bv[k] + (add_input ? hist[TAPS - 1][k] : 0.f);
-#pragma unroll
-      for (int j = 0; j < TAPS; ++j) acc[k] += wv[j][k] * hist[j][k];
-      if (act == 1) acc[k] = acc[k] / (1.0f + __expf(-acc[k]));
-      if (slot < 0) acc[k] = 0.f;           // padding row of a captured bucket
-    }
-    Vec8<T>::store(out + (long)row * width + c, acc);
-    if (single_rows && slot >= 0) {
-      T* st = state + (long)slot * (TAPS - 1) * width + c;
-#pragma unroll
-      for (int j = 0; j < TAPS - 1; ++j) Vec8<T>::store(st + (long)j * width, hist[j + 1]);
-    }
-#pragma unroll
-    for (int j = 0; j + 1 < TAPS; ++j)
-#pragma unroll
-      for (int k = 0; k < 8; ++k) hist[j][k] = hist[j + 1][k];
-  }
   }
 }
 

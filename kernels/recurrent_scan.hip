@@ -218,36 +218,36 @@ __global__ __launch_bounds__(256) void matrix_scan_kernel(ScanArgs a) {
         for (int i = 0; i < NPT; ++i) S[c][i] = alpha * S[c][i] + u[c] * kk[i];
       }
     } else {
-    float dot[VPT], ndot = 0.f;
+      float dot[VPT], ndot = 0.f;
 #pragma unroll
-    for (int c = 0; c < VPT; ++c) dot[c] = 0.f;
+      for (int c = 0; c < VPT; ++c) dot[c] = 0.f;
 #pragma unroll
-    for (int i = 0; i < NPT; ++i) {
-      const float al = KIND == KIND_HGRN2 ? kk[i] : KIND == KIND_GLA ? dd[i < ND ? i : 0] : alpha;
-      const float bk = KIND == KIND_HGRN2 ? 1.0f - kk[i] : KIND == KIND_GLA ? kk[i] : beta * kk[i];
+      for (int i = 0; i < NPT; ++i) {
+        const float al = KIND == KIND_HGRN2 ? kk[i] : KIND == KIND_GLA ? dd[i < ND ? i : 0] : alpha;
+        const float bk = KIND == KIND_HGRN2 ? 1.0f - kk[i] : KIND == KIND_GLA ? kk[i] : beta * kk[i];
+        if (KIND == KIND_MLSTM) {
+          nst[i] = alpha * nst[i] + bk;
+          ndot += nst[i] * qq[i];
+        }
+#pragma unroll
+        for (int c = 0; c < VPT; ++c) {
+          S[c][i] = al * S[c][i] + bk * vj[c];
+          dot[c] += S[c][i] * qq[i];
+        }
+      }
+      float den = 1.f;    // mLSTM: the query scale is applied to the two sums
       if (KIND == KIND_MLSTM) {
-        nst[i] = alpha * nst[i] + bk;
-        ndot += nst[i] * qq[i];
+        ndot = lanes_sum<NSP>(ndot) * a.q_scale;
+        den = a.q_scale / (fmaxf(fabsf(ndot), gt.z) + 1e-6f);
       }
 #pragma unroll
       for (int c = 0; c < VPT; ++c) {
-        S[c][i] = al * S[c][i] + bk * vj[c];
-        dot[c] += S[c][i] * qq[i];
+        const float d = lanes_sum<NSP>(dot[c]);
+        const float yv = KIND == KIND_MLSTM ? d * den
+                         : KIND == KIND_GLA ? d * a.q_scale : d + c2 * vj[c];
+        if (ns == 0 && jbase + c < a.vdim)
+          a.y[row * a.y_st + (long)h * a.vdim + jbase + c] = yv;
       }
-    }
-    float den = 1.f;    // mLSTM: the query scale is applied to the two sums
-    if (KIND == KIND_MLSTM) {
-      ndot = lanes_sum<NSP>(ndot) * a.q_scale;
-      den = a.q_scale / (fmaxf(fabsf(ndot), gt.z) + 1e-6f);
-    }
-#pragma unroll
-    for (int c = 0; c < VPT; ++c) {
-      const float d = lanes_sum<NSP>(dot[c]);
-      const float yv = KIND == KIND_MLSTM ? d * den
-                       : KIND == KIND_GLA ? d * a.q_scale : d + c2 * vj[c];
-      if (ns == 0 && jbase + c < a.vdim)
-        a.y[row * a.y_st + (long)h * a.vdim + jbase + c] = yv;
-    }
     }
     if (more) {
 #pragma unroll
